@@ -32,6 +32,12 @@ InferenceState *inference_state_create_from_ref(const SFTModelRef *model, int ma
  * fp32 copy of the model in host memory: tensor bytes are uploaded as stored and converted on the GPU, and F16 / Q8_0
  * tensors that already have the wanted format are used bit for bit (no dequantise -> requantise). */
 InferenceState *inference_state_create_from_file(const char *path, ModelType model_type, int max_seq_len, int use_fp16);
+/* MODEL_NEVURAX: a decoder whose config.json (beside the weights) lists its layers one by one -- mixer 'delta' or
+ * 'channel_delta' (gated delta rule, one decay per head or per key channel) or 'latent_attention' (sliding window), each
+ * with an optional mixture of experts.  It is created from safetensors files only; use_fp16 is 1 (F16 weights, F16
+ * operands of the products of several rows, everything else fp32) or 2 (weights, products and sums in 32-bit).  It has
+ * no end tokens unless config.json gives eos_token_id (inference_state_load_eos) or the caller sets some, takes no
+ * adapters, and has no training path. */
 
 /* src/nn/fast_inference.h:49 (impl src/nn/fast_inference.c:527-610, owns_weights = 0 at :596-603): the state owns no
  * weights.  It reads the SFT state's own operands in place -- the F16 or Q8_0 tiles of its forward products, embedding
@@ -70,6 +76,12 @@ int inference_generate_batch(InferenceState *state, const uint32_t *prompt_token
  * may be NULL.  pos = 0 starts new sequences; otherwise pos must follow the step before on the same batch_size (a step
  * of this call or the end of inference_generate_batch).  Returns 0, -1 when the arguments do not fit. */
 int inference_step_batch(InferenceState *state, const int *tokens, int batch_size, int pos, float *logits);
+
+/* The next n tokens at the current position, which advances by n, and the logits [n_want][vocab] (host) at the places
+ * want[0 .. n_want) among them, ascending; n_want may be 0.  A prompt may be cut into calls anywhere.  MODEL_NEVURAX runs
+ * them as one step (long prompts: a few), the other models token by token.  No counterpart in the reference.  Returns 0,
+ * -1 when the arguments do not fit. */
+int  inference_forward_tokens(InferenceState *state, const int *tokens, int n, const int *want, int n_want, float *logits);
 
 ModelType inference_state_model_type(InferenceState *state);         /* src/nn/fast_inference.h:31 */
 int  inference_state_vocab_size(InferenceState *state);              /* src/nn/fast_inference.h:34 */

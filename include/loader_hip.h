@@ -48,6 +48,11 @@ float *model_file_load_f32(ModelFile *f, const char *name, size_t *n_elements);
  * (src/nn/wmat.c:19-75) applied to the widened values. */
 WMat *model_file_load_wmat(ModelFile *f, const char *name, int use_fp16);
 
+/* main.c:286-324: which model the config.json inside the directory `path` (or next to the file) describes; Qwen3 when it
+ * says nothing or is absent.  A design that lists its layers is recognised by its "architecture". */
+ModelType model_type_detect(const char *path);
+const char *model_type_name(ModelType model_type);
+
 /* qwen3_load_safetensors / qwen3_load_gguf (src/nn/qwen3.c:211-371) and gemma3_load_safetensors
  * (src/nn/gemma3.c:176-285) up to the point where the model struct is filled: every tensor as fp32, the LM head tied to
  * the embedding when the file has none, Gemma3's norm weights + 1.0 (its RMSNorm is (1 + w) * norm(x)).  Shapes

@@ -10,6 +10,7 @@
 #include "backend.h"
 #include "devutil.h"
 #include "fused.h"
+#include "stack.h"
 #include "../../include/inference_hip.h"
 #include "../../include/loader_hip.h"
 
@@ -28,10 +29,13 @@ extern "C" MetalBuf *sft_get_token_emb_buf(SFTState *s);
 namespace {
 struct BatchRun;
 void batch_release(BatchRun *r);
-// a state on a training state's tiles: one token through the lock-step path with a run of one sequence
-void step_on_tiles(InferenceState *s, int token, int pos);
-const float *logits_on_tiles(InferenceState *s);
-int argmax_on_tiles(InferenceState *s);
+// a state on a training state's tiles, or of a layer-by-layer model: one token through the lock-step path with a run of
+// one sequence
+void step_on_run(InferenceState *s, int token, int pos);
+const float *logits_on_run(InferenceState *s);
+int argmax_on_run(InferenceState *s);
+void prefill_on_run(InferenceState *s, const uint32_t *tokens, int n, int pos);
+int forward_rows(InferenceState *s, const int *tokens, int n, const int *want, int n_want, float *logits);
 }
 
 struct InferenceState {
@@ -56,6 +60,9 @@ struct InferenceState {
     std::vector<BorrowedLayer> borrowed;
     WeightOp borrowed_lm;
     BatchRun *single;
+    // A model that is described layer by layer (stack.h): its configuration and weights; every step goes through a run
+    // here as well.  NULL for the other models.
+    LayerStack *stack;
     std::vector<Layer> layers;
     WMat *lm_head;
     MetalBuf *g_final, *emb;
@@ -374,11 +381,28 @@ int argmax_to_host(InferenceState *s)
     return *s->best_host;
 }
 
+// every step of the state is one of a run (BatchRun), also with a single sequence
+bool steps_on_run(const InferenceState *s) { return s->borrows_tiles || s->stack; }
+
 void default_eos(InferenceState *s)
 {
+    if (s->stack) { s->n_eos = 0; return; }                           // a design without end tokens of its own
     if (s->model_type == MODEL_GEMMA3) { s->eos[0] = 1; s->eos[1] = 106; }            // <eos>, <end_of_turn>
     else { s->eos[0] = 151645; s->eos[1] = 151643; }
     s->n_eos = 2;
+}
+
+// what every state has: sizes, end tokens, the host copies of logits and argmax
+InferenceState *base_state(ModelType mt, int D, int V, int NL, int max_seq, LayerStack *stack = nullptr)
+{
+    InferenceState *s = new InferenceState();
+    s->D = D; s->V = V; s->NL = NL;
+    s->max_seq = max_seq; s->cur_len = 0; s->model_type = mt;
+    s->stack = stack;
+    default_eos(s);
+    HIP_CHECK(hipHostMalloc((void **)&s->logits_host, (size_t)V * 4, hipHostMallocDefault));
+    HIP_CHECK(hipHostMalloc((void **)&s->best_host, sizeof(int), hipHostMallocDefault));
+    return s;
 }
 
 InferenceState *new_state(ModelType mt, int D, int Hq, int Hkv, int hd, int IS, int V, int NL, int max_seq, int use_fp16,
@@ -390,9 +414,8 @@ InferenceState *new_state(ModelType mt, int D, int Hq, int Hkv, int hd, int IS, 
         fast_metal_shutdown();
         return nullptr;
     }
-    InferenceState *s = new InferenceState();
-    s->D = D; s->Hq = Hq; s->Hkv = Hkv; s->hd = hd; s->IS = IS; s->V = V; s->NL = NL;
-    s->max_seq = max_seq; s->cur_len = 0; s->use_fp16 = use_fp16; s->model_type = mt;
+    InferenceState *s = base_state(mt, D, V, NL, max_seq);
+    s->Hq = Hq; s->Hkv = Hkv; s->hd = hd; s->IS = IS; s->use_fp16 = use_fp16;
     s->emb_scale = mt == MODEL_GEMMA3 ? sqrtf((float)D) : 1.0f;
     s->eps = 1e-6f;                                                       // src/nn/fast_inference.c:383
     s->thetas.assign(thetas, thetas + NL);
@@ -408,10 +431,7 @@ InferenceState *new_state(ModelType mt, int D, int Hq, int Hkv, int hd, int IS, 
         s->rope_tabs = metal_buf_create(distinct.size() * per * sizeof(float2));
         for (size_t k = 0; k < distinct.size(); k++) launch_rope_table(dptr_as<float2>(s->rope_tabs) + k * per, max_seq, hd, distinct[k]);
     }
-    default_eos(s);
     const int qd = Hq * hd, kd = Hkv * hd;
-    HIP_CHECK(hipHostMalloc((void **)&s->logits_host, (size_t)V * 4, hipHostMallocDefault));
-    HIP_CHECK(hipHostMalloc((void **)&s->best_host, sizeof(int), hipHostMallocDefault));
     if (matvec_path) {                                                    // scratch and caches of the matrix-vector pipeline
         s->x = fbuf(D); s->x2 = fbuf(D); s->branch = fbuf(D); s->ln = fbuf(D);
         s->qkv = fbuf(qd + 2 * kd); s->att = fbuf(qd);
@@ -501,8 +521,12 @@ InferenceState *inference_state_create_from_ref(const SFTModelRef *m, int max_se
 
 // Straight from the file to HBM: every matrix is uploaded as stored and converted on the GPU (F16 and Q8_0 tensors that
 // already have the wanted format are used bit for bit); Q|K|V and gate|up are joined by device copies of whole rows.
+static InferenceState *stack_state_from_file(const char *path, int max_seq_len, int weight_format);
+
 InferenceState *inference_state_create_from_file(const char *path, ModelType model_type, int max_seq_len, int use_fp16)
 {
+    if (model_type == MODEL_NEVURAX) return stack_state_from_file(path, max_seq_len, use_fp16);
+    if (use_fp16 == 2) { fprintf(stderr, "[FastGen] %s weights are F16 or Q8_0\n", model_type_name(model_type)); return nullptr; }
     ModelFile *f = model_file_open(path);
     if (!f) return nullptr;
     const bool gg = model_file_is_gguf(f);
@@ -584,6 +608,31 @@ InferenceState *inference_state_create_from_file(const char *path, ModelType mod
     return s;
 }
 
+// A model described layer by layer: config.json beside the weights says what the layers are.
+static InferenceState *stack_state_from_file(const char *path, int max_seq_len, int weight_format)
+{
+    if (weight_format != 1 && weight_format != 2) { fprintf(stderr, "[FastGen] Nevurax weights are F16 or 32-bit\n"); return nullptr; }
+    if (max_seq_len <= 0) return nullptr;
+    const std::string cfg_path = config_path_of(path);
+    std::ifstream in(cfg_path);
+    std::stringstream text;
+    if (in) text << in.rdbuf();
+    StackConfig cfg;
+    std::string why;
+    if (!in || !read_stack_config(text.str(), cfg, why)) {
+        fprintf(stderr, "[FastGen] %s: %s\n", cfg_path.c_str(), in ? why.c_str() : "cannot be read");
+        return nullptr;
+    }
+    if (fast_metal_init() != 0) { fprintf(stderr, "[FastGen] no GPU: fast_metal_init failed\n"); return nullptr; }
+    ModelFile *f = model_file_open(path);
+    LayerStack *st = f ? stack_load(f, cfg, weight_format == 2, max_seq_len) : nullptr;
+    model_file_close(f);
+    if (!st) { fast_metal_shutdown(); return nullptr; }
+    InferenceState *s = base_state(MODEL_NEVURAX, cfg.width, cfg.vocab, (int)cfg.layers.size(), max_seq_len, st);
+    s->use_fp16 = weight_format;
+    return s;
+}
+
 InferenceState *inference_state_create_from_sft(SFTState *sft, int max_seq_len)
 {
     InferenceState *s = new_state(sft_get_model_type(sft), sft_get_d_model(sft), sft_get_n_q_heads(sft), sft_get_n_kv_heads(sft),
@@ -614,6 +663,7 @@ void inference_state_refresh_from_sft(InferenceState *s) { (void)s; }
 
 void inference_state_set_lora(InferenceState *s, SFTState *sft)
 {
+    if (s->stack) { fprintf(stderr, "[FastGen] %s takes no adapters\n", model_type_name(s->model_type)); return; }
     const int R = sft_get_lora_rank(sft);
     if (R == 0) return;                                                   // full-parameter state: no adapters
     if (!s->lora_t && !s->borrows_tiles) s->lora_t = fbuf(2 * (size_t)R);
@@ -631,6 +681,7 @@ void inference_state_free(InferenceState *s)
     metal_flush();
     batch_release(s->batch);
     batch_release(s->single);
+    stack_free(s->stack);
     for (MetalBuf *b : {s->gate_v, s->up_v, s->x, s->x2, s->branch, s->ln, s->qkv, s->att, s->gu, s->logits, s->best, s->lora_t, s->rope_tabs})
         metal_buf_free(b);
     for (MetalBuf *b : s->kc) metal_buf_free(b);
@@ -668,17 +719,18 @@ static bool token_ok(InferenceState *s, int token)
 
 static void step_token(InferenceState *s, int token, int pos)
 {
-    if (s->borrows_tiles) step_on_tiles(s, token, pos);
+    if (steps_on_run(s)) step_on_run(s, token, pos);
     else forward_token(s, token, pos);
 }
-static int argmax_host(InferenceState *s) { return s->borrows_tiles ? argmax_on_tiles(s) : argmax_to_host(s); }
+static int argmax_host(InferenceState *s) { return steps_on_run(s) ? argmax_on_run(s) : argmax_to_host(s); }
+static const float *logits_host(InferenceState *s) { return steps_on_run(s) ? logits_on_run(s) : logits_to_host(s); }
 
 const float *inference_forward_token(InferenceState *s, int token)
 {
     if (!token_ok(s, token)) return nullptr;
     step_token(s, token, s->cur_len);
     s->cur_len++;
-    return s->borrows_tiles ? logits_on_tiles(s) : logits_to_host(s);
+    return logits_host(s);
 }
 
 int inference_forward_token_argmax(InferenceState *s, int token)
@@ -689,15 +741,36 @@ int inference_forward_token_argmax(InferenceState *s, int token)
     return argmax_host(s);
 }
 
+// The next n tokens of the sequence from the current position on, and the logits at the places want[0 .. n_want)
+// (ascending) among them.
+int inference_forward_tokens(InferenceState *s, const int *tokens, int n, const int *want, int n_want, float *logits)
+{
+    if (!s || !tokens || n <= 0 || n_want < 0 || (n_want && (!want || !logits))) return -1;
+    if (n > s->max_seq - s->cur_len) { fprintf(stderr, "[FastGen] %d more tokens do not fit %d positions\n", n, s->max_seq); return -1; }
+    for (int i = 0; i < n; i++) if (!token_ok(s, tokens[i])) return -1;
+    for (int i = 0; i < n_want; i++)
+        if (want[i] < 0 || want[i] >= n || (i && want[i] <= want[i - 1])) { fprintf(stderr, "[FastGen] wanted places must ascend inside the portion\n"); return -1; }
+    if (s->stack) return forward_rows(s, tokens, n, want, n_want, logits);
+    for (int i = 0, w = 0; i < n; i++) {                                  // the other models take one token per step
+        step_token(s, tokens[i], s->cur_len);
+        s->cur_len++;
+        if (w < n_want && want[w] == i) memcpy(logits + (size_t)w++ * s->V, logits_host(s), (size_t)s->V * sizeof(float));
+    }
+    metal_flush();
+    return 0;
+}
+
 int inference_generate(InferenceState *s, const uint32_t *prompt_tokens, int prompt_len, uint32_t *output_tokens, int max_gen_len)
 {
     s->cur_len = 0;
     if (prompt_len <= 0 || max_gen_len <= 0 || prompt_len > s->max_seq) return 0;
     for (int i = 0; i < prompt_len; i++) {
         if (!token_ok(s, (int)prompt_tokens[i])) return 0;
+        if (s->stack) continue;                                       // takes the prompt at once, below
         step_token(s, (int)prompt_tokens[i], i);                      // prefill: only the last logits are looked at
         s->cur_len = i + 1;
     }
+    if (s->stack) { prefill_on_run(s, prompt_tokens, prompt_len, 0); s->cur_len = prompt_len; }
     int next = argmax_host(s);
     output_tokens[0] = (uint32_t)next;
     int n_gen = 1;
@@ -748,6 +821,7 @@ __global__ __launch_bounds__(AM_WGS) void k_argmax_final_batch(const float *__re
 
 // Scratch and KV caches of a batch of B sequences decoded in lock step (BatchState of src/nn/fast_inference.c:699-776).
 struct BatchRun {
+    StackRun *stk;                                                       // a layer-by-layer model's caches, states and scratch (then only logits and best besides)
     int B, R, len;                                                       // sequences; adapter rank the scratch was sized for; positions held by the caches
     MetalBuf *x, *ln, *qkv, *att, *act, *logits, *best, *lora_t;
     MetalBuf *a16, *inv_ln, *inv_br, *planes;                            // a product's operand, its factors (of ln | of att and act), its planes
@@ -758,6 +832,7 @@ struct BatchRun {
 void batch_release(BatchRun *r)
 {
     if (!r) return;
+    stack_run_free(r->stk);
     for (MetalBuf *b : {r->x, r->ln, r->qkv, r->att, r->act, r->logits, r->best, r->lora_t, r->a16, r->inv_ln, r->inv_br, r->planes}) metal_buf_free(b);
     for (MetalBuf *b : r->kc) metal_buf_free(b);
     for (MetalBuf *b : r->vc) metal_buf_free(b);
@@ -772,6 +847,11 @@ void batch_release(BatchRun *r)
 // that consumes them and the norm kernel writes the next product's operand itself, where a row is one workgroup's.
 void forward_token_batch(InferenceState *s, BatchRun &r, const int *tokens, int pos)
 {
+    if (s->stack) {
+        stack_forward(s->stack, r.stk, tokens, 1, pos);
+        stack_logits(s->stack, r.stk, nullptr, r.B, dptr_as<float>(r.logits));
+        return;
+    }
     const int D = s->D, Hq = s->Hq, Hkv = s->Hkv, hd = s->hd, IS = s->IS, B = r.B;
     const int qd = Hq * hd, kd = Hkv * hd, nqkv = qd + 2 * kd;
     const bool gemma = s->model_type == MODEL_GEMMA3;
@@ -871,6 +951,14 @@ BatchRun &batch_acquire(InferenceState *s, BatchRun *&slot, int B)
     batch_release(slot);
     slot = new BatchRun{};
     BatchRun &r = *slot;
+    if (s->stack) {
+        r.B = B;
+        r.stk = stack_run_create(s->stack, B);
+        r.logits = fbuf((size_t)std::max(B, STACK_WANT) * s->V);
+        r.best = metal_buf_create(((size_t)B + (size_t)B * 2 * AM_WGS) * sizeof(int));
+        HIP_CHECK(hipHostMalloc((void **)&r.best_host, (size_t)B * sizeof(int), hipHostMallocDefault));
+        return r;
+    }
     const int D = s->D, qd = s->Hq * s->hd, kd = s->Hkv * s->hd, IS = s->IS, V = s->V;
     r.B = B; r.R = R; r.len = 0;
     r.x = fbuf((size_t)B * D); r.ln = fbuf((size_t)B * D);
@@ -902,19 +990,57 @@ BatchRun &batch_acquire(InferenceState *s, BatchRun *&slot, int B)
     return r;
 }
 
-void step_on_tiles(InferenceState *s, int token, int pos)
+void step_on_run(InferenceState *s, int token, int pos)
 {
     BatchRun &r = batch_acquire(s, s->single, 1);
     forward_token_batch(s, r, &token, pos);
     r.len = pos + 1;
 }
-const float *logits_on_tiles(InferenceState *s)
+// A prompt, or a portion of one, for every sequence of the run, in as few steps as its scratch allows; the logits of the
+// last token stay in the run.
+void prefill_rows(InferenceState *s, BatchRun &r, const uint32_t *tokens, int n, int pos)
+{
+    const int portion = stack_portion(r.stk);
+    std::vector<int> ids;
+    for (int at = 0; at < n; at += portion) {
+        const int T = std::min(portion, n - at);
+        ids.resize((size_t)r.B * T);
+        for (int b = 0; b < r.B; b++) for (int t = 0; t < T; t++) ids[(size_t)b * T + t] = (int)tokens[at + t];
+        stack_forward(s->stack, r.stk, ids.data(), T, pos + at);
+    }
+    stack_logits(s->stack, r.stk, nullptr, r.B, dptr_as<float>(r.logits));
+    r.len = pos + n;
+}
+void prefill_on_run(InferenceState *s, const uint32_t *tokens, int n, int pos) { prefill_rows(s, batch_acquire(s, s->single, 1), tokens, n, pos); }
+int forward_rows(InferenceState *s, const int *tokens, int n, const int *want, int n_want, float *logits)
+{
+    BatchRun &r = batch_acquire(s, s->single, 1);
+    const int portion = stack_portion(r.stk);
+    int w = 0;
+    for (int at = 0; at < n; at += portion) {
+        const int T = std::min(portion, n - at);
+        stack_forward(s->stack, r.stk, tokens + at, T, s->cur_len);
+        s->cur_len += T;
+        r.len = s->cur_len;
+        while (w < n_want && want[w] < at + T) {                          // the wanted rows of this step, STACK_WANT at a time
+            int rows[STACK_WANT], k = 0;
+            while (w + k < n_want && k < STACK_WANT && want[w + k] < at + T) { rows[k] = want[w + k] - at; k++; }
+            stack_logits(s->stack, r.stk, rows, k, dptr_as<float>(r.logits));
+            HIP_CHECK(hipMemcpyAsync(logits + (size_t)w * s->V, dptr(r.logits), (size_t)k * s->V * sizeof(float), hipMemcpyDeviceToHost, stream()));
+            HIP_CHECK(hipStreamSynchronize(stream()));
+            w += k;
+        }
+    }
+    HIP_CHECK(hipStreamSynchronize(stream()));
+    return 0;
+}
+const float *logits_on_run(InferenceState *s)
 {
     HIP_CHECK(hipMemcpyAsync(s->logits_host, dptr(s->single->logits), (size_t)s->V * 4, hipMemcpyDeviceToHost, stream()));
     HIP_CHECK(hipStreamSynchronize(stream()));
     return s->logits_host;
 }
-int argmax_on_tiles(InferenceState *s)
+int argmax_on_run(InferenceState *s)
 {
     int best = 0;
     argmax_batch(s, *s->single, &best);
@@ -923,6 +1049,7 @@ int argmax_on_tiles(InferenceState *s)
 
 bool batch_args_ok(InferenceState *s, int B)
 {
+    if (s->stack) return B >= 1 && B <= 32;
     if (!s->use_fp16 && !s->borrows_tiles) { fprintf(stderr, "[BatchGen] F16 weights only\n"); return false; }
     if (B < 1 || B > 32) return false;
     if (s->D > 8192) { fprintf(stderr, "[BatchGen] hidden size %d not supported (<= 8192)\n", s->D); return false; }
@@ -946,7 +1073,8 @@ int inference_generate_batch(InferenceState *s, const uint32_t *prompt_tokens, i
         if (prompt_tokens[i] >= (uint32_t)s->V) { fprintf(stderr, "[BatchGen] token %u outside the vocabulary (%d)\n", prompt_tokens[i], s->V); return 0; }
     BatchRun &r = batch_acquire(s, s->batch, B);
     int tokens[32], next[32], active[32];
-    for (int i = 0; i < prompt_len; i++) {                               // prefill: the same token for every sequence (:910-916)
+    if (s->stack) prefill_rows(s, r, prompt_tokens, prompt_len, 0);
+    else for (int i = 0; i < prompt_len; i++) {                               // prefill: the same token for every sequence (:910-916)
         for (int b = 0; b < B; b++) tokens[b] = (int)prompt_tokens[i];
         forward_token_batch(s, r, tokens, i);
     }
@@ -957,7 +1085,7 @@ int inference_generate_batch(InferenceState *s, const uint32_t *prompt_tokens, i
     for (int gen = 1; gen < max_gen_len && cur_len < s->max_seq; gen++) {
         int any_active = 0;
         for (int b = 0; b < B; b++) {
-            bool ended = next[b] == 0;
+            bool ended = next[b] == 0 && !s->stack;                      // (token 0 is the reference's rule for its models)
             for (int e = 0; e < s->n_eos; e++) ended |= next[b] == s->eos[e];
             if (active[b] && ended) active[b] = 0;
             any_active |= active[b];
@@ -1005,13 +1133,7 @@ void inference_state_set_eos(InferenceState *s, const int *eos_tokens, int n_eos
 // src/nn/fast_inference.c:13-49, 324-342: config.json inside model_path when that is a directory, else next to it
 void inference_state_load_eos(InferenceState *s, const char *model_path)
 {
-    std::string path = model_path ? model_path : "";
-    struct stat st;
-    if (stat(path.c_str(), &st) == 0 && S_ISDIR(st.st_mode)) path += "/config.json";
-    else {
-        const size_t sl = path.rfind('/');
-        path = sl == std::string::npos ? "config.json" : path.substr(0, sl) + "/config.json";
-    }
+    const std::string path = config_path_of(model_path);
     int ids[4], n = 0;
     std::ifstream f(path);
     if (f) {

@@ -3,6 +3,7 @@
 // conversion done on the GPU.  Interface and reference citations: include/loader_hip.h.
 #include "backend.h"
 #include "devutil.h"
+#include "json.h"
 #include "../../include/loader_hip.h"
 
 #include <algorithm>
@@ -88,53 +89,6 @@ size_t bytes_of(int dtype, uint64_t n)
 }
 
 // ---------------------------------------------------------------- safetensors header (JSON)
-
-// A cursor over the header text.  The header is one object: tensor name -> {"dtype", "shape", "data_offsets"}, plus
-// an optional "__metadata__" object of strings.
-struct Json {
-    const char *p, *end;
-    void ws() { while (p < end && (*p == ' ' || *p == '\n' || *p == '\r' || *p == '\t')) p++; }
-    bool eat(char c) { ws(); if (p < end && *p == c) { p++; return true; } return false; }
-    bool string(std::string &out)
-    {
-        ws();
-        if (p >= end || *p != '"') return false;
-        out.clear();
-        for (p++; p < end && *p != '"'; p++) {
-            if (*p == '\\' && p + 1 < end) p++;
-            out.push_back(*p);
-        }
-        if (p >= end) return false;
-        p++;
-        return true;
-    }
-    bool number(uint64_t &v)
-    {
-        ws();
-        if (p >= end || *p < '0' || *p > '9') return false;
-        v = 0;
-        while (p < end && *p >= '0' && *p <= '9') v = v * 10 + (uint64_t)(*p++ - '0');
-        return true;
-    }
-    bool skip()                    // any value
-    {
-        ws();
-        if (p >= end) return false;
-        if (*p == '"') { std::string s; return string(s); }
-        if (*p == '{' || *p == '[') {
-            const char open = *p, close = open == '{' ? '}' : ']';
-            p++;
-            if (eat(close)) return true;
-            do {
-                if (open == '{') { std::string k; if (!string(k) || !eat(':')) return false; }
-                if (!skip()) return false;
-            } while (eat(','));
-            return eat(close);
-        }
-        while (p < end && *p != ',' && *p != '}' && *p != ']') p++;
-        return true;
-    }
-};
 
 bool parse_safetensors_header(const char *text, size_t len, int shard, std::vector<TensorInfo> &out)
 {
@@ -332,6 +286,26 @@ __global__ __launch_bounds__(256) void k_widen16(const uint16_t *__restrict__ sr
     dst[i] = bf16 ? __uint_as_float((uint32_t)h << 16) : (float)__builtin_bit_cast(half_t, h);
 }
 
+// Tensor elements of a raw image as F16 or fp32 into rows of a wider matrix.  An F16 result that is infinite where the
+// value was not sets *overflow.
+__global__ __launch_bounds__(256) void k_place(const void *__restrict__ src, int dtype, int rows, int cols, void *__restrict__ dst, int f32,
+                                               size_t off, int ld, int *overflow)
+{
+    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= (size_t)rows * cols) return;
+    float v;
+    if (dtype == MF_F32) v = ((const float *)src)[i];
+    else {
+        const uint16_t h = ((const uint16_t *)src)[i];
+        v = dtype == MF_BF16 ? __uint_as_float((uint32_t)h << 16) : (float)__builtin_bit_cast(half_t, h);
+    }
+    const size_t o = off + (i / cols) * (size_t)ld + i % cols;
+    if (f32) { ((float *)dst)[o] = v; return; }
+    const half_t h = f2h(v);
+    ((half_t *)dst)[o] = h;
+    if (fabsf((float)h) > 65504.f && fabsf(v) < 3.0e38f) *overflow = 1;
+}
+
 // ---------------------------------------------------------------- model description
 
 struct OwnedRef {
@@ -351,6 +325,35 @@ std::string layer_name(bool gguf, int L, const char *hf, const char *gg)
 }
 
 }  // namespace
+
+namespace lmhip {
+
+// Tensor `name`, which must be [rows, cols] (a vector: 1 x cols), into dst from element elem_off on, rows ld elements
+// apart, as fp32 (f32) or F16.  false, with a message, when it is absent or of another shape or type.
+bool model_file_place(ModelFile *f, const char *name, int rows, int cols, MetalBuf *dst, int f32, size_t elem_off, int ld, int *overflow)
+{
+    const TensorInfo *t = find(f, name);
+    int r = 0, c = 0;
+    if (!t || !model_file_matrix_shape(f, name, &r, &c)) { fprintf(stderr, "[Loader] tensor '%s' not found\n", name); return false; }
+    if (r != rows || c != cols || (t->dtype != MF_F32 && t->dtype != MF_F16 && t->dtype != MF_BF16)) {
+        fprintf(stderr, "[Loader] tensor '%s' is %d x %d, expected %d x %d (F32, F16 or BF16)\n", name, r, c, rows, cols);
+        return false;
+    }
+    const size_t n = (size_t)rows * cols;
+    if (n == 0 || (elem_off + (size_t)(rows - 1) * ld + cols) * (f32 ? 4 : 2) > dst->size || ld < cols) {
+        fprintf(stderr, "[Loader] tensor '%s' does not fit its place\n", name);
+        return false;
+    }
+    MetalBuf *raw = metal_buf_from_data(bytes(f, t), t->nbytes);
+    hipLaunchKernelGGL(k_place, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, stream(), dptr(raw), t->dtype, rows, cols, dptr(dst), f32,
+                       elem_off, ld, overflow);
+    HIP_CHECK(hipGetLastError());
+    mark_written(dst);
+    metal_buf_free(raw);                                      // synchronises the stream first
+    return true;
+}
+
+}  // namespace lmhip
 
 extern "C" {
 

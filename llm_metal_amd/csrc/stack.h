@@ -1,0 +1,192 @@
+// A decoder described layer by layer: every layer names its mixer (gated delta rule with one decay per head or per key
+// channel, latent attention) and its feed-forward (mixture of experts, or none), both fed by one norm.  This header is
+// the configuration, the weights as the kernels read them, what a sequence keeps between steps, and the launches.
+// The steps themselves are driven by the generation state (inference.hip) like those of the other models.
+#pragma once
+#include "backend.h"
+#include "devutil.h"
+#include "gemm.h"
+#include "../../include/loader_hip.h"
+#include <string>
+#include <vector>
+
+namespace lmhip {
+
+// ---------------------------------------------------------------- configuration (config.json)
+
+enum MixerKind { MIX_DELTA, MIX_CHANNEL_DELTA, MIX_LATENT };
+
+struct LayerConfig {
+    int mixer = MIX_DELTA;
+    int heads = 0, dim = 0, vdim = 0;
+    int kv_heads = 0, taps = 0;                          // delta rule
+    int rot_dim = 0, kv_rank = 0, window = 0, rot_dims = 0;   // latent attention; rot_dims: how many of the rot_dim turn
+    double rot_base = 0.0;
+    float scale = 0.f;
+    int experts = 0, top = 0, ff = 0, shared_ff = 0;     // experts == 0: no feed-forward; shared_ff == 0: no shared expert
+};
+
+struct StackConfig {
+    int vocab = 0, width = 0;
+    float emb_scale = 1.f, eps = 0.f;
+    std::vector<LayerConfig> layers;
+};
+
+// config.json inside `path` when that is a directory, else next to it
+std::string config_path_of(const char *path);
+// false, with the reason in `why`, when the text is not a description this build can run
+bool read_stack_config(const std::string &json_text, StackConfig &out, std::string &why);
+
+// ---------------------------------------------------------------- weights
+
+// Row-major weight matrix, F16 or fp32 by the state's precision; columns padded with zeros to a multiple of 8, so that
+// every row starts on 16 bytes and the padded entries of the vectors (zero too) add nothing.
+struct StackMat {
+    MetalBuf *buf = nullptr;
+    int rows = 0, cols = 0;
+};
+inline int pad8(int n) { return (n + 7) & ~7; }
+
+struct StackLayer {
+    LayerConfig c;
+    MetalBuf *g_norm = nullptr;                          // [width padded]
+    // One product serves everything that reads the normed vector; each part starts at a multiple of four rows.
+    //   delta: q | k | v | b | a (or a1) | g (or g1);  latent: q | dkv;  then router | shared up
+    StackMat in;
+    int o_q = 0, o_k = 0, o_v = 0, o_b = 0, o_a = 0, o_g = 0, o_dkv = 0, o_router = 0, o_shared = 0;
+    int rank_a = 0, rank_g = 0;                          // per-channel decay: widths of the two low-rank products
+    // One product for everything added to the residual by the dense part: columns [mixer output | shared activation]
+    StackMat out;
+    int hv = 0, o_sh = 0;                                // width of the mixer output; column where the shared activation starts
+    MetalBuf *conv = nullptr, *a_exp = nullptr, *dt_bias = nullptr, *g_out = nullptr;   // fp32: filters [channels][taps], exp(A_log), bias, head norm
+    StackMat a2, g2;
+    MetalBuf *g_c = nullptr, *rope = nullptr;            // latent norm weight; (cos, sin) [max_seq][rot_dims / 2]
+    StackMat uk, uv;                                     // [heads * dim, rank], [heads * vdim, rank]
+    StackMat up, down;                                   // experts one after the other: [E * ff, width], [E * width, ff]
+    int channels() const { return 2 * c.kv_heads * c.dim + c.heads * c.vdim; }
+    bool delta() const { return c.mixer != MIX_LATENT; }
+};
+
+struct LayerStack {
+    StackConfig cfg;
+    int f32 = 0;                                         // weights and products in 32-bit; else F16 weights
+    int D = 0, Dp = 0, V = 0, max_seq = 0;
+    std::vector<StackLayer> layers;
+    StackMat head;
+    MetalBuf *g_final = nullptr, *emb = nullptr;         // emb: fp32 [V][D]
+    std::vector<MetalBuf *> ropes;                       // the distinct rotation tables
+};
+
+// NULL, with a message, when a tensor is missing or mis-shaped or the weights do not fit F16
+LayerStack *stack_load(ModelFile *f, const StackConfig &cfg, int f32, int max_seq);
+void stack_free(LayerStack *st);
+
+// ---------------------------------------------------------------- what sequences keep, and a run's scratch
+
+struct StackRun {
+    int B = 0, rows = 0;                                 // sequences; token rows the scratch holds
+    // per layer.  delta: state [B][heads][vdim][dim] and the last `taps` inputs of the convolutions [B][taps][channels];
+    // latent: ring of (latent | rotated key) rows [B][ring][row width].  Row of position p: p % taps, p % ring.
+    // Nothing is cleared between sequences: what lies before position 0 is never read.
+    struct Layer { MetalBuf *S = nullptr, *conv = nullptr, *ring = nullptr; int ring_rows = 0; };
+    std::vector<Layer> layers;
+    MetalBuf *tok = nullptr, *want = nullptr;
+    int *tok_host = nullptr, *want_host = nullptr;       // pinned; tok_host [B * max_seq], each portion in its own place
+    MetalBuf *x = nullptr, *h = nullptr, *cin = nullptr, *cat = nullptr, *cout = nullptr;
+    MetalBuf *a16 = nullptr, *inv = nullptr;             // F16 operand of a product and its row factors
+    MetalBuf *aux = nullptr;                             // the mixer's intermediates
+    MetalBuf *route_idx = nullptr, *route_w = nullptr, *act = nullptr, *ymoe = nullptr;
+    MetalBuf *moe = nullptr;                             // grouped experts: tables, operands and results
+    int T = 0, pending = 0;                              // tokens per sequence of the last step; its last layer's sum still waits in cout (1) and ymoe (2)
+};
+StackRun *stack_run_create(const LayerStack *st, int B);
+void stack_run_free(StackRun *r);
+// most tokens per sequence that one call of stack_forward takes
+int stack_portion(const StackRun *r);
+
+// One step: T tokens of each of the run's sequences, tokens[b * T + t] entering sequence b at position pos + t (a host
+// array).  A sequence begins at pos 0; any other pos continues where the run's steps before it ended.
+void stack_forward(LayerStack *st, StackRun *r, const int *tokens, int T, int pos);
+// Logits of rows of the last step (b * T + t) into logits [n][V] on the device: the rows listed in `want` (host array, at
+// most STACK_WANT of them; the stream must be synchronised before the next call), or with NULL the last token of each
+// sequence.
+constexpr int STACK_WANT = 64;
+void stack_logits(LayerStack *st, StackRun *r, const int *want, int n, float *logits);
+
+// ---------------------------------------------------------------- launches (rows: B * T tokens, row m = b * T + t)
+
+struct Rows { int B, T, pos; int n() const { return B * T; } };
+
+// norm.hip: x[src] += cout[src] + ymoe[src] (either may be null), kept in x when `keep`; then layer norm with weight g,
+// written as the tiled F16 operand a16 with its row factors inv (when a16) and / or as fp32 h [rows][Dp] (when h).
+// src = want[m] when `want`, else m * step + first.
+struct NormRows {
+    float *x; const float *cout, *ymoe;
+    const float *g; half_t *a16; float *inv, *h;
+    const int *want;
+    int step, first, D, Dp, keep; float eps;
+    // grouped experts: instead of ymoe the sum over s of route_w[row][s] * moe_y[moe_pos[row][s]]
+    const float *moe_y, *route_w; const int *moe_pos; int top;
+};
+void launch_norm_rows(const NormRows &a, int rows);
+void launch_embed_rows(const float *emb, const int *tok, float scale, float *x, int D, int Dp, int rows);
+
+// gemm_f32.hip: C[m][n] = sum_k A[m][k] W[n][k], fp32 throughout
+void launch_gemm_f32(const float *A, int lda, const float *W, int ldw, float *C, int ldc, int M, int N, int K);
+
+// delta.hip
+struct DeltaRows {
+    Rows r;
+    int H, KV, dim, vdim, taps, per_channel;
+    const float *cin; int ldc, o_q, o_k, o_v, o_b, o_a;  // the input product
+    const float *filters, *a_exp, *dt_bias;
+    float *conv, *S;                                     // state
+    float *q, *k, *v, *kq, *beta, *g;                    // intermediates: [rows][KV][dim] x 2, [rows][H][vdim], [rows][KV], [rows][H], [rows][H] or [rows][H][dim]
+    const float *a2;                                     // per channel: W_a2 (W_a1 h) [rows][H * dim]
+    float *o;                                            // [rows][H][vdim]
+};
+void launch_delta_inputs(const DeltaRows &a);            // convolutions, unit norms, step sizes, decays
+void launch_delta_scan(const DeltaRows &a);              // the recurrence; also moves the convolution's last inputs into the state
+
+// The operand of the output product: mixer output (head norm and gate applied when g_out) | squared-ReLU of the shared
+// up product, as fp32 cat [rows][ldk] and / or as a16 with inv
+struct CatRows {
+    const float *o; int H, vdim;                         // mixer output [rows][H * vdim]
+    const float *g_out, *gate; int ld_gate, gate_silu; float eps;   // head norm weight, gate rows (silu or sigmoid)
+    const float *shared; int ld_shared, shared_ff, o_sh; // shared up rows
+    float *cat; half_t *a16; float *inv; int ldk;
+};
+void launch_cat_rows(const CatRows &a, int rows);
+
+// latent.hip
+struct LatentRows {
+    Rows r;
+    int H, dim, rot, vdim, rank, window, ring_rows, rot_dims;
+    float scale, eps;
+    const float *cin; int ldc, o_q, o_dkv;
+    const float *g_c; const float2 *rope;
+    float *ring;                                         // [B][ring_rows][w], w = both parts padded to 8
+    float *q;                                            // absorbed query [rows][H][w]
+    float *part_o, *part_ml;                             // slices (scratch of the launch)
+    float *o;                                            // [rows][H * vdim]
+    int f32; const void *uk, *uv; int ldu;               // weights and their row stride
+};
+void launch_latent_cache(const LatentRows &a);           // latent norm and key rotation into the ring
+void launch_latent_attend(const LatentRows &a);          // any number of rows, over the latents themselves
+
+void launch_rope_interleaved(float2 *tab, int max_seq, int dims, double base);
+
+// moe.hip
+struct MoeRows {
+    int rows, E, top, ff, ffp, D, Dp, f32;
+    const float *z; int ldz;                             // router logits
+    int *idx; float *w;                                  // [rows][top]
+    const float *h;                                      // [rows][Dp]
+    const void *up, *down;
+    float *act;                                          // [rows][top][ffp]
+    float *y;                                            // [rows][Dp]
+};
+void launch_route(const MoeRows &a);
+void launch_experts_per_row(const MoeRows &a);           // each row reads its own experts
+
+}  // namespace lmhip

@@ -1,0 +1,446 @@
+// A layer-by-layer model on the device: weights from the checkpoint into the matrices of stack.h, what the sequences of
+// a run keep, and one step over any number of tokens.  The generation state (inference.hip) owns both and drives them.
+#include "stack.h"
+#include "rows.h"
+
+#include <algorithm>
+#include <math.h>
+#include <string.h>
+
+namespace lmhip {
+
+// loader.hip
+bool model_file_place(ModelFile *f, const char *name, int rows, int cols, MetalBuf *dst, int f32, size_t elem_off, int ld, int *overflow);
+
+namespace {
+
+MetalBuf *fbuf(size_t n) { return metal_buf_create(n * sizeof(float)); }
+MetalBuf *zeroed(size_t bytes)
+{
+    MetalBuf *b = metal_buf_create(bytes);
+    HIP_CHECK(hipMemsetAsync(dptr(b), 0, bytes, stream()));
+    return b;
+}
+int pad4(int n) { return (n + 3) & ~3; }
+
+// ---------------------------------------------------------------- loading
+
+struct Loading {
+    ModelFile *f;
+    LayerStack *st;
+    MetalBuf *overflow;                                   // set by a weight that F16 cannot hold
+    bool ok = true;
+
+    size_t esize() const { return st->f32 ? 4 : 2; }
+    bool shape(const std::string &name, int *rows, int *cols)
+    {
+        if (model_file_matrix_shape(f, name.c_str(), rows, cols)) return true;
+        fprintf(stderr, "[FastGen] tensor '%s' not found or not a matrix\n", name.c_str());
+        return ok = false;
+    }
+    StackMat matrix(int rows, int cols)
+    {
+        StackMat m;
+        m.rows = rows; m.cols = pad8(cols);
+        m.buf = zeroed((size_t)m.rows * m.cols * esize());
+        return m;
+    }
+    // tensor [rows, cols] into rows row0 .. of a matrix, its columns from col0 on
+    void place(const std::string &name, int rows, int cols, StackMat &m, int row0 = 0, int col0 = 0)
+    {
+        if (!ok) return;
+        ok = model_file_place(f, name.c_str(), rows, cols, m.buf, st->f32, (size_t)row0 * m.cols + col0, m.cols, dptr_as<int>(overflow));
+    }
+    // fp32 vector (a matrix is taken row by row), padded with zeros
+    MetalBuf *vector(const std::string &name, size_t n, size_t padded = 0)
+    {
+        size_t got = 0;
+        float *v = ok ? model_file_load_f32(f, name.c_str(), &got) : nullptr;
+        if (!v || got != n) {
+            if (ok) fprintf(stderr, "[FastGen] tensor '%s': %zu elements, expected %zu\n", name.c_str(), got, n);
+            free(v);
+            ok = false;
+            return nullptr;
+        }
+        std::vector<float> p(std::max(n, padded), 0.f);
+        memcpy(p.data(), v, n * sizeof(float));
+        free(v);
+        return metal_buf_from_data(p.data(), p.size() * sizeof(float));
+    }
+};
+
+void load_delta(Loading &ld, StackLayer &L, const std::string &p, int rows_before)
+{
+    const LayerConfig &c = L.c;
+    const int D = ld.st->D, qd = c.kv_heads * c.dim, vd = c.heads * c.vdim;
+    const bool pc = c.mixer == MIX_CHANNEL_DELTA;
+    ld.place(p + "q", qd, D, L.in, L.o_q); ld.place(p + "k", qd, D, L.in, L.o_k); ld.place(p + "v", vd, D, L.in, L.o_v);
+    ld.place(p + "b", c.heads, D, L.in, L.o_b);
+    ld.place(p + (pc ? "a1" : "a"), pc ? L.rank_a : c.heads, D, L.in, L.o_a);
+    ld.place(p + (pc ? "g1" : "g"), pc ? L.rank_g : vd, D, L.in, L.o_g);
+    (void)rows_before;
+    if (pc) {
+        L.a2 = ld.matrix(c.heads * c.dim, L.rank_a); ld.place(p + "a2", c.heads * c.dim, L.rank_a, L.a2);
+        L.g2 = ld.matrix(vd, L.rank_g); ld.place(p + "g2", vd, L.rank_g, L.g2);
+    }
+    L.conv = fbuf((size_t)L.channels() * c.taps);
+    int at = 0;
+    const char *names[3] = {"q.conv", "k.conv", "v.conv"};
+    const int chans[3] = {qd, qd, vd};
+    for (int i = 0; i < 3 && ld.ok; i++) {
+        size_t n = 0;
+        float *w = model_file_load_f32(ld.f, (p + names[i]).c_str(), &n);
+        if (!w || n != (size_t)chans[i] * c.taps) { fprintf(stderr, "[FastGen] tensor '%s%s' is missing or mis-shaped\n", p.c_str(), names[i]); ld.ok = false; }
+        else metal_buf_write(L.conv, (size_t)at * c.taps * sizeof(float), w, n * sizeof(float));
+        free(w);
+        at += chans[i];
+    }
+    L.a_exp = ld.vector(p + "A_log", c.heads);
+    if (L.a_exp) {
+        std::vector<float> a(c.heads);
+        metal_buf_read(L.a_exp, 0, a.data(), a.size() * sizeof(float));
+        for (float &v : a) v = (float)exp((double)v);
+        metal_buf_write(L.a_exp, 0, a.data(), a.size() * sizeof(float));
+    }
+    L.dt_bias = ld.vector(p + "dt_bias", pc ? (size_t)c.heads * c.dim : c.heads);
+    L.g_out = ld.vector(p + "norm", c.vdim);
+}
+
+void load_latent(Loading &ld, StackLayer &L, const std::string &p)
+{
+    const LayerConfig &c = L.c;
+    const int D = ld.st->D;
+    ld.place(p + "q", c.heads * (c.dim + c.rot_dim), D, L.in, L.o_q);
+    ld.place(p + "dkv", c.kv_rank + c.rot_dim, D, L.in, L.o_dkv);
+    L.g_c = ld.vector(p + "dkv.norm", c.kv_rank);
+    L.uk = ld.matrix(c.heads * c.dim, c.kv_rank); ld.place(p + "uk", c.heads * c.dim, c.kv_rank, L.uk);
+    L.uv = ld.matrix(c.heads * c.vdim, c.kv_rank); ld.place(p + "uv", c.heads * c.vdim, c.kv_rank, L.uv);
+}
+
+void load_layer(Loading &ld, StackLayer &L, int i)
+{
+    const LayerConfig &c = L.c;
+    const int D = ld.st->D;
+    const std::string p = "l" + std::to_string(i) + ".", mix = p + "mix.", mlp = p + "mlp.";
+    L.g_norm = ld.vector(p + "norm1", D, ld.st->Dp);
+    // the parts of the input product
+    int at = 0, cols = 0;
+    auto part = [&](int &o, int n) { o = at; at = pad4(at + n); };
+    if (L.delta()) {
+        const int qd = c.kv_heads * c.dim, vd = c.heads * c.vdim;
+        const bool pc = c.mixer == MIX_CHANNEL_DELTA;
+        if (pc && (!ld.shape(mix + "a1", &L.rank_a, &cols) || !ld.shape(mix + "g1", &L.rank_g, &cols))) return;
+        part(L.o_q, qd); part(L.o_k, qd); part(L.o_v, vd); part(L.o_b, c.heads);
+        part(L.o_a, pc ? pad8(L.rank_a) : c.heads);       // read as rows of pad8 columns by the second low-rank product
+        part(L.o_g, pc ? pad8(L.rank_g) : vd);
+    } else {
+        part(L.o_q, c.heads * (c.dim + c.rot_dim)); part(L.o_dkv, c.kv_rank + c.rot_dim);
+    }
+    if (c.experts) { part(L.o_router, c.experts); if (c.shared_ff) part(L.o_shared, c.shared_ff); }
+    L.in = ld.matrix(at, D);
+    L.hv = c.heads * c.vdim;
+    L.o_sh = pad8(L.hv);
+    L.out = ld.matrix(ld.st->Dp, L.o_sh + c.shared_ff);
+    if (L.delta()) load_delta(ld, L, mix, 0); else load_latent(ld, L, mix);
+    ld.place(mix + "o", D, L.hv, L.out);
+    if (!c.experts) return;
+    ld.place(mlp + "router", c.experts, D, L.in, L.o_router);
+    if (c.shared_ff) {
+        ld.place(mlp + "shared.up", c.shared_ff, D, L.in, L.o_shared);
+        ld.place(mlp + "shared.down", D, c.shared_ff, L.out, 0, L.o_sh);
+    }
+    L.up = ld.matrix(c.experts * c.ff, D);
+    L.down = ld.matrix(c.experts * D, c.ff);
+    for (int e = 0; e < c.experts && ld.ok; e++) {
+        const std::string ex = mlp + "e" + std::to_string(e) + ".";
+        ld.place(ex + "up", c.ff, D, L.up, e * c.ff);
+        ld.place(ex + "down", D, c.ff, L.down, e * D);
+    }
+}
+
+}  // namespace
+
+LayerStack *stack_load(ModelFile *f, const StackConfig &cfg, int f32, int max_seq)
+{
+    LayerStack *st = new LayerStack();
+    st->cfg = cfg; st->f32 = f32; st->D = cfg.width; st->Dp = pad8(cfg.width); st->V = cfg.vocab; st->max_seq = max_seq;
+    Loading ld{f, st, zeroed(sizeof(int))};
+    std::vector<std::pair<double, int>> tables;           // (base, dims) of st->ropes
+    st->layers.resize(cfg.layers.size());
+    for (size_t i = 0; i < st->layers.size() && ld.ok; i++) {
+        StackLayer &L = st->layers[i];
+        L.c = cfg.layers[i];
+        load_layer(ld, L, (int)i);
+        if (L.delta() || !ld.ok) continue;
+        size_t k = 0;
+        while (k < tables.size() && tables[k] != std::make_pair(L.c.rot_base, L.c.rot_dims)) k++;
+        if (k == tables.size()) {
+            tables.emplace_back(L.c.rot_base, L.c.rot_dims);
+            st->ropes.push_back(metal_buf_create(std::max<size_t>(8, (size_t)max_seq * (L.c.rot_dims / 2) * sizeof(float2))));
+            launch_rope_interleaved(dptr_as<float2>(st->ropes[k]), max_seq, L.c.rot_dims, L.c.rot_base);
+        }
+        L.rope = st->ropes[k];
+    }
+    if (ld.ok) {
+        st->g_final = ld.vector("final.norm", st->D, st->Dp);
+        st->head = ld.matrix(st->V, st->D);
+        ld.place("head", st->V, st->D, st->head);
+        st->emb = fbuf((size_t)st->V * st->D);
+        if (ld.ok) ld.ok = model_file_place(f, "embed", st->V, st->D, st->emb, 1, 0, st->D, nullptr);
+    }
+    int over = 0;
+    if (ld.ok) metal_buf_read(ld.overflow, 0, &over, sizeof over);
+    metal_buf_free(ld.overflow);
+    if (over) { fprintf(stderr, "[FastGen] a weight lies outside the F16 range; load the model in 32-bit precision\n"); ld.ok = false; }
+    if (!ld.ok) { stack_free(st); return nullptr; }
+    return st;
+}
+
+void stack_free(LayerStack *st)
+{
+    if (!st) return;
+    for (StackLayer &L : st->layers)
+        for (MetalBuf *b : {L.g_norm, L.in.buf, L.out.buf, L.conv, L.a_exp, L.dt_bias, L.g_out, L.a2.buf, L.g2.buf, L.g_c, L.uk.buf, L.uv.buf,
+                            L.up.buf, L.down.buf}) metal_buf_free(b);
+    for (MetalBuf *b : st->ropes) metal_buf_free(b);
+    for (MetalBuf *b : {st->head.buf, st->g_final, st->emb}) metal_buf_free(b);
+    delete st;
+}
+
+// ---------------------------------------------------------------- runs
+
+namespace {
+
+constexpr int PORTION_ROWS = 2048;
+
+// floats of a layer's intermediates for `rows` rows, in the order the step hands them out (each piece a multiple of 4)
+struct Aux {
+    float *base = nullptr;
+    size_t at = 0;
+    float *take(size_t n) { float *p = base ? base + at : nullptr; at += (n + 3) & ~(size_t)3; return p; }
+};
+
+struct DeltaAux { float *q, *k, *v, *kq, *beta, *g, *a2, *g2, *o; };
+DeltaAux delta_aux(Aux &x, const LayerConfig &c, size_t rows)
+{
+    const bool pc = c.mixer == MIX_CHANNEL_DELTA;
+    DeltaAux d{};
+    d.q = x.take(rows * c.kv_heads * c.dim); d.k = x.take(rows * c.kv_heads * c.dim); d.v = x.take(rows * c.heads * c.vdim);
+    d.kq = x.take(rows * c.kv_heads); d.beta = x.take(rows * c.heads);
+    d.g = x.take(rows * c.heads * (pc ? c.dim : 1));
+    d.a2 = x.take(pc ? rows * c.heads * c.dim : 0); d.g2 = x.take(pc ? rows * c.heads * c.vdim : 0);
+    d.o = x.take(rows * c.heads * c.vdim);
+    return d;
+}
+
+struct LatentAux { float *q, *o; };
+LatentAux latent_aux(Aux &x, const LayerConfig &c, size_t rows)
+{
+    LatentAux d{};
+    d.q = x.take(rows * c.heads * (pad8(c.kv_rank) + pad8(c.rot_dim)));
+    d.o = x.take(rows * c.heads * c.vdim);
+    return d;
+}
+
+// C [M][w.rows] = A x w^T; A as the run's F16 operand (a16, inv) or, in 32-bit, as fp32 rows
+void product(const LayerStack *st, const StackMat &w, const half_t *a16, const float *inv, const float *A, int lda, float *C, int M)
+{
+    const int N = w.rows, K = w.cols;
+    if (st->f32) { launch_gemm_f32(A, lda, dptr_as<float>(w.buf), K, C, N, M, N, K); return; }
+    const WeightOp op = weight_f16(tiled_weight_of(w.buf, N, K));
+    const size_t plane = (size_t)M * N;
+    if (use_big_gemm(M, N, K, 0)) {
+        const int chunks = big_gemm_chunks(M, N, K, 0);
+        if (chunks == 1) { launch_gemm_big(a16, inv, op, C, N, M, N, K); return; }
+        float *P = (float *)scratch(SCR_PARTIAL, plane * chunks * sizeof(float));
+        const int S = launch_gemm_big(a16, nullptr, op, P, N, M, N, K, chunks, plane);
+        launch_reduce_planes(P, S, plane, N, inv, C, M, N);
+        return;
+    }
+    const GemmPlan p = plan_gemm(M, N, K);
+    if (p.S == 1) { launch_gemm(a16, inv, op, C, N, 0, M, N, K, p); return; }
+    float *P = (float *)scratch(SCR_PARTIAL, plane * p.S * sizeof(float));
+    launch_gemm(a16, nullptr, op, P, N, plane, M, N, K, p);
+    launch_reduce_planes(P, p.S, plane, N, inv, C, M, N);
+}
+
+}  // namespace
+
+StackRun *stack_run_create(const LayerStack *st, int B)
+{
+    StackRun *r = new StackRun();
+    r->B = B;
+    r->rows = std::max(1, std::min(PORTION_ROWS / B, st->max_seq)) * B;
+    const int portion = r->rows / B;
+    size_t n_in = 0, ko = 0, aux = 0, act = 0, top = 0;
+    int kmax = st->Dp;
+    bool moe = false;
+    for (const StackLayer &L : st->layers) {
+        const LayerConfig &c = L.c;
+        StackRun::Layer k;
+        Aux a;
+        if (L.delta()) {
+            k.S = fbuf((size_t)B * c.heads * c.vdim * c.dim);
+            k.conv = fbuf((size_t)B * c.taps * L.channels());
+            delta_aux(a, c, r->rows);
+            kmax = std::max({kmax, L.a2.cols, L.g2.cols});
+        } else {
+            k.ring_rows = std::min(st->max_seq, c.window - 1 + portion);
+            k.ring = fbuf((size_t)B * k.ring_rows * (pad8(c.kv_rank) + pad8(c.rot_dim)));
+            latent_aux(a, c, r->rows);
+        }
+        r->layers.push_back(k);
+        n_in = std::max<size_t>(n_in, L.in.rows); ko = std::max<size_t>(ko, L.out.cols); aux = std::max(aux, a.at);
+        if (c.experts) { moe = true; top = std::max<size_t>(top, c.top); act = std::max<size_t>(act, (size_t)c.top * pad8(c.ff)); }
+    }
+    kmax = std::max<int>(kmax, (int)ko);
+    r->tok = metal_buf_create((size_t)r->rows * sizeof(int));
+    r->want = metal_buf_create(STACK_WANT * sizeof(int));
+    HIP_CHECK(hipHostMalloc((void **)&r->tok_host, (size_t)B * st->max_seq * sizeof(int), hipHostMallocDefault));
+    HIP_CHECK(hipHostMalloc((void **)&r->want_host, STACK_WANT * sizeof(int), hipHostMallocDefault));
+    r->x = fbuf((size_t)r->rows * st->Dp);
+    r->cin = fbuf((size_t)r->rows * n_in);
+    r->cout = fbuf((size_t)r->rows * st->Dp);
+    r->aux = fbuf(aux);
+    r->h = fbuf((size_t)std::max(r->rows, STACK_WANT) * st->Dp);
+    if (st->f32) r->cat = fbuf((size_t)r->rows * ko);
+    else {
+        r->a16 = metal_buf_create(tiled_elems(std::max(r->rows, STACK_WANT), kmax) * sizeof(half_t));
+        r->inv = fbuf(std::max(r->rows, STACK_WANT));
+    }
+    if (moe) {
+        r->route_idx = metal_buf_create((size_t)r->rows * top * sizeof(int));
+        r->route_w = fbuf((size_t)r->rows * top);
+        r->act = fbuf((size_t)r->rows * act);
+        r->ymoe = fbuf((size_t)r->rows * st->Dp);
+    }
+    return r;
+}
+
+void stack_run_free(StackRun *r)
+{
+    if (!r) return;
+    for (StackRun::Layer &k : r->layers) for (MetalBuf *b : {k.S, k.conv, k.ring}) metal_buf_free(b);
+    for (MetalBuf *b : {r->tok, r->want, r->x, r->h, r->cin, r->cat, r->cout, r->a16, r->inv, r->aux, r->route_idx, r->route_w, r->act, r->ymoe, r->moe})
+        metal_buf_free(b);
+    if (r->tok_host) hipHostFree(r->tok_host);
+    if (r->want_host) hipHostFree(r->want_host);
+    delete r;
+}
+
+int stack_portion(const StackRun *r) { return r->rows / r->B; }
+
+// ---------------------------------------------------------------- the step
+
+namespace {
+
+template <typename T> T *ptr(MetalBuf *b) { return b ? dptr_as<T>(b) : nullptr; }
+
+// the norm ahead of a product over all rows of the step (or, with want / step, some of them), the pending sum added first
+void norm(LayerStack *st, StackRun *r, MetalBuf *g, int rows, int keep, bool need_h, const int *want = nullptr, int step = 1, int first = 0)
+{
+    NormRows n{};
+    n.x = ptr<float>(r->x);
+    if (r->pending & 1) n.cout = ptr<float>(r->cout);
+    if (r->pending & 2) n.ymoe = ptr<float>(r->ymoe);
+    n.g = ptr<float>(g); n.a16 = ptr<half_t>(r->a16); n.inv = ptr<float>(r->inv); n.h = need_h || st->f32 ? ptr<float>(r->h) : nullptr;
+    n.want = want; n.step = step; n.first = first; n.D = st->D; n.Dp = st->Dp; n.keep = keep; n.eps = st->cfg.eps;
+    launch_norm_rows(n, rows);
+}
+
+float *mix_delta(LayerStack *st, StackRun *r, StackLayer &L, StackRun::Layer &k, const Rows &rows, CatRows &cat)
+{
+    const LayerConfig &c = L.c;
+    const int n = rows.n(), ldc = L.in.rows;
+    const bool pc = c.mixer == MIX_CHANNEL_DELTA;
+    Aux ax{ptr<float>(r->aux)};
+    const DeltaAux d = delta_aux(ax, c, n);
+    const float *cin = ptr<float>(r->cin);
+    if (pc) {                                             // the second halves of the two low-rank products
+        auto low_rank = [&](const StackMat &w, int col, float *out) {
+            if (!st->f32) launch_rows_to_f16(cin + col, ldc, ptr<half_t>(r->a16), ptr<float>(r->inv), n, w.cols);
+            product(st, w, ptr<half_t>(r->a16), ptr<float>(r->inv), cin + col, ldc, out, n);
+        };
+        low_rank(L.a2, L.o_a, d.a2);
+        low_rank(L.g2, L.o_g, d.g2);
+    }
+    DeltaRows a{};
+    a.r = rows; a.H = c.heads; a.KV = c.kv_heads; a.dim = c.dim; a.vdim = c.vdim; a.taps = c.taps; a.per_channel = pc;
+    a.cin = cin; a.ldc = ldc; a.o_q = L.o_q; a.o_k = L.o_k; a.o_v = L.o_v; a.o_b = L.o_b; a.o_a = L.o_a;
+    a.filters = ptr<float>(L.conv); a.a_exp = ptr<float>(L.a_exp); a.dt_bias = ptr<float>(L.dt_bias);
+    a.conv = ptr<float>(k.conv); a.S = ptr<float>(k.S);
+    a.q = d.q; a.k = d.k; a.v = d.v; a.kq = d.kq; a.beta = d.beta; a.g = d.g; a.a2 = d.a2; a.o = d.o;
+    launch_delta_inputs(a);
+    launch_delta_scan(a);
+    cat.g_out = ptr<float>(L.g_out);
+    cat.gate = pc ? d.g2 : cin + L.o_g; cat.ld_gate = pc ? L.hv : ldc; cat.gate_silu = pc ? 0 : 1;
+    return d.o;
+}
+
+float *mix_latent(LayerStack *st, StackRun *r, StackLayer &L, StackRun::Layer &k, const Rows &rows)
+{
+    const LayerConfig &c = L.c;
+    Aux ax{ptr<float>(r->aux)};
+    const LatentAux d = latent_aux(ax, c, rows.n());
+    LatentRows a{};
+    a.r = rows; a.H = c.heads; a.dim = c.dim; a.rot = c.rot_dim; a.vdim = c.vdim; a.rank = c.kv_rank; a.window = c.window;
+    a.ring_rows = k.ring_rows; a.rot_dims = c.rot_dims; a.scale = c.scale; a.eps = st->cfg.eps;
+    a.cin = ptr<float>(r->cin); a.ldc = L.in.rows; a.o_q = L.o_q; a.o_dkv = L.o_dkv;
+    a.g_c = ptr<float>(L.g_c); a.rope = ptr<float2>(L.rope); a.ring = ptr<float>(k.ring);
+    a.q = d.q; a.o = d.o; a.f32 = st->f32; a.uk = dptr(L.uk.buf); a.uv = dptr(L.uv.buf); a.ldu = L.uk.cols;
+    launch_latent_cache(a);
+    launch_latent_attend(a);
+    return d.o;
+}
+
+}  // namespace
+
+void stack_forward(LayerStack *st, StackRun *r, const int *tokens, int T, int pos)
+{
+    const Rows rows{r->B, T, pos};
+    const int n = rows.n();
+    // tokens travel through pinned memory, every position in a place of its own: only a new sequence writes a place again
+    if (pos == 0) HIP_CHECK(hipStreamSynchronize(stream()));
+    int *th = r->tok_host + (size_t)pos * r->B;
+    memcpy(th, tokens, (size_t)n * sizeof(int));
+    HIP_CHECK(hipMemcpyAsync(dptr(r->tok), th, (size_t)n * sizeof(int), hipMemcpyHostToDevice, stream()));
+    launch_embed_rows(ptr<float>(st->emb), ptr<int>(r->tok), st->cfg.emb_scale, ptr<float>(r->x), st->D, st->Dp, n);
+    r->T = T; r->pending = 0;
+    for (size_t i = 0; i < st->layers.size(); i++) {
+        StackLayer &L = st->layers[i];
+        const LayerConfig &c = L.c;
+        norm(st, r, L.g_norm, n, 1, c.experts > 0);
+        product(st, L.in, ptr<half_t>(r->a16), ptr<float>(r->inv), ptr<float>(r->h), st->Dp, ptr<float>(r->cin), n);
+        CatRows cat{};
+        cat.o = L.delta() ? mix_delta(st, r, L, r->layers[i], rows, cat) : mix_latent(st, r, L, r->layers[i], rows);
+        cat.H = c.heads; cat.vdim = c.vdim; cat.eps = st->cfg.eps;
+        cat.shared = ptr<float>(r->cin) + L.o_shared; cat.ld_shared = L.in.rows; cat.shared_ff = c.shared_ff; cat.o_sh = L.o_sh;
+        cat.cat = ptr<float>(r->cat); cat.a16 = ptr<half_t>(r->a16); cat.inv = ptr<float>(r->inv); cat.ldk = L.out.cols;
+        launch_cat_rows(cat, n);
+        product(st, L.out, cat.a16, cat.inv, cat.cat, cat.ldk, ptr<float>(r->cout), n);
+        r->pending = 1;
+        if (!c.experts) continue;
+        MoeRows m{};
+        m.rows = n; m.E = c.experts; m.top = c.top; m.ff = c.ff; m.ffp = L.down.cols; m.D = st->D; m.Dp = st->Dp; m.f32 = st->f32;
+        m.z = ptr<float>(r->cin) + L.o_router; m.ldz = L.in.rows; m.idx = ptr<int>(r->route_idx); m.w = ptr<float>(r->route_w);
+        m.h = ptr<float>(r->h); m.up = dptr(L.up.buf); m.down = dptr(L.down.buf); m.act = ptr<float>(r->act); m.y = ptr<float>(r->ymoe);
+        launch_route(m);
+        launch_experts_per_row(m);
+        r->pending = 3;
+    }
+}
+
+void stack_logits(LayerStack *st, StackRun *r, const int *want, int n, float *logits)
+{
+    if (n <= 0) return;
+    const int *list = nullptr;
+    if (want) {
+        memcpy(r->want_host, want, (size_t)n * sizeof(int));
+        HIP_CHECK(hipMemcpyAsync(dptr(r->want), r->want_host, (size_t)n * sizeof(int), hipMemcpyHostToDevice, stream()));
+        list = ptr<int>(r->want);
+    }
+    norm(st, r, st->g_final, n, 0, false, list, r->T, r->T - 1);
+    product(st, st->head, ptr<half_t>(r->a16), ptr<float>(r->inv), ptr<float>(r->h), st->Dp, logits, n);
+}
+
+}  // namespace lmhip

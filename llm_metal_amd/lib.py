@@ -19,6 +19,12 @@ def build(jobs=8):
     return LIB_PATH
 
 
+def build_library(jobs=8):
+    """Compile only the library, and only what is not built yet (no driver program)."""
+    subprocess.check_call(["make", "-C", os.path.join(_HERE, "csrc"), f"-j{jobs}", "../libllm_metal_hip.so"], stdout=subprocess.DEVNULL)
+    return LIB_PATH
+
+
 def declared_symbols():
     """Function names declared in include/*.h (used to check the exports)."""
     names = []
@@ -146,7 +152,8 @@ def load():
         "inference_state_reset": (None, [vp]), "inference_forward_token": (C.POINTER(C.c_float), [vp, i]),
         "inference_forward_token_argmax": (i, [vp, i]), "inference_state_set_lora": (None, [vp, vp]),
         "inference_state_set_eos": (None, [vp, vp, i]), "inference_state_load_eos": (None, [vp, C.c_char_p]),
-        "inference_state_position": (i, [vp]),
+        "inference_state_position": (i, [vp]), "inference_forward_tokens": (i, [vp, vp, i, vp, i, vp]),
+        "model_type_detect": (i, [C.c_char_p]), "model_type_name": (C.c_char_p, [i]),
         "inference_state_create_from_file": (vp, [C.c_char_p, i, i, i]),
         "model_file_open": (vp, [C.c_char_p]), "model_file_close": (None, [vp]), "model_file_is_gguf": (i, [vp]),
         "model_file_count": (i, [vp]), "model_file_name": (C.c_char_p, [vp, i]),

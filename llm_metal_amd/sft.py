@@ -240,11 +240,16 @@ class InferenceState:
     """inference_state_create_from_ref / _from_sft ... inference_state_free (include/inference_hip.h)."""
 
     def __init__(self, c: SFTConfig = None, model=None, max_seq=256, use_fp16=True, sft: "SFTState" = None, path=None,
-                 model_type=0):
+                 model_type=0, weight_format=None):
+        """model_type None (with path): as the config.json there says.  weight_format, with path: "f16", "q8_0" or "f32"
+        instead of use_fp16."""
         self.L = _lib.load()
         if path is not None:                               # inference_state_create_from_file
             self.c, self._keep = c, []
-            self.h = self.L.inference_state_create_from_file(str(path).encode(), model_type, max_seq, 1 if use_fp16 else 0)
+            if model_type is None:
+                model_type = self.L.model_type_detect(str(path).encode())
+            fmt = {"q8_0": 0, "f16": 1, "f32": 2}[weight_format] if weight_format else 1 if use_fp16 else 0
+            self.h = self.L.inference_state_create_from_file(str(path).encode(), model_type, max_seq, fmt)
         elif sft is not None:
             self.c, self._keep = sft.c, [sft]
             self.h = self.L.inference_state_create_from_sft(sft.h, max_seq)
@@ -266,6 +271,15 @@ class InferenceState:
         if not p:
             raise RuntimeError("inference_forward_token refused the token (outside the vocabulary or cache full)")
         return np.ctypeslib.as_array(p, shape=(self.V,)).copy()
+
+    def forward_tokens(self, tokens, want=()):
+        """The next tokens at the current position; logits [len(want), V] at the places `want` (ascending) among them."""
+        t = np.ascontiguousarray(tokens, dtype=np.int32)
+        w = np.ascontiguousarray(want, dtype=np.int32)
+        out = np.empty((len(w), self.V), dtype=np.float32)
+        if self.L.inference_forward_tokens(self.h, _vp(t), len(t), _vp(w), len(w), _vp(out)) != 0:
+            raise RuntimeError("inference_forward_tokens refused its arguments")
+        return out
 
     def forward_token_argmax(self, token):
         return int(self.L.inference_forward_token_argmax(self.h, int(token)))
