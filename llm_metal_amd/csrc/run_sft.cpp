@@ -1,10 +1,12 @@
-// run_sft — the reference's `--mode sft` driver (main.c:204-278 options, :286-324 model-type detection, :366-524 loop)
+// run_sft — the reference's `--mode sft` driver (and `--mode generate`: greedy generation from token ids) (main.c:204-278 options, :286-324 model-type detection, :366-524 loop)
 // over the HIP library: load a checkpoint (safetensors file / shard directory or GGUF), build the SFT state (LoRA or
 // full-parameter), feed batches from a pre-tokenized int32 file (or the reference's synthetic fallback), print
 // `step | loss | lr | tok/s`, save the adapters or the full checkpoint.
 #include "../../include/data_hip.h"
+#include "../../include/inference_hip.h"
 #include "../../include/loader_hip.h"
 
+#include <ctype.h>
 #include <stdio.h>
 #include <stdlib.h>
 #include <string.h>
@@ -17,6 +19,8 @@ namespace {
 
 struct Options {
     std::string model, train_data, lora_adapter, checkpoint_dir = "checkpoints";
+    std::string mode = "sft", prompt;
+    int max_gen = 64, max_seq = 0, f32 = 0;
     int lora_rank = 16, seq_len = 512, batch = 1, max_steps = 10000, log_interval = 1, full_param = 0, use_q8 = 0;
     float lora_alpha = 32.0f, lr = 0.0f;
 };
@@ -36,25 +40,47 @@ void usage(const char *prog)
            "  --full-param          full-parameter SGD inside the backward (no LoRA)\n"
            "  --q8                  keep the frozen weights as Q8_0 in HBM (LoRA only)\n"
            "  --checkpoint <dir>    where lora_adapter.bin / full_checkpoint.bin go (default checkpoints)\n"
-           "  --log-interval <n>    print every n steps (default 1)\n", prog);
+           "  --log-interval <n>    print every n steps (default 1)\n"
+           "  --mode sft|generate   train (default), or emit greedy tokens after a prompt\n"
+           "generate: --prompt <ids>  token ids with commas between them\n"
+           "          --max-gen <n>   tokens to emit (default 64);  --max-seq <n>  positions to reserve\n"
+           "          --q8 | --f32    Q8_0 or 32-bit weights instead of F16 (32-bit: Nevurax models)\n", prog);
 }
 
-// main.c:286-324: "gemma3" / "gemma2" in the config.json next to (or inside) the model path, else Qwen3
+// which model the path holds, reported as the reference reports it (main.c:286-324)
 ModelType detect_model_type(const std::string &path)
 {
-    struct stat st;
-    std::string cfg;
-    if (stat(path.c_str(), &st) == 0 && S_ISDIR(st.st_mode)) cfg = path + "/config.json";
-    else { const size_t sl = path.rfind('/'); cfg = sl == std::string::npos ? "config.json" : path.substr(0, sl) + "/config.json"; }
-    FILE *fp = fopen(cfg.c_str(), "r");
-    if (!fp) return MODEL_QWEN3;
-    char buf[4096];
-    const size_t n = fread(buf, 1, sizeof buf - 1, fp);
-    buf[n] = 0;
-    fclose(fp);
-    if (strstr(buf, "\"gemma3") || strstr(buf, "\"gemma2")) { printf("[Model] Detected model_type: gemma3 (from config.json)\n"); return MODEL_GEMMA3; }
-    if (strstr(buf, "\"qwen3") || strstr(buf, "\"qwen2")) printf("[Model] Detected model_type: qwen3 (from config.json)\n");
-    return MODEL_QWEN3;
+    const ModelType t = model_type_detect(path.c_str());
+    std::string name = model_type_name(t);
+    for (char &c : name) c = (char)tolower(c);
+    printf("[Model] Detected model_type: %s\n", name.c_str());
+    return t;
+}
+
+// --mode generate: greedy tokens after a prompt of token ids (any model the library generates with)
+int generate(const std::string &model, const std::string &prompt, int max_gen, int max_seq, int weight_format)
+{
+    std::vector<uint32_t> ids;
+    for (const char *p = prompt.c_str(); *p;) {
+        char *e = nullptr;
+        const unsigned long v = strtoul(p, &e, 10);
+        if (e == p) { fprintf(stderr, "[Generate] the prompt is a list of token ids: 5,17,3\n"); return 2; }
+        ids.push_back((uint32_t)v);
+        p = *e == ',' ? e + 1 : e;
+        if (p == e && *p) { fprintf(stderr, "[Generate] the prompt is a list of token ids: 5,17,3\n"); return 2; }
+    }
+    if (ids.empty()) { fprintf(stderr, "[Generate] Error: --prompt is required\n"); return 2; }
+    InferenceState *s = inference_state_create_from_file(model.c_str(), detect_model_type(model), max_seq ? max_seq : (int)ids.size() + max_gen, weight_format);
+    if (!s) { fprintf(stderr, "[Generate] Failed to load model\n"); return 1; }
+    inference_state_load_eos(s, model.c_str());
+    std::vector<uint32_t> out(max_gen);
+    const int n = inference_generate(s, ids.data(), (int)ids.size(), out.data(), max_gen);
+    inference_state_free(s);
+    if (n <= 0) { fprintf(stderr, "[Generate] the prompt was refused\n"); return 1; }
+    printf("tokens:");
+    for (int i = 0; i < n; i++) printf(" %u", out[i]);
+    printf("\n");
+    return 0;
 }
 
 double seconds_since(const timespec &t0)
@@ -86,14 +112,23 @@ int main(int argc, char **argv)
         else if (a == "--log-interval" && has) o.log_interval = atoi(argv[++i]);
         else if (a == "--full-param" || a == "--accurate") o.full_param = 1;
         else if (a == "--q8") o.use_q8 = 1;
-        else if (a == "--mode" && has) { if (strcmp(argv[++i], "sft") != 0) { fprintf(stderr, "[SFT] this driver only has --mode sft\n"); return 2; } }
+        else if (a == "--mode" && has) { o.mode = argv[++i]; if (o.mode != "sft" && o.mode != "generate") { fprintf(stderr, "[SFT] this driver has --mode sft and --mode generate\n"); return 2; } }
+        else if (a == "--prompt" && has) o.prompt = argv[++i];
+        else if (a == "--max-gen" && has) o.max_gen = atoi(argv[++i]);
+        else if (a == "--max-seq" && has) o.max_seq = atoi(argv[++i]);
+        else if (a == "--f32") o.f32 = 1;
         else { fprintf(stderr, "[SFT] unknown option %s\n", a.c_str()); usage(argv[0]); return 2; }
     }
     if (o.model.empty()) { fprintf(stderr, "[SFT] Error: --model is required for SFT mode\n"); return 2; }
+    if (o.mode == "generate") {
+        if (o.max_gen <= 0 || o.max_seq < 0) { fprintf(stderr, "[Generate] Error: --max-gen must be positive\n"); return 2; }
+        return generate(o.model, o.prompt, o.max_gen, o.max_seq, o.f32 ? 2 : o.use_q8 ? 0 : 1);
+    }
     if (o.seq_len <= 0 || o.batch <= 0 || o.max_steps < 0 || o.log_interval <= 0) { fprintf(stderr, "[SFT] Error: --seq, --batch, --log-interval must be positive\n"); return 2; }
     const float lr = o.lr > 0 ? o.lr : 1e-5f;
     const ModelType mtype = detect_model_type(o.model);
-    printf("=== %s Fast %s SFT ===\n", mtype == MODEL_GEMMA3 ? "Gemma3" : "Qwen3", o.full_param ? "Full-param SGD" : "LoRA");
+    if (mtype == MODEL_NEVURAX) { fprintf(stderr, "[SFT] %s has no training path (--mode generate)\n", model_type_name(mtype)); return 2; }
+    printf("=== %s Fast %s SFT ===\n", model_type_name(mtype), o.full_param ? "Full-param SGD" : "LoRA");
     printf("  Model: %s\n", o.model.c_str());
     if (!o.full_param) printf("  LoRA rank: %d, alpha: %.1f\n", o.lora_rank, o.lora_alpha);
     printf("  Seq: %d, Steps: %d\n  LR: %.2e\n\n", o.seq_len, o.max_steps, lr);

@@ -116,3 +116,96 @@ def make_batch(c: SFTConfig, seed=1):
     tok = rng.integers(0, c.V, size=(c.batch, c.seq), dtype=np.uint32)
     tgt = np.roll(tok, -1, axis=1)
     return tok.reshape(-1).copy(), tgt.reshape(-1).copy()
+
+
+# ---------------------------------------------------------------- models described layer by layer (Nevurax)
+
+def stack_shapes(cfg, rank_a=24, rank_g=24):
+    """Tensor names and shapes of a layer-by-layer model; cfg is the dictionary that becomes its config.json.  rank_a and
+    rank_g: widths of the two low-rank products of a per-channel decay (tensor shapes, not configuration)."""
+    D = cfg["width"]
+    out = {"embed": (cfg["vocab"], D)}
+    for i, L in enumerate(cfg["layers"]):
+        m, p = L["mixer"], f"l{i}."
+        H, d, dv = m["heads"], m["dim"], m["vdim"]
+        out[p + "norm1"] = (D,)
+        x = p + "mix."
+        if L["type"] == "latent_attention":
+            r, R = m["rot_dim"], m["kv_rank"]
+            out.update({x + "q": (H * (d + r), D), x + "dkv": (R + r, D), x + "dkv.norm": (R,), x + "uk": (H * d, R), x + "uv": (H * dv, R)})
+        else:
+            kd = m["kv_heads"] * d
+            for n, c in (("q", kd), ("k", kd), ("v", H * dv)):
+                out.update({x + n: (c, D), x + n + ".conv": (c, m["conv"])})
+            out.update({x + "b": (H, D), x + "A_log": (H,), x + "norm": (dv,)})
+            if L["type"] == "channel_delta":
+                out.update({x + "a1": (rank_a, D), x + "a2": (H * d, rank_a), x + "dt_bias": (H * d,),
+                            x + "g1": (rank_g, D), x + "g2": (H * dv, rank_g)})
+            else:
+                out.update({x + "a": (H, D), x + "dt_bias": (H,), x + "g": (H * dv, D)})
+        out[x + "o"] = (D, H * dv)
+        if L.get("mlp"):
+            e, f, y = L["mlp"]["router"]["experts"], L["mlp"]["expert"]["ff"], p + "mlp."
+            for k in range(e):
+                out.update({f"{y}e{k}.up": (f, D), f"{y}e{k}.down": (D, f)})
+            out[y + "router"] = (e, D)
+            if L["mlp"].get("shared"):
+                s = L["mlp"]["shared"]["ff"]
+                out.update({y + "shared.up": (s, D), y + "shared.down": (D, s)})
+    out.update({"final.norm": (D,), "head": (cfg["vocab"], D)})
+    return out
+
+
+def make_stack_tensor(name, shape, rng):
+    """Matrices ~ N(0, 1 / columns) (down and output projections half of that), norms around 1, filters and decay
+    parameters spread so that states remember from a few tokens to a few hundred."""
+    leaf = name.rsplit(".", 1)[-1]
+    if leaf in ("norm", "norm1"):
+        return (1.0 + 0.1 * rng.standard_normal(shape)).astype(np.float32)
+    if leaf == "conv":
+        return (rng.standard_normal(shape) / np.sqrt(shape[1])).astype(np.float32)
+    if leaf == "A_log":
+        return rng.uniform(-3.0, 0.5, shape).astype(np.float32)
+    if leaf == "dt_bias":
+        return rng.uniform(-3.0, 0.0, shape).astype(np.float32)
+    if leaf == "embed":
+        return rng.standard_normal(shape, dtype=np.float32)
+    scale = (0.5 if leaf in ("down", "o") else 1.0) / np.sqrt(shape[-1])
+    a = rng.standard_normal(shape, dtype=np.float32)
+    a *= np.float32(scale)
+    return a
+
+
+def to_bf16_bits(a):
+    b = np.ascontiguousarray(a, np.float32).view(np.uint32)
+    return ((b + np.uint32(0x7FFF) + ((b >> np.uint32(16)) & np.uint32(1))) >> np.uint32(16)).astype(np.uint16)
+
+
+def write_stack_checkpoint(path, cfg, seed=0, rank_a=24, rank_g=24, keep=False, edit=None):
+    """config.json and model.safetensors (bfloat16) of a random model in the folder `path`.  keep: return the values the
+    file holds, fp32 by name.  edit(name, array): may replace a tensor before it is rounded."""
+    import json
+    import struct
+    shapes = stack_shapes(cfg, rank_a, rank_g)
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    header, off = {}, 0
+    for name, shape in shapes.items():
+        n = 2 * int(np.prod(shape))
+        header[name] = {"dtype": "BF16", "shape": list(shape), "data_offsets": [off, off + n]}
+        off += n
+    text = json.dumps(header).encode()
+    text += b" " * (-len(text) % 8)
+    kept = {}
+    with open(os.path.join(path, "model.safetensors"), "wb") as f:
+        f.write(struct.pack("<Q", len(text)) + text)
+        for i, (name, shape) in enumerate(shapes.items()):
+            a = make_stack_tensor(name, shape, np.random.default_rng([seed, i]))
+            if edit is not None:
+                a = edit(name, a)
+            bits = to_bf16_bits(a)
+            f.write(bits.tobytes())
+            if keep:
+                kept[name] = (bits.astype(np.uint32) << np.uint32(16)).view(np.float32)
+    return kept

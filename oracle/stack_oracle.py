@@ -150,6 +150,11 @@ def new_state(cfg):
     return {"pos": 0, "layers": [{} for _ in cfg["layers"]]}
 
 
+def copy_state(state):
+    """Steps replace what a state holds and append to its lists; they never write into an array."""
+    return {"pos": state["pos"], "layers": [{k: list(v) if isinstance(v, list) else v for k, v in L.items()} for L in state["layers"]]}
+
+
 def step(cfg, W, state, token, trace=None):
     """One token through every layer; returns the logits.  `trace`: list that receives x after each layer."""
     eps, pos = cfg["norm"]["eps"], state["pos"]
