@@ -28,6 +28,7 @@
 #include "fused.h"
 #include "planes.h"
 #include "bf16pair.h"
+#include "lds_copy.h"
 
 namespace lmhip {
 namespace {
@@ -283,17 +284,6 @@ struct FaArgs {
     float *dkp, *dvp;                    // [Hq / Hkv][rows][Hkv * HD]: per query head of a group
 };
 
-// One wave-wide copy of 1 KB from memory into LDS without passing registers: lane i's 16 bytes land at lds_base + 16 i
-// (M0 holds the wave-uniform base).  Written as assembly so that the compiler does not count it among its own loads:
-// it cannot tell which LDS bytes a pending copy will write and would wait for ALL copies in flight before every LDS
-// read.  The kernels wait for their copies themselves, once per step (FA_WAIT_AND_BARRIER); loads retire in order, so
-// a wait that the compiler inserts for a load of its own can only wait longer than it has to, never too short.
-__device__ __forceinline__ void copy_to_lds_1k(const uint4 *src_lane, uint4 *lds_base)
-{
-    const uint32_t base = __builtin_amdgcn_readfirstlane((uint32_t)(uintptr_t)(lds_void *)lds_base);
-    asm volatile("s_mov_b32 m0, %1\n\tglobal_load_lds_dwordx4 %0, off" :: "v"(src_lane), "s"(base) : "memory", "m0");
-}
-
 // The tiles of the next step go into the other LDS buffer while the current one is multiplied; every wave requests a
 // quarter of the fragments.  NT tiles per step; tile t of block `blk` sits at src[t] + blk * TILE.
 template <int HD, int NT>
@@ -407,7 +397,6 @@ __device__ __forceinline__ void touch_b_rows(const bf16x8 (&bh)[HD / 16], const 
 // carries it in ordinary registers and copies all of it in and out around the matrix instructions of every step).
 #define FA_PIN_ACC(x) asm volatile("" : "+a"(x))
 
-#define FA_WAIT_AND_BARRIER() asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory")
 
 // grid (blocks of 128 queries * Hq * batch), block 256; LDS: two buffers of [RT(K) | PT(V)]
 template <int HD>

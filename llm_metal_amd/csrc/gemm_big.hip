@@ -257,7 +257,12 @@ __global__ __launch_bounds__(256) void gemm_big(GemmKArgs g)
 // every LDS read); the wait before the barrier is written by hand: the barrier that ends half step h - 1 finds h and
 // h + 1 in LDS -- every wave has waited for its own copies of them -- so slice 0 of h + 1 is read under the MFMAs of
 // slice 1 of h and no half step starts by waiting out an LDS round trip; h + 5 is requested into the buffer h - 1 left.
-__global__ __launch_bounds__(256) void gemm_big_f16(GemmKArgs g)
+//
+// GROUPED: the 128-row blocks of A belong to different weights of one shape, laid group.stride halves apart: block mt is
+// multiplied with number group.of[mt]; a negative number is a block without rows, and its workgroups leave at once.
+struct GroupArgs { const int *of; size_t stride; };
+template <bool GROUPED>
+__global__ __launch_bounds__(256) void gemm_big_f16(GemmKArgs g, GroupArgs group)
 {
     constexpr int HB = 12 * 2 * 64;                       // half8 per buffer: [4 A + 8 W row blocks][2 slices][64 lanes]
     __shared__ half8 lb0[HB], lb1[HB], lb2[HB], lb3[HB], lb4[HB], lb5[HB];
@@ -276,6 +281,11 @@ __global__ __launch_bounds__(256) void gemm_big_f16(GemmKArgs g)
         if (mt >= MT || nt >= NT) return;
     }
     const int nb0 = nt * 8, mb0 = mt * 4;
+    if (GROUPED) {
+        const int e = __builtin_amdgcn_readfirstlane(group.of[mt]);
+        if (e < 0) return;
+        g.W.w16 += (size_t)e * group.stride;
+    }
     const int wm = wave >> 1, wn = wave & 1;
     const int k_beg = chunk * g.steps_per_chunk, nsteps = min(g.Kb, k_beg + g.steps_per_chunk) - k_beg;
     const int nhalf = 2 * nsteps, last = nhalf - 1;
@@ -857,7 +867,11 @@ int launch_gemm_big(const half_t *A, const float *a_inv_scale, const WeightOp &W
             const dim3 grid = w ? grid_of(a, 256, 256) : grid_of(a, 128, 128 * WPW);
 #define BIG_LAUNCH(KERNEL) do { if (prof) hipExtLaunchKernelGGL((KERNEL), grid, block, 0, stream(), e0, e1, 0, a); \
                                 else hipLaunchKernelGGL((KERNEL), grid, block, 0, stream(), a); } while (0)
-            if (W.fmt == 0) { if (w) BIG_LAUNCH(gemm_big_f16_256); else BIG_LAUNCH(gemm_big_f16); }
+            if (W.fmt == 0) {
+                if (w) BIG_LAUNCH(gemm_big_f16_256);
+                else if (prof) hipExtLaunchKernelGGL((gemm_big_f16<false>), grid, block, 0, stream(), e0, e1, 0, a, GroupArgs{});
+                else hipLaunchKernelGGL((gemm_big_f16<false>), grid, block, 0, stream(), a, GroupArgs{});
+            }
             else if (W.fmt == 1) { if (a.W.nbq < a.Nb) BIG_LAUNCH((gemm_big_q8<1, 256, true>)); else BIG_LAUNCH((gemm_big_q8<1, 256>)); }
             else BIG_LAUNCH((gemm_big_q8<2, 256>));
 #undef BIG_LAUNCH
@@ -892,6 +906,27 @@ int launch_gemm_big(const half_t *A, const float *a_inv_scale, const WeightOp &W
     }
     HIP_CHECK(hipGetLastError());
     return 1;
+}
+
+void launch_gemm_groups(const half_t *A, const float *a_inv_scale, const half_t *W, size_t group_stride, const int *group_of, float *C, int ldc,
+                        int M, int N, int K, int groups)
+{
+    if (M <= 0 || N <= 0 || K <= 0) return;
+    if (ldc < N || (M & 127) || !A || !W || !group_of || group_stride < tiled_elems(N, K)) {
+        fprintf(stderr, "[fast_hip] gemm_groups: bad launch M=%d N=%d K=%d ldc=%d\n", M, N, K, ldc);
+        abort();
+    }
+    GemmKArgs g{};
+    g.A = reinterpret_cast<const half8 *>(A); g.a_inv_scale = a_inv_scale; g.W = weight_f16(W);
+    g.P = C; g.ldp = ldc; g.M = M; g.N = N; g.Mb = tiled_rb(M); g.Nb = tiled_rb(N); g.Kb = tiled_kb(K);
+    g.steps_per_chunk = g.Kb; g.S = 1;
+    const int mt = M / 128, nt = (N + 255) / 256;
+    const dim3 grid(8 * 32 * ((mt + 7) / 8) * (((nt + 7) / 8 + 3) / 4));
+    hipEvent_t ev_a = nullptr, ev_b = nullptr;
+    if (gemm_prof_begin(2.0 * groups * N * K, 2.0 * M * N * K, &ev_a, &ev_b))
+        hipExtLaunchKernelGGL((gemm_big_f16<true>), grid, dim3(256), 0, stream(), ev_a, ev_b, 0, g, GroupArgs{group_of, group_stride});
+    else hipLaunchKernelGGL((gemm_big_f16<true>), grid, dim3(256), 0, stream(), g, GroupArgs{group_of, group_stride});
+    HIP_CHECK(hipGetLastError());
 }
 
 void set_big_gemm_split(int mode) { g_big_split = mode; }

@@ -61,7 +61,7 @@ __global__ __launch_bounds__(256) void k_latent_query(LatentRows a, int m0)
     for (int i = tid; i < a.dim; i += 256) qs[i] = q[i];
     __syncthreads();
     float *out = a.q + ((size_t)m * a.H + h) * w;
-    const WT *uk = (const WT *)a.uk + (size_t)h * a.dim * a.ldu;
+    const WT *uk = (const WT *)a.ukv + (size_t)h * a.dim * a.ldu;
     for (int c = tid; c < rp; c += 256) {                 // the weight's padding columns are zero
         float s = 0.f;
         for (int d = 0; d < a.dim; d++) s = fmaf((float)uk[(size_t)d * a.ldu + c], qs[d], s);
@@ -160,7 +160,7 @@ __global__ __launch_bounds__(256) void k_latent_values(LatentRows a, int m0, int
     }
     __syncthreads();
     for (int i = wave; i < a.vdim; i += 4) {
-        const WT *uv = (const WT *)a.uv + ((size_t)h * a.vdim + i) * a.ldu;
+        const WT *uv = (const WT *)a.ukv + ((size_t)a.H * a.dim + (size_t)h * a.vdim + i) * a.ldu;
         float s = 0.f;
         for (int c = lane; c < rp; c += 64) s = fmaf((float)uv[c], ctx[c], s);
         s = wave_sum(s);

@@ -88,7 +88,7 @@ __global__ __launch_bounds__(256) void k_expert_up(MoeRows a)
     if (i >= a.ffp) return;
     const size_t slot = (size_t)m * a.top + s;
     float v = 0.f;
-    if (i < a.ff) v = wave_sum(dot_part((const WT *)a.up + ((size_t)a.idx[slot] * a.ff + i) * a.Dp, a.h + (size_t)m * a.Dp, a.Dp, lane));
+    if (i < a.ff) v = wave_sum(dot_part((const WT *)a.up + ((size_t)a.idx[slot] * a.up_rows + i) * a.Dp, a.h + (size_t)m * a.Dp, a.Dp, lane));
     if (lane == 0) a.act[slot * a.ffp + i] = relu2(v);   // the padding is written too: zero
 }
 
@@ -102,13 +102,117 @@ __global__ __launch_bounds__(256) void k_expert_down(MoeRows a)
     if (d < a.D)
         for (int s = 0; s < a.top; s++) {
             const size_t slot = (size_t)m * a.top + s;
-            y = fmaf(a.w[slot], dot_part((const WT *)a.down + ((size_t)a.idx[slot] * a.D + d) * a.ffp, a.act + slot * a.ffp, a.ffp, lane), y);
+            y = fmaf(a.w[slot], dot_part((const WT *)a.down + ((size_t)a.idx[slot] * a.down_rows + d) * a.ffp, a.act + slot * a.ffp, a.ffp, lane), y);
         }
     y = wave_sum(y);
     if (lane == 0) a.y[(size_t)m * a.Dp + d] = y;
 }
 
+// ---------------------------------------------------------------- pairs sorted by expert
+
+// grid (E), block 256: how many pairs chose expert blockIdx.x
+__global__ __launch_bounds__(256) void k_moe_count(const int *__restrict__ idx, int n, int *__restrict__ count)
+{
+    __shared__ float sm[16];
+    int c = 0;
+    for (int i = threadIdx.x; i < n; i += 256) c += idx[i] == (int)blockIdx.x;
+    const float total = block_sum((float)c, sm);          // exact: far below 2^24
+    if (threadIdx.x == 0) count[blockIdx.x] = (int)total;
+}
+
+// grid (E), block 256: the expert's blocks, and its pairs in order of row into them
+__global__ __launch_bounds__(256) void k_moe_place(const int *__restrict__ idx, int n, int top, int E, MoeGroups g)
+{
+    __shared__ float sm[16];
+    __shared__ int wave_n[4];
+    const int e = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    int before = 0;                                       // blocks of the experts ahead
+    for (int i = tid; i < e; i += 256) before += (g.count[i] + 127) >> 7;
+    const int t0 = (int)block_sum((float)before, sm), mine = g.count[e], nt = (mine + 127) >> 7;
+    for (int i = tid; i < nt; i += 256) g.of[t0 + i] = e;
+    for (int i = mine + tid; i < nt * 128; i += 256) g.src[t0 * 128 + i] = -1;
+    if (e == E - 1)                                       // blocks behind the last expert's
+        for (int i = t0 + nt + tid; i < g.tiles; i += 256) g.of[i] = -1;
+    if (!mine) return;
+    int at = t0 * 128;
+    for (int i0 = 0; i0 < n; i0 += 256) {
+        const int i = i0 + tid;
+        const bool hit = i < n && idx[i] == e;
+        const unsigned long long b = __ballot(hit);
+        if (lane == 0) wave_n[wave] = __popcll(b);
+        __syncthreads();
+        int o = at;
+        for (int w = 0; w < wave; w++) o += wave_n[w];
+        if (hit) {
+            const int p = o + __popcll(b & ((1ull << lane) - 1ull));
+            g.src[p] = i / top;
+            g.pos[i] = p;
+        }
+        at += wave_n[0] + wave_n[1] + wave_n[2] + wave_n[3];
+        __syncthreads();
+    }
+}
+
+// grid (rows of the groups), block 256: one row of a tiled operand to another place, 16 bytes per thread and trip
+__global__ __launch_bounds__(256) void k_moe_gather(MoeGroups g, const half_t *__restrict__ a16, const float *__restrict__ inv,
+                                                    half_t *__restrict__ out16, float *__restrict__ out_inv, int Kb)
+{
+    const int p = blockIdx.x;
+    if (g.of[p >> 7] < 0) return;
+    const int m = g.src[p];
+    if (m < 0) return;
+    for (int k = threadIdx.x * 8; k < Kb * 64; k += 2048)
+        *reinterpret_cast<half8 *>(&out16[tiled_a_index(p, k, Kb)]) = *reinterpret_cast<const half8 *>(&a16[tiled_a_index(m, k, Kb)]);
+    if (threadIdx.x == 0) out_inv[p] = inv[m];
+}
+
+// grid (rows of the groups), block 256
+__global__ __launch_bounds__(256) void k_moe_act(MoeGroups g, const float *__restrict__ up, int ld, int n, half_t *__restrict__ out16,
+                                                 float *__restrict__ out_inv, int K)
+{
+    extern __shared__ float row[];                        // [K]
+    __shared__ float sm[16];
+    const int p = blockIdx.x;
+    if (g.of[p >> 7] < 0 || g.src[p] < 0) return;
+    float mx = 0.f;
+    for (int i = threadIdx.x; i < K; i += 256) {
+        const float v = i < n ? relu2(up[(size_t)p * ld + i]) : 0.f;
+        row[i] = v;
+        mx = fmaxf(mx, v);
+    }
+    const float s = row_scale_for(block_max(mx, sm));     // its barriers publish the row
+    store_row_f16(row, K, out16, p, tiled_kb(K), s);
+    if (threadIdx.x == 0) out_inv[p] = 1.f / s;
+}
+
 }  // namespace
+
+int moe_group_tiles(int rows, int top, int E) { const int n = rows * top; return n / 128 + (E < n ? E : n); }
+size_t moe_group_ints(int rows, int top, int E) { const size_t t = moe_group_tiles(rows, top, E); return (size_t)E + t + t * 128 + (size_t)rows * top; }
+MoeGroups moe_groups_at(int *base, int rows, int top, int E)
+{
+    MoeGroups g{};
+    g.tiles = moe_group_tiles(rows, top, E);
+    g.count = base; g.of = g.count + E; g.src = g.of + g.tiles; g.pos = g.src + (size_t)g.tiles * 128;
+    return g;
+}
+
+void launch_moe_groups(const MoeRows &a, const MoeGroups &g)
+{
+    const int n = a.rows * a.top;
+    LAUNCH(k_moe_count, dim3(a.E), dim3(256), 0, a.idx, n, g.count);
+    LAUNCH(k_moe_place, dim3(a.E), dim3(256), 0, a.idx, n, a.top, a.E, g);
+}
+
+void launch_moe_gather(const MoeGroups &g, const half_t *a16, const float *inv, half_t *out16, float *out_inv, int K)
+{
+    LAUNCH(k_moe_gather, dim3(g.tiles * 128), dim3(256), 0, g, a16, inv, out16, out_inv, tiled_kb(K));
+}
+
+void launch_moe_act(const MoeGroups &g, const float *up, int ld, int n, half_t *out16, float *out_inv, int K)
+{
+    LAUNCH(k_moe_act, dim3(g.tiles * 128), dim3(256), (size_t)K * 4, g, up, ld, n, out16, out_inv, K);
+}
 
 void launch_route(const MoeRows &a) { LAUNCH(k_route, dim3((a.rows + 3) / 4), dim3(256), 0, a); }
 

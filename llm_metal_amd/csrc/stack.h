@@ -61,8 +61,9 @@ struct StackLayer {
     MetalBuf *conv = nullptr, *a_exp = nullptr, *dt_bias = nullptr, *g_out = nullptr;   // fp32: filters [channels][taps], exp(A_log), bias, head norm
     StackMat a2, g2;
     MetalBuf *g_c = nullptr, *rope = nullptr;            // latent norm weight; (cos, sin) [max_seq][rot_dims / 2]
-    StackMat uk, uv;                                     // [heads * dim, rank], [heads * vdim, rank]
-    StackMat up, down;                                   // experts one after the other: [E * ff, width], [E * width, ff]
+    StackMat ukv;                                        // [heads * dim | heads * vdim, rank]: key and value projections
+    StackMat up, down;                                   // experts one after the other: [E * up_rows, width], [E * down_rows, ff]
+    int up_rows = 0, down_rows = 0;                      // ff and width padded to the 32 rows of a tile
     int channels() const { return 2 * c.kv_heads * c.dim + c.heads * c.vdim; }
     bool delta() const { return c.mixer != MIX_LATENT; }
 };
@@ -83,6 +84,15 @@ void stack_free(LayerStack *st);
 
 // ---------------------------------------------------------------- what sequences keep, and a run's scratch
 
+// The (row, choice) pairs sorted by expert, each expert's share padded to whole blocks of 128 rows, so that every expert's
+// weights meet all their rows in one product.
+struct MoeGroups {
+    int tiles;                                           // blocks of 128 rows at most
+    int *count;                                          // [E]
+    int *of;                                             // [tiles]: expert of a block, -1: no rows
+    int *src;                                            // [tiles * 128]: row of the step, -1: padding
+    int *pos;                                            // [rows][top]: where the pair's result lies
+};
 struct StackRun {
     int B = 0, rows = 0;                                 // sequences; token rows the scratch holds
     // per layer.  delta: state [B][heads][vdim][dim] and the last `taps` inputs of the convolutions [B][taps][channels];
@@ -93,11 +103,16 @@ struct StackRun {
     MetalBuf *tok = nullptr, *want = nullptr;
     int *tok_host = nullptr, *want_host = nullptr;       // pinned; tok_host [B * max_seq], each portion in its own place
     MetalBuf *x = nullptr, *h = nullptr, *cin = nullptr, *cat = nullptr, *cout = nullptr;
-    MetalBuf *a16 = nullptr, *inv = nullptr;             // F16 operand of a product and its row factors
+    MetalBuf *a16 = nullptr, *inv = nullptr;             // F16 operand of a product and its row factors: the normed rows
+    MetalBuf *b16 = nullptr, *binv = nullptr;            // the same of every other product
     MetalBuf *aux = nullptr;                             // the mixer's intermediates
     MetalBuf *route_idx = nullptr, *route_w = nullptr, *act = nullptr, *ymoe = nullptr;
-    MetalBuf *moe = nullptr;                             // grouped experts: tables, operands and results
-    int T = 0, pending = 0;                              // tokens per sequence of the last step; its last layer's sum still waits in cout (1) and ymoe (2)
+    MetalBuf *moe_tab = nullptr, *moe_a16 = nullptr, *moe_inv = nullptr, *moe_up = nullptr, *moe_act = nullptr, *moe_y = nullptr;   // grouped experts
+    MetalBuf *lat_a16 = nullptr, *lat_inv = nullptr, *lat_kv = nullptr, *lat_frags = nullptr;   // prompt attention: expanded keys and values
+    int moe_rows = 0;                                    // rows those hold
+    int T = 0, pending = 0;                              // tokens per sequence of the last step; its last layer's sum still waits in cout (1) and ymoe (2) or moe_y (4, by `groups`)
+    MoeGroups groups{};
+    int groups_top = 0;
 };
 StackRun *stack_run_create(const LayerStack *st, int B);
 void stack_run_free(StackRun *r);
@@ -169,16 +184,26 @@ struct LatentRows {
     float *q;                                            // absorbed query [rows][H][w]
     float *part_o, *part_ml;                             // slices (scratch of the launch)
     float *o;                                            // [rows][H * vdim]
-    int f32; const void *uk, *uv; int ldu;               // weights and their row stride
+    int f32; const void *ukv; int ldu;                   // projections (keys, then values) and their row stride
 };
 void launch_latent_cache(const LatentRows &a);           // latent norm and key rotation into the ring
 void launch_latent_attend(const LatentRows &a);          // any number of rows, over the latents themselves
+
+// latent_prompt.hip: many rows of 16-bit precision with keys and values expanded once per step.  The step's visible keys
+// are positions first .. pos + T - 1; kv holds W_uk c | W_uv c of them, [B][n_keys][H * (dim + vdim)].
+bool latent_prompt_fits(const LatentRows &a);            // head sizes that kernel is built for, rows enough to pay
+int latent_prompt_first(const LatentRows &a);
+inline int latent_prompt_keys(const LatentRows &a) { return a.r.pos + a.r.T - latent_prompt_first(a); }
+size_t latent_prompt_frag_halfs(const LatentRows &a, int B, int n_keys);
+void launch_latent_operand(const LatentRows &a, half_t *a16, float *inv);        // the visible latents as a product's operand
+void launch_latent_prompt(const LatentRows &a, const float *kv, half_t *frags);
 
 void launch_rope_interleaved(float2 *tab, int max_seq, int dims, double base);
 
 // moe.hip
 struct MoeRows {
     int rows, E, top, ff, ffp, D, Dp, f32;
+    int up_rows, down_rows;                              // rows from one expert to the next
     const float *z; int ldz;                             // router logits
     int *idx; float *w;                                  // [rows][top]
     const float *h;                                      // [rows][Dp]
@@ -188,5 +213,14 @@ struct MoeRows {
 };
 void launch_route(const MoeRows &a);
 void launch_experts_per_row(const MoeRows &a);           // each row reads its own experts
+
+int moe_group_tiles(int rows, int top, int E);
+size_t moe_group_ints(int rows, int top, int E);
+MoeGroups moe_groups_at(int *base, int rows, int top, int E);
+void launch_moe_groups(const MoeRows &a, const MoeGroups &g);
+// rows of the tiled operand a16 (K columns, factors inv) gathered into the groups' order
+void launch_moe_gather(const MoeGroups &g, const half_t *a16, const float *inv, half_t *out16, float *out_inv, int K);
+// squared ReLU of [tiles * 128][ld] as the next product's operand of K columns (n of them real)
+void launch_moe_act(const MoeGroups &g, const float *up, int ld, int n, half_t *out16, float *out_inv, int K);
 
 }  // namespace lmhip

@@ -69,7 +69,7 @@ struct Loading {
     }
 };
 
-void load_delta(Loading &ld, StackLayer &L, const std::string &p, int rows_before)
+void load_delta(Loading &ld, StackLayer &L, const std::string &p)
 {
     const LayerConfig &c = L.c;
     const int D = ld.st->D, qd = c.kv_heads * c.dim, vd = c.heads * c.vdim;
@@ -78,7 +78,6 @@ void load_delta(Loading &ld, StackLayer &L, const std::string &p, int rows_befor
     ld.place(p + "b", c.heads, D, L.in, L.o_b);
     ld.place(p + (pc ? "a1" : "a"), pc ? L.rank_a : c.heads, D, L.in, L.o_a);
     ld.place(p + (pc ? "g1" : "g"), pc ? L.rank_g : vd, D, L.in, L.o_g);
-    (void)rows_before;
     if (pc) {
         L.a2 = ld.matrix(c.heads * c.dim, L.rank_a); ld.place(p + "a2", c.heads * c.dim, L.rank_a, L.a2);
         L.g2 = ld.matrix(vd, L.rank_g); ld.place(p + "g2", vd, L.rank_g, L.g2);
@@ -113,8 +112,9 @@ void load_latent(Loading &ld, StackLayer &L, const std::string &p)
     ld.place(p + "q", c.heads * (c.dim + c.rot_dim), D, L.in, L.o_q);
     ld.place(p + "dkv", c.kv_rank + c.rot_dim, D, L.in, L.o_dkv);
     L.g_c = ld.vector(p + "dkv.norm", c.kv_rank);
-    L.uk = ld.matrix(c.heads * c.dim, c.kv_rank); ld.place(p + "uk", c.heads * c.dim, c.kv_rank, L.uk);
-    L.uv = ld.matrix(c.heads * c.vdim, c.kv_rank); ld.place(p + "uv", c.heads * c.vdim, c.kv_rank, L.uv);
+    L.ukv = ld.matrix(c.heads * (c.dim + c.vdim), c.kv_rank);
+    ld.place(p + "uk", c.heads * c.dim, c.kv_rank, L.ukv);
+    ld.place(p + "uv", c.heads * c.vdim, c.kv_rank, L.ukv, c.heads * c.dim);
 }
 
 void load_layer(Loading &ld, StackLayer &L, int i)
@@ -141,7 +141,7 @@ void load_layer(Loading &ld, StackLayer &L, int i)
     L.hv = c.heads * c.vdim;
     L.o_sh = pad8(L.hv);
     L.out = ld.matrix(ld.st->Dp, L.o_sh + c.shared_ff);
-    if (L.delta()) load_delta(ld, L, mix, 0); else load_latent(ld, L, mix);
+    if (L.delta()) load_delta(ld, L, mix); else load_latent(ld, L, mix);
     ld.place(mix + "o", D, L.hv, L.out);
     if (!c.experts) return;
     ld.place(mlp + "router", c.experts, D, L.in, L.o_router);
@@ -149,12 +149,13 @@ void load_layer(Loading &ld, StackLayer &L, int i)
         ld.place(mlp + "shared.up", c.shared_ff, D, L.in, L.o_shared);
         ld.place(mlp + "shared.down", D, c.shared_ff, L.out, 0, L.o_sh);
     }
-    L.up = ld.matrix(c.experts * c.ff, D);
-    L.down = ld.matrix(c.experts * D, c.ff);
+    L.up_rows = (c.ff + 31) & ~31; L.down_rows = (ld.st->Dp + 31) & ~31;
+    L.up = ld.matrix(c.experts * L.up_rows, D);
+    L.down = ld.matrix(c.experts * L.down_rows, c.ff);
     for (int e = 0; e < c.experts && ld.ok; e++) {
         const std::string ex = mlp + "e" + std::to_string(e) + ".";
-        ld.place(ex + "up", c.ff, D, L.up, e * c.ff);
-        ld.place(ex + "down", D, c.ff, L.down, e * D);
+        ld.place(ex + "up", c.ff, D, L.up, e * L.up_rows);
+        ld.place(ex + "down", D, c.ff, L.down, e * L.down_rows);
     }
 }
 
@@ -200,7 +201,7 @@ void stack_free(LayerStack *st)
 {
     if (!st) return;
     for (StackLayer &L : st->layers)
-        for (MetalBuf *b : {L.g_norm, L.in.buf, L.out.buf, L.conv, L.a_exp, L.dt_bias, L.g_out, L.a2.buf, L.g2.buf, L.g_c, L.uk.buf, L.uv.buf,
+        for (MetalBuf *b : {L.g_norm, L.in.buf, L.out.buf, L.conv, L.a_exp, L.dt_bias, L.g_out, L.a2.buf, L.g2.buf, L.g_c, L.ukv.buf,
                             L.up.buf, L.down.buf}) metal_buf_free(b);
     for (MetalBuf *b : st->ropes) metal_buf_free(b);
     for (MetalBuf *b : {st->head.buf, st->g_final, st->emb}) metal_buf_free(b);
@@ -272,7 +273,8 @@ StackRun *stack_run_create(const LayerStack *st, int B)
     r->B = B;
     r->rows = std::max(1, std::min(PORTION_ROWS / B, st->max_seq)) * B;
     const int portion = r->rows / B;
-    size_t n_in = 0, ko = 0, aux = 0, act = 0, top = 0;
+    size_t n_in = 0, ko = 0, aux = 0, act = 0, top = 0, tab = 0;
+    int up_ld = 0, ffp = 0;
     int kmax = st->Dp;
     bool moe = false;
     for (const StackLayer &L : st->layers) {
@@ -291,6 +293,12 @@ StackRun *stack_run_create(const LayerStack *st, int B)
         }
         r->layers.push_back(k);
         n_in = std::max<size_t>(n_in, L.in.rows); ko = std::max<size_t>(ko, L.out.cols); aux = std::max(aux, a.at);
+        if (c.experts) {
+            const int tiles = moe_group_tiles(r->rows, c.top, c.experts);
+            r->moe_rows = std::max(r->moe_rows, tiles * 128);
+            tab = std::max(tab, moe_group_ints(r->rows, c.top, c.experts));
+            up_ld = std::max(up_ld, L.up_rows); ffp = std::max(ffp, L.down.cols);
+        }
         if (c.experts) { moe = true; top = std::max<size_t>(top, c.top); act = std::max<size_t>(act, (size_t)c.top * pad8(c.ff)); }
     }
     kmax = std::max<int>(kmax, (int)ko);
@@ -305,14 +313,24 @@ StackRun *stack_run_create(const LayerStack *st, int B)
     r->h = fbuf((size_t)std::max(r->rows, STACK_WANT) * st->Dp);
     if (st->f32) r->cat = fbuf((size_t)r->rows * ko);
     else {
-        r->a16 = metal_buf_create(tiled_elems(std::max(r->rows, STACK_WANT), kmax) * sizeof(half_t));
+        r->a16 = metal_buf_create(tiled_elems(std::max(r->rows, STACK_WANT), st->Dp) * sizeof(half_t));
+        r->b16 = metal_buf_create(tiled_elems(r->rows, kmax) * sizeof(half_t));
         r->inv = fbuf(std::max(r->rows, STACK_WANT));
+        r->binv = fbuf(r->rows);
     }
     if (moe) {
         r->route_idx = metal_buf_create((size_t)r->rows * top * sizeof(int));
         r->route_w = fbuf((size_t)r->rows * top);
         r->act = fbuf((size_t)r->rows * act);
         r->ymoe = fbuf((size_t)r->rows * st->Dp);
+        if (!st->f32) {
+            r->moe_tab = metal_buf_create(tab * sizeof(int));
+            r->moe_a16 = metal_buf_create(tiled_elems(r->moe_rows, st->Dp) * sizeof(half_t));
+            r->moe_inv = fbuf((size_t)2 * r->moe_rows);   // of the gathered rows | of the activations
+            r->moe_up = fbuf((size_t)r->moe_rows * up_ld);
+            r->moe_act = metal_buf_create(tiled_elems(r->moe_rows, ffp) * sizeof(half_t));
+            r->moe_y = fbuf((size_t)r->moe_rows * st->Dp);
+        }
     }
     return r;
 }
@@ -321,7 +339,8 @@ void stack_run_free(StackRun *r)
 {
     if (!r) return;
     for (StackRun::Layer &k : r->layers) for (MetalBuf *b : {k.S, k.conv, k.ring}) metal_buf_free(b);
-    for (MetalBuf *b : {r->tok, r->want, r->x, r->h, r->cin, r->cat, r->cout, r->a16, r->inv, r->aux, r->route_idx, r->route_w, r->act, r->ymoe, r->moe})
+    for (MetalBuf *b : {r->tok, r->want, r->x, r->h, r->cin, r->cat, r->cout, r->a16, r->inv, r->b16, r->binv, r->aux, r->route_idx, r->route_w, r->act, r->ymoe,
+                        r->moe_tab, r->moe_a16, r->moe_inv, r->moe_up, r->moe_act, r->moe_y, r->lat_a16, r->lat_inv, r->lat_kv, r->lat_frags})
         metal_buf_free(b);
     if (r->tok_host) hipHostFree(r->tok_host);
     if (r->want_host) hipHostFree(r->want_host);
@@ -343,6 +362,7 @@ void norm(LayerStack *st, StackRun *r, MetalBuf *g, int rows, int keep, bool nee
     n.x = ptr<float>(r->x);
     if (r->pending & 1) n.cout = ptr<float>(r->cout);
     if (r->pending & 2) n.ymoe = ptr<float>(r->ymoe);
+    if (r->pending & 4) { n.moe_y = ptr<float>(r->moe_y); n.moe_pos = r->groups.pos; n.route_w = ptr<float>(r->route_w); n.top = r->groups_top; }
     n.g = ptr<float>(g); n.a16 = ptr<half_t>(r->a16); n.inv = ptr<float>(r->inv); n.h = need_h || st->f32 ? ptr<float>(r->h) : nullptr;
     n.want = want; n.step = step; n.first = first; n.D = st->D; n.Dp = st->Dp; n.keep = keep; n.eps = st->cfg.eps;
     launch_norm_rows(n, rows);
@@ -358,8 +378,8 @@ float *mix_delta(LayerStack *st, StackRun *r, StackLayer &L, StackRun::Layer &k,
     const float *cin = ptr<float>(r->cin);
     if (pc) {                                             // the second halves of the two low-rank products
         auto low_rank = [&](const StackMat &w, int col, float *out) {
-            if (!st->f32) launch_rows_to_f16(cin + col, ldc, ptr<half_t>(r->a16), ptr<float>(r->inv), n, w.cols);
-            product(st, w, ptr<half_t>(r->a16), ptr<float>(r->inv), cin + col, ldc, out, n);
+            if (!st->f32) launch_rows_to_f16(cin + col, ldc, ptr<half_t>(r->b16), ptr<float>(r->binv), n, w.cols);
+            product(st, w, ptr<half_t>(r->b16), ptr<float>(r->binv), cin + col, ldc, out, n);
         };
         low_rank(L.a2, L.o_a, d.a2);
         low_rank(L.g2, L.o_g, d.g2);
@@ -387,9 +407,18 @@ float *mix_latent(LayerStack *st, StackRun *r, StackLayer &L, StackRun::Layer &k
     a.ring_rows = k.ring_rows; a.rot_dims = c.rot_dims; a.scale = c.scale; a.eps = st->cfg.eps;
     a.cin = ptr<float>(r->cin); a.ldc = L.in.rows; a.o_q = L.o_q; a.o_dkv = L.o_dkv;
     a.g_c = ptr<float>(L.g_c); a.rope = ptr<float2>(L.rope); a.ring = ptr<float>(k.ring);
-    a.q = d.q; a.o = d.o; a.f32 = st->f32; a.uk = dptr(L.uk.buf); a.uv = dptr(L.uv.buf); a.ldu = L.uk.cols;
+    a.q = d.q; a.o = d.o; a.f32 = st->f32; a.ukv = dptr(L.ukv.buf); a.ldu = L.ukv.cols;
     launch_latent_cache(a);
-    launch_latent_attend(a);
+    if (!latent_prompt_fits(a)) { launch_latent_attend(a); return d.o; }
+    const int nk = latent_prompt_keys(a), most = k.ring_rows;            // grown to what any step of this layer needs
+    auto room = [&](MetalBuf *&b, size_t bytes) { if (!b || b->size < bytes) { metal_buf_free(b); b = metal_buf_create(bytes); } };
+    room(r->lat_a16, tiled_elems(r->B * most, c.kv_rank) * sizeof(half_t));
+    room(r->lat_inv, (size_t)r->B * most * sizeof(float));
+    room(r->lat_kv, (size_t)r->B * most * L.ukv.rows * sizeof(float));
+    room(r->lat_frags, latent_prompt_frag_halfs(a, r->B, most) * sizeof(half_t));
+    launch_latent_operand(a, ptr<half_t>(r->lat_a16), ptr<float>(r->lat_inv));
+    product(st, L.ukv, ptr<half_t>(r->lat_a16), ptr<float>(r->lat_inv), nullptr, 0, ptr<float>(r->lat_kv), r->B * nk);
+    launch_latent_prompt(a, ptr<float>(r->lat_kv), ptr<half_t>(r->lat_frags));
     return d.o;
 }
 
@@ -409,24 +438,38 @@ void stack_forward(LayerStack *st, StackRun *r, const int *tokens, int T, int po
     for (size_t i = 0; i < st->layers.size(); i++) {
         StackLayer &L = st->layers[i];
         const LayerConfig &c = L.c;
-        norm(st, r, L.g_norm, n, 1, c.experts > 0);
+        // from a few rows per expert on, each expert's weights are read once for all its rows
+        const bool grouped = c.experts && !st->f32 && n >= 16 && n * c.top >= c.experts;
+        norm(st, r, L.g_norm, n, 1, c.experts && !grouped);
         product(st, L.in, ptr<half_t>(r->a16), ptr<float>(r->inv), ptr<float>(r->h), st->Dp, ptr<float>(r->cin), n);
         CatRows cat{};
         cat.o = L.delta() ? mix_delta(st, r, L, r->layers[i], rows, cat) : mix_latent(st, r, L, r->layers[i], rows);
         cat.H = c.heads; cat.vdim = c.vdim; cat.eps = st->cfg.eps;
         cat.shared = ptr<float>(r->cin) + L.o_shared; cat.ld_shared = L.in.rows; cat.shared_ff = c.shared_ff; cat.o_sh = L.o_sh;
-        cat.cat = ptr<float>(r->cat); cat.a16 = ptr<half_t>(r->a16); cat.inv = ptr<float>(r->inv); cat.ldk = L.out.cols;
+        cat.cat = ptr<float>(r->cat); cat.a16 = ptr<half_t>(r->b16); cat.inv = ptr<float>(r->binv); cat.ldk = L.out.cols;
         launch_cat_rows(cat, n);
         product(st, L.out, cat.a16, cat.inv, cat.cat, cat.ldk, ptr<float>(r->cout), n);
         r->pending = 1;
         if (!c.experts) continue;
         MoeRows m{};
         m.rows = n; m.E = c.experts; m.top = c.top; m.ff = c.ff; m.ffp = L.down.cols; m.D = st->D; m.Dp = st->Dp; m.f32 = st->f32;
+        m.up_rows = L.up_rows; m.down_rows = L.down_rows;
         m.z = ptr<float>(r->cin) + L.o_router; m.ldz = L.in.rows; m.idx = ptr<int>(r->route_idx); m.w = ptr<float>(r->route_w);
         m.h = ptr<float>(r->h); m.up = dptr(L.up.buf); m.down = dptr(L.down.buf); m.act = ptr<float>(r->act); m.y = ptr<float>(r->ymoe);
         launch_route(m);
-        launch_experts_per_row(m);
-        r->pending = 3;
+        if (!grouped) { launch_experts_per_row(m); r->pending = 3; continue; }
+        const MoeGroups g = moe_groups_at(ptr<int>(r->moe_tab), n, c.top, c.experts);
+        const int M = g.tiles * 128;
+        float *up = ptr<float>(r->moe_up), *inv = ptr<float>(r->moe_inv), *inv_act = inv + r->moe_rows;
+        half_t *rows16 = ptr<half_t>(r->moe_a16), *act16 = ptr<half_t>(r->moe_act);
+        launch_moe_groups(m, g);
+        launch_moe_gather(g, ptr<half_t>(r->a16), ptr<float>(r->inv), rows16, inv, st->Dp);
+        launch_gemm_groups(rows16, inv, tiled_weight_of(L.up.buf, L.up.rows, L.up.cols), tiled_elems(L.up_rows, L.up.cols), g.of, up, L.up_rows,
+                           M, c.ff, L.up.cols, c.experts);
+        launch_moe_act(g, up, L.up_rows, c.ff, act16, inv_act, m.ffp);
+        launch_gemm_groups(act16, inv_act, tiled_weight_of(L.down.buf, L.down.rows, L.down.cols), tiled_elems(L.down_rows, L.down.cols), g.of,
+                           ptr<float>(r->moe_y), st->Dp, M, st->Dp, L.down.cols, c.experts);
+        r->pending = 5; r->groups = g; r->groups_top = c.top;
     }
 }
 
