@@ -215,6 +215,69 @@ def decode_bench(args, cfg, L):
     emit(out)
 
 
+def nevurax_bench(args, L):
+    """Prompt and decoding throughput of Nevurax models (random weights), each beside the Qwen3 shape of the same width: its
+    greedy decoding, and as its many-row pass the training state's forward over as many rows (generation takes Qwen3 prompts
+    token by token).  One JSON line for all sizes."""
+    import tempfile
+    from llm_metal_amd.configs import NEVURAX_SIZES, qwen3_beside
+    from llm_metal_amd.sft import InferenceState, SFTState
+    from llm_metal_amd.synth import write_stack_checkpoint
+    rows, rng = args.nevurax_prompt, np.random.default_rng(5)
+    out = []
+    for size in args.nevurax.split(","):
+        cfg = NEVURAX_SIZES[size]
+        toks = rng.integers(0, cfg["vocab"], rows)
+
+        def decode_ms(inf, tok):
+            for _ in range(args.warmup):
+                tok = inf.forward_token_argmax(tok)
+            t0 = time.perf_counter()
+            for _ in range(args.steps):
+                tok = inf.forward_token_argmax(tok)
+            return (time.perf_counter() - t0) / args.steps * 1e3
+
+        max_seq = rows + args.warmup + args.steps + 8
+        with tempfile.TemporaryDirectory() as d:
+            write_stack_checkpoint(d, cfg, seed=1, rank_a=128, rank_g=128, repeat=True)
+            inf = InferenceState(path=d, model_type=None, max_seq=max_seq)
+        res = {"size": size, "width": cfg["width"], "layers": len(cfg["layers"]), "prompt_rows": rows}
+        best = []
+        for i in range(2 + args.warmup):
+            inf.reset()
+            t0 = time.perf_counter()
+            inf.forward_tokens(toks, [rows - 1])
+            best.append((time.perf_counter() - t0) * 1e3)
+        res["prompt_ms"] = round(min(best[1:]), 3)
+        res["prompt_tokens_per_s"] = round(rows / res["prompt_ms"] * 1e3)
+        res["decode_ms"] = round(decode_ms(inf, 1), 4)
+        res["decode_tokens_per_s"] = round(1e3 / res["decode_ms"], 1)
+        inf.free()
+        if not args.nevurax_alone:
+            q = qwen3_beside(cfg)
+            model = make_model(q, seed=0, lora_b_std=0.0)
+            inf = InferenceState(q, model, max_seq=max_seq)
+            for t in toks[:args.nevurax_context]:
+                tok = inf.forward_token_argmax(int(t))
+            ref = {"ffn_width": q.IS, "decode_ms": round(decode_ms(inf, tok), 4)}
+            inf.free()
+            with SFTState(q.with_(batch=1, seq=rows), model) as st:
+                st.x_cpu()[:] = model["token_emb"][toks]
+                best = []
+                for i in range(2 + args.warmup):
+                    L.metal_flush()
+                    t0 = time.perf_counter()
+                    st.forward_to_logits()
+                    L.metal_flush()
+                    best.append((time.perf_counter() - t0) * 1e3)
+            ref["forward_ms"] = round(min(best[1:]), 3)
+            del model
+            res["qwen3"] = ref
+        out.append(res)
+    emit({"metric": "Nevurax prompt and greedy decode tokens/s", "unit": "tokens/s", "n_gpus": 1, "data": "synthetic", "steps": args.steps,
+          "dtype": "f16 weights, f32 accumulate", "sizes": out})
+
+
 class _LibraryStdoutToStderr:
     """The library reports like the reference does, with printf on stdout ("[FastSFT] Grad accum buffers allocated ...").
     While this is active, file descriptor 1 is stderr, so that the one JSON line is all this program writes to stdout."""
@@ -286,6 +349,11 @@ def _main():
                     help="with --decode: a generation state made from a training state (inference_state_create_from_sft)")
     ap.add_argument("--decode-batch", type=int, default=0,
                     help="with --decode: also time this many copies of one prompt decoded in lock step")
+    ap.add_argument("--nevurax", nargs="?", const="1k,2k,4k", default=None, metavar="SIZES",
+                    help="time prompts and decoding of Nevurax models of these sizes (1k,2k,4k) beside a Qwen3 shape of equal size")
+    ap.add_argument("--nevurax-prompt", type=int, default=2048, help="with --nevurax: tokens of the prompt")
+    ap.add_argument("--nevurax-context", type=int, default=256, help="with --nevurax: tokens before the Qwen3 shape's timed decoding")
+    ap.add_argument("--nevurax-alone", action="store_true", help="with --nevurax: without the Qwen3 shape")
     ap.add_argument("--gemm-shapes", action="store_true",
                     help="time every product shape of the configuration alone, with cold weights: the weight loads only, gemm_ring, gemm_tiled")
     ap.add_argument("--copy-calibration", action="store_true",
@@ -293,9 +361,9 @@ def _main():
                          "the known-size reference for scaling FETCH_SIZE / WRITE_SIZE counters")
     args = ap.parse_args()
     if args.steps is None:
-        args.steps = 20 if args.decode else 200
+        args.steps = 20 if args.decode or args.nevurax else 200
     if args.warmup is None:
-        args.warmup = 3 if args.decode else 20
+        args.warmup = 3 if args.decode or args.nevurax else 20
     if args.gpus != 1:
         print("bench.py: this build runs on one GPU only (the step has no multi-GPU path); use --gpus 1",
               file=sys.stderr)
@@ -323,6 +391,8 @@ def _main():
                                    "bytes_written_per_launch": 4 * n, "launches": 5}})
         return
 
+    if args.nevurax:
+        return nevurax_bench(args, L)
     if args.decode:
         return decode_bench(args, cfg, L)
     if args.gemm_shapes:

@@ -78,3 +78,31 @@ C3Q = C3.with_(name="c3_qwen3_4b_q8_seq64", weight_format="q8_0")
 TINY_GEMMA3 = SFTConfig("tiny_gemma3", GEMMA3, NL=7, D=128, Hq=4, Hkv=1, hd=32, IS=384, V=2048, tied=True, seq=32)
 
 CONFIGS = {c.name: c for c in (C1, C2, C3, C4, C5, C3Q, TINY_GEMMA3)}
+
+
+def nevurax_config(width, heads, ff, experts, top, shared_ff, vocab=32768, head_dim=128, rot_dim=64, kv_rank=512, window=1024,
+                   order=("channel_delta", "latent_attention", "delta", "channel_delta")):
+    """config.json of a Nevurax model with layers of a real model's proportions (one width of heads for all mixers)."""
+    mlp = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}, "shared": {"ff": shared_ff}}
+    rule = {"heads": heads, "kv_heads": heads, "dim": head_dim, "vdim": head_dim, "conv": 4}
+    latent = {"heads": heads, "dim": head_dim, "rot_dim": rot_dim, "vdim": head_dim, "kv_rank": kv_rank, "mask": {"size": window},
+              "rot": {"base": 1e4, "dims": rot_dim}, "scale": (head_dim + rot_dim) ** -0.5}
+    return {"architecture": "Nevurax", "vocab": vocab, "width": width, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-6},
+            "layers": [{"type": t, "mixer": latent if t == "latent_attention" else rule, "mlp": mlp} for t in order]}
+
+
+# benchmark sizes: four layers each, beside a Qwen3-shaped model of the same width, heads and active FFN weights per token
+NEVURAX_SIZES = {
+    "1k": nevurax_config(1024, 8, 512, 32, 4, 1024),
+    "2k": nevurax_config(2048, 16, 768, 64, 6, 1536),
+    "4k": nevurax_config(4096, 32, 1024, 32, 8, 2048),
+}
+
+
+def qwen3_beside(cfg):
+    """The Qwen3 shape with a Nevurax configuration's width, layers, heads and feed-forward weights per token."""
+    L = cfg["layers"][0]["mlp"]
+    active = 2 * (L["router"]["top"] * L["expert"]["ff"] + L["shared"]["ff"])
+    heads = cfg["layers"][0]["mixer"]["heads"]
+    return SFTConfig("qwen3_beside_nevurax", QWEN3, NL=len(cfg["layers"]), D=cfg["width"], Hq=heads, Hkv=max(1, heads // 4),
+                     hd=cfg["layers"][0]["mixer"]["dim"], IS=active // 3 // 64 * 64, V=cfg["vocab"])

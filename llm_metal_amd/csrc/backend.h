@@ -68,9 +68,12 @@ struct NormIn {
     const float *xr, *br, *g;
     float *x_out;
     float eps;
+    int dim;                             // layer norm only: entries of xr that count
 };
 // infer_kernels.hip: y = W . RMSNorm(xr + br; g) (glu 0), or the gated pair product of matvec_glu over it (1 SiLU, 2 GELU)
 void matvec_norm(MetalBuf *W, const NormIn &nin, MetalBuf *y, int rows, int cols, int q8, int glu);
+// infer_kernels.hip: y = W . LayerNorm(x; g) over the first dim of cols entries (F16 rows)
+void matvec_layernorm(MetalBuf *W, const float *x, const float *g, int dim, float eps, float *y, int rows, int cols);
 
 }  // namespace lmhip
 

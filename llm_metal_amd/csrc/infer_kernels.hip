@@ -96,7 +96,8 @@ const int8_t *q8_split_of(MetalBuf *W, int rows, int nb, const half_t **scales)
 // NORM (with XLDS): the vector is RMSNorm(v; g) of v = xr + br (br may be null), which every workgroup forms for itself
 // while its first weights are on their way: v g goes to LDS, the sum of squares through one block reduction, and the
 // factor rsqrt(mean + eps) onto the finished sums; workgroup 0 also writes v to x_out (not xr: the others still read it).
-// residual_add + rms_norm of shaders/q8_kernels.metal:133-158, 369-375 without a launch of their own.
+// residual_add + rms_norm of shaders/q8_kernels.metal:133-158, 369-375 without a launch of their own.  NORM 2: a layer norm
+// of the first `dim` entries of xr instead (mean taken off, no branch, the padding behind them zero).
 // REPS (NORM only): row groups a wave takes one after the other, so that fewer workgroups form the vector.
 template <int FMT, int R, int U, int XLDS, int GLU = 0, int NORM = 0, int REPS = 1>
 __global__ __launch_bounds__(TB) void k_matvec(const void *__restrict__ Wp, const half_t *__restrict__ scales,
@@ -112,7 +113,7 @@ __global__ __launch_bounds__(TB) void k_matvec(const void *__restrict__ Wp, cons
         float   dsc[FMT == 1 ? R : 1][U];
         float4v x0[XLDS ? 1 : U], x1[XLDS ? 1 : U];
     };
-    static_assert(REPS == 1 || NORM == 1, "row groups in turn only where the vector is formed in the kernel");
+    static_assert(REPS == 1 || NORM != 0, "row groups in turn only where the vector is formed in the kernel");
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     int row0 = ((blockIdx.x * REPS) * 4 + wave) * (GLU ? 1 : R);
     size_t roff[R];                                             // element offset of each row (clamped: extra rows are not stored)
@@ -184,7 +185,24 @@ __global__ __launch_bounds__(TB) void k_matvec(const void *__restrict__ Wp, cons
     Stage cur;
     load(cur, lane * 8);
     float norm_inv = 1.f;
-    if (NORM) {
+    if (NORM == 2) {
+        float sum = 0.f;
+        for (int i = tid * 4; i < cols; i += TB * 4) {
+            const float4v v = *reinterpret_cast<const float4v *>(&nin.xr[i]);
+            sum += (v[0] + v[1]) + (v[2] + v[3]);
+            *reinterpret_cast<float4v *>(&xs[i]) = v;
+        }
+        const float mean = block_sum(sum, red) / (float)nin.dim;
+        float ss = 0.f;
+        for (int i = tid * 4; i < cols; i += TB * 4) {          // the thread's own entries
+            float4v v = *reinterpret_cast<const float4v *>(&xs[i]);
+            const float4v gg = *reinterpret_cast<const float4v *>(&nin.g[i]);
+#pragma unroll
+            for (int e = 0; e < 4; e++) { v[e] = i + e < nin.dim ? v[e] - mean : 0.f; ss += v[e] * v[e]; }
+            *reinterpret_cast<float4v *>(&xs[i]) = v * gg;
+        }
+        norm_inv = 1.f / sqrtf(block_sum(ss, red) / (float)nin.dim + nin.eps);
+    } else if (NORM) {
         float ss = 0.f;
         for (int i0 = tid * 4; i0 < cols; i0 += TB * 16) {      // four groups of a thread requested together
             float4v v[4], b[4], gg[4];
@@ -925,6 +943,27 @@ void matvec_glu(MetalBuf *W, MetalBuf *x, MetalBuf *y, int rows, int cols, int q
         launch_matvec_glu<0>(dptr(W), nullptr, dptr_as<float>(x), dptr_as<float>(y), rows, cols, gelu);
     }
     mark_written(y);
+}
+
+// y = W . LayerNorm(x; g), the norm of the first `dim` entries formed inside the launch (F16 rows of `cols` columns)
+void matvec_layernorm(MetalBuf *W, const float *x, const float *g, int dim, float eps, float *y, int rows, int cols)
+{
+    if (rows <= 0 || dim <= 0 || dim > cols || (cols & 7) || cols > 15360 || !aligned16(dptr(W)) || !x || !g || !aligned16(x) || !aligned16(g)) {
+        fprintf(stderr, "[fast_hip] matvec_layernorm: unsupported shape %d x %d or operands\n", rows, cols); abort();
+    }
+    REQUIRE_BYTES(W, (size_t)rows * cols * 2, "matvec_layernorm");
+    const NormIn nin{x, nullptr, g, nullptr, eps, dim};
+    hipEvent_t ev_a = nullptr, ev_b = nullptr;
+    const bool prof = gemm_prof_begin(2.0 * rows * cols, 2.0 * rows * cols, &ev_a, &ev_b);
+    const size_t lds = (size_t)cols * 4;
+    const half_t *scales = nullptr;
+#define LN_LAUNCH(REPS_) do { \
+    const dim3 grid((rows + 8 * REPS_ - 1) / (8 * REPS_)); \
+    if (prof) hipExtLaunchKernelGGL((k_matvec<0, 2, 2, 1, 0, 2, REPS_>), grid, dim3(TB), lds, stream(), ev_a, ev_b, 0, dptr(W), scales, nullptr, y, rows, cols, nin); \
+    else hipLaunchKernelGGL((k_matvec<0, 2, 2, 1, 0, 2, REPS_>), grid, dim3(TB), lds, stream(), dptr(W), scales, nullptr, y, rows, cols, nin); \
+    HIP_CHECK(hipGetLastError()); } while (0)
+    if (rows >= 16384) LN_LAUNCH(4); else LN_LAUNCH(1);      // many rows: fewer workgroups form the vector
+#undef LN_LAUNCH
 }
 
 // The same products (glu 0: y[i] = W_i . ln for `rows` rows) over ln = RMSNorm(xr + br; g), the sum and the norm formed

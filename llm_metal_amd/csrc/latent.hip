@@ -2,7 +2,7 @@
 // projection is moved to the query (q_u . W_uk c = (W_uk^T q_u) . c) and the value projection behind the weighted sum,
 // so a key row is read once for several heads and never expanded.  Scores, weights and sums are fp32.
 #include "stack.h"
-#include "rows.h"
+#include "latent_rows.h"
 #include <algorithm>
 
 namespace lmhip {
@@ -12,7 +12,6 @@ namespace {
     hipLaunchKernelGGL(kern, grid, block, lds, stream(), __VA_ARGS__); HIP_CHECK(hipGetLastError()); } while (0)
 
 constexpr int HG = 4;        // heads that share the reading of a key row
-constexpr int SLK = 64;      // keys per workgroup
 
 __global__ __launch_bounds__(256) void k_rope_interleaved(float2 *tab, int n, int pairs, int dims, double base)
 {
@@ -22,57 +21,24 @@ __global__ __launch_bounds__(256) void k_rope_interleaved(float2 *tab, int n, in
     tab[i] = make_float2((float)cos(angle), (float)sin(angle));
 }
 
-// element i of a rotated vector: pairs (2p, 2p + 1) of the first `dims` turn, the rest passes
-__device__ __forceinline__ float rotated(const float *x, int i, int dims, const float2 *cs)
-{
-    if (i >= dims) return x[i];
-    const float2 c = cs[i >> 1];
-    return (i & 1) ? x[i] * c.x + x[i - 1] * c.y : x[i] * c.x - x[i + 1] * c.y;
-}
-
-// widths of a ring row / an absorbed query: latent part and rotated part, each padded to 8 with zeros
-__device__ __forceinline__ int rank_pad(const LatentRows &a) { return (a.rank + 7) & ~7; }
-__device__ __forceinline__ int row_width(const LatentRows &a) { return rank_pad(a) + ((a.rot + 7) & ~7); }
-
-// grid (rows): the row's latent and key part into the ring
+// grid (rows)
 __global__ __launch_bounds__(256) void k_latent_cache(LatentRows a)
 {
     __shared__ float sm[16];
-    const int m = blockIdx.x, b = m / a.r.T, p = a.r.pos + m % a.r.T, tid = threadIdx.x;
-    const int rp = rank_pad(a), w = row_width(a);
-    const float *c = a.cin + (size_t)m * a.ldc + a.o_dkv, *k = c + a.rank;
-    float *dst = a.ring + ((size_t)b * a.ring_rows + p % a.ring_rows) * w;
-    const float2 *cs = a.rope + (size_t)p * (a.rot_dims / 2);
-    float ss = 0.f;
-    for (int i = tid; i < a.rank; i += 256) ss += c[i] * c[i];
-    const float inv = 1.f / sqrtf(block_sum(ss, sm) / (float)a.rank + a.eps);
-    for (int i = tid; i < w; i += 256)
-        dst[i] = i < rp ? (i < a.rank ? c[i] * inv * a.g_c[i] : 0.f) : (i - rp < a.rot ? rotated(k, i - rp, a.rot_dims, cs) : 0.f);
+    latent_cache_row(a, blockIdx.x, sm);
 }
 
-// grid (H, rows): the query moved into the latent space, and its rotated part behind it
+// grid (H, rows)
 template <typename WT>
 __global__ __launch_bounds__(256) void k_latent_query(LatentRows a, int m0)
 {
-    extern __shared__ float qs[];                         // [dim]
-    const int h = blockIdx.x, m = m0 + blockIdx.y, p = a.r.pos + m % a.r.T, tid = threadIdx.x;
-    const int rp = rank_pad(a), w = row_width(a);
-    const float *q = a.cin + (size_t)m * a.ldc + a.o_q + h * (a.dim + a.rot);
-    for (int i = tid; i < a.dim; i += 256) qs[i] = q[i];
-    __syncthreads();
-    float *out = a.q + ((size_t)m * a.H + h) * w;
-    const WT *uk = (const WT *)a.ukv + (size_t)h * a.dim * a.ldu;
-    for (int c = tid; c < rp; c += 256) {                 // the weight's padding columns are zero
-        float s = 0.f;
-        for (int d = 0; d < a.dim; d++) s = fmaf((float)uk[(size_t)d * a.ldu + c], qs[d], s);
-        out[c] = s;
-    }
-    const float2 *cs = a.rope + (size_t)p * (a.rot_dims / 2);
-    for (int i = tid; i < w - rp; i += 256) out[rp + i] = i < a.rot ? rotated(q + a.dim, i, a.rot_dims, cs) : 0.f;
+    extern __shared__ float lds[];
+    latent_query_row<WT>(a, m0 + blockIdx.y, blockIdx.x, lds);
 }
 
-// grid (slices, ceil(H / HG), rows): softmax statistics and weighted latent sum of HG heads over one slice of the
+// SLK (up to 64): keys per workgroup.  grid (slices, ceil(H / HG), rows): softmax statistics and weighted latent sum of HG heads over one slice of the
 // row's visible keys.  LDS: queries [HG][w], scores [HG][SLK], partial sums [parts][HG][rp]
+template <int SLK>
 __global__ __launch_bounds__(256) void k_latent_attend(LatentRows a, int m0, int nsplit)
 {
     extern __shared__ float lds[];
@@ -111,7 +77,7 @@ __global__ __launch_bounds__(256) void k_latent_attend(LatentRows a, int m0, int
     __syncthreads();
     if (wave < HG) {                                      // one wave per head
         const float s = lane < nj ? sc[wave * SLK + lane] : -3.0e38f, mx = wave_max(s), e = lane < nj ? expf(s - mx) : 0.f, l = wave_sum(e);
-        sc[wave * SLK + lane] = e;
+        if (lane < SLK) sc[wave * SLK + lane] = e;
         if (lane == 0 && h0 + wave < a.H) { float *ml = a.part_ml + (slot0 + (size_t)wave * nsplit) * 2; ml[0] = mx; ml[1] = l; }
     }
     __syncthreads();
@@ -141,38 +107,37 @@ __global__ __launch_bounds__(256) void k_latent_attend(LatentRows a, int m0, int
     }
 }
 
-// grid (H, rows): the slices of one head merged, then the value projection
+// grid (H, rows, ceil(vdim / VR)): the slices of one head merged, then VR rows of the value projection
+constexpr int VR = 16;
 template <typename WT>
 __global__ __launch_bounds__(256) void k_latent_values(LatentRows a, int m0, int nsplit)
 {
-    extern __shared__ float ctx[];                        // [rp]
+    extern __shared__ float ctx[];                        // [rp], then the slices' factors [nsplit]
     const int h = blockIdx.x, m = m0 + blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, rp = rank_pad(a);
+    float *fac = ctx + rp;
     const size_t slot0 = ((size_t)(m - m0) * a.H + h) * nsplit;
     const float *ml = a.part_ml + slot0 * 2;
-    float mx = -3.0e38f, l = 0.f;
-    for (int s = 0; s < nsplit; s++) mx = fmaxf(mx, ml[2 * s]);
-    for (int s = 0; s < nsplit; s++) l = fmaf(ml[2 * s + 1], expf(ml[2 * s] - mx), l);
+    float mx = -3.0e38f;
+    for (int s = lane; s < nsplit; s += 64) mx = fmaxf(mx, ml[2 * s]);
+    mx = wave_max(mx);
+    float l = 0.f;
+    for (int s = lane; s < nsplit; s += 64) l += ml[2 * s + 1] > 0.f ? ml[2 * s + 1] * expf(ml[2 * s] - mx) : 0.f;
+    l = wave_total(l);
+    for (int s = tid; s < nsplit; s += 256) fac[s] = ml[2 * s + 1] > 0.f ? expf(ml[2 * s] - mx) / l : 0.f;
+    __syncthreads();
     for (int c = tid; c < rp; c += 256) {
         float o = 0.f;
-        for (int s = 0; s < nsplit; s++)
-            if (ml[2 * s + 1] > 0.f) o = fmaf(a.part_o[(slot0 + s) * rp + c], expf(ml[2 * s] - mx), o);
-        ctx[c] = o / l;
+#pragma unroll 8
+        for (int s = 0; s < nsplit; s++)                  // (a slice without keys has left nothing to read)
+            if (fac[s] > 0.f) o = fmaf(a.part_o[(slot0 + s) * rp + c], fac[s], o);
+        ctx[c] = o;
     }
     __syncthreads();
-    for (int i = wave; i < a.vdim; i += 4) {
+    for (int i = blockIdx.z * VR + wave; i < min(a.vdim, (int)(blockIdx.z + 1) * VR); i += 4) {
         const WT *uv = (const WT *)a.ukv + ((size_t)a.H * a.dim + (size_t)h * a.vdim + i) * a.ldu;
-        float s = 0.f;
-        for (int c = lane; c < rp; c += 64) s = fmaf((float)uv[c], ctx[c], s);
-        s = wave_sum(s);
+        const float s = wave_sum(dot_part(uv, ctx, rp, lane));
         if (lane == 0) a.o[((size_t)m * a.H + h) * a.vdim + i] = s;
     }
-}
-
-int slices_of(const LatentRows &a) { return (std::min(a.window, a.r.pos + a.r.T) + SLK - 1) / SLK; }
-int rows_per_launch(const LatentRows &a)
-{
-    const size_t per_row = (size_t)a.H * slices_of(a) * (size_t)pad8(a.rank);
-    return (int)std::max<size_t>(1, std::min<size_t>((size_t)a.r.n(), ((size_t)32 << 20) / per_row));
 }
 
 }  // namespace
@@ -185,22 +150,46 @@ void launch_rope_interleaved(float2 *tab, int max_seq, int dims, double base)
 
 void launch_latent_cache(const LatentRows &a) { LAUNCH(k_latent_cache, dim3(a.r.n()), dim3(256), 0, a); }
 
+LatentSlices latent_slices(const LatentRows &a)
+{
+    LatentSlices s;
+    s.keys = a.r.T == 1 ? 32 : 64;                        // decoding: more workgroups on fewer keys each
+    s.n = (std::min(a.window, a.r.pos + a.r.T) + s.keys - 1) / s.keys;
+    const size_t per_row = (size_t)a.H * s.n * (size_t)pad8(a.rank);
+    s.rows = (int)std::max<size_t>(1, std::min<size_t>((size_t)a.r.n(), ((size_t)32 << 20) / per_row));
+    return s;
+}
+
+// what the slices of `rows` rows leave for the value kernel
+void latent_partials(LatentRows &a, const LatentSlices &s)
+{
+    const size_t po = (size_t)s.rows * a.H * s.n * pad8(a.rank), pml = (size_t)s.rows * a.H * s.n * 2;
+    a.part_o = (float *)scratch(SCR_PARTIAL, (po + pml) * sizeof(float));
+    a.part_ml = a.part_o + po;
+}
+
+void launch_latent_slices(const LatentRows &a, const LatentSlices &s, int m0, int nr)
+{
+    const int rp = pad8(a.rank), w = rp + pad8(a.rot), parts = std::max(1, 256 / (rp / 4));
+    const size_t lds = ((size_t)HG * w + (size_t)HG * s.keys + (size_t)parts * HG * rp) * sizeof(float);
+    const dim3 grid(s.n, (a.H + HG - 1) / HG, nr), vgrid(a.H, nr, (a.vdim + VR - 1) / VR);
+    if (s.keys == 32) LAUNCH(k_latent_attend<32>, grid, dim3(256), lds, a, m0, s.n);
+    else LAUNCH(k_latent_attend<64>, grid, dim3(256), lds, a, m0, s.n);
+    if (a.f32) LAUNCH(k_latent_values<float>, vgrid, dim3(256), (size_t)(rp + s.n) * 4, a, m0, s.n);
+    else LAUNCH(k_latent_values<half_t>, vgrid, dim3(256), (size_t)(rp + s.n) * 4, a, m0, s.n);
+}
+
 void launch_latent_attend(const LatentRows &in)
 {
     LatentRows a = in;
-    const int nsplit = slices_of(a), step = rows_per_launch(a), rp = pad8(a.rank), w = rp + pad8(a.rot);
-    const size_t po = (size_t)step * a.H * nsplit * rp, pml = (size_t)step * a.H * nsplit * 2;
-    a.part_o = (float *)scratch(SCR_PARTIAL, (po + pml) * sizeof(float));
-    a.part_ml = a.part_o + po;
-    const int parts = std::max(1, 256 / (rp / 4));
-    const size_t lds = ((size_t)HG * w + (size_t)HG * SLK + (size_t)parts * HG * rp) * sizeof(float);
-    for (int m0 = 0; m0 < a.r.n(); m0 += step) {
-        const int nr = std::min(step, a.r.n() - m0);
-        if (a.f32) LAUNCH(k_latent_query<float>, dim3(a.H, nr), dim3(256), (size_t)a.dim * 4, a, m0);
-        else LAUNCH(k_latent_query<half_t>, dim3(a.H, nr), dim3(256), (size_t)a.dim * 4, a, m0);
-        LAUNCH(k_latent_attend, dim3(nsplit, (a.H + HG - 1) / HG, nr), dim3(256), lds, a, m0, nsplit);
-        if (a.f32) LAUNCH(k_latent_values<float>, dim3(a.H, nr), dim3(256), (size_t)rp * 4, a, m0, nsplit);
-        else LAUNCH(k_latent_values<half_t>, dim3(a.H, nr), dim3(256), (size_t)rp * 4, a, m0, nsplit);
+    const LatentSlices s = latent_slices(a);
+    latent_partials(a, s);
+    for (int m0 = 0; m0 < a.r.n(); m0 += s.rows) {
+        const int nr = std::min(s.rows, a.r.n() - m0);
+        const size_t qlds = latent_query_lds(a);
+        if (a.f32) LAUNCH(k_latent_query<float>, dim3(a.H, nr), dim3(256), qlds, a, m0);
+        else LAUNCH(k_latent_query<half_t>, dim3(a.H, nr), dim3(256), qlds, a, m0);
+        launch_latent_slices(a, s, m0, nr);
     }
 }
 

@@ -2,7 +2,7 @@
 // per step (one product of the latents with both projections), laid out as matrix-core fragments, and met by 128 queries
 // of a head per workgroup.  Scores, running maximum and sums are fp32; the operands of the two products are F16.
 #include "stack.h"
-#include "rows.h"
+#include "latent_rows.h"
 #include "lds_copy.h"
 #include <algorithm>
 
@@ -20,14 +20,6 @@ struct PromptArgs {
     const float *kv;
     half_t *frags;                                       // [B][H][blocks][NJ + 2 NDB fragments][64 lanes][8]
 };
-
-// element d of head h's rotated query or of the key part: pairs (2i, 2i + 1) of the first `dims`
-__device__ __forceinline__ float turned(const float *x, int i, int dims, const float2 *cs)
-{
-    if (i >= dims) return x[i];
-    const float2 c = cs[i >> 1];
-    return (i & 1) ? x[i] * c.x + x[i - 1] * c.y : x[i] * c.x - x[i + 1] * c.y;
-}
 
 // grid (n_keys, B): the latent of one visible position as a row of the expansion's operand
 __global__ __launch_bounds__(256) void k_latent_operand(PromptArgs p, half_t *a16, float *inv)
@@ -107,7 +99,7 @@ __global__ __launch_bounds__(256) void k_latent_prompt(PromptArgs p)
 #pragma unroll
             for (int e = 0; e < 8; e++) {
                 const int d = 16 * j + 8 * hh + e;
-                qf[j][e] = (half_t)(d < a.dim ? q[d] * f : d < a.dim + a.rot ? turned(q + a.dim, d - a.dim, a.rot_dims, cs) * f : 0.f);
+                qf[j][e] = (half_t)(d < a.dim ? q[d] * f : d < a.dim + a.rot ? rotated(q + a.dim, d - a.dim, a.rot_dims, cs) * f : 0.f);
             }
     }
     float16v O[NDB];

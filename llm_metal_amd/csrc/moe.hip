@@ -1,6 +1,6 @@
 // Mixture of experts: softmax router with the largest scores chosen, squared-ReLU experts.
 #include "stack.h"
-#include "rows.h"
+#include "expert.h"
 
 namespace lmhip {
 namespace {
@@ -8,76 +8,12 @@ namespace {
 #define LAUNCH(kern, grid, block, lds, ...) do { \
     hipLaunchKernelGGL(kern, grid, block, lds, stream(), __VA_ARGS__); HIP_CHECK(hipGetLastError()); } while (0)
 
-// One wave per row: softmax over all experts, the `top` largest scores in order (of equals the lower index), not
-// renormalised.  A lane holds experts lane, lane + 64, ...
+// One wave per row: its experts and their weights
 __global__ __launch_bounds__(256) void k_route(MoeRows a)
 {
     const int m = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
     if (m >= a.rows) return;
-    const float *z = a.z + (size_t)m * a.ldz;
-    float v[16], mx = -3.0e38f;
-#pragma unroll
-    for (int i = 0; i < 16; i++) {
-        const int e = lane + 64 * i;
-        v[i] = e < a.E ? z[e] : -3.0e38f;
-        mx = fmaxf(mx, v[i]);
-    }
-    mx = wave_max(mx);
-    float sum = 0.f;
-#pragma unroll
-    for (int i = 0; i < 16; i++) {
-        const bool in = lane + 64 * i < a.E;
-        v[i] = in ? expf(v[i] - mx) : -1.f;
-        sum += in ? v[i] : 0.f;
-    }
-    sum = wave_sum(sum);
-    for (int s = 0; s < a.top; s++) {
-        float best = -2.f;
-        int idx = 0x7fffffff;
-#pragma unroll
-        for (int i = 0; i < 16; i++) if (v[i] > best) { best = v[i]; idx = lane + 64 * i; }
-#pragma unroll
-        for (int o = 32; o > 0; o >>= 1) {
-            const float ob = __shfl_xor(best, o, WAVE);
-            const int oi = __shfl_xor(idx, o, WAVE);
-            if (ob > best || (ob == best && oi < idx)) { best = ob; idx = oi; }
-        }
-        if (lane == 0) { a.idx[(size_t)m * a.top + s] = idx; a.w[(size_t)m * a.top + s] = best / sum; }
-#pragma unroll
-        for (int i = 0; i < 16; i++) if (lane + 64 * i == idx) v[i] = -1.f;
-    }
-}
-
-template <typename WT> struct Vec8;
-template <> struct Vec8<half_t> {
-    static __device__ __forceinline__ void load(const half_t *p, float (&w)[8])
-    {
-        const half8 v = *reinterpret_cast<const half8 *>(p);
-#pragma unroll
-        for (int e = 0; e < 8; e++) w[e] = (float)v[e];
-    }
-};
-template <> struct Vec8<float> {
-    static __device__ __forceinline__ void load(const float *p, float (&w)[8])
-    {
-        const float4 a = *reinterpret_cast<const float4 *>(p), b = *reinterpret_cast<const float4 *>(p + 4);
-        w[0] = a.x; w[1] = a.y; w[2] = a.z; w[3] = a.w; w[4] = b.x; w[5] = b.y; w[6] = b.z; w[7] = b.w;
-    }
-};
-
-// lane's part of W[row] . x over `cols` (a multiple of 8)
-template <typename WT>
-__device__ __forceinline__ float dot_part(const WT *w, const float *x, int cols, int lane)
-{
-    float s = 0.f;
-    for (int c = lane * 8; c < cols; c += 512) {
-        float wv[8];
-        Vec8<WT>::load(w + c, wv);
-        const float4 x0 = *reinterpret_cast<const float4 *>(x + c), x1 = *reinterpret_cast<const float4 *>(x + c + 4);
-        s = fmaf(wv[0], x0.x, s); s = fmaf(wv[1], x0.y, s); s = fmaf(wv[2], x0.z, s); s = fmaf(wv[3], x0.w, s);
-        s = fmaf(wv[4], x1.x, s); s = fmaf(wv[5], x1.y, s); s = fmaf(wv[6], x1.z, s); s = fmaf(wv[7], x1.w, s);
-    }
-    return s;
+    route_row(a.z + (size_t)m * a.ldz, a.E, a.top, lane, a.idx + (size_t)m * a.top, a.w + (size_t)m * a.top);
 }
 
 // act[m][s][i] = relu(up_e[i] . h[m])^2 for the s-th chosen expert e of row m; a wave per i.  grid (ceil(ffp / 4), top, rows)
@@ -115,6 +51,7 @@ __global__ __launch_bounds__(256) void k_moe_count(const int *__restrict__ idx, 
 {
     __shared__ float sm[16];
     int c = 0;
+#pragma unroll 8
     for (int i = threadIdx.x; i < n; i += 256) c += idx[i] == (int)blockIdx.x;
     const float total = block_sum((float)c, sm);          // exact: far below 2^24
     if (threadIdx.x == 0) count[blockIdx.x] = (int)total;
@@ -135,35 +72,53 @@ __global__ __launch_bounds__(256) void k_moe_place(const int *__restrict__ idx, 
         for (int i = t0 + nt + tid; i < g.tiles; i += 256) g.of[i] = -1;
     if (!mine) return;
     int at = t0 * 128;
-    for (int i0 = 0; i0 < n; i0 += 256) {
-        const int i = i0 + tid;
-        const bool hit = i < n && idx[i] == e;
-        const unsigned long long b = __ballot(hit);
-        if (lane == 0) wave_n[wave] = __popcll(b);
+    constexpr int U = 8;                                  // 256 U pairs per trip, their reads in flight together
+    for (int i0 = 0; i0 < n; i0 += 256 * U) {
+        bool hit[U];
+        int rank[U], in_wave = 0;
+#pragma unroll
+        for (int u = 0; u < U; u++) { const int i = i0 + (wave * U + u) * 64 + lane; hit[u] = i < n && idx[min(i, n - 1)] == e; }
+#pragma unroll
+        for (int u = 0; u < U; u++) {
+            const unsigned long long b = __ballot(hit[u]);
+            rank[u] = in_wave + __popcll(b & ((1ull << lane) - 1ull));
+            in_wave += __popcll(b);
+        }
+        if (lane == 0) wave_n[wave] = in_wave;
         __syncthreads();
         int o = at;
         for (int w = 0; w < wave; w++) o += wave_n[w];
-        if (hit) {
-            const int p = o + __popcll(b & ((1ull << lane) - 1ull));
-            g.src[p] = i / top;
-            g.pos[i] = p;
-        }
+#pragma unroll
+        for (int u = 0; u < U; u++)
+            if (hit[u]) {
+                const int i = i0 + (wave * U + u) * 64 + lane;
+                g.src[o + rank[u]] = i / top;
+                g.pos[i] = o + rank[u];
+            }
         at += wave_n[0] + wave_n[1] + wave_n[2] + wave_n[3];
         __syncthreads();
     }
 }
 
-// grid (rows of the groups), block 256: one row of a tiled operand to another place, 16 bytes per thread and trip
+// grid (row blocks of 32, chunks of K blocks), block 256: rows of a tiled operand to other places.  A wave writes whole 1 KB
+// slices; a row is 32 contiguous bytes of its source slice.
 __global__ __launch_bounds__(256) void k_moe_gather(MoeGroups g, const half_t *__restrict__ a16, const float *__restrict__ inv,
-                                                    half_t *__restrict__ out16, float *__restrict__ out_inv, int Kb)
+                                                    half_t *__restrict__ out16, float *__restrict__ out_inv, int Kb, int per)
 {
-    const int p = blockIdx.x;
-    if (g.of[p >> 7] < 0) return;
-    const int m = g.src[p];
-    if (m < 0) return;
-    for (int k = threadIdx.x * 8; k < Kb * 64; k += 2048)
-        *reinterpret_cast<half8 *>(&out16[tiled_a_index(p, k, Kb)]) = *reinterpret_cast<const half8 *>(&a16[tiled_a_index(m, k, Kb)]);
-    if (threadIdx.x == 0) out_inv[p] = inv[m];
+    const int rb = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    if (g.of[rb >> 2] < 0) return;
+    const int m = g.src[rb * 32 + (lane >> 1)], src = max(m, 0);
+    const half8 *from = reinterpret_cast<const half8 *>(a16) + ((size_t)(src >> 5) * Kb) * 256 + ((src & 31) << 1) + (lane & 1);
+    half8 *to = reinterpret_cast<half8 *>(out16) + (size_t)rb * Kb * 256 + lane;
+    const int s0 = blockIdx.y * per * 4, s1 = min(s0 + per * 4, Kb * 4);
+    for (int s = s0 + wave; s < s1; s += 4 * 4) {         // four slices of a wave in flight
+        half8 v[4];
+#pragma unroll
+        for (int u = 0; u < 4; u++) v[u] = from[(size_t)min(s + 4 * u, s1 - 1) * 64];
+#pragma unroll
+        for (int u = 0; u < 4; u++) if (s + 4 * u < s1) to[(size_t)(s + 4 * u) * 64] = v[u];
+    }
+    if (blockIdx.y == 0 && threadIdx.x < 32) { const int r = g.src[rb * 32 + threadIdx.x]; if (r >= 0) out_inv[rb * 32 + threadIdx.x] = inv[r]; }
 }
 
 // grid (rows of the groups), block 256
@@ -206,7 +161,8 @@ void launch_moe_groups(const MoeRows &a, const MoeGroups &g)
 
 void launch_moe_gather(const MoeGroups &g, const half_t *a16, const float *inv, half_t *out16, float *out_inv, int K)
 {
-    LAUNCH(k_moe_gather, dim3(g.tiles * 128), dim3(256), 0, g, a16, inv, out16, out_inv, tiled_kb(K));
+    const int Kb = tiled_kb(K), per = 16;
+    LAUNCH(k_moe_gather, dim3(g.tiles * 4, (Kb + per - 1) / per), dim3(256), 0, g, a16, inv, out16, out_inv, Kb, per);
 }
 
 void launch_moe_act(const MoeGroups &g, const float *up, int ld, int n, half_t *out16, float *out_inv, int K)

@@ -41,4 +41,12 @@ __device__ __forceinline__ float group_sum(float v)
     return v;
 }
 
+// sum over the wave, left in every lane
+__device__ __forceinline__ float wave_total(float v)
+{
+    v = group_sum<16>(v);
+    v += __shfl_xor(v, 16, WAVE);
+    return v + __shfl_xor(v, 32, WAVE);
+}
+
 }  // namespace lmhip

@@ -111,6 +111,7 @@ struct StackRun {
     MetalBuf *lat_a16 = nullptr, *lat_inv = nullptr, *lat_kv = nullptr, *lat_frags = nullptr;   // prompt attention: expanded keys and values
     int moe_rows = 0;                                    // rows those hold
     int T = 0, pending = 0;                              // tokens per sequence of the last step; its last layer's sum still waits in cout (1) and ymoe (2) or moe_y (4, by `groups`)
+    bool fused = false, one = false;                     // single tokens take the fused steps; the last step was one
     MoeGroups groups{};
     int groups_top = 0;
 };
@@ -188,6 +189,10 @@ struct LatentRows {
 };
 void launch_latent_cache(const LatentRows &a);           // latent norm and key rotation into the ring
 void launch_latent_attend(const LatentRows &a);          // any number of rows, over the latents themselves
+struct LatentSlices { int keys, n, rows; };              // keys per workgroup, slices of a row's keys, rows per launch
+LatentSlices latent_slices(const LatentRows &a);
+void latent_partials(LatentRows &a, const LatentSlices &s);
+void launch_latent_slices(const LatentRows &a, const LatentSlices &s, int m0, int nr);   // behind the absorbed queries: attention and values
 
 // latent_prompt.hip: many rows of 16-bit precision with keys and values expanded once per step.  The step's visible keys
 // are positions first .. pos + T - 1; kv holds W_uk c | W_uv c of them, [B][n_keys][H * (dim + vdim)].

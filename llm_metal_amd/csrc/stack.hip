@@ -2,6 +2,7 @@
 // a run keep, and one step over any number of tokens.  The generation state (inference.hip) owns both and drives them.
 #include "stack.h"
 #include "rows.h"
+#include "stack_decode.h"
 
 #include <algorithm>
 #include <math.h>
@@ -271,6 +272,8 @@ StackRun *stack_run_create(const LayerStack *st, int B)
 {
     StackRun *r = new StackRun();
     r->B = B;
+    r->fused = !st->f32 && B == 1 && st->Dp <= 15360;
+    for (const StackLayer &L : st->layers) r->fused = r->fused && decode_fits(L.out.cols, L.c.top, L.down.cols, st->Dp);
     r->rows = std::max(1, std::min(PORTION_ROWS / B, st->max_seq)) * B;
     const int portion = r->rows / B;
     size_t n_in = 0, ko = 0, aux = 0, act = 0, top = 0, tab = 0;
@@ -368,6 +371,41 @@ void norm(LayerStack *st, StackRun *r, MetalBuf *g, int rows, int keep, bool nee
     launch_norm_rows(n, rows);
 }
 
+DeltaRows delta_rows(const LayerStack *st, const StackRun *r, const StackLayer &L, const StackRun::Layer &k, const Rows &rows, const DeltaAux &d)
+{
+    const LayerConfig &c = L.c;
+    DeltaRows a{};
+    a.r = rows; a.H = c.heads; a.KV = c.kv_heads; a.dim = c.dim; a.vdim = c.vdim; a.taps = c.taps; a.per_channel = c.mixer == MIX_CHANNEL_DELTA;
+    a.cin = ptr<float>(r->cin); a.ldc = L.in.rows; a.o_q = L.o_q; a.o_k = L.o_k; a.o_v = L.o_v; a.o_b = L.o_b; a.o_a = L.o_a;
+    a.filters = ptr<float>(L.conv); a.a_exp = ptr<float>(L.a_exp); a.dt_bias = ptr<float>(L.dt_bias);
+    a.conv = ptr<float>(k.conv); a.S = ptr<float>(k.S);
+    a.q = d.q; a.k = d.k; a.v = d.v; a.kq = d.kq; a.beta = d.beta; a.g = d.g; a.a2 = d.a2; a.o = d.o;
+    return a;
+}
+
+LatentRows latent_rows(const LayerStack *st, const StackRun *r, const StackLayer &L, const StackRun::Layer &k, const Rows &rows, const LatentAux &d)
+{
+    const LayerConfig &c = L.c;
+    LatentRows a{};
+    a.r = rows; a.H = c.heads; a.dim = c.dim; a.rot = c.rot_dim; a.vdim = c.vdim; a.rank = c.kv_rank; a.window = c.window;
+    a.ring_rows = k.ring_rows; a.rot_dims = c.rot_dims; a.scale = c.scale; a.eps = st->cfg.eps;
+    a.cin = ptr<float>(r->cin); a.ldc = L.in.rows; a.o_q = L.o_q; a.o_dkv = L.o_dkv;
+    a.g_c = ptr<float>(L.g_c); a.rope = ptr<float2>(L.rope); a.ring = ptr<float>(k.ring);
+    a.q = d.q; a.o = d.o; a.f32 = st->f32; a.ukv = dptr(L.ukv.buf); a.ldu = L.ukv.cols;
+    return a;
+}
+
+// mixer output | shared activation of a layer, without the mixer's own part
+CatRows cat_rows(const LayerStack *st, const StackRun *r, const StackLayer &L)
+{
+    const LayerConfig &c = L.c;
+    CatRows cat{};
+    cat.H = c.heads; cat.vdim = c.vdim; cat.eps = st->cfg.eps; cat.g_out = ptr<float>(L.g_out); cat.gate_silu = c.mixer == MIX_DELTA;
+    cat.shared = ptr<float>(r->cin) + L.o_shared; cat.ld_shared = L.in.rows; cat.shared_ff = c.shared_ff; cat.o_sh = L.o_sh;
+    cat.cat = ptr<float>(r->cat); cat.a16 = ptr<half_t>(r->b16); cat.inv = ptr<float>(r->binv); cat.ldk = L.out.cols;
+    return cat;
+}
+
 float *mix_delta(LayerStack *st, StackRun *r, StackLayer &L, StackRun::Layer &k, const Rows &rows, CatRows &cat)
 {
     const LayerConfig &c = L.c;
@@ -384,16 +422,10 @@ float *mix_delta(LayerStack *st, StackRun *r, StackLayer &L, StackRun::Layer &k,
         low_rank(L.a2, L.o_a, d.a2);
         low_rank(L.g2, L.o_g, d.g2);
     }
-    DeltaRows a{};
-    a.r = rows; a.H = c.heads; a.KV = c.kv_heads; a.dim = c.dim; a.vdim = c.vdim; a.taps = c.taps; a.per_channel = pc;
-    a.cin = cin; a.ldc = ldc; a.o_q = L.o_q; a.o_k = L.o_k; a.o_v = L.o_v; a.o_b = L.o_b; a.o_a = L.o_a;
-    a.filters = ptr<float>(L.conv); a.a_exp = ptr<float>(L.a_exp); a.dt_bias = ptr<float>(L.dt_bias);
-    a.conv = ptr<float>(k.conv); a.S = ptr<float>(k.S);
-    a.q = d.q; a.k = d.k; a.v = d.v; a.kq = d.kq; a.beta = d.beta; a.g = d.g; a.a2 = d.a2; a.o = d.o;
+    const DeltaRows a = delta_rows(st, r, L, k, rows, d);
     launch_delta_inputs(a);
     launch_delta_scan(a);
-    cat.g_out = ptr<float>(L.g_out);
-    cat.gate = pc ? d.g2 : cin + L.o_g; cat.ld_gate = pc ? L.hv : ldc; cat.gate_silu = pc ? 0 : 1;
+    cat.gate = pc ? d.g2 : cin + L.o_g; cat.ld_gate = pc ? L.hv : ldc;
     return d.o;
 }
 
@@ -402,12 +434,7 @@ float *mix_latent(LayerStack *st, StackRun *r, StackLayer &L, StackRun::Layer &k
     const LayerConfig &c = L.c;
     Aux ax{ptr<float>(r->aux)};
     const LatentAux d = latent_aux(ax, c, rows.n());
-    LatentRows a{};
-    a.r = rows; a.H = c.heads; a.dim = c.dim; a.rot = c.rot_dim; a.vdim = c.vdim; a.rank = c.kv_rank; a.window = c.window;
-    a.ring_rows = k.ring_rows; a.rot_dims = c.rot_dims; a.scale = c.scale; a.eps = st->cfg.eps;
-    a.cin = ptr<float>(r->cin); a.ldc = L.in.rows; a.o_q = L.o_q; a.o_dkv = L.o_dkv;
-    a.g_c = ptr<float>(L.g_c); a.rope = ptr<float2>(L.rope); a.ring = ptr<float>(k.ring);
-    a.q = d.q; a.o = d.o; a.f32 = st->f32; a.ukv = dptr(L.ukv.buf); a.ldu = L.ukv.cols;
+    const LatentRows a = latent_rows(st, r, L, k, rows, d);
     launch_latent_cache(a);
     if (!latent_prompt_fits(a)) { launch_latent_attend(a); return d.o; }
     const int nk = latent_prompt_keys(a), most = k.ring_rows;            // grown to what any step of this layer needs
@@ -424,6 +451,48 @@ float *mix_latent(LayerStack *st, StackRun *r, StackLayer &L, StackRun::Layer &k
 
 }  // namespace
 
+namespace {
+
+// decoding one sequence with F16 weights: the fused steps of stack_decode.hip
+void decode_layers(LayerStack *st, StackRun *r, int pos)
+{
+    const Rows rows{1, 1, pos};
+    float *x = ptr<float>(r->x), *cin = ptr<float>(r->cin);
+    for (size_t i = 0; i < st->layers.size(); i++) {
+        StackLayer &L = st->layers[i];
+        StackRun::Layer &k = r->layers[i];
+        const LayerConfig &c = L.c;
+        matvec_layernorm(L.in.buf, x, ptr<float>(L.g_norm), st->D, st->cfg.eps, cin, L.in.rows, L.in.cols);
+        DecodeMoe e{};
+        e.x = x; e.g = ptr<float>(L.g_norm); e.D = st->D; e.Dp = st->Dp; e.eps = st->cfg.eps;
+        if (c.experts) {
+            e.z = cin + L.o_router; e.E = c.experts; e.top = c.top; e.idx = ptr<int>(r->route_idx); e.w = ptr<float>(r->route_w);
+            e.up = ptr<half_t>(L.up.buf); e.down = ptr<half_t>(L.down.buf); e.up_rows = L.up_rows; e.down_rows = L.down_rows;
+            e.ff = c.ff; e.ffp = L.down.cols; e.act = ptr<float>(r->act);
+        }
+        DecodeOut o{};
+        o.cat = cat_rows(st, r, L);
+        o.out = ptr<half_t>(L.out.buf); o.x = x; o.D = st->D;
+        Aux ax{ptr<float>(r->aux)};
+        if (L.delta()) {
+            const DeltaAux d = delta_aux(ax, c, 1);
+            DecodeDelta s{};
+            s.a = delta_rows(st, r, L, k, rows, d);
+            s.a2 = ptr<half_t>(L.a2.buf); s.g2 = ptr<half_t>(L.g2.buf); s.lda2 = L.a2.cols; s.ldg2 = L.g2.cols; s.o_g = L.o_g;
+            s.gate = d.v;                                 // (the values stay in registers here)
+            launch_delta_decode(s, e);
+            o.cat.o = d.o; o.cat.gate = s.gate;
+        } else {
+            const LatentAux d = latent_aux(ax, c, 1);
+            launch_latent_decode(latent_rows(st, r, L, k, rows, d), e);
+            o.cat.o = d.o;
+        }
+        launch_out_decode(o, e);
+    }
+}
+
+}  // namespace
+
 void stack_forward(LayerStack *st, StackRun *r, const int *tokens, int T, int pos)
 {
     const Rows rows{r->B, T, pos};
@@ -435,6 +504,8 @@ void stack_forward(LayerStack *st, StackRun *r, const int *tokens, int T, int po
     HIP_CHECK(hipMemcpyAsync(dptr(r->tok), th, (size_t)n * sizeof(int), hipMemcpyHostToDevice, stream()));
     launch_embed_rows(ptr<float>(st->emb), ptr<int>(r->tok), st->cfg.emb_scale, ptr<float>(r->x), st->D, st->Dp, n);
     r->T = T; r->pending = 0;
+    r->one = n == 1 && r->fused;
+    if (r->one) { decode_layers(st, r, pos); return; }
     for (size_t i = 0; i < st->layers.size(); i++) {
         StackLayer &L = st->layers[i];
         const LayerConfig &c = L.c;
@@ -442,11 +513,8 @@ void stack_forward(LayerStack *st, StackRun *r, const int *tokens, int T, int po
         const bool grouped = c.experts && !st->f32 && n >= 16 && n * c.top >= c.experts;
         norm(st, r, L.g_norm, n, 1, c.experts && !grouped);
         product(st, L.in, ptr<half_t>(r->a16), ptr<float>(r->inv), ptr<float>(r->h), st->Dp, ptr<float>(r->cin), n);
-        CatRows cat{};
+        CatRows cat = cat_rows(st, r, L);
         cat.o = L.delta() ? mix_delta(st, r, L, r->layers[i], rows, cat) : mix_latent(st, r, L, r->layers[i], rows);
-        cat.H = c.heads; cat.vdim = c.vdim; cat.eps = st->cfg.eps;
-        cat.shared = ptr<float>(r->cin) + L.o_shared; cat.ld_shared = L.in.rows; cat.shared_ff = c.shared_ff; cat.o_sh = L.o_sh;
-        cat.cat = ptr<float>(r->cat); cat.a16 = ptr<half_t>(r->b16); cat.inv = ptr<float>(r->binv); cat.ldk = L.out.cols;
         launch_cat_rows(cat, n);
         product(st, L.out, cat.a16, cat.inv, cat.cat, cat.ldk, ptr<float>(r->cout), n);
         r->pending = 1;
@@ -476,6 +544,10 @@ void stack_forward(LayerStack *st, StackRun *r, const int *tokens, int T, int po
 void stack_logits(LayerStack *st, StackRun *r, const int *want, int n, float *logits)
 {
     if (n <= 0) return;
+    if (r->one) {                                         // whatever `want` says, it is the one row
+        matvec_layernorm(st->head.buf, ptr<float>(r->x), ptr<float>(st->g_final), st->D, st->cfg.eps, logits, st->head.rows, st->head.cols);
+        return;
+    }
     const int *list = nullptr;
     if (want) {
         memcpy(r->want_host, want, (size_t)n * sizeof(int));

@@ -181,9 +181,10 @@ def to_bf16_bits(a):
     return ((b + np.uint32(0x7FFF) + ((b >> np.uint32(16)) & np.uint32(1))) >> np.uint32(16)).astype(np.uint16)
 
 
-def write_stack_checkpoint(path, cfg, seed=0, rank_a=24, rank_g=24, keep=False, edit=None):
+def write_stack_checkpoint(path, cfg, seed=0, rank_a=24, rank_g=24, keep=False, edit=None, repeat=False):
     """config.json and model.safetensors (bfloat16) of a random model in the folder `path`.  keep: return the values the
-    file holds, fp32 by name.  edit(name, array): may replace a tensor before it is rounded."""
+    file holds, fp32 by name.  edit(name, array): may replace a tensor before it is rounded.  repeat: every matrix of the
+    experts is the same one (large models for timing, written in a fraction of the time)."""
     import json
     import struct
     shapes = stack_shapes(cfg, rank_a, rank_g)
@@ -197,15 +198,21 @@ def write_stack_checkpoint(path, cfg, seed=0, rank_a=24, rank_g=24, keep=False, 
         off += n
     text = json.dumps(header).encode()
     text += b" " * (-len(text) % 8)
-    kept = {}
+    kept, drawn = {}, {}
     with open(os.path.join(path, "model.safetensors"), "wb") as f:
         f.write(struct.pack("<Q", len(text)) + text)
         for i, (name, shape) in enumerate(shapes.items()):
+            kind = (name.rsplit(".", 1)[-1], shape)
+            if repeat and ".e" in name and kind in drawn:
+                f.write(drawn[kind])
+                continue
             a = make_stack_tensor(name, shape, np.random.default_rng([seed, i]))
             if edit is not None:
                 a = edit(name, a)
             bits = to_bf16_bits(a)
             f.write(bits.tobytes())
+            if repeat and ".e" in name:
+                drawn[kind] = bits.tobytes()
             if keep:
                 kept[name] = (bits.astype(np.uint32) << np.uint32(16)).view(np.float32)
     return kept
