@@ -9,19 +9,16 @@ namespace {
 #define LAUNCH(kern, grid, block, lds, ...) do { \
     hipLaunchKernelGGL(kern, grid, block, lds, stream(), __VA_ARGS__); HIP_CHECK(hipGetLastError()); } while (0)
 
-// silu of the convolution at one channel for the tokens t0 .. t0 + TW - 1 of sequence b, one after the other: `use(i, value)`.
-// Up to four taps the inputs slide through registers, each read once; more taps are gathered token by token.
+// silu of the convolutions at NE channels for the tokens t0 .. t0 + TW - 1 of sequence b: y[token][channel], zeros past the
+// end.  Up to four taps the inputs slide through registers, each read once; more taps are gathered token by token.
 constexpr int TW = 8;        // tokens per wave
-template <int NE, typename F>
-__device__ __forceinline__ void conv_tokens(const DeltaRows &a, int b, int t0, const int (&ch)[NE], const int (&col)[NE], const bool (&in)[NE], F use)
+template <int NE>
+__device__ __forceinline__ void conv_tokens(const DeltaRows &a, int b, int t0, const int (&ch)[NE], const int (&col)[NE], const bool (&in)[NE],
+                                            float (&y)[TW][NE])
 {
     const int T = a.r.T, nt = min(TW, T - t0), C = 2 * a.KV * a.dim + a.H * a.vdim;
     if (a.taps <= 4) {
         float f[NE][4], x[NE][TW + 3];
-#pragma unroll
-        for (int e = 0; e < NE; e++)
-#pragma unroll
-            for (int i = 0; i < 4; i++) f[e][i] = in[e] && i >= 4 - a.taps ? a.filters[(size_t)ch[e] * a.taps + i - (4 - a.taps)] : 0.f;
 #pragma unroll
         for (int i = 0; i < TW + 3; i++) {
             const int tt = t0 - 3 + i, p = a.r.pos + tt;
@@ -36,34 +33,34 @@ __device__ __forceinline__ void conv_tokens(const DeltaRows &a, int b, int t0, c
             }
         }
 #pragma unroll
-        for (int i = 0; i < TW; i++) {
-            if (i >= nt) break;
-            float y[NE];
+        for (int e = 0; e < NE; e++)
 #pragma unroll
-            for (int e = 0; e < NE; e++) y[e] = in[e] ? silu(fmaf(f[e][3], x[e][i + 3], fmaf(f[e][2], x[e][i + 2], fmaf(f[e][1], x[e][i + 1], f[e][0] * x[e][i])))) : 0.f;
-            use(i, y);
-        }
-    } else
-        for (int i = 0; i < nt; i++) {
-            float y[NE];
+            for (int i = 0; i < 4; i++) f[e][i] = in[e] && i >= 4 - a.taps ? a.filters[(size_t)ch[e] * a.taps + i - (4 - a.taps)] : 0.f;
 #pragma unroll
-            for (int e = 0; e < NE; e++) y[e] = in[e] ? silu(conv_at(a, b * T + t0 + i, ch[e], col[e])) : 0.f;
-            use(i, y);
-        }
+        for (int i = 0; i < TW; i++)
+#pragma unroll
+            for (int e = 0; e < NE; e++)
+                y[i][e] = silu(fmaf(f[e][3], x[e][i + 3], fmaf(f[e][2], x[e][i + 2], fmaf(f[e][1], x[e][i + 1], f[e][0] * x[e][i]))));
+    } else {
+#pragma unroll
+        for (int i = 0; i < TW; i++)
+#pragma unroll
+            for (int e = 0; e < NE; e++) y[i][e] = in[e] && i < nt ? silu(conv_at(a, b * T + t0 + i, ch[e], col[e])) : 0.f;
+    }
 }
 
-// One wave per (unit, TW tokens): units 0 .. KV-1 finish q and k of a key head (and their dot product), the next H the value
-// head, its step size and its decay.  A lane holds channels lane, lane + 64, ... (E of them).  grid (ceil(units / 4),
-// ceil(T / TW), B)
+// One wave per (unit, TW tokens): units 0 .. KV-1 finish q and k of a key head, the others 64 channels of the values.  A
+// lane holds channels lane, lane + 64, ... (E of them).  grid (ceil(units / 4), ceil(T / TW), B)
 template <int E>
 __global__ __launch_bounds__(256) void k_delta_inputs(DeltaRows a)
 {
     const int lane = threadIdx.x & 63, u = blockIdx.x * 4 + (threadIdx.x >> 6), t0 = blockIdx.y * TW, b = blockIdx.z;
-    if (u >= a.KV + a.H) return;
-    const int qd = a.KV * a.dim, m0 = b * a.r.T + t0;
+    const int qd = a.KV * a.dim, vd = a.H * a.vdim, m0 = b * a.r.T + t0, nt = min(TW, a.r.T - t0);
+    if (u >= a.KV + (vd + 63) / 64) return;
     if (u < a.KV) {
         int ch[2 * E], col[2 * E];
         bool in[2 * E];
+        float y[TW][2 * E];
 #pragma unroll
         for (int e = 0; e < E; e++) {
             const int d = lane + 64 * e;
@@ -71,61 +68,130 @@ __global__ __launch_bounds__(256) void k_delta_inputs(DeltaRows a)
             ch[e] = u * a.dim + d; col[e] = a.o_q + ch[e];
             ch[E + e] = qd + u * a.dim + d; col[E + e] = a.o_k + u * a.dim + d;
         }
-        conv_tokens<2 * E>(a, b, t0, ch, col, in, [&](int i, const float (&y)[2 * E]) {
-            float sq = 0.f, sk = 0.f, dot = 0.f;
+        conv_tokens<2 * E>(a, b, t0, ch, col, in, y);
+        float iq[TW], ik[TW];
 #pragma unroll
-            for (int e = 0; e < E; e++) { sq += y[e] * y[e]; sk += y[E + e] * y[E + e]; dot += y[e] * y[E + e]; }
-            sq = wave_total(sq); sk = wave_total(sk); dot = wave_total(dot);
-            const float iq = 1.f / (sqrtf(sq + 1e-6f) * sqrtf((float)a.dim)), ik = 1.f / sqrtf(sk + 1e-6f);
-            const size_t o = ((size_t)(m0 + i) * a.KV + u) * a.dim;
+        for (int i = 0; i < TW; i++) {
+            float sq = 0.f, sk = 0.f;
+#pragma unroll
+            for (int e = 0; e < E; e++) { sq += y[i][e] * y[i][e]; sk += y[i][E + e] * y[i][E + e]; }
+            iq[i] = wave_total(sq); ik[i] = wave_total(sk);
+        }
+#pragma unroll
+        for (int i = 0; i < TW; i++) {
+            if (i >= nt) break;
+            const float fq = 1.f / (sqrtf(iq[i] + 1e-6f) * sqrtf((float)a.dim)), fk = 1.f / sqrtf(ik[i] + 1e-6f);
+            const size_t o = ((size_t)(m0 + i) * a.KV + u) * a.dim + lane;
 #pragma unroll
             for (int e = 0; e < E; e++)
-                if (in[e]) { a.q[o + lane + 64 * e] = y[e] * iq; a.k[o + lane + 64 * e] = y[E + e] * ik; }
-            if (lane == 0) a.kq[(size_t)(m0 + i) * a.KV + u] = dot * iq * ik;
-        });
+                if (in[e]) { a.q[o + 64 * e] = y[i][e] * fq; a.k[o + 64 * e] = y[i][E + e] * fk; }
+        }
         return;
     }
-    const int h = u - a.KV;
-    for (int d0 = 0; d0 < a.vdim; d0 += 64) {
-        const int d = d0 + lane, ch[1] = {2 * qd + h * a.vdim + d}, col[1] = {a.o_v + h * a.vdim + d};
-        const bool in[1] = {d < a.vdim};
-        conv_tokens<1>(a, b, t0, ch, col, in, [&](int i, const float (&y)[1]) { if (in[0]) a.v[((size_t)(m0 + i) * a.H + h) * a.vdim + d] = y[0]; });
-    }
-    const int nt = min(TW, a.r.T - t0);
-    if (lane < nt) {
-        const float *row = a.cin + (size_t)(m0 + lane) * a.ldc;
-        a.beta[(size_t)(m0 + lane) * a.H + h] = sigmoid(row[a.o_b + h]);
-        if (!a.per_channel) a.g[(size_t)(m0 + lane) * a.H + h] = expf(-a.a_exp[h] * softplus(row[a.o_a + h] + a.dt_bias[h]));
-    }
-    if (a.per_channel)
-        for (int d = lane; d < a.dim; d += 64) {
-            const float ae = a.a_exp[h], bias = a.dt_bias[h * a.dim + d];
+    const int c = (u - a.KV) * 64 + lane, ch[1] = {2 * qd + c}, col[1] = {a.o_v + c};
+    const bool in[1] = {c < vd};
+    float y[TW][1];
+    conv_tokens<1>(a, b, t0, ch, col, in, y);
 #pragma unroll
-            for (int i = 0; i < TW; i++) {
-                if (i >= nt) break;
-                const size_t o = ((size_t)(m0 + i) * a.H + h) * a.dim + d;
-                a.g[o] = expf(-ae * softplus(a.a2[o] + bias));
+    for (int i = 0; i < TW; i++) if (i < nt && in[0]) a.v[(size_t)(m0 + i) * vd + c] = y[i][0];
+}
+
+// ---------------------------------------------------------------- tokens in groups of four
+//
+// Four tokens are taken through the recurrence together.  With S the state ahead of them, d(j, i) the decay between
+// writing token j and reading token i (the product of the decays of j + 1 .. i) and d(0-, i) the one from S to i:
+//     p_i = S^T (d(0-, i) k_i)          w_i = S^T (d(0-, i) q_i)
+//     u_i = beta_i (v_i - p_i - sum_{j < i} A_ij u_j)      A_ij = k_i . d(j, i) k_j
+//     o_i = w_i + sum_{j <= i} B_ij u_j                    B_ij = q_i . d(j, i) k_j
+//     S  <- d(0-, 3) S + sum_j d(j, 3) k_j u_j^T
+// which is the token-by-token recurrence with the sums written out: all eight products with the state run side by side,
+// and the state is written once.  The numbers that do not depend on the state are made ahead, 32 per group and head:
+//     0 .. 3 beta | 4 .. 9 A10 A20 A21 A30 A31 A32 | 12 .. 21 B00 B10 B11 B20 B21 B22 B30 B31 B32 B33
+//     | 24 .. 27 d(0-, i) | 28 .. 31 d(i, 3)  (the last two with one decay per head only)
+constexpr int GT = 4, GS = 32;
+
+// One wave per (group, head): decays, step sizes and the pair products.  grid (ceil(H / 4), groups, B)
+template <int E, int PC>
+__global__ __launch_bounds__(256) void k_delta_pairs(DeltaRows a)
+{
+    const int lane = threadIdx.x & 63, h = blockIdx.x * 4 + (threadIdx.x >> 6), grp = blockIdx.y, b = blockIdx.z, T = a.r.T;
+    if (h >= a.H) return;
+    const int kvh = h / (a.H / a.KV), t0 = grp * GT, nt = min(GT, T - t0);
+    const size_t m0 = (size_t)b * T + t0;
+    float k[GT][E], q[GT][E], g[GT][E], gh[GT];
+    const float ae = a.a_exp[h];
+#pragma unroll
+    for (int i = 0; i < GT; i++) {
+        gh[i] = 1.f;
+        if (!PC && i < nt) gh[i] = expf(-ae * softplus(a.cin[(m0 + i) * a.ldc + a.o_a + h] + a.dt_bias[h]));
+#pragma unroll
+        for (int e = 0; e < E; e++) {
+            const int d = lane + 64 * e;
+            const bool in = d < a.dim && i < nt;
+            const size_t o = ((m0 + i) * a.KV + kvh) * a.dim + d;
+            k[i][e] = in ? a.k[o] : 0.f;
+            q[i][e] = in ? a.q[o] : 0.f;
+            g[i][e] = gh[i];
+            if (PC && in) {
+                const size_t og = ((m0 + i) * a.H + h) * a.dim + d;
+                g[i][e] = expf(-ae * softplus(a.a2[og] + a.dt_bias[h * a.dim + d]));
+                a.g[og] = g[i][e];
             }
         }
+    }
+    float A[6], B[10];
+    int na = 0, nb = 0;
+#pragma unroll
+    for (int i = 0; i < GT; i++)
+#pragma unroll
+        for (int j = 0; j <= i; j++) {
+            float sa = 0.f, sb = 0.f;
+#pragma unroll
+            for (int e = 0; e < E; e++) {
+                float kj = k[j][e];
+#pragma unroll
+                for (int x = j + 1; x <= i; x++) kj *= g[x][e];
+                sa = fmaf(k[i][e], kj, sa); sb = fmaf(q[i][e], kj, sb);
+            }
+            if (j < i) A[na++] = wave_total(sa);
+            B[nb++] = wave_total(sb);
+        }
+    // lane n keeps number n
+    float mine = 0.f;
+#pragma unroll
+    for (int i = 0; i < GT; i++) {
+        if (lane == i && i < nt) mine = sigmoid(a.cin[(m0 + i) * a.ldc + a.o_b + h]);
+        if (!PC) {
+            float c = 1.f, r = 1.f;
+#pragma unroll
+            for (int x = 0; x < GT; x++) { if (x <= i) c *= gh[x]; else r *= gh[x]; }
+            if (lane == 24 + i) mine = c;
+            if (lane == 28 + i) mine = r;
+        }
+    }
+#pragma unroll
+    for (int n = 0; n < 6; n++) if (lane == 4 + n) mine = A[n];
+#pragma unroll
+    for (int n = 0; n < 10; n++) if (lane == 12 + n) mine = B[n];
+    if (lane < GS) a.pairs[(((size_t)b * ((T + GT - 1) / GT) + grp) * a.H + h) * GS + lane] = mine;
 }
 
 // The recurrence.  The columns of a head's state (one per value channel) do not meet: a column is G lanes of a wave, each
-// with R of its rows -- lane l of the group has rows 4 l .. 4 l + 3 of every block of 4 G -- so a token costs no barrier:
-// with both dot products taken before the update (o = (g S)^T q + u (k . q), the read-out after the write) they are reduced
-// side by side.  Tokens are staged through LDS TC at a time, the next TC on their way in registers; a token's LDS reads are
-// issued two tokens ahead.  The lane numbered like the token keeps its output until the stage is over.
+// with R of its rows -- lane l of the group has rows 4 l .. 4 l + 3 of every block of 4 G -- so no token costs a barrier.
+// Tokens are staged through LDS TC at a time with the decays already on the keys and queries, the next TC on their way in
+// registers; a group's LDS reads are issued one group ahead.  The lane numbered like a token keeps its output until the
+// stage is over.
 // grid (column blocks of 256 / G, H, B), block 256.  VEC: dim is a multiple of 4 (16-byte loads).
 template <int G, int R, int PC, int VEC>
 __global__ __launch_bounds__(256) void k_delta_scan(DeltaRows a)
 {
-    constexpr int TC = 16, DP = G * R, COLS = 256 / G, RB = R / 4;
-    constexpr int NV = (TC * DP / 4 + 255) / 256;         // 16-byte pieces per thread and array of one stage
+    constexpr int TC = 16, NG = TC / GT, DP = G * R, COLS = 256 / G, RB = R / 4;
     constexpr int NC = (TC * COLS + 255) / 256, NK = (TC + G - 1) / G;
-    __shared__ float ks[2][TC * DP], qs[2][TC * DP], gs[2][PC ? TC * DP : TC];
-    __shared__ float vs[2][TC * COLS];
-    __shared__ float2 bs[2][TC];                          // (step size, k . q)
+    static_assert(DP <= 256, "a thread stages four columns of one group");
+    __shared__ float ks[2][TC * DP], qs[2][TC * DP], us[2][PC ? TC * DP : 4], gs[2][PC ? NG * DP : 4];
+    __shared__ float vs[2][COLS * TC], ps[2][NG * GS];
     const int tid = threadIdx.x, l = tid % G, col = tid / G;
-    const int h = blockIdx.y, b = blockIdx.z, kvh = h / (a.H / a.KV), T = a.r.T;
+    const int h = blockIdx.y, b = blockIdx.z, kvh = h / (a.H / a.KV), T = a.r.T, groups = (T + GT - 1) / GT;
     const int j0 = blockIdx.x * COLS, j = j0 + col;
     const size_t r0 = (size_t)b * T;
     float S[R];
@@ -135,27 +201,31 @@ __global__ __launch_bounds__(256) void k_delta_scan(DeltaRows a)
         const int d = (e >> 2) * 4 * G + 4 * l + (e & 3);
         S[e] = (a.r.pos > 0 && d < a.dim) ? Sg[d] : 0.f;  // position 0 starts from nothing, whatever the state held
     }
-    float4 kr[NV], qr[NV], gr[PC ? NV : 1];
-    float vr[NC], gsr = 0.f;
-    float2 br = make_float2(0.f, 0.f);
+    const int sd = (tid % (DP / 4)) * 4, sgrp = tid / (DP / 4);          // staging: four columns of one group (tid < DP)
+    float4 kr[GT], qr[GT], gr[PC ? GT : 1];
+    float vr[NC], pr = 0.f;
     // tokens past the end leave the state alone: no key, no step, decay 1
-    auto fetch = [&](int t0) {
+    auto load4 = [&](const float *p, float4 none) __attribute__((always_inline)) {
+        if (VEC) return *reinterpret_cast<const float4 *>(p);
+        float4 v = none;
+        v.x = p[0];
+        if (sd + 1 < a.dim) v.y = p[1];
+        if (sd + 2 < a.dim) v.z = p[2];
+        if (sd + 3 < a.dim) v.w = p[3];
+        return v;
+    };
+    auto fetch = [&](int t0) __attribute__((always_inline)) {
+        if (tid < DP) {
 #pragma unroll
-        for (int i = 0; i < NV; i++) {
-            const int e = (tid + 256 * i) * 4, t = e / DP, d = e % DP;
-            const bool in = t0 + t < T && t < TC && d < a.dim;
-            kr[i] = qr[i] = make_float4(0.f, 0.f, 0.f, 0.f);
-            if (PC) gr[PC ? i : 0] = make_float4(1.f, 1.f, 1.f, 1.f);
-            if (in) {
-                const float *k = a.k + ((r0 + t0 + t) * a.KV + kvh) * a.dim + d, *q = a.q + ((r0 + t0 + t) * a.KV + kvh) * a.dim + d;
-                const float *g = PC ? a.g + ((r0 + t0 + t) * a.H + h) * a.dim + d : nullptr;
-                if (VEC) {
-                    kr[i] = *reinterpret_cast<const float4 *>(k); qr[i] = *reinterpret_cast<const float4 *>(q);
-                    if (PC) gr[PC ? i : 0] = *reinterpret_cast<const float4 *>(g);
-                } else {
-                    float *kd = &kr[i].x, *qd = &qr[i].x, *gd = &gr[PC ? i : 0].x;
-#pragma unroll
-                    for (int u = 0; u < 4; u++) if (d + u < a.dim) { kd[u] = k[u]; qd[u] = q[u]; if (PC) gd[u] = g[u]; }
+            for (int i = 0; i < GT; i++) {
+                const int t = t0 + sgrp * GT + i;
+                const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f), one = make_float4(1.f, 1.f, 1.f, 1.f);
+                kr[i] = qr[i] = zero;
+                if (PC) gr[PC ? i : 0] = one;
+                if (t < T && sd < a.dim) {
+                    const size_t o = ((r0 + t) * a.KV + kvh) * a.dim + sd;
+                    kr[i] = load4(a.k + o, zero); qr[i] = load4(a.q + o, zero);
+                    if (PC) gr[PC ? i : 0] = load4(a.g + ((r0 + t) * a.H + h) * a.dim + sd, one);
                 }
             }
         }
@@ -164,95 +234,119 @@ __global__ __launch_bounds__(256) void k_delta_scan(DeltaRows a)
             const int e = tid + 256 * i, t = e / COLS, c = e % COLS;
             vr[i] = (t < TC && t0 + t < T && j0 + c < a.vdim) ? a.v[((r0 + t0 + t) * a.H + h) * a.vdim + j0 + c] : 0.f;
         }
-        if (tid < TC) {
-            br = make_float2(0.f, 0.f); gsr = 1.f;
-            if (t0 + tid < T) {
-                const size_t m = r0 + t0 + tid;
-                br = make_float2(a.beta[m * a.H + h], a.kq[m * a.KV + kvh]);
-                if (!PC) gsr = a.g[m * a.H + h];
+        if (tid < NG * GS) {
+            const int grp = t0 / GT + tid / GS;
+            pr = grp < groups ? a.pairs[(((size_t)b * groups + grp) * a.H + h) * GS + tid % GS] : 0.f;
+        }
+    };
+    auto mul4 = [](const float4 &x, const float4 &y) __attribute__((always_inline)) { return make_float4(x.x * y.x, x.y * y.y, x.z * y.z, x.w * y.w); };
+    auto park = [&](int s) __attribute__((always_inline)) {
+        if (tid < DP) {
+            float4 c = make_float4(1.f, 1.f, 1.f, 1.f), r = c;
+#pragma unroll
+            for (int i = 0; i < GT; i++) {
+                if (PC) c = mul4(c, gr[PC ? i : 0]);
+                const int at = (sgrp * GT + i) * DP + sd;
+                *reinterpret_cast<float4 *>(&ks[s][at]) = PC ? mul4(kr[i], c) : kr[i];
+                *reinterpret_cast<float4 *>(&qs[s][at]) = PC ? mul4(qr[i], c) : qr[i];
+            }
+            if (PC) {
+                *reinterpret_cast<float4 *>(&gs[s][sgrp * DP + sd]) = c;
+#pragma unroll
+                for (int i = GT - 1; i >= 0; i--) {
+                    *reinterpret_cast<float4 *>(&us[s][(sgrp * GT + i) * DP + sd]) = mul4(kr[i], r);
+                    r = mul4(r, gr[PC ? i : 0]);
+                }
             }
         }
-    };
-    auto park = [&](int s) {
 #pragma unroll
-        for (int i = 0; i < NV; i++) {
-            const int e = (tid + 256 * i) * 4;
-            if (e < TC * DP) {
-                *reinterpret_cast<float4 *>(&ks[s][e]) = kr[i]; *reinterpret_cast<float4 *>(&qs[s][e]) = qr[i];
-                if (PC) *reinterpret_cast<float4 *>(&gs[s][e]) = gr[PC ? i : 0];
+        for (int i = 0; i < NC; i++) { const int e = tid + 256 * i, t = e / COLS, c = e % COLS; if (t < TC) vs[s][c * TC + t] = vr[i]; }
+        if (tid < NG * GS) ps[s][tid] = pr;
+    };
+    struct Group { float4 k[GT][RB], q[GT][RB]; };
+    auto read = [&](Group &x, int s, int grp) __attribute__((always_inline)) {
+#pragma unroll
+        for (int i = 0; i < GT; i++)
+#pragma unroll
+            for (int r = 0; r < RB; r++) {
+                const int at = (grp * GT + i) * DP + r * 4 * G + 4 * l;
+                x.k[i][r] = *reinterpret_cast<const float4 *>(&ks[s][at]);
+                x.q[i][r] = *reinterpret_cast<const float4 *>(&qs[s][at]);
+            }
+    };
+    auto dot = [&](const float4 (&x)[RB]) __attribute__((always_inline)) {
+        float y[RB];
+#pragma unroll
+        for (int r = 0; r < RB; r++) y[r] = fmaf(S[4 * r + 3], x[r].w, fmaf(S[4 * r + 2], x[r].z, fmaf(S[4 * r + 1], x[r].y, S[4 * r] * x[r].x)));
+#pragma unroll
+        for (int r = 1; r < RB; r++) y[0] += y[r];
+        return y[0];
+    };
+    float keep[NK];
+    auto take = [&](const Group &x, int s, int grp) __attribute__((always_inline)) {
+        const float4 *n = reinterpret_cast<const float4 *>(&ps[s][grp * GS]);
+        const float4 be = n[0], a0 = n[1], a1 = n[2], b0 = n[3], b1 = n[4], b2 = n[5];
+        const float4 v = *reinterpret_cast<const float4 *>(&vs[s][col * TC + grp * GT]);
+        float p[GT], w[GT];
+#pragma unroll
+        for (int i = 0; i < GT; i++) { p[i] = dot(x.k[i]); w[i] = dot(x.q[i]); }
+#pragma unroll
+        for (int i = 0; i < GT; i++) { p[i] = group_sum<G>(p[i]); w[i] = group_sum<G>(w[i]); }
+        float u[GT];
+        float4 dr = make_float4(1.f, 1.f, 1.f, 1.f);
+        float all = 1.f;
+        if (!PC) {
+            const float4 dc = n[6];
+            dr = n[7];
+            p[0] *= dc.x; p[1] *= dc.y; p[2] *= dc.z; p[3] *= dc.w;
+            w[0] *= dc.x; w[1] *= dc.y; w[2] *= dc.z; w[3] *= dc.w;
+            all = dc.w;
+        }
+        u[0] = be.x * (v.x - p[0]);
+        u[1] = be.y * (v.y - p[1] - a0.x * u[0]);
+        u[2] = be.z * (v.z - p[2] - a0.y * u[0] - a0.z * u[1]);
+        u[3] = be.w * (v.w - p[3] - a0.w * u[0] - a1.x * u[1] - a1.y * u[2]);
+        const float o[GT] = {fmaf(b0.x, u[0], w[0]), fmaf(b0.z, u[1], fmaf(b0.y, u[0], w[1])),
+                             fmaf(b1.y, u[2], fmaf(b1.x, u[1], fmaf(b0.w, u[0], w[2]))),
+                             fmaf(b2.y, u[3], fmaf(b2.x, u[2], fmaf(b1.w, u[1], fmaf(b1.z, u[0], w[3]))))};
+        if (!PC) { u[0] *= dr.x; u[1] *= dr.y; u[2] *= dr.z; u[3] *= dr.w; }
+#pragma unroll
+        for (int r = 0; r < RB; r++) {
+            float4 g = make_float4(all, all, all, all);
+            if (PC) g = *reinterpret_cast<const float4 *>(&gs[s][grp * DP + r * 4 * G + 4 * l]);
+            float *z = &S[4 * r];
+            z[0] *= g.x; z[1] *= g.y; z[2] *= g.z; z[3] *= g.w;
+#pragma unroll
+            for (int i = 0; i < GT; i++) {
+                const float4 k = PC ? *reinterpret_cast<const float4 *>(&us[s][PC ? (grp * GT + i) * DP + r * 4 * G + 4 * l : 0]) : x.k[i][r];
+                z[0] = fmaf(k.x, u[i], z[0]); z[1] = fmaf(k.y, u[i], z[1]); z[2] = fmaf(k.z, u[i], z[2]); z[3] = fmaf(k.w, u[i], z[3]);
             }
         }
 #pragma unroll
-        for (int i = 0; i < NC; i++) { const int e = tid + 256 * i; if (e < TC * COLS) vs[s][e] = vr[i]; }
-        if (tid < TC) { bs[s][tid] = br; if (!PC) gs[s][tid] = gsr; }
-    };
-    struct Tok { float4 k[RB], q[RB], g[PC ? RB : 1]; float gv, v; float2 b; };
-    auto read = [&](Tok &x, int s, int t) __attribute__((always_inline)) {
-#pragma unroll
-        for (int i = 0; i < RB; i++) {
-            x.k[i] = *reinterpret_cast<const float4 *>(&ks[s][t * DP + i * 4 * G + 4 * l]);
-            x.q[i] = *reinterpret_cast<const float4 *>(&qs[s][t * DP + i * 4 * G + 4 * l]);
-            if (PC) x.g[PC ? i : 0] = *reinterpret_cast<const float4 *>(&gs[s][t * DP + i * 4 * G + 4 * l]);
+        for (int i = 0; i < GT; i++) {
+            const int t = grp * GT + i;
+            keep[t / G] = l == t % G ? o[i] : keep[t / G];
         }
-        if (!PC) x.gv = gs[s][t];
-        x.v = vs[s][t * COLS + col];
-        x.b = bs[s][t];
-    };
-    auto token = [&](const Tok &x) __attribute__((always_inline)) -> float {
-        float p[RB], w[RB];
-#pragma unroll
-        for (int i = 0; i < RB; i++) {
-            const float k[4] = {x.k[i].x, x.k[i].y, x.k[i].z, x.k[i].w}, q[4] = {x.q[i].x, x.q[i].y, x.q[i].z, x.q[i].w};
-            const float g[4] = {PC ? x.g[PC ? i : 0].x : x.gv, PC ? x.g[PC ? i : 0].y : x.gv, PC ? x.g[PC ? i : 0].z : x.gv, PC ? x.g[PC ? i : 0].w : x.gv};
-#pragma unroll
-            for (int e = 0; e < 4; e++) S[4 * i + e] *= g[e];
-            p[i] = S[4 * i] * k[0]; w[i] = S[4 * i] * q[0];
-#pragma unroll
-            for (int e = 1; e < 4; e++) { p[i] = fmaf(S[4 * i + e], k[e], p[i]); w[i] = fmaf(S[4 * i + e], q[e], w[i]); }
-        }
-#pragma unroll
-        for (int i = 1; i < RB; i++) { p[0] += p[i]; w[0] += w[i]; }
-        const float ps = group_sum<G>(p[0]), ws = group_sum<G>(w[0]);
-        const float u = x.b.x * (x.v - ps);
-#pragma unroll
-        for (int i = 0; i < RB; i++) {
-            const float k[4] = {x.k[i].x, x.k[i].y, x.k[i].z, x.k[i].w};
-#pragma unroll
-            for (int e = 0; e < 4; e++) S[4 * i + e] = fmaf(k[e], u, S[4 * i + e]);
-        }
-        return fmaf(u, x.b.y, ws);
     };
     fetch(0);
     park(0);
     __syncthreads();
     for (int t0 = 0, s = 0; t0 < T; t0 += TC, s ^= 1) {
         if (t0 + TC < T) fetch(t0 + TC);
-        float keep[NK];
 #pragma unroll
         for (int i = 0; i < NK; i++) keep[i] = 0.f;
-        if (T - t0 >= TC) {
-            Tok x[3];
-            read(x[0], s, 0); read(x[1], s, 1);
+        Group x[2];
+        read(x[0], s, 0);
 #pragma unroll
-            for (int t = 0; t < TC; t++) {
-                if (t + 2 < TC) read(x[(t + 2) % 3], s, t + 2);
-                const float o = token(x[t % 3]);
-                keep[t / G] = l == t % G ? o : keep[t / G];
-            }
-        } else {
-#pragma unroll 1
-            for (int t = 0; t < T - t0; t++) {
-                Tok x;
-                read(x, s, t);
-                const float o = token(x);
-#pragma unroll
-                for (int i = 0; i < NK; i++) if (t == i * G + l) keep[i] = o;
-            }
+        for (int grp = 0; grp < NG; grp++) {
+            if (t0 + grp * GT >= T) break;                // uniform
+            if (grp + 1 < NG) read(x[(grp + 1) & 1], s, grp + 1);
+            take(x[grp & 1], s, grp);
         }
 #pragma unroll
         for (int i = 0; i < NK; i++) {
-            const int t = t0 + i * G + l;
-            if (i * G + l < TC && t < T && j < a.vdim) a.o[((r0 + t) * a.H + h) * a.vdim + j] = keep[i];
+            const int t = i * G + l;
+            if (t < TC && t0 + t < T && j < a.vdim) a.o[((r0 + t0 + t) * a.H + h) * a.vdim + j] = keep[i];
         }
         if (t0 + TC < T) park(s ^ 1);                     // the other stage: its readers passed the barrier below
         __syncthreads();
@@ -308,12 +402,17 @@ __global__ __launch_bounds__(256) void k_cat_rows(CatRows a)
 
 }  // namespace
 
+int delta_groups(int T) { return (T + GT - 1) / GT; }
+size_t delta_pair_floats(int B, int T, int H) { return (size_t)B * delta_groups(T) * H * GS; }
+
 void launch_delta_inputs(const DeltaRows &a)
 {
-    const dim3 grid((a.KV + a.H + 3) / 4, (a.r.T + TW - 1) / TW, a.r.B);
-    if (a.dim <= 64) LAUNCH(k_delta_inputs<1>, grid, dim3(256), 0, a);
-    else if (a.dim <= 128) LAUNCH(k_delta_inputs<2>, grid, dim3(256), 0, a);
-    else LAUNCH(k_delta_inputs<4>, grid, dim3(256), 0, a);
+    const dim3 grid((a.KV + (a.H * a.vdim + 63) / 64 + 3) / 4, (a.r.T + TW - 1) / TW, a.r.B), pgrid((a.H + 3) / 4, delta_groups(a.r.T), a.r.B);
+#define INPUTS(E_) do { \
+    LAUNCH(k_delta_inputs<E_>, grid, dim3(256), 0, a); \
+    if (a.per_channel) LAUNCH((k_delta_pairs<E_, 1>), pgrid, dim3(256), 0, a); else LAUNCH((k_delta_pairs<E_, 0>), pgrid, dim3(256), 0, a); } while (0)
+    if (a.dim <= 64) INPUTS(1); else if (a.dim <= 128) INPUTS(2); else INPUTS(4);
+#undef INPUTS
 }
 
 void launch_delta_scan(const DeltaRows &a)

@@ -42,6 +42,7 @@ __device__ __forceinline__ void route_row(const float *z, int E, int top, int la
 }
 
 template <typename WT> struct Vec8;
+// eight consecutive weights of a row as fp32
 template <> struct Vec8<half_t> {
     static __device__ __forceinline__ void load(const half_t *p, float (&w)[8])
     {
@@ -58,19 +59,40 @@ template <> struct Vec8<float> {
     }
 };
 
-// lane's part of W[row] . x over `cols` (a multiple of 8)
+// eight products of a piece added to s
+__device__ __forceinline__ float dot8(const float (&w)[8], const float *x, float s)
+{
+    const float4 a = *reinterpret_cast<const float4 *>(x), b = *reinterpret_cast<const float4 *>(x + 4);
+    s = fmaf(w[0], a.x, s); s = fmaf(w[1], a.y, s); s = fmaf(w[2], a.z, s); s = fmaf(w[3], a.w, s);
+    s = fmaf(w[4], b.x, s); s = fmaf(w[5], b.y, s); s = fmaf(w[6], b.z, s); s = fmaf(w[7], b.w, s);
+    return s;
+}
+
+// lane's part of N rows . x over `cols` (a multiple of 8), added to s[]; U pieces of every row in flight.  The loads past
+// the end of a row ask for its last piece again and count nothing.
+template <int N, int U, typename WT>
+__device__ __forceinline__ void dot_rows(const WT *const (&w)[N], const float *x, int cols, int lane, float (&s)[N])
+{
+    for (int c0 = lane * 8; c0 - lane * 8 < cols; c0 += 512 * U) {
+        float wv[N][U][8];
+#pragma unroll
+        for (int u = 0; u < U; u++)
+#pragma unroll
+            for (int n = 0; n < N; n++) Vec8<WT>::load(w[n] + min(c0 + 512 * u, cols - 8), wv[n][u]);
+#pragma unroll
+        for (int u = 0; u < U; u++)
+            if (c0 + 512 * u < cols)
+#pragma unroll
+                for (int n = 0; n < N; n++) s[n] = dot8(wv[n][u], x + c0 + 512 * u, s[n]);
+    }
+}
 template <typename WT>
 __device__ __forceinline__ float dot_part(const WT *w, const float *x, int cols, int lane)
 {
-    float s = 0.f;
-    for (int c = lane * 8; c < cols; c += 512) {
-        float wv[8];
-        Vec8<WT>::load(w + c, wv);
-        const float4 x0 = *reinterpret_cast<const float4 *>(x + c), x1 = *reinterpret_cast<const float4 *>(x + c + 4);
-        s = fmaf(wv[0], x0.x, s); s = fmaf(wv[1], x0.y, s); s = fmaf(wv[2], x0.z, s); s = fmaf(wv[3], x0.w, s);
-        s = fmaf(wv[4], x1.x, s); s = fmaf(wv[5], x1.y, s); s = fmaf(wv[6], x1.z, s); s = fmaf(wv[7], x1.w, s);
-    }
-    return s;
+    const WT *const rows[1] = {w};
+    float s[1] = {0.f};
+    dot_rows<1, 4>(rows, x, cols, lane, s);
+    return s[0];
 }
 
 }  // namespace lmhip

@@ -55,11 +55,17 @@ __global__ __launch_bounds__(256) void k_latent_attend(LatentRows a, int m0, int
     for (int i = tid; i < HG * w; i += 256) qs[i] = a.q[((size_t)m * a.H + min(h0 + i / w, a.H - 1)) * w + i % w];
     __syncthreads();
     const float *ring = a.ring + (size_t)b * a.ring_rows * w;
+    const int slot_j0 = j0 % a.ring_rows;                 // row of key j0; the slice wraps at most once
+    auto key_row = [&](int jj) __attribute__((always_inline)) {
+        const int r = slot_j0 + jj;
+        return ring + (size_t)(r >= a.ring_rows ? r - a.ring_rows : r) * w;
+    };
     // scores: sixteen lanes per key
     for (int jj = tid >> 4; jj < SLK; jj += 16) {
         if (jj >= nj) break;                              // uniform over the sixteen lanes of the key
-        const float *key = ring + (size_t)((j0 + jj) % a.ring_rows) * w;
+        const float *key = key_row(jj);
         float s[HG] = {};
+#pragma unroll 4
         for (int c = (tid & 15) * 4; c < w; c += 64) {
             const float4 k = *reinterpret_cast<const float4 *>(key + c);
 #pragma unroll
@@ -86,8 +92,9 @@ __global__ __launch_bounds__(256) void k_latent_attend(LatentRows a, int m0, int
         float4 o[HG];
 #pragma unroll
         for (int u = 0; u < HG; u++) o[u] = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll 8
         for (int jj = part; jj < nj; jj += parts) {
-            const float4 v = *reinterpret_cast<const float4 *>(ring + (size_t)((j0 + jj) % a.ring_rows) * w + c);
+            const float4 v = *reinterpret_cast<const float4 *>(key_row(jj) + c);
 #pragma unroll
             for (int u = 0; u < HG; u++) {
                 const float e = sc[u * SLK + jj];
@@ -112,7 +119,7 @@ constexpr int VR = 16;
 template <typename WT>
 __global__ __launch_bounds__(256) void k_latent_values(LatentRows a, int m0, int nsplit)
 {
-    extern __shared__ float ctx[];                        // [rp], then the slices' factors [nsplit]
+    extern __shared__ float ctx[];                        // [rp], the slices' factors [nsplit], sums [shares][rp]
     const int h = blockIdx.x, m = m0 + blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, rp = rank_pad(a);
     float *fac = ctx + rp;
     const size_t slot0 = ((size_t)(m - m0) * a.H + h) * nsplit;
@@ -125,18 +132,36 @@ __global__ __launch_bounds__(256) void k_latent_values(LatentRows a, int m0, int
     l = wave_total(l);
     for (int s = tid; s < nsplit; s += 256) fac[s] = ml[2 * s + 1] > 0.f ? expf(ml[2 * s] - mx) / l : 0.f;
     __syncthreads();
-    for (int c = tid; c < rp; c += 256) {
-        float o = 0.f;
+    // four columns of a share of the slices per thread (a slice without keys holds nothing that counts)
+    float *red = fac + ((nsplit + 3) & ~3);
+    const int nc = rp / 4, shares = max(1, min(8, 256 / nc)), part = tid / nc, c = (tid % nc) * 4;
+    if (part < shares) {
+        float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
 #pragma unroll 8
-        for (int s = 0; s < nsplit; s++)                  // (a slice without keys has left nothing to read)
-            if (fac[s] > 0.f) o = fmaf(a.part_o[(slot0 + s) * rp + c], fac[s], o);
-        ctx[c] = o;
+        for (int s = part; s < nsplit; s += shares) {
+            const float f = fac[s];
+            const float4 v = *reinterpret_cast<const float4 *>(a.part_o + (slot0 + s) * rp + c);
+            if (f > 0.f) { o.x = fmaf(v.x, f, o.x); o.y = fmaf(v.y, f, o.y); o.z = fmaf(v.z, f, o.z); o.w = fmaf(v.w, f, o.w); }
+        }
+        *reinterpret_cast<float4 *>(red + part * rp + c) = o;
     }
     __syncthreads();
-    for (int i = blockIdx.z * VR + wave; i < min(a.vdim, (int)(blockIdx.z + 1) * VR); i += 4) {
-        const WT *uv = (const WT *)a.ukv + ((size_t)a.H * a.dim + (size_t)h * a.vdim + i) * a.ldu;
-        const float s = wave_sum(dot_part(uv, ctx, rp, lane));
-        if (lane == 0) a.o[((size_t)m * a.H + h) * a.vdim + i] = s;
+    for (int i = tid; i < rp; i += 256) {
+        float o = 0.f;
+        for (int k = 0; k < shares; k++) o += red[k * rp + i];
+        ctx[i] = o;
+    }
+    __syncthreads();
+    const int i0 = blockIdx.z * VR + wave * (VR / 4);
+    const WT *uv[VR / 4];
+    float y[VR / 4] = {};
+#pragma unroll
+    for (int k = 0; k < VR / 4; k++) uv[k] = (const WT *)a.ukv + ((size_t)a.H * a.dim + (size_t)h * a.vdim + min(i0 + k, a.vdim - 1)) * a.ldu;
+    dot_rows<VR / 4, 1>(uv, ctx, rp, lane, y);
+#pragma unroll
+    for (int k = 0; k < VR / 4; k++) {
+        const float t = wave_total(y[k]);
+        if (lane == 0 && i0 + k < a.vdim) a.o[((size_t)m * a.H + h) * a.vdim + i0 + k] = t;
     }
 }
 
@@ -172,11 +197,12 @@ void launch_latent_slices(const LatentRows &a, const LatentSlices &s, int m0, in
 {
     const int rp = pad8(a.rank), w = rp + pad8(a.rot), parts = std::max(1, 256 / (rp / 4));
     const size_t lds = ((size_t)HG * w + (size_t)HG * s.keys + (size_t)parts * HG * rp) * sizeof(float);
+    const size_t vlds = ((size_t)rp + ((s.n + 3) & ~3) + (size_t)std::max(1, std::min(8, 256 / (rp / 4))) * rp) * sizeof(float);
     const dim3 grid(s.n, (a.H + HG - 1) / HG, nr), vgrid(a.H, nr, (a.vdim + VR - 1) / VR);
     if (s.keys == 32) LAUNCH(k_latent_attend<32>, grid, dim3(256), lds, a, m0, s.n);
     else LAUNCH(k_latent_attend<64>, grid, dim3(256), lds, a, m0, s.n);
-    if (a.f32) LAUNCH(k_latent_values<float>, vgrid, dim3(256), (size_t)(rp + s.n) * 4, a, m0, s.n);
-    else LAUNCH(k_latent_values<half_t>, vgrid, dim3(256), (size_t)(rp + s.n) * 4, a, m0, s.n);
+    if (a.f32) LAUNCH(k_latent_values<float>, vgrid, dim3(256), vlds, a, m0, s.n);
+    else LAUNCH(k_latent_values<half_t>, vgrid, dim3(256), vlds, a, m0, s.n);
 }
 
 void launch_latent_attend(const LatentRows &in)

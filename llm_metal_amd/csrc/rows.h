@@ -30,6 +30,18 @@ __device__ __forceinline__ float dpp_add(float v)
 {
     return v + __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, true));
 }
+// v of this lane plus v of the lane 16 (32) away: the swaps exchange the rows of sixteen (halves) of two registers, here
+// two copies of v
+__device__ __forceinline__ float swap16_add(float v)
+{
+    const auto t = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    return __uint_as_float(t[0]) + __uint_as_float(t[1]);
+}
+__device__ __forceinline__ float swap32_add(float v)
+{
+    const auto t = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    return __uint_as_float(t[0]) + __uint_as_float(t[1]);
+}
 template <int G>
 __device__ __forceinline__ float group_sum(float v)
 {
@@ -37,16 +49,14 @@ __device__ __forceinline__ float group_sum(float v)
     v = dpp_add<0x4E>(v);                                 // quad lanes 2 3 0 1
     if (G >= 8) v = dpp_add<0x141>(v);                    // mirror of eight lanes
     if (G >= 16) v = dpp_add<0x140>(v);                   // mirror of sixteen lanes
-    if (G >= 32) v += __shfl_xor(v, 16, WAVE);
+    if (G >= 32) v = swap16_add(v);
     return v;
 }
 
 // sum over the wave, left in every lane
 __device__ __forceinline__ float wave_total(float v)
 {
-    v = group_sum<16>(v);
-    v += __shfl_xor(v, 16, WAVE);
-    return v + __shfl_xor(v, 32, WAVE);
+    return swap32_add(group_sum<32>(v));
 }
 
 }  // namespace lmhip

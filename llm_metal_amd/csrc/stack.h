@@ -157,10 +157,11 @@ struct DeltaRows {
     const float *cin; int ldc, o_q, o_k, o_v, o_b, o_a;  // the input product
     const float *filters, *a_exp, *dt_bias;
     float *conv, *S;                                     // state
-    float *q, *k, *v, *kq, *beta, *g;                    // intermediates: [rows][KV][dim] x 2, [rows][H][vdim], [rows][KV], [rows][H], [rows][H] or [rows][H][dim]
+    float *q, *k, *v, *g, *pairs;                        // intermediates: [rows][KV][dim] x 2, [rows][H][vdim], [rows][H][dim] (per channel), [groups][H][..]
     const float *a2;                                     // per channel: W_a2 (W_a1 h) [rows][H * dim]
     float *o;                                            // [rows][H][vdim]
 };
+size_t delta_pair_floats(int B, int T, int H);           // size of `pairs`
 void launch_delta_inputs(const DeltaRows &a);            // convolutions, unit norms, step sizes, decays
 void launch_delta_scan(const DeltaRows &a);              // the recurrence; also moves the convolution's last inputs into the state
 

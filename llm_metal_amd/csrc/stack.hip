@@ -222,14 +222,15 @@ struct Aux {
     float *take(size_t n) { float *p = base ? base + at : nullptr; at += (n + 3) & ~(size_t)3; return p; }
 };
 
-struct DeltaAux { float *q, *k, *v, *kq, *beta, *g, *a2, *g2, *o; };
-DeltaAux delta_aux(Aux &x, const LayerConfig &c, size_t rows)
+struct DeltaAux { float *q, *k, *v, *g, *pairs, *a2, *g2, *o; };
+DeltaAux delta_aux(Aux &x, const LayerConfig &c, int B, int T)
 {
+    const size_t rows = (size_t)B * T;
     const bool pc = c.mixer == MIX_CHANNEL_DELTA;
     DeltaAux d{};
     d.q = x.take(rows * c.kv_heads * c.dim); d.k = x.take(rows * c.kv_heads * c.dim); d.v = x.take(rows * c.heads * c.vdim);
-    d.kq = x.take(rows * c.kv_heads); d.beta = x.take(rows * c.heads);
-    d.g = x.take(rows * c.heads * (pc ? c.dim : 1));
+    d.g = x.take(pc ? rows * c.heads * c.dim : 0);
+    d.pairs = x.take(delta_pair_floats(B, T, c.heads));
     d.a2 = x.take(pc ? rows * c.heads * c.dim : 0); d.g2 = x.take(pc ? rows * c.heads * c.vdim : 0);
     d.o = x.take(rows * c.heads * c.vdim);
     return d;
@@ -287,7 +288,7 @@ StackRun *stack_run_create(const LayerStack *st, int B)
         if (L.delta()) {
             k.S = fbuf((size_t)B * c.heads * c.vdim * c.dim);
             k.conv = fbuf((size_t)B * c.taps * L.channels());
-            delta_aux(a, c, r->rows);
+            delta_aux(a, c, B, portion);
             kmax = std::max({kmax, L.a2.cols, L.g2.cols});
         } else {
             k.ring_rows = std::min(st->max_seq, c.window - 1 + portion);
@@ -379,7 +380,7 @@ DeltaRows delta_rows(const LayerStack *st, const StackRun *r, const StackLayer &
     a.cin = ptr<float>(r->cin); a.ldc = L.in.rows; a.o_q = L.o_q; a.o_k = L.o_k; a.o_v = L.o_v; a.o_b = L.o_b; a.o_a = L.o_a;
     a.filters = ptr<float>(L.conv); a.a_exp = ptr<float>(L.a_exp); a.dt_bias = ptr<float>(L.dt_bias);
     a.conv = ptr<float>(k.conv); a.S = ptr<float>(k.S);
-    a.q = d.q; a.k = d.k; a.v = d.v; a.kq = d.kq; a.beta = d.beta; a.g = d.g; a.a2 = d.a2; a.o = d.o;
+    a.q = d.q; a.k = d.k; a.v = d.v; a.g = d.g; a.pairs = d.pairs; a.a2 = d.a2; a.o = d.o;
     return a;
 }
 
@@ -412,7 +413,7 @@ float *mix_delta(LayerStack *st, StackRun *r, StackLayer &L, StackRun::Layer &k,
     const int n = rows.n(), ldc = L.in.rows;
     const bool pc = c.mixer == MIX_CHANNEL_DELTA;
     Aux ax{ptr<float>(r->aux)};
-    const DeltaAux d = delta_aux(ax, c, n);
+    const DeltaAux d = delta_aux(ax, c, rows.B, rows.T);
     const float *cin = ptr<float>(r->cin);
     if (pc) {                                             // the second halves of the two low-rank products
         auto low_rank = [&](const StackMat &w, int col, float *out) {
@@ -475,7 +476,7 @@ void decode_layers(LayerStack *st, StackRun *r, int pos)
         o.out = ptr<half_t>(L.out.buf); o.x = x; o.D = st->D;
         Aux ax{ptr<float>(r->aux)};
         if (L.delta()) {
-            const DeltaAux d = delta_aux(ax, c, 1);
+            const DeltaAux d = delta_aux(ax, c, 1, 1);
             DecodeDelta s{};
             s.a = delta_rows(st, r, L, k, rows, d);
             s.a2 = ptr<half_t>(L.a2.buf); s.g2 = ptr<half_t>(L.g2.buf); s.lda2 = L.a2.cols; s.ldg2 = L.g2.cols; s.o_g = L.o_g;

@@ -45,12 +45,21 @@ __device__ __forceinline__ void experts_up(const DecodeMoe &a, int blk, float *l
     const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)a.D + a.eps);
     if (blk == 0 && tid < a.top) { a.idx[tid] = idx[tid]; a.w[tid] = w[tid]; }
     const int n = a.top * a.ffp;
-    for (int k = 0; k < UP_ROWS / 4; k++) {
-        const int r = blk * UP_ROWS + wave * (UP_ROWS / 4) + k, s = r / a.ffp, i = r % a.ffp;
-        if (r >= n) break;
-        float v = 0.f;
-        if (i < a.ff) v = wave_total(dot_part(a.up + ((size_t)idx[s] * a.up_rows + i) * a.Dp, lds, a.Dp, lane)) * inv;
-        if (lane == 0) a.act[r] = relu2(v);               // the padding is written too: zero
+    constexpr int PER = UP_ROWS / 4;
+    const int r0 = blk * UP_ROWS + wave * PER;
+    const half_t *rows[PER];
+    float y[PER];
+#pragma unroll
+    for (int k = 0; k < PER; k++) {
+        const int r = min(r0 + k, n - 1), s = r / a.ffp, i = min(r % a.ffp, a.ff - 1);
+        rows[k] = a.up + ((size_t)idx[s] * a.up_rows + i) * a.Dp;
+        y[k] = 0.f;
+    }
+    dot_rows<PER, 2>(rows, lds, a.Dp, lane, y);
+#pragma unroll
+    for (int k = 0; k < PER; k++) {
+        const float v = wave_total(y[k]) * inv;
+        if (lane == 0 && r0 + k < n) a.act[r0 + k] = (r0 + k) % a.ffp < a.ff ? relu2(v) : 0.f;   // the padding is written too
     }
 }
 
@@ -153,9 +162,9 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentRows a, DecodeMoe e
 }
 
 // x[d] += out[d] . (mixer output | shared activation) + sum over the chosen experts of w * down_e[d] . act_e; a wave takes
-// `per` values of d.  lds: [ldk] then [top * ffp]
-template <int TPB>
-__global__ __launch_bounds__(TPB) void k_out_decode(DecodeOut a, DecodeMoe e, int per)
+// PER values of d.  lds: [ldk] then [top * ffp]
+template <int TPB, int PER>
+__global__ __launch_bounds__(TPB) void k_out_decode(DecodeOut a, DecodeMoe e)
 {
     extern __shared__ float lds[];
     constexpr int NW = TPB / 64;
@@ -179,13 +188,39 @@ __global__ __launch_bounds__(TPB) void k_out_decode(DecodeOut a, DecodeMoe e, in
         cat[i] = s >= 0 && s < c.shared_ff ? relu2(c.shared[s]) : 0.f;
     }
     __syncthreads();
-    const int d0 = (blockIdx.x * NW + wave) * per;
-    for (int d = d0; d < min(d0 + per, a.D); d++) {
-        float y = dot_part(a.out + (size_t)d * c.ldk, cat, c.ldk, lane);
-        for (int s = 0; s < e.top; s++)
-            y = fmaf(e.w[s], dot_part(e.down + ((size_t)e.idx[s] * e.down_rows + d) * e.ffp, act + s * e.ffp, e.ffp, lane), y);
-        y = wave_total(y);
-        if (lane == 0) a.x[d] += y;
+    // PER rows of one wave at a time, the pieces of four experts (or of the dense row) in flight together
+    const int d0 = (blockIdx.x * NW + wave) * PER;
+    if (d0 >= a.D) return;
+    float y[PER] = {};
+    const half_t *rows[PER];
+#pragma unroll
+    for (int k = 0; k < PER; k++) rows[k] = a.out + (size_t)min(d0 + k, a.D - 1) * c.ldk;
+    dot_rows<PER, 8 / PER>(rows, cat, c.ldk, lane, y);
+    for (int s0 = 0; s0 < e.top; s0 += 4) {
+        const half_t *base[4];
+        float wt[4];
+#pragma unroll
+        for (int u = 0; u < 4; u++) {
+            const int s = min(s0 + u, e.top - 1);
+            base[u] = e.down + ((size_t)e.idx[s] * e.down_rows) * e.ffp;
+            wt[u] = s0 + u < e.top ? e.w[s] : 0.f;
+        }
+        for (int cc = lane * 8; cc < e.ffp; cc += 512) {
+            float wv[PER][4][8];
+#pragma unroll
+            for (int k = 0; k < PER; k++)
+#pragma unroll
+                for (int u = 0; u < 4; u++) Vec8<half_t>::load(base[u] + (size_t)min(d0 + k, a.D - 1) * e.ffp + cc, wv[k][u]);
+#pragma unroll
+            for (int u = 0; u < 4; u++)
+#pragma unroll
+                for (int k = 0; k < PER; k++) y[k] = fmaf(wt[u], dot8(wv[k][u], act + min(s0 + u, e.top - 1) * e.ffp + cc, 0.f), y[k]);
+        }
+    }
+#pragma unroll
+    for (int k = 0; k < PER; k++) {
+        const float t = wave_total(y[k]);
+        if (lane == 0 && d0 + k < a.D) a.x[d0 + k] += t;
     }
 }
 
@@ -224,15 +259,15 @@ void launch_out_decode(const DecodeOut &a, const DecodeMoe &e)
     const size_t lds = ((size_t)a.cat.ldk + (size_t)e.top * e.ffp) * sizeof(float);
     static bool set = false;
     if (!set) {                                           // more than the default 64 KB
-        HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void *>(&k_out_decode<512>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)DECODE_LDS));
-        HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void *>(&k_out_decode<256>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)DECODE_LDS));
+        for (const void *k : {reinterpret_cast<const void *>(&k_out_decode<512, 2>), reinterpret_cast<const void *>(&k_out_decode<512, 1>), reinterpret_cast<const void *>(&k_out_decode<256, 1>)})
+            HIP_CHECK(hipFuncSetAttribute(k, hipFuncAttributeMaxDynamicSharedMemorySize, (int)DECODE_LDS));
         set = true;
     }
     // as many rows per workgroup as still give every CU one: each stages both vectors
     const int cus = num_cus() > 0 ? num_cus() : 256;
-    if (a.D >= 16 * cus) LAUNCH(k_out_decode<512>, dim3((a.D + 15) / 16), dim3(512), lds, a, e, 2);
-    else if (a.D >= 8 * cus) LAUNCH(k_out_decode<512>, dim3((a.D + 7) / 8), dim3(512), lds, a, e, 1);
-    else LAUNCH(k_out_decode<256>, dim3((a.D + 3) / 4), dim3(256), lds, a, e, 1);
+    if (a.D >= 16 * cus) LAUNCH((k_out_decode<512, 2>), dim3((a.D + 15) / 16), dim3(512), lds, a, e);
+    else if (a.D >= 8 * cus) LAUNCH((k_out_decode<512, 1>), dim3((a.D + 7) / 8), dim3(512), lds, a, e);
+    else LAUNCH((k_out_decode<256, 1>), dim3((a.D + 3) / 4), dim3(256), lds, a, e);
 }
 
 }  // namespace lmhip
