@@ -178,8 +178,8 @@ __global__ __launch_bounds__(256) void k_delta_pairs(DeltaRows a)
 
 // The recurrence.  The columns of a head's state (one per value channel) do not meet: a column is G lanes of a wave, each
 // with R of its rows -- lane l of the group has rows 4 l .. 4 l + 3 of every block of 4 G -- so no token costs a barrier.
-// Tokens are staged through LDS TC at a time with the decays already on the keys and queries, the next TC on their way in
-// registers; a group's LDS reads are issued one group ahead.  The lane numbered like a token keeps its output until the
+// Tokens are staged through LDS TC at a time with the decays already on the keys and queries, the next two stages on their
+// way in registers; a group's LDS reads are issued one group ahead.  The lane numbered like a token keeps its output until the
 // stage is over.
 // grid (column blocks of 256 / G, H, B), block 256.  VEC: dim is a multiple of 4 (16-byte loads).
 template <int G, int R, int PC, int VEC>
@@ -201,67 +201,66 @@ __global__ __launch_bounds__(256) void k_delta_scan(DeltaRows a)
         const int d = (e >> 2) * 4 * G + 4 * l + (e & 3);
         S[e] = (a.r.pos > 0 && d < a.dim) ? Sg[d] : 0.f;  // position 0 starts from nothing, whatever the state held
     }
-    const int sd = (tid % (DP / 4)) * 4, sgrp = tid / (DP / 4);          // staging: four columns of one group (tid < DP)
-    float4 kr[GT], qr[GT], gr[PC ? GT : 1];
-    float vr[NC], pr = 0.f;
-    // tokens past the end leave the state alone: no key, no step, decay 1
-    auto load4 = [&](const float *p, float4 none) __attribute__((always_inline)) {
-        if (VEC) return *reinterpret_cast<const float4 *>(p);
-        float4 v = none;
-        v.x = p[0];
-        if (sd + 1 < a.dim) v.y = p[1];
-        if (sd + 2 < a.dim) v.z = p[2];
-        if (sd + 3 < a.dim) v.w = p[3];
-        return v;
+    // staging: a thread brings four columns of the four tokens of one group (threads from DP on repeat others' reads and
+    // park nothing).  Two register sets, a stage's loads are asked for two stages ahead.  Every load is unconditional, past
+    // the end for the last token again: under a condition the compiler could not tell the two sets' loads apart and would
+    // wait for both.  What lies past the end is taken out when it is parked: no key, no step, decay 1.
+    const int sd = (tid % (DP / 4)) * 4, sgrp = tid / (DP / 4) % NG;
+    struct Stage { float4 k[GT], q[GT], g[PC ? GT : 1]; float v[NC], p; };
+    auto at = [](const float *base, uint32_t i) __attribute__((always_inline)) { return reinterpret_cast<const float *>(reinterpret_cast<const char *>(base) + 4u * i); };
+    auto load4 = [&](const float *base, uint32_t i) __attribute__((always_inline)) {
+        if (VEC) return *reinterpret_cast<const float4 *>(at(base, i));
+        const uint32_t last = (uint32_t)(a.dim - 1 - min(sd, a.dim - 1));
+        return make_float4(*at(base, i), *at(base, i + min(1u, last)), *at(base, i + min(2u, last)), *at(base, i + min(3u, last)));
     };
-    auto fetch = [&](int t0) __attribute__((always_inline)) {
-        if (tid < DP) {
+    const uint32_t kq0 = (uint32_t)((r0 * a.KV + kvh) * a.dim + min(sd, a.dim - (VEC ? 4 : 1)));
+    const uint32_t g0 = (uint32_t)((r0 * a.H + h) * a.dim + min(sd, a.dim - (VEC ? 4 : 1)));
+    auto fetch = [&](Stage &x, int t0) __attribute__((always_inline)) {
 #pragma unroll
-            for (int i = 0; i < GT; i++) {
-                const int t = t0 + sgrp * GT + i;
-                const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f), one = make_float4(1.f, 1.f, 1.f, 1.f);
-                kr[i] = qr[i] = zero;
-                if (PC) gr[PC ? i : 0] = one;
-                if (t < T && sd < a.dim) {
-                    const size_t o = ((r0 + t) * a.KV + kvh) * a.dim + sd;
-                    kr[i] = load4(a.k + o, zero); qr[i] = load4(a.q + o, zero);
-                    if (PC) gr[PC ? i : 0] = load4(a.g + ((r0 + t) * a.H + h) * a.dim + sd, one);
-                }
-            }
+        for (int i = 0; i < GT; i++) {
+            const uint32_t t = (uint32_t)min(t0 + sgrp * GT + i, T - 1);
+            const uint32_t o = kq0 + t * (uint32_t)(a.KV * a.dim);
+            x.k[i] = load4(a.k, o); x.q[i] = load4(a.q, o);
+            if (PC) x.g[PC ? i : 0] = load4(a.g, g0 + t * (uint32_t)(a.H * a.dim));
         }
 #pragma unroll
         for (int i = 0; i < NC; i++) {
-            const int e = tid + 256 * i, t = e / COLS, c = e % COLS;
-            vr[i] = (t < TC && t0 + t < T && j0 + c < a.vdim) ? a.v[((r0 + t0 + t) * a.H + h) * a.vdim + j0 + c] : 0.f;
+            const int e = tid + 256 * i, t = e / COLS % TC, c = e % COLS;
+            x.v[i] = *at(a.v, (uint32_t)(((r0 + min(t0 + t, T - 1)) * a.H + h) * a.vdim + min(j0 + c, a.vdim - 1)));
         }
-        if (tid < NG * GS) {
-            const int grp = t0 / GT + tid / GS;
-            pr = grp < groups ? a.pairs[(((size_t)b * groups + grp) * a.H + h) * GS + tid % GS] : 0.f;
-        }
+        const int grp = min(t0 / GT + tid / GS % NG, groups - 1);
+        x.p = *at(a.pairs, (uint32_t)((((size_t)b * groups + grp) * a.H + h) * GS + tid % GS));
     };
     auto mul4 = [](const float4 &x, const float4 &y) __attribute__((always_inline)) { return make_float4(x.x * y.x, x.y * y.y, x.z * y.z, x.w * y.w); };
-    auto park = [&](int s) __attribute__((always_inline)) {
+    auto park = [&](const Stage &x, int t0, int s) __attribute__((always_inline)) {
         if (tid < DP) {
-            float4 c = make_float4(1.f, 1.f, 1.f, 1.f), r = c;
+            const float4 one = make_float4(1.f, 1.f, 1.f, 1.f);
+            float4 c = one, r = one, k[GT], g[GT];
 #pragma unroll
             for (int i = 0; i < GT; i++) {
-                if (PC) c = mul4(c, gr[PC ? i : 0]);
-                const int at = (sgrp * GT + i) * DP + sd;
-                *reinterpret_cast<float4 *>(&ks[s][at]) = PC ? mul4(kr[i], c) : kr[i];
-                *reinterpret_cast<float4 *>(&qs[s][at]) = PC ? mul4(qr[i], c) : qr[i];
+                const bool in = t0 + sgrp * GT + i < T;
+                const float f0 = in && sd < a.dim ? 1.f : 0.f, f1 = in && (VEC ? sd : sd + 1) < a.dim ? 1.f : 0.f;
+                const float f2 = in && (VEC ? sd : sd + 2) < a.dim ? 1.f : 0.f, f3 = in && (VEC ? sd : sd + 3) < a.dim ? 1.f : 0.f;
+                const float4 f = make_float4(f0, f1, f2, f3);
+                k[i] = mul4(x.k[i], f);
+                g[i] = PC && in ? x.g[PC ? i : 0] : one;
+                c = mul4(c, g[i]);
+                const int to = (sgrp * GT + i) * DP + sd;
+                *reinterpret_cast<float4 *>(&ks[s][to]) = PC ? mul4(k[i], c) : k[i];
+                *reinterpret_cast<float4 *>(&qs[s][to]) = PC ? mul4(mul4(x.q[i], f), c) : mul4(x.q[i], f);
             }
             if (PC) {
                 *reinterpret_cast<float4 *>(&gs[s][sgrp * DP + sd]) = c;
 #pragma unroll
                 for (int i = GT - 1; i >= 0; i--) {
-                    *reinterpret_cast<float4 *>(&us[s][(sgrp * GT + i) * DP + sd]) = mul4(kr[i], r);
-                    r = mul4(r, gr[PC ? i : 0]);
+                    *reinterpret_cast<float4 *>(&us[s][(sgrp * GT + i) * DP + sd]) = mul4(k[i], r);
+                    r = mul4(r, g[i]);
                 }
             }
         }
 #pragma unroll
-        for (int i = 0; i < NC; i++) { const int e = tid + 256 * i, t = e / COLS, c = e % COLS; if (t < TC) vs[s][c * TC + t] = vr[i]; }
-        if (tid < NG * GS) ps[s][tid] = pr;
+        for (int i = 0; i < NC; i++) { const int e = tid + 256 * i, t = e / COLS, c = e % COLS; if (t < TC) vs[s][c * TC + t] = x.v[i]; }
+        if (tid < NG * GS) ps[s][tid] = x.p;              // (step sizes past the end are zero already)
     };
     struct Group { float4 k[GT][RB], q[GT][RB]; };
     auto read = [&](Group &x, int s, int grp) __attribute__((always_inline)) {
@@ -328,11 +327,9 @@ __global__ __launch_bounds__(256) void k_delta_scan(DeltaRows a)
             keep[t / G] = l == t % G ? o[i] : keep[t / G];
         }
     };
-    fetch(0);
-    park(0);
-    __syncthreads();
-    for (int t0 = 0, s = 0; t0 < T; t0 += TC, s ^= 1) {
-        if (t0 + TC < T) fetch(t0 + TC);
+    Stage even, odd;
+    auto stage = [&](int t0, int s, Stage &ahead, const Stage &next) __attribute__((always_inline)) {
+        fetch(ahead, t0 + 2 * TC);
 #pragma unroll
         for (int i = 0; i < NK; i++) keep[i] = 0.f;
         Group x[2];
@@ -343,13 +340,21 @@ __global__ __launch_bounds__(256) void k_delta_scan(DeltaRows a)
             if (grp + 1 < NG) read(x[(grp + 1) & 1], s, grp + 1);
             take(x[grp & 1], s, grp);
         }
+        park(next, t0 + TC, s ^ 1);                       // the other stage: its readers passed the barrier before this one
 #pragma unroll
         for (int i = 0; i < NK; i++) {
             const int t = i * G + l;
             if (t < TC && t0 + t < T && j < a.vdim) a.o[((r0 + t0 + t) * a.H + h) * a.vdim + j] = keep[i];
         }
-        if (t0 + TC < T) park(s ^ 1);                     // the other stage: its readers passed the barrier below
         __syncthreads();
+    };
+    fetch(even, 0);
+    fetch(odd, TC);
+    park(even, 0, 0);
+    __syncthreads();
+    for (int t0 = 0; t0 < T; t0 += 2 * TC) {
+        stage(t0, 0, even, odd);
+        if (t0 + TC < T) stage(t0 + TC, 1, odd, even);
     }
     if (j < a.vdim)
 #pragma unroll
