@@ -1,5 +1,5 @@
 // Gated delta rule: short causal convolutions, unit norms, decays, the recurrence over tokens, the gated head norm.
-// Everything here is fp32.
+// Everything here is fp32, the matrix instructions of the recurrence included.
 #include "stack.h"
 #include "delta_rows.h"
 
@@ -96,272 +96,214 @@ __global__ __launch_bounds__(256) void k_delta_inputs(DeltaRows a)
     for (int i = 0; i < TW; i++) if (i < nt && in[0]) a.v[(size_t)(m0 + i) * vd + c] = y[i][0];
 }
 
-// ---------------------------------------------------------------- tokens in groups of four
+// ---------------------------------------------------------------- tokens in chunks of sixteen
 //
-// Four tokens are taken through the recurrence together.  With S the state ahead of them, d(j, i) the decay between
-// writing token j and reading token i (the product of the decays of j + 1 .. i) and d(0-, i) the one from S to i:
-//     p_i = S^T (d(0-, i) k_i)          w_i = S^T (d(0-, i) q_i)
+// Sixteen tokens are taken through the recurrence together.  With S the state ahead of them, d(j, i) the decay between
+// writing token j and reading token i (the product of the decays of j + 1 .. i) and d(-, i) the one from S to i:
+//     p_i = S^T (d(-, i) k_i)           w_i = S^T (d(-, i) q_i)
 //     u_i = beta_i (v_i - p_i - sum_{j < i} A_ij u_j)      A_ij = k_i . d(j, i) k_j
 //     o_i = w_i + sum_{j <= i} B_ij u_j                    B_ij = q_i . d(j, i) k_j
-//     S  <- d(0-, 3) S + sum_j d(j, 3) k_j u_j^T
-// which is the token-by-token recurrence with the sums written out: all eight products with the state run side by side,
-// and the state is written once.  The numbers that do not depend on the state are made ahead, 32 per group and head:
-//     0 .. 3 beta | 4 .. 9 A10 A20 A21 A30 A31 A32 | 12 .. 21 B00 B10 B11 B20 B21 B22 B30 B31 B32 B33
-//     | 24 .. 27 d(0-, i) | 28 .. 31 d(i, 3)  (the last two with one decay per head only)
-constexpr int GT = 4, GS = 32;
+//     S  <- d(-, 15) S + sum_j d(j, 15) k_j u_j^T
+// which is the token-by-token recurrence with the sums written out.  All decays enter as products of factors up to 1 --
+// nothing is divided by a decay that may have vanished.  The u_i are U = M (V - P) with M = (I + diag(beta) A)^-1
+// diag(beta), so a chunk is a few small matrix products.  What does not depend on the state (M, B, the decayed keys and
+// queries) is made for all chunks at once by k_delta_prepare; k_delta_chunks then goes through them in order.
+//
+// Layouts, per (sequence, chunk, head), dimensions padded with zeros to DP (whole tiles of 16, the same number per wave):
+//   kd, qd [tiles][lane][4]: lane -> token lane & 15, dimensions 4 (lane >> 4) + 0 .. 3 of the tile
+//   ku     [tiles][lane][4]: lane -> dimension lane & 15 of the tile, tokens 4 (lane >> 4) + 0 .. 3
+//   gc     [DP]: d(-, 15);  mb [2][16][16]: M, B
+constexpr int CT = DELTA_CHUNK;
+static_assert(CT == 16, "a chunk is one tile of the matrix instruction");
 
-// One wave per (group, head): decays, step sizes and the pair products.  grid (ceil(H / 4), groups, B)
-template <int E, int PC>
-__global__ __launch_bounds__(256) void k_delta_pairs(DeltaRows a)
+// grid (H, chunks, B), block 256.  LDS: k, q, g [16][DP + 4], A, B [16][17], beta [16]
+__global__ __launch_bounds__(256) void k_delta_prepare(DeltaRows a, int DP)
 {
-    const int lane = threadIdx.x & 63, h = blockIdx.x * 4 + (threadIdx.x >> 6), grp = blockIdx.y, b = blockIdx.z, T = a.r.T;
-    if (h >= a.H) return;
-    const int kvh = h / (a.H / a.KV), t0 = grp * GT, nt = min(GT, T - t0);
-    const size_t m0 = (size_t)b * T + t0;
-    float k[GT][E], q[GT][E], g[GT][E], gh[GT];
+    extern __shared__ float lds[];
+    const int LD = DP + 4;
+    float *ks = lds, *qs = ks + CT * LD, *gs = qs + CT * LD, *A = gs + CT * LD, *Bm = A + CT * 17, *beta = Bm + CT * 17;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int h = blockIdx.x, ck = blockIdx.y, b = blockIdx.z, T = a.r.T, kvh = h / (a.H / a.KV), t0 = ck * CT, nt = min(CT, T - t0);
+    const size_t m0 = (size_t)b * T + t0, chunk = ((size_t)b * gridDim.y + ck) * a.H + h;
     const float ae = a.a_exp[h];
+    // tokens past the end leave the state alone: no key, no step, decay 1
+    for (int e = tid; e < CT * DP; e += 256) {
+        const int t = e / DP, d = e % DP;
+        const bool in = t < nt && d < a.dim;
+        const size_t o = ((m0 + t) * a.KV + kvh) * a.dim + d;
+        ks[t * LD + d] = in ? a.k[o] : 0.f;
+        qs[t * LD + d] = in ? a.q[o] : 0.f;
+        float g = 1.f;
+        if (t < nt) {
+            if (!a.per_channel) g = a.cin[(m0 + t) * a.ldc + a.o_a + h] + a.dt_bias[h];
+            else if (in) g = a.a2[((m0 + t) * a.H + h) * a.dim + d] + a.dt_bias[h * a.dim + d];
+            g = a.per_channel && !in ? 1.f : expf(-ae * softplus(g));
+        }
+        gs[t * LD + d] = g;
+    }
+    if (tid < CT) beta[tid] = tid < nt ? sigmoid(a.cin[(m0 + tid) * a.ldc + a.o_b + h]) : 0.f;
+    __syncthreads();
+    {   // A and B: sixteen lanes share a row j of keys, each with every 16th piece of four dimensions, and walk the tokens i
+        // from j on while the decay between builds up
+        const int j = wave * 4 + (lane >> 4), part = lane & 15;
+        float sa[CT], sb[CT];
 #pragma unroll
-    for (int i = 0; i < GT; i++) {
-        gh[i] = 1.f;
-        if (!PC && i < nt) gh[i] = expf(-ae * softplus(a.cin[(m0 + i) * a.ldc + a.o_a + h] + a.dt_bias[h]));
+        for (int i = 0; i < CT; i++) sa[i] = sb[i] = 0.f;
+        for (int d = part * 4; d < DP; d += 64) {
+            float4 c = *reinterpret_cast<const float4 *>(&ks[j * LD + d]);
 #pragma unroll
-        for (int e = 0; e < E; e++) {
-            const int d = lane + 64 * e;
-            const bool in = d < a.dim && i < nt;
-            const size_t o = ((m0 + i) * a.KV + kvh) * a.dim + d;
-            k[i][e] = in ? a.k[o] : 0.f;
-            q[i][e] = in ? a.q[o] : 0.f;
-            g[i][e] = gh[i];
-            if (PC && in) {
-                const size_t og = ((m0 + i) * a.H + h) * a.dim + d;
-                g[i][e] = expf(-ae * softplus(a.a2[og] + a.dt_bias[h * a.dim + d]));
-                a.g[og] = g[i][e];
+            for (int i = 0; i < CT; i++) {
+                if (i < wave * 4) continue;               // (the wave's first j; what lies below a lane's own j is not kept)
+                const float4 k = *reinterpret_cast<const float4 *>(&ks[i * LD + d]), q = *reinterpret_cast<const float4 *>(&qs[i * LD + d]);
+                const float4 g = *reinterpret_cast<const float4 *>(&gs[i * LD + d]);
+                const bool later = i > j;
+                c.x *= later ? g.x : 1.f; c.y *= later ? g.y : 1.f; c.z *= later ? g.z : 1.f; c.w *= later ? g.w : 1.f;
+                sa[i] = fmaf(k.x, c.x, fmaf(k.y, c.y, fmaf(k.z, c.z, fmaf(k.w, c.w, sa[i]))));
+                sb[i] = fmaf(q.x, c.x, fmaf(q.y, c.y, fmaf(q.z, c.z, fmaf(q.w, c.w, sb[i]))));
             }
         }
-    }
-    float A[6], B[10];
-    int na = 0, nb = 0;
 #pragma unroll
-    for (int i = 0; i < GT; i++)
-#pragma unroll
-        for (int j = 0; j <= i; j++) {
-            float sa = 0.f, sb = 0.f;
-#pragma unroll
-            for (int e = 0; e < E; e++) {
-                float kj = k[j][e];
-#pragma unroll
-                for (int x = j + 1; x <= i; x++) kj *= g[x][e];
-                sa = fmaf(k[i][e], kj, sa); sb = fmaf(q[i][e], kj, sb);
-            }
-            if (j < i) A[na++] = wave_total(sa);
-            B[nb++] = wave_total(sb);
-        }
-    // lane n keeps number n
-    float mine = 0.f;
-#pragma unroll
-    for (int i = 0; i < GT; i++) {
-        if (lane == i && i < nt) mine = sigmoid(a.cin[(m0 + i) * a.ldc + a.o_b + h]);
-        if (!PC) {
-            float c = 1.f, r = 1.f;
-#pragma unroll
-            for (int x = 0; x < GT; x++) { if (x <= i) c *= gh[x]; else r *= gh[x]; }
-            if (lane == 24 + i) mine = c;
-            if (lane == 28 + i) mine = r;
+        for (int i = 0; i < CT; i++) {
+            const float va = group_sum<16>(sa[i]), vb = group_sum<16>(sb[i]);
+            if (part == 0) { A[i * 17 + j] = i > j ? va : 0.f; Bm[i * 17 + j] = i >= j ? vb : 0.f; }
         }
     }
+    // decayed keys and queries: a thread per (token, four dimensions)
+    for (int e = tid; e < CT * DP / 4; e += 256) {
+        const int t = e % CT, d = (e / CT) * 4;
+        float4 c = make_float4(1.f, 1.f, 1.f, 1.f);
+        for (int x = 0; x <= t; x++) {
+            const float4 g = *reinterpret_cast<const float4 *>(&gs[x * LD + d]);
+            c.x *= g.x; c.y *= g.y; c.z *= g.z; c.w *= g.w;
+        }
+        const float4 k = *reinterpret_cast<const float4 *>(&ks[t * LD + d]), q = *reinterpret_cast<const float4 *>(&qs[t * LD + d]);
+        const size_t o = chunk * DP * CT + ((size_t)(d / 16) * 64 + ((d % 16) / 4) * 16 + t) * 4;
+        *reinterpret_cast<float4 *>(a.kd + o) = make_float4(k.x * c.x, k.y * c.y, k.z * c.z, k.w * c.w);
+        *reinterpret_cast<float4 *>(a.qd + o) = make_float4(q.x * c.x, q.y * c.y, q.z * c.z, q.w * c.w);
+        if (t == CT - 1) *reinterpret_cast<float4 *>(a.gc + chunk * DP + d) = c;
+    }
+    // keys as the state's update takes them: a thread per (dimension, four tokens)
+    for (int e = tid; e < CT * DP / 4; e += 256) {
+        const int d = e % DP, t4 = (e / DP) * 4;
+        float r = 1.f, v[4];
+        for (int x = CT - 1; x > t4 + 3; x--) r *= gs[x * LD + d];
 #pragma unroll
-    for (int n = 0; n < 6; n++) if (lane == 4 + n) mine = A[n];
+        for (int x = 3; x >= 0; x--) { v[x] = ks[(t4 + x) * LD + d] * r; r *= gs[(t4 + x) * LD + d]; }
+        const size_t o = chunk * DP * CT + ((size_t)(d / 16) * 64 + (t4 / 4) * 16 + d % 16) * 4;
+        *reinterpret_cast<float4 *>(a.ku + o) = make_float4(v[0], v[1], v[2], v[3]);
+    }
+    __syncthreads();
+    float *mb = a.mb + chunk * 2 * CT * CT;
+    if (tid < CT) {                                       // column tid of M by forward substitution
+        float x[CT];
 #pragma unroll
-    for (int n = 0; n < 10; n++) if (lane == 12 + n) mine = B[n];
-    if (lane < GS) a.pairs[(((size_t)b * ((T + GT - 1) / GT) + grp) * a.H + h) * GS + lane] = mine;
+        for (int i = 0; i < CT; i++) {
+            float s = i == tid ? 1.f : 0.f;
+#pragma unroll
+            for (int j = 0; j < i; j++) s = fmaf(-A[i * 17 + j], x[j], s);
+            x[i] = beta[i] * s;
+            mb[i * CT + tid] = x[i];
+        }
+    } else if (tid >= 64) {
+        for (int e = tid - 64; e < CT * CT; e += 192) mb[CT * CT + e] = Bm[(e / CT) * 17 + e % CT];
+    }
 }
 
-// The recurrence.  The columns of a head's state (one per value channel) do not meet: a column is G lanes of a wave, each
-// with R of its rows -- lane l of the group has rows 4 l .. 4 l + 3 of every block of 4 G -- so no token costs a barrier.
-// Tokens are staged through LDS TC at a time with the decays already on the keys and queries, the next two stages on their
-// way in registers; a group's LDS reads are issued one group ahead.  The lane numbered like a token keeps its output until the
-// stage is over.
-// grid (column blocks of 256 / G, H, B), block 256.  VEC: dim is a multiple of 4 (16-byte loads).
-template <int G, int R, int PC, int VEC>
-__global__ __launch_bounds__(256) void k_delta_scan(DeltaRows a)
+// grid (ceil(vdim / 16), H, B); a workgroup owns sixteen columns of a head's state, each of its waves TPW tiles of sixteen
+// rows, held as the accumulators of v_mfma_f32_16x16x4_f32 (fp32 operands and sums).  The register order of an accumulator
+// -- column lane & 15, rows 4 (lane >> 4) + 0 .. 3 -- is also a legal order of the reduction index of an operand, so S, U
+// and V - P go from one product into the next as they are.  Per chunk the waves add their parts of P and W through LDS (one
+// barrier); everything from memory is asked for SETS chunks ahead.
+template <int TPW, int SETS>
+__global__ __launch_bounds__(256) void k_delta_chunks(DeltaRows a, int DP, int chunks)
 {
-    constexpr int TC = 16, NG = TC / GT, DP = G * R, COLS = 256 / G, RB = R / 4;
-    constexpr int NC = (TC * COLS + 255) / 256, NK = (TC + G - 1) / G;
-    static_assert(DP <= 256, "a thread stages four columns of one group");
-    __shared__ float ks[2][TC * DP], qs[2][TC * DP], us[2][PC ? TC * DP : 4], gs[2][PC ? NG * DP : 4];
-    __shared__ float vs[2][COLS * TC], ps[2][NG * GS];
-    const int tid = threadIdx.x, l = tid % G, col = tid / G;
-    const int h = blockIdx.y, b = blockIdx.z, kvh = h / (a.H / a.KV), T = a.r.T, groups = (T + GT - 1) / GT;
-    const int j0 = blockIdx.x * COLS, j = j0 + col;
-    const size_t r0 = (size_t)b * T;
-    float S[R];
-    float *Sg = a.S + (((size_t)b * a.H + h) * a.vdim + min(j, a.vdim - 1)) * a.dim;
+    __shared__ float4v red[2][4][2][64];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6, c = lane & 15, r4 = lane >> 4;
+    const int h = blockIdx.y, b = blockIdx.z, T = a.r.T, j = blockIdx.x * 16 + c, jc = min(j, a.vdim - 1);
+    const int vd = a.H * a.vdim;
+    float *Sg = a.S + (((size_t)b * a.H + h) * a.vdim + jc) * a.dim;
+    const int d0 = wave * TPW * 16 + 4 * r4;              // rows d0 + 16 tile + 0 .. 3
+    float4v S[TPW];
 #pragma unroll
-    for (int e = 0; e < R; e++) {
-        const int d = (e >> 2) * 4 * G + 4 * l + (e & 3);
-        S[e] = (a.r.pos > 0 && d < a.dim) ? Sg[d] : 0.f;  // position 0 starts from nothing, whatever the state held
-    }
-    // staging: a thread brings four columns of the four tokens of one group (threads from DP on repeat others' reads and
-    // park nothing).  Two register sets, a stage's loads are asked for two stages ahead.  Every load is unconditional, past
-    // the end for the last token again: under a condition the compiler could not tell the two sets' loads apart and would
-    // wait for both.  What lies past the end is taken out when it is parked: no key, no step, decay 1.
-    const int sd = (tid % (DP / 4)) * 4, sgrp = tid / (DP / 4) % NG;
-    struct Stage { float4 k[GT], q[GT], g[PC ? GT : 1]; float v[NC], p; };
-    auto at = [](const float *base, uint32_t i) __attribute__((always_inline)) { return reinterpret_cast<const float *>(reinterpret_cast<const char *>(base) + 4u * i); };
-    auto load4 = [&](const float *base, uint32_t i) __attribute__((always_inline)) {
-        if (VEC) return *reinterpret_cast<const float4 *>(at(base, i));
-        const uint32_t last = (uint32_t)(a.dim - 1 - min(sd, a.dim - 1));
-        return make_float4(*at(base, i), *at(base, i + min(1u, last)), *at(base, i + min(2u, last)), *at(base, i + min(3u, last)));
-    };
-    const uint32_t kq0 = (uint32_t)((r0 * a.KV + kvh) * a.dim + min(sd, a.dim - (VEC ? 4 : 1)));
-    const uint32_t g0 = (uint32_t)((r0 * a.H + h) * a.dim + min(sd, a.dim - (VEC ? 4 : 1)));
-    auto fetch = [&](Stage &x, int t0) __attribute__((always_inline)) {
+    for (int i = 0; i < TPW; i++)
 #pragma unroll
-        for (int i = 0; i < GT; i++) {
-            const uint32_t t = (uint32_t)min(t0 + sgrp * GT + i, T - 1);
-            const uint32_t o = kq0 + t * (uint32_t)(a.KV * a.dim);
-            x.k[i] = load4(a.k, o); x.q[i] = load4(a.q, o);
-            if (PC) x.g[PC ? i : 0] = load4(a.g, g0 + t * (uint32_t)(a.H * a.dim));
+        for (int v = 0; v < 4; v++) {                     // position 0 starts from nothing, whatever the state held
+            const int d = d0 + 16 * i + v;
+            S[i][v] = (a.r.pos > 0 && d < a.dim) ? Sg[d] : 0.f;
         }
-#pragma unroll
-        for (int i = 0; i < NC; i++) {
-            const int e = tid + 256 * i, t = e / COLS % TC, c = e % COLS;
-            x.v[i] = *at(a.v, (uint32_t)(((r0 + min(t0 + t, T - 1)) * a.H + h) * a.vdim + min(j0 + c, a.vdim - 1)));
-        }
-        const int grp = min(t0 / GT + tid / GS % NG, groups - 1);
-        x.p = *at(a.pairs, (uint32_t)((((size_t)b * groups + grp) * a.H + h) * GS + tid % GS));
+    auto at4 = [](const float *base, uint32_t i) __attribute__((always_inline)) {
+        return *reinterpret_cast<const float4v *>(reinterpret_cast<const char *>(base) + 4u * i);
     };
-    auto mul4 = [](const float4 &x, const float4 &y) __attribute__((always_inline)) { return make_float4(x.x * y.x, x.y * y.y, x.z * y.z, x.w * y.w); };
-    auto park = [&](const Stage &x, int t0, int s) __attribute__((always_inline)) {
-        if (tid < DP) {
-            const float4 one = make_float4(1.f, 1.f, 1.f, 1.f);
-            float4 c = one, r = one, k[GT], g[GT];
+    auto at1 = [](const float *base, uint32_t i) __attribute__((always_inline)) {
+        return *reinterpret_cast<const float *>(reinterpret_cast<const char *>(base) + 4u * i);
+    };
+    struct Set { float4v k[TPW], q[TPW], u[TPW], g[TPW], m, b, v; };
+    auto fetch = [&](Set &x, int ck) __attribute__((always_inline)) {
+        const uint32_t chunk = (uint32_t)((b * chunks + min(ck, chunks - 1)) * a.H + h);
+        const uint32_t f = chunk * (uint32_t)(DP * CT) + (uint32_t)(wave * TPW * 256 + lane * 4);
 #pragma unroll
-            for (int i = 0; i < GT; i++) {
-                const bool in = t0 + sgrp * GT + i < T;
-                const float f0 = in && sd < a.dim ? 1.f : 0.f, f1 = in && (VEC ? sd : sd + 1) < a.dim ? 1.f : 0.f;
-                const float f2 = in && (VEC ? sd : sd + 2) < a.dim ? 1.f : 0.f, f3 = in && (VEC ? sd : sd + 3) < a.dim ? 1.f : 0.f;
-                const float4 f = make_float4(f0, f1, f2, f3);
-                k[i] = mul4(x.k[i], f);
-                g[i] = PC && in ? x.g[PC ? i : 0] : one;
-                c = mul4(c, g[i]);
-                const int to = (sgrp * GT + i) * DP + sd;
-                *reinterpret_cast<float4 *>(&ks[s][to]) = PC ? mul4(k[i], c) : k[i];
-                *reinterpret_cast<float4 *>(&qs[s][to]) = PC ? mul4(mul4(x.q[i], f), c) : mul4(x.q[i], f);
+        for (int i = 0; i < TPW; i++) {
+            x.k[i] = at4(a.kd, f + 256 * i); x.q[i] = at4(a.qd, f + 256 * i); x.u[i] = at4(a.ku, f + 256 * i);
+            x.g[i] = at4(a.gc, chunk * (uint32_t)DP + (uint32_t)(d0 + 16 * i));
+        }
+        const uint32_t mb = chunk * (uint32_t)(2 * CT * CT) + (uint32_t)(c * CT + 4 * r4);
+        x.m = at4(a.mb, mb); x.b = at4(a.mb, mb + CT * CT);
+#pragma unroll
+        for (int v = 0; v < 4; v++)
+            x.v[v] = at1(a.v, (uint32_t)((b * T + min(min(ck, chunks - 1) * CT + 4 * r4 + v, T - 1)) * vd + h * a.vdim + jc));
+    };
+    auto take = [&](const Set &x, int ck) __attribute__((always_inline)) {
+        float4v p = {0.f, 0.f, 0.f, 0.f}, w = p;
+#pragma unroll
+        for (int i = 0; i < TPW; i++)
+#pragma unroll
+            for (int v = 0; v < 4; v++) {
+                p = __builtin_amdgcn_mfma_f32_16x16x4f32(x.k[i][v], S[i][v], p, 0, 0, 0);
+                w = __builtin_amdgcn_mfma_f32_16x16x4f32(x.q[i][v], S[i][v], w, 0, 0, 0);
             }
-            if (PC) {
-                *reinterpret_cast<float4 *>(&gs[s][sgrp * DP + sd]) = c;
-#pragma unroll
-                for (int i = GT - 1; i >= 0; i--) {
-                    *reinterpret_cast<float4 *>(&us[s][(sgrp * GT + i) * DP + sd]) = mul4(k[i], r);
-                    r = mul4(r, g[i]);
-                }
-            }
-        }
-#pragma unroll
-        for (int i = 0; i < NC; i++) { const int e = tid + 256 * i, t = e / COLS, c = e % COLS; if (t < TC) vs[s][c * TC + t] = x.v[i]; }
-        if (tid < NG * GS) ps[s][tid] = x.p;              // (step sizes past the end are zero already)
-    };
-    struct Group { float4 k[GT][RB], q[GT][RB]; };
-    auto read = [&](Group &x, int s, int grp) __attribute__((always_inline)) {
-#pragma unroll
-        for (int i = 0; i < GT; i++)
-#pragma unroll
-            for (int r = 0; r < RB; r++) {
-                const int at = (grp * GT + i) * DP + r * 4 * G + 4 * l;
-                x.k[i][r] = *reinterpret_cast<const float4 *>(&ks[s][at]);
-                x.q[i][r] = *reinterpret_cast<const float4 *>(&qs[s][at]);
-            }
-    };
-    auto dot = [&](const float4 (&x)[RB]) __attribute__((always_inline)) {
-        float y[RB];
-#pragma unroll
-        for (int r = 0; r < RB; r++) y[r] = fmaf(S[4 * r + 3], x[r].w, fmaf(S[4 * r + 2], x[r].z, fmaf(S[4 * r + 1], x[r].y, S[4 * r] * x[r].x)));
-#pragma unroll
-        for (int r = 1; r < RB; r++) y[0] += y[r];
-        return y[0];
-    };
-    float keep[NK];
-    auto take = [&](const Group &x, int s, int grp) __attribute__((always_inline)) {
-        const float4 *n = reinterpret_cast<const float4 *>(&ps[s][grp * GS]);
-        const float4 be = n[0], a0 = n[1], a1 = n[2], b0 = n[3], b1 = n[4], b2 = n[5];
-        const float4 v = *reinterpret_cast<const float4 *>(&vs[s][col * TC + grp * GT]);
-        float p[GT], w[GT];
-#pragma unroll
-        for (int i = 0; i < GT; i++) { p[i] = dot(x.k[i]); w[i] = dot(x.q[i]); }
-#pragma unroll
-        for (int i = 0; i < GT; i++) { p[i] = group_sum<G>(p[i]); w[i] = group_sum<G>(w[i]); }
-        float u[GT];
-        float4 dr = make_float4(1.f, 1.f, 1.f, 1.f);
-        float all = 1.f;
-        if (!PC) {
-            const float4 dc = n[6];
-            dr = n[7];
-            p[0] *= dc.x; p[1] *= dc.y; p[2] *= dc.z; p[3] *= dc.w;
-            w[0] *= dc.x; w[1] *= dc.y; w[2] *= dc.z; w[3] *= dc.w;
-            all = dc.w;
-        }
-        u[0] = be.x * (v.x - p[0]);
-        u[1] = be.y * (v.y - p[1] - a0.x * u[0]);
-        u[2] = be.z * (v.z - p[2] - a0.y * u[0] - a0.z * u[1]);
-        u[3] = be.w * (v.w - p[3] - a0.w * u[0] - a1.x * u[1] - a1.y * u[2]);
-        const float o[GT] = {fmaf(b0.x, u[0], w[0]), fmaf(b0.z, u[1], fmaf(b0.y, u[0], w[1])),
-                             fmaf(b1.y, u[2], fmaf(b1.x, u[1], fmaf(b0.w, u[0], w[2]))),
-                             fmaf(b2.y, u[3], fmaf(b2.x, u[2], fmaf(b1.w, u[1], fmaf(b1.z, u[0], w[3]))))};
-        if (!PC) { u[0] *= dr.x; u[1] *= dr.y; u[2] *= dr.z; u[3] *= dr.w; }
-#pragma unroll
-        for (int r = 0; r < RB; r++) {
-            float4 g = make_float4(all, all, all, all);
-            if (PC) g = *reinterpret_cast<const float4 *>(&gs[s][grp * DP + r * 4 * G + 4 * l]);
-            float *z = &S[4 * r];
-            z[0] *= g.x; z[1] *= g.y; z[2] *= g.z; z[3] *= g.w;
-#pragma unroll
-            for (int i = 0; i < GT; i++) {
-                const float4 k = PC ? *reinterpret_cast<const float4 *>(&us[s][PC ? (grp * GT + i) * DP + r * 4 * G + 4 * l : 0]) : x.k[i][r];
-                z[0] = fmaf(k.x, u[i], z[0]); z[1] = fmaf(k.y, u[i], z[1]); z[2] = fmaf(k.z, u[i], z[2]); z[3] = fmaf(k.w, u[i], z[3]);
-            }
-        }
-#pragma unroll
-        for (int i = 0; i < GT; i++) {
-            const int t = grp * GT + i;
-            keep[t / G] = l == t % G ? o[i] : keep[t / G];
-        }
-    };
-    Stage even, odd;
-    auto stage = [&](int t0, int s, Stage &ahead, const Stage &next) __attribute__((always_inline)) {
-        fetch(ahead, t0 + 2 * TC);
-#pragma unroll
-        for (int i = 0; i < NK; i++) keep[i] = 0.f;
-        Group x[2];
-        read(x[0], s, 0);
-#pragma unroll
-        for (int grp = 0; grp < NG; grp++) {
-            if (t0 + grp * GT >= T) break;                // uniform
-            if (grp + 1 < NG) read(x[(grp + 1) & 1], s, grp + 1);
-            take(x[grp & 1], s, grp);
-        }
-        park(next, t0 + TC, s ^ 1);                       // the other stage: its readers passed the barrier before this one
-#pragma unroll
-        for (int i = 0; i < NK; i++) {
-            const int t = i * G + l;
-            if (t < TC && t0 + t < T && j < a.vdim) a.o[((r0 + t0 + t) * a.H + h) * a.vdim + j] = keep[i];
-        }
+        float4v(&rd)[4][2][64] = red[ck & 1];
+        rd[wave][0][lane] = p; rd[wave][1][lane] = w;
         __syncthreads();
+        p = rd[0][0][lane]; w = rd[0][1][lane];
+        for (int n = 1; n < nw; n++) { p += rd[n][0][lane]; w += rd[n][1][lane]; }
+        const float4v z = x.v - p;
+        float4v u = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int v = 0; v < 4; v++) u = __builtin_amdgcn_mfma_f32_16x16x4f32(x.m[v], z[v], u, 0, 0, 0);
+#pragma unroll
+        for (int i = 0; i < TPW; i++) {
+            S[i] *= x.g[i];
+#pragma unroll
+            for (int v = 0; v < 4; v++) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.u[i][v], u[v], S[i], 0, 0, 0);
+        }
+        if (ck % nw == wave) {                            // the waves take the outputs in turn
+#pragma unroll
+            for (int v = 0; v < 4; v++) w = __builtin_amdgcn_mfma_f32_16x16x4f32(x.b[v], u[v], w, 0, 0, 0);
+#pragma unroll
+            for (int v = 0; v < 4; v++) {
+                const int t = ck * CT + 4 * r4 + v;
+                if (t < T && j < a.vdim) a.o[((size_t)b * T + t) * vd + h * a.vdim + j] = w[v];
+            }
+        }
     };
-    fetch(even, 0);
-    fetch(odd, TC);
-    park(even, 0, 0);
-    __syncthreads();
-    for (int t0 = 0; t0 < T; t0 += 2 * TC) {
-        stage(t0, 0, even, odd);
-        if (t0 + TC < T) stage(t0 + TC, 1, odd, even);
-    }
+    Set x[SETS];
+#pragma unroll
+    for (int n = 0; n < SETS - 1; n++) fetch(x[n], n);
+    for (int ck = 0; ck < chunks; ck += SETS)
+#pragma unroll
+        for (int n = 0; n < SETS; n++) {
+            if (ck + n >= chunks) break;                  // uniform
+            fetch(x[(n + SETS - 1) % SETS], ck + n + SETS - 1);
+            take(x[n], ck + n);
+        }
     if (j < a.vdim)
 #pragma unroll
-        for (int e = 0; e < R; e++) {
-            const int d = (e >> 2) * 4 * G + 4 * l + (e & 3);
-            if (d < a.dim) Sg[d] = S[e];
-        }
+        for (int i = 0; i < TPW; i++)
+#pragma unroll
+            for (int v = 0; v < 4; v++) {
+                const int d = d0 + 16 * i + v;
+                if (d < a.dim) Sg[d] = S[i][v];
+            }
 }
 
 // The last `taps` inputs of this step's convolutions into the state's ring.  grid (ceil(channels / 256), taps, B)
@@ -407,32 +349,34 @@ __global__ __launch_bounds__(256) void k_cat_rows(CatRows a)
 
 }  // namespace
 
-int delta_groups(int T) { return (T + GT - 1) / GT; }
-size_t delta_pair_floats(int B, int T, int H) { return (size_t)B * delta_groups(T) * H * GS; }
+// waves of a workgroup of k_delta_chunks and tiles of each
+struct ChunkShape { int nw, tpw; int dp() const { return nw * tpw * 16; } };
+static ChunkShape chunk_shape(int dim)
+{
+    const int tiles = (dim + 15) / 16, nw = tiles < 4 ? tiles : 4, per = (tiles + nw - 1) / nw;
+    return ChunkShape{nw, per <= 1 ? 1 : per <= 2 ? 2 : 4};
+}
+int delta_chunks(int T) { return (T + CT - 1) / CT; }
+int delta_padded_dim(int dim) { return chunk_shape(dim).dp(); }
 
 void launch_delta_inputs(const DeltaRows &a)
 {
-    const dim3 grid((a.KV + (a.H * a.vdim + 63) / 64 + 3) / 4, (a.r.T + TW - 1) / TW, a.r.B), pgrid((a.H + 3) / 4, delta_groups(a.r.T), a.r.B);
-#define INPUTS(E_) do { \
-    LAUNCH(k_delta_inputs<E_>, grid, dim3(256), 0, a); \
-    if (a.per_channel) LAUNCH((k_delta_pairs<E_, 1>), pgrid, dim3(256), 0, a); else LAUNCH((k_delta_pairs<E_, 0>), pgrid, dim3(256), 0, a); } while (0)
-    if (a.dim <= 64) INPUTS(1); else if (a.dim <= 128) INPUTS(2); else INPUTS(4);
-#undef INPUTS
+    const dim3 grid((a.KV + (a.H * a.vdim + 63) / 64 + 3) / 4, (a.r.T + TW - 1) / TW, a.r.B);
+    if (a.dim <= 64) LAUNCH(k_delta_inputs<1>, grid, dim3(256), 0, a);
+    else if (a.dim <= 128) LAUNCH(k_delta_inputs<2>, grid, dim3(256), 0, a);
+    else LAUNCH(k_delta_inputs<4>, grid, dim3(256), 0, a);
+    const int DP = delta_padded_dim(a.dim);
+    LAUNCH(k_delta_prepare, dim3(a.H, delta_chunks(a.r.T), a.r.B), dim3(256), (size_t)(3 * CT * (DP + 4) + 2 * CT * 17 + CT) * sizeof(float), a, DP);
 }
 
 void launch_delta_scan(const DeltaRows &a)
 {
-    // eight rows per lane; four where the columns would otherwise leave most of the SIMDs without a wave
-    const int g8 = a.dim <= 32 ? 4 : a.dim <= 64 ? 8 : a.dim <= 128 ? 16 : 32;
-    const bool few = (long)a.r.B * a.H * a.vdim * g8 / 64 <= 2 * num_cus() && a.dim <= 128;
-    const int G = few ? 2 * g8 : g8, cols = 256 / G;
-    const dim3 grid((a.vdim + cols - 1) / cols, a.H, a.r.B);
-#define SCAN(G_, R_) do { \
-    if (a.dim % 4 == 0) { if (a.per_channel) LAUNCH((k_delta_scan<G_, R_, 1, 1>), grid, dim3(256), 0, a); else LAUNCH((k_delta_scan<G_, R_, 0, 1>), grid, dim3(256), 0, a); } \
-    else { if (a.per_channel) LAUNCH((k_delta_scan<G_, R_, 1, 0>), grid, dim3(256), 0, a); else LAUNCH((k_delta_scan<G_, R_, 0, 0>), grid, dim3(256), 0, a); } } while (0)
-    if (few) { if (G == 8) SCAN(8, 4); else if (G == 16) SCAN(16, 4); else SCAN(32, 4); }
-    else if (G == 4) SCAN(4, 8); else if (G == 8) SCAN(8, 8); else if (G == 16) SCAN(16, 8); else SCAN(32, 8);
-#undef SCAN
+    const ChunkShape cs = chunk_shape(a.dim);
+    const dim3 grid((a.vdim + 15) / 16, a.H, a.r.B), block(64 * cs.nw);
+    const int chunks = delta_chunks(a.r.T);
+    if (cs.tpw == 1) LAUNCH((k_delta_chunks<1, 4>), grid, block, 0, a, cs.dp(), chunks);
+    else if (cs.tpw == 2) LAUNCH((k_delta_chunks<2, 4>), grid, block, 0, a, cs.dp(), chunks);
+    else LAUNCH((k_delta_chunks<4, 2>), grid, block, 0, a, cs.dp(), chunks);
     const int C = 2 * a.KV * a.dim + a.H * a.vdim;
     LAUNCH(k_conv_keep, dim3((C + 255) / 256, a.taps, a.r.B), dim3(256), 0, a);
 }

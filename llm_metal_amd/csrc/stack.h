@@ -157,12 +157,15 @@ struct DeltaRows {
     const float *cin; int ldc, o_q, o_k, o_v, o_b, o_a;  // the input product
     const float *filters, *a_exp, *dt_bias;
     float *conv, *S;                                     // state
-    float *q, *k, *v, *g, *pairs;                        // intermediates: [rows][KV][dim] x 2, [rows][H][vdim], [rows][H][dim] (per channel), [groups][H][..]
+    float *q, *k, *v;                                    // intermediates: [rows][KV][dim] x 2, [rows][H][vdim]
+    float *kd, *qd, *ku, *gc, *mb;                       // per chunk of tokens and head (delta.hip)
     const float *a2;                                     // per channel: W_a2 (W_a1 h) [rows][H * dim]
     float *o;                                            // [rows][H][vdim]
 };
-size_t delta_pair_floats(int B, int T, int H);           // size of `pairs`
-void launch_delta_inputs(const DeltaRows &a);            // convolutions, unit norms, step sizes, decays
+int delta_chunks(int T);                                 // chunks of a sequence's T tokens
+int delta_padded_dim(int dim);
+constexpr int DELTA_CHUNK = 16;
+void launch_delta_inputs(const DeltaRows &a);            // convolutions and unit norms, then what the chunks need ahead
 void launch_delta_scan(const DeltaRows &a);              // the recurrence; also moves the convolution's last inputs into the state
 
 // The operand of the output product: mixer output (head norm and gate applied when g_out) | squared-ReLU of the shared

@@ -222,15 +222,16 @@ struct Aux {
     float *take(size_t n) { float *p = base ? base + at : nullptr; at += (n + 3) & ~(size_t)3; return p; }
 };
 
-struct DeltaAux { float *q, *k, *v, *g, *pairs, *a2, *g2, *o; };
+struct DeltaAux { float *q, *k, *v, *kd, *qd, *ku, *gc, *mb, *a2, *g2, *o; };
 DeltaAux delta_aux(Aux &x, const LayerConfig &c, int B, int T)
 {
     const size_t rows = (size_t)B * T;
     const bool pc = c.mixer == MIX_CHANNEL_DELTA;
     DeltaAux d{};
     d.q = x.take(rows * c.kv_heads * c.dim); d.k = x.take(rows * c.kv_heads * c.dim); d.v = x.take(rows * c.heads * c.vdim);
-    d.g = x.take(pc ? rows * c.heads * c.dim : 0);
-    d.pairs = x.take(delta_pair_floats(B, T, c.heads));
+    const size_t parts = (size_t)B * delta_chunks(T) * c.heads, dp = delta_padded_dim(c.dim);
+    d.kd = x.take(parts * dp * DELTA_CHUNK); d.qd = x.take(parts * dp * DELTA_CHUNK); d.ku = x.take(parts * dp * DELTA_CHUNK);
+    d.gc = x.take(parts * dp); d.mb = x.take(parts * 2 * DELTA_CHUNK * DELTA_CHUNK);
     d.a2 = x.take(pc ? rows * c.heads * c.dim : 0); d.g2 = x.take(pc ? rows * c.heads * c.vdim : 0);
     d.o = x.take(rows * c.heads * c.vdim);
     return d;
@@ -380,7 +381,7 @@ DeltaRows delta_rows(const LayerStack *st, const StackRun *r, const StackLayer &
     a.cin = ptr<float>(r->cin); a.ldc = L.in.rows; a.o_q = L.o_q; a.o_k = L.o_k; a.o_v = L.o_v; a.o_b = L.o_b; a.o_a = L.o_a;
     a.filters = ptr<float>(L.conv); a.a_exp = ptr<float>(L.a_exp); a.dt_bias = ptr<float>(L.dt_bias);
     a.conv = ptr<float>(k.conv); a.S = ptr<float>(k.S);
-    a.q = d.q; a.k = d.k; a.v = d.v; a.g = d.g; a.pairs = d.pairs; a.a2 = d.a2; a.o = d.o;
+    a.q = d.q; a.k = d.k; a.v = d.v; a.kd = d.kd; a.qd = d.qd; a.ku = d.ku; a.gc = d.gc; a.mb = d.mb; a.a2 = d.a2; a.o = d.o;
     return a;
 }
 
