@@ -127,19 +127,28 @@ __global__ __launch_bounds__(256) void k_delta_prepare(DeltaRows a, int DP)
     const size_t m0 = (size_t)b * T + t0, chunk = ((size_t)b * gridDim.y + ck) * a.H + h;
     const float ae = a.a_exp[h];
     // tokens past the end leave the state alone: no key, no step, decay 1
-    for (int e = tid; e < CT * DP; e += 256) {
-        const int t = e / DP, d = e % DP;
-        const bool in = t < nt && d < a.dim;
-        const size_t o = ((m0 + t) * a.KV + kvh) * a.dim + d;
-        ks[t * LD + d] = in ? a.k[o] : 0.f;
-        qs[t * LD + d] = in ? a.q[o] : 0.f;
-        float g = 1.f;
-        if (t < nt) {
-            if (!a.per_channel) g = a.cin[(m0 + t) * a.ldc + a.o_a + h] + a.dt_bias[h];
-            else if (in) g = a.a2[((m0 + t) * a.H + h) * a.dim + d] + a.dt_bias[h * a.dim + d];
-            g = a.per_channel && !in ? 1.f : expf(-ae * softplus(g));
+    const int n4 = DP / 4, step = 256 / n4, d = tid % n4 * 4;
+    const bool vec = a.dim % 4 == 0;                      // the rows of k, q and a2 then start on 16 bytes
+    for (int t = tid / n4; t < CT && tid < step * n4; t += step) {
+        float4 k = make_float4(0.f, 0.f, 0.f, 0.f), q = k, z = k, g = make_float4(1.f, 1.f, 1.f, 1.f);
+        if (t < nt && d < a.dim) {
+            const float *kp = a.k + ((m0 + t) * a.KV + kvh) * a.dim + d, *qp = a.q + ((m0 + t) * a.KV + kvh) * a.dim + d;
+            const float *zp = a.per_channel ? a.a2 + ((m0 + t) * a.H + h) * a.dim + d : nullptr;
+            if (vec) {
+                k = *reinterpret_cast<const float4 *>(kp); q = *reinterpret_cast<const float4 *>(qp);
+                if (zp) z = *reinterpret_cast<const float4 *>(zp);
+            } else
+                for (int u = 0; u < 4 && d + u < a.dim; u++) { (&k.x)[u] = kp[u]; (&q.x)[u] = qp[u]; if (zp) (&z.x)[u] = zp[u]; }
+            if (zp) {
+                const float *bias = a.dt_bias + h * a.dim + d;
+#pragma unroll
+                for (int u = 0; u < 4; u++) if (d + u < a.dim) (&g.x)[u] = expf(-ae * softplus((&z.x)[u] + bias[u]));
+            }
         }
-        gs[t * LD + d] = g;
+        if (!a.per_channel && t < nt) g.x = g.y = g.z = g.w = expf(-ae * softplus(a.cin[(m0 + t) * a.ldc + a.o_a + h] + a.dt_bias[h]));
+        *reinterpret_cast<float4 *>(&ks[t * LD + d]) = k;
+        *reinterpret_cast<float4 *>(&qs[t * LD + d]) = q;
+        *reinterpret_cast<float4 *>(&gs[t * LD + d]) = g;
     }
     if (tid < CT) beta[tid] = tid < nt ? sigmoid(a.cin[(m0 + tid) * a.ldc + a.o_b + h]) : 0.f;
     __syncthreads();
@@ -170,7 +179,7 @@ __global__ __launch_bounds__(256) void k_delta_prepare(DeltaRows a, int DP)
     }
     // decayed keys and queries: a thread per (token, four dimensions)
     for (int e = tid; e < CT * DP / 4; e += 256) {
-        const int t = e % CT, d = (e / CT) * 4;
+        const int t = e % CT, d = (e / CT) * 4;           // (sixteen tokens side by side: their fragments are contiguous)
         float4 c = make_float4(1.f, 1.f, 1.f, 1.f);
         for (int x = 0; x <= t; x++) {
             const float4 g = *reinterpret_cast<const float4 *>(&gs[x * LD + d]);
@@ -214,11 +223,11 @@ __global__ __launch_bounds__(256) void k_delta_prepare(DeltaRows a, int DP)
 // -- column lane & 15, rows 4 (lane >> 4) + 0 .. 3 -- is also a legal order of the reduction index of an operand, so S, U
 // and V - P go from one product into the next as they are.  Per chunk the waves add their parts of P and W through LDS (one
 // barrier); everything from memory is asked for SETS chunks ahead.
-template <int TPW, int SETS>
-__global__ __launch_bounds__(256) void k_delta_chunks(DeltaRows a, int DP, int chunks)
+template <int TPW, int SETS, int NW>
+__global__ __launch_bounds__(64 * NW) void k_delta_chunks(DeltaRows a, int DP, int chunks)
 {
-    __shared__ float4v red[2][4][2][64];
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6, c = lane & 15, r4 = lane >> 4;
+    __shared__ float4v red[2][NW][2][64];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, r4 = lane >> 4;
     const int h = blockIdx.y, b = blockIdx.z, T = a.r.T, j = blockIdx.x * 16 + c, jc = min(j, a.vdim - 1);
     const int vd = a.H * a.vdim;
     float *Sg = a.S + (((size_t)b * a.H + h) * a.vdim + jc) * a.dim;
@@ -237,6 +246,7 @@ __global__ __launch_bounds__(256) void k_delta_chunks(DeltaRows a, int DP, int c
     auto at1 = [](const float *base, uint32_t i) __attribute__((always_inline)) {
         return *reinterpret_cast<const float *>(reinterpret_cast<const char *>(base) + 4u * i);
     };
+    const uint32_t out0 = (uint32_t)((b * T + 4 * r4) * vd + h * a.vdim + jc);
     struct Set { float4v k[TPW], q[TPW], u[TPW], g[TPW], m, b, v; };
     auto fetch = [&](Set &x, int ck) __attribute__((always_inline)) {
         const uint32_t chunk = (uint32_t)((b * chunks + min(ck, chunks - 1)) * a.H + h);
@@ -250,7 +260,7 @@ __global__ __launch_bounds__(256) void k_delta_chunks(DeltaRows a, int DP, int c
         x.m = at4(a.mb, mb); x.b = at4(a.mb, mb + CT * CT);
 #pragma unroll
         for (int v = 0; v < 4; v++)
-            x.v[v] = at1(a.v, (uint32_t)((b * T + min(min(ck, chunks - 1) * CT + 4 * r4 + v, T - 1)) * vd + h * a.vdim + jc));
+            x.v[v] = at1(a.v, (uint32_t)(b * T + min(min(ck, chunks - 1) * CT + 4 * r4 + v, T - 1)) * (uint32_t)vd + (uint32_t)(h * a.vdim + jc));
     };
     auto take = [&](const Set &x, int ck) __attribute__((always_inline)) {
         float4v p = {0.f, 0.f, 0.f, 0.f}, w = p;
@@ -261,11 +271,17 @@ __global__ __launch_bounds__(256) void k_delta_chunks(DeltaRows a, int DP, int c
                 p = __builtin_amdgcn_mfma_f32_16x16x4f32(x.k[i][v], S[i][v], p, 0, 0, 0);
                 w = __builtin_amdgcn_mfma_f32_16x16x4f32(x.q[i][v], S[i][v], w, 0, 0, 0);
             }
-        float4v(&rd)[4][2][64] = red[ck & 1];
+        float4v(&rd)[NW][2][64] = red[ck & 1];
         rd[wave][0][lane] = p; rd[wave][1][lane] = w;
         __syncthreads();
-        p = rd[0][0][lane]; w = rd[0][1][lane];
-        for (int n = 1; n < nw; n++) { p += rd[n][0][lane]; w += rd[n][1][lane]; }
+        float4v pn[NW], wn[NW];
+#pragma unroll
+        for (int n = 0; n < NW; n++) pn[n] = rd[n][0][lane];
+#pragma unroll
+        for (int n = 0; n < NW; n++) wn[n] = rd[n][1][lane];
+        p = pn[0]; w = wn[0];
+#pragma unroll
+        for (int n = 1; n < NW; n++) { p += pn[n]; w += wn[n]; }
         const float4v z = x.v - p;
         float4v u = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -276,13 +292,17 @@ __global__ __launch_bounds__(256) void k_delta_chunks(DeltaRows a, int DP, int c
 #pragma unroll
             for (int v = 0; v < 4; v++) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.u[i][v], u[v], S[i], 0, 0, 0);
         }
-        if (ck % nw == wave) {                            // the waves take the outputs in turn
+        if (ck % NW == wave) {                            // the waves take the outputs in turn
 #pragma unroll
             for (int v = 0; v < 4; v++) w = __builtin_amdgcn_mfma_f32_16x16x4f32(x.b[v], u[v], w, 0, 0, 0);
+            char *to = reinterpret_cast<char *>(a.o) + 4u * (out0 + (uint32_t)(ck * CT) * (uint32_t)vd);
+            if (j < a.vdim) {
+                if (ck * CT + CT <= T) {
 #pragma unroll
-            for (int v = 0; v < 4; v++) {
-                const int t = ck * CT + 4 * r4 + v;
-                if (t < T && j < a.vdim) a.o[((size_t)b * T + t) * vd + h * a.vdim + j] = w[v];
+                    for (int v = 0; v < 4; v++) *reinterpret_cast<float *>(to + 4u * (uint32_t)(v * vd)) = w[v];
+                } else
+#pragma unroll
+                    for (int v = 0; v < 4; v++) if (ck * CT + 4 * r4 + v < T) *reinterpret_cast<float *>(to + 4u * (uint32_t)(v * vd)) = w[v];
             }
         }
     };
@@ -374,9 +394,10 @@ void launch_delta_scan(const DeltaRows &a)
     const ChunkShape cs = chunk_shape(a.dim);
     const dim3 grid((a.vdim + 15) / 16, a.H, a.r.B), block(64 * cs.nw);
     const int chunks = delta_chunks(a.r.T);
-    if (cs.tpw == 1) LAUNCH((k_delta_chunks<1, 4>), grid, block, 0, a, cs.dp(), chunks);
-    else if (cs.tpw == 2) LAUNCH((k_delta_chunks<2, 4>), grid, block, 0, a, cs.dp(), chunks);
-    else LAUNCH((k_delta_chunks<4, 2>), grid, block, 0, a, cs.dp(), chunks);
+#define CHUNKS(T_, S_, N_) LAUNCH((k_delta_chunks<T_, S_, N_>), grid, block, 0, a, cs.dp(), chunks)
+    if (cs.tpw == 2) CHUNKS(2, 4, 4); else if (cs.tpw == 4) CHUNKS(4, 2, 4);
+    else if (cs.nw == 1) CHUNKS(1, 4, 1); else if (cs.nw == 2) CHUNKS(1, 4, 2); else if (cs.nw == 3) CHUNKS(1, 4, 3); else CHUNKS(1, 4, 4);
+#undef CHUNKS
     const int C = 2 * a.KV * a.dim + a.H * a.vdim;
     LAUNCH(k_conv_keep, dim3((C + 255) / 256, a.taps, a.r.B), dim3(256), 0, a);
 }
