@@ -130,8 +130,8 @@ void set_big_gemm_block(int mode);     // F16 tiles: 0 block shape by the measur
 int launch_gemm_big(const half_t *A_tiled, const float *a_inv_scale, const WeightOp &W, float *C, int ldc, int M, int N, int K,
                     int chunks = 1, size_t plane_stride = 0);
 // The same with F16 tiles for rows that belong to different weights [N, K] of one shape (the experts of a mixture), their
-// tiled images group_stride halves apart: row block i of 128 rows is multiplied with weight group_of[i] (device), a negative
-// number marking a block without rows, whose part of C is not written.  M is a multiple of 128; `groups`: how many weights.
+// tiled images group_stride halves apart: row block i of 128 rows is multiplied with weight group_of[i] (device), and only the
+// first group_of[M / 128] blocks have rows (the rest of C is not written).  M is a multiple of 128; `groups`: how many weights.
 void launch_gemm_groups(const half_t *A_tiled, const float *a_inv_scale, const half_t *W_tiled, size_t group_stride, const int *group_of,
                         float *C, int ldc, int M, int N, int K, int groups);
 // true when the large-M kernel is the faster one for this product

@@ -259,7 +259,7 @@ __global__ __launch_bounds__(256) void gemm_big(GemmKArgs g)
 // slice 1 of h and no half step starts by waiting out an LDS round trip; h + 5 is requested into the buffer h - 1 left.
 //
 // GROUPED: the 128-row blocks of A belong to different weights of one shape, laid group.stride halves apart: block mt is
-// multiplied with number group.of[mt]; a negative number is a block without rows, and its workgroups leave at once.
+// multiplied with number group.of[mt]; only the first group.of[M / 128] blocks have rows.
 struct GroupArgs { const int *of; size_t stride; };
 template <bool GROUPED>
 __global__ __launch_bounds__(256) void gemm_big_f16(GemmKArgs g, GroupArgs group)
@@ -271,7 +271,13 @@ __global__ __launch_bounds__(256) void gemm_big_f16(GemmKArgs g, GroupArgs group
     const int MT = (g.M + 127) >> 7, NT = (g.N + 255) >> 8;
     const int m_patches = (MT + 7) >> 3;
     int mt, nt, chunk = 0;
-    if (g.S > 1) {
+    if (GROUPED) {
+        // the blocks that have rows, column blocks first, dealt to the XCDs in contiguous shares: the row blocks of a weight
+        // meet in one L2, and few column blocks leave no XCD without work
+        const int total = group.of[MT] * NT, share = (total + 7) >> 3, seq = blockIdx.x >> 3, t = (blockIdx.x & 7) * share + seq;
+        if (seq >= share || t >= total) return;
+        mt = t / NT; nt = t % NT;
+    } else if (g.S > 1) {
         const int t = blockIdx.x % (MT * NT);
         chunk = blockIdx.x / (MT * NT); mt = t % MT; nt = t / MT;
     } else {
@@ -283,7 +289,6 @@ __global__ __launch_bounds__(256) void gemm_big_f16(GemmKArgs g, GroupArgs group
     const int nb0 = nt * 8, mb0 = mt * 4;
     if (GROUPED) {
         const int e = __builtin_amdgcn_readfirstlane(group.of[mt]);
-        if (e < 0) return;
         g.W.w16 += (size_t)e * group.stride;
     }
     const int wm = wave >> 1, wn = wave & 1;
@@ -921,7 +926,7 @@ void launch_gemm_groups(const half_t *A, const float *a_inv_scale, const half_t 
     g.P = C; g.ldp = ldc; g.M = M; g.N = N; g.Mb = tiled_rb(M); g.Nb = tiled_rb(N); g.Kb = tiled_kb(K);
     g.steps_per_chunk = g.Kb; g.S = 1;
     const int mt = M / 128, nt = (N + 255) / 256;
-    const dim3 grid(8 * 32 * ((mt + 7) / 8) * (((nt + 7) / 8 + 3) / 4));
+    const dim3 grid(8 * ((mt * nt + 7) / 8));
     hipEvent_t ev_a = nullptr, ev_b = nullptr;
     if (gemm_prof_begin(2.0 * groups * N * K, 2.0 * M * N * K, &ev_a, &ev_b))
         hipExtLaunchKernelGGL((gemm_big_f16<true>), grid, dim3(256), 0, stream(), ev_a, ev_b, 0, g, GroupArgs{group_of, group_stride});

@@ -68,6 +68,7 @@ __global__ __launch_bounds__(256) void k_moe_place(const int *__restrict__ idx, 
     const int t0 = (int)block_sum((float)before, sm), mine = g.count[e], nt = (mine + 127) >> 7;
     for (int i = tid; i < nt; i += 256) g.of[t0 + i] = e;
     for (int i = mine + tid; i < nt * 128; i += 256) g.src[t0 * 128 + i] = -1;
+    if (e == E - 1 && tid == 0) g.of[g.tiles] = t0 + nt;
     if (e == E - 1)                                       // blocks behind the last expert's
         for (int i = t0 + nt + tid; i < g.tiles; i += 256) g.of[i] = -1;
     if (!mine) return;
@@ -143,12 +144,12 @@ __global__ __launch_bounds__(256) void k_moe_act(MoeGroups g, const float *__res
 }  // namespace
 
 int moe_group_tiles(int rows, int top, int E) { const int n = rows * top; return n / 128 + (E < n ? E : n); }
-size_t moe_group_ints(int rows, int top, int E) { const size_t t = moe_group_tiles(rows, top, E); return (size_t)E + t + t * 128 + (size_t)rows * top; }
+size_t moe_group_ints(int rows, int top, int E) { const size_t t = moe_group_tiles(rows, top, E); return (size_t)E + t + 1 + t * 128 + (size_t)rows * top; }
 MoeGroups moe_groups_at(int *base, int rows, int top, int E)
 {
     MoeGroups g{};
     g.tiles = moe_group_tiles(rows, top, E);
-    g.count = base; g.of = g.count + E; g.src = g.of + g.tiles; g.pos = g.src + (size_t)g.tiles * 128;
+    g.count = base; g.of = g.count + E; g.src = g.of + g.tiles + 1; g.pos = g.src + (size_t)g.tiles * 128;
     return g;
 }
 

@@ -89,7 +89,7 @@ void stack_free(LayerStack *st);
 struct MoeGroups {
     int tiles;                                           // blocks of 128 rows at most
     int *count;                                          // [E]
-    int *of;                                             // [tiles]: expert of a block, -1: no rows
+    int *of;                                             // [tiles]: expert of a block, -1: no rows; then how many have rows
     int *src;                                            // [tiles * 128]: row of the step, -1: padding
     int *pos;                                            // [rows][top]: where the pair's result lies
 };
