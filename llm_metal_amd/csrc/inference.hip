@@ -480,6 +480,7 @@ extern "C" {
 
 InferenceState *inference_state_create_from_ref(const SFTModelRef *m, int max_seq_len, int use_fp16)
 {
+    if (m->model_type == MODEL_NEVURAX) { fprintf(stderr, "[FastGen] Nevurax models are created by inference_state_create_from_file\n"); return nullptr; }
     InferenceState *s = new_state(m->model_type, m->d_model, m->n_q_heads, m->n_kv_heads, m->head_dim, m->intermediate_size,
                                   m->vocab_size, m->n_layers, max_seq_len, use_fp16, m->rope_thetas);
     if (!s) return nullptr;

@@ -16,6 +16,14 @@ __global__ __launch_bounds__(256) void k_embed_rows(const float *__restrict__ em
     if (i < Dp) x[(size_t)m * Dp + i] = i < D ? emb[(size_t)tok[m] * D + i] * scale : 0.f;
 }
 
+// the same for tokens that travel with the launch
+struct FewTokens { int id[STACK_FEW]; };
+__global__ __launch_bounds__(256) void k_embed_few(const float *__restrict__ emb, FewTokens tok, float scale, float *__restrict__ x, int D, int Dp)
+{
+    const int m = blockIdx.y, i = blockIdx.x * 256 + threadIdx.x;
+    if (i < Dp) x[(size_t)m * Dp + i] = i < D ? emb[(size_t)tok.id[m] * D + i] * scale : 0.f;
+}
+
 // One workgroup per row; the row waits in LDS between the passes (mean, squared deviations, output).
 __global__ __launch_bounds__(256) void k_norm_rows(NormRows a)
 {
@@ -71,6 +79,13 @@ __global__ __launch_bounds__(256) void k_norm_rows(NormRows a)
 void launch_embed_rows(const float *emb, const int *tok, float scale, float *x, int D, int Dp, int rows)
 {
     LAUNCH(k_embed_rows, dim3((Dp + 255) / 256, rows), dim3(256), 0, emb, tok, scale, x, D, Dp);
+}
+
+void launch_embed_few(const float *emb, const int *tok, float scale, float *x, int D, int Dp, int rows)
+{
+    FewTokens t{};
+    for (int i = 0; i < rows; i++) t.id[i] = tok[i];
+    LAUNCH(k_embed_few, dim3((Dp + 255) / 256, rows), dim3(256), 0, emb, t, scale, x, D, Dp);
 }
 
 void launch_norm_rows(const NormRows &a, int rows) { LAUNCH(k_norm_rows, dim3(rows), dim3(256), (size_t)a.Dp * 4, a); }

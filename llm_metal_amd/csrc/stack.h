@@ -109,6 +109,7 @@ struct StackRun {
     MetalBuf *route_idx = nullptr, *route_w = nullptr, *act = nullptr, *ymoe = nullptr;
     MetalBuf *moe_tab = nullptr, *moe_a16 = nullptr, *moe_inv = nullptr, *moe_up = nullptr, *moe_act = nullptr, *moe_y = nullptr;   // grouped experts
     MetalBuf *lat_a16 = nullptr, *lat_inv = nullptr, *lat_kv = nullptr, *lat_frags = nullptr;   // prompt attention: expanded keys and values
+    int tok_end = 0;                                     // end of the positions whose tokens have been put there
     int moe_rows = 0;                                    // rows those hold
     int T = 0, pending = 0;                              // tokens per sequence of the last step; its last layer's sum still waits in cout (1) and ymoe (2) or moe_y (4, by `groups`)
     bool fused = false, one = false;                     // single tokens take the fused steps; the last step was one
@@ -146,6 +147,8 @@ struct NormRows {
 };
 void launch_norm_rows(const NormRows &a, int rows);
 void launch_embed_rows(const float *emb, const int *tok, float scale, float *x, int D, int Dp, int rows);
+constexpr int STACK_FEW = 32;
+void launch_embed_few(const float *emb, const int *tok, float scale, float *x, int D, int Dp, int rows);   // tok: host array of at most STACK_FEW
 
 // gemm_f32.hip: C[m][n] = sum_k A[m][k] W[n][k], fp32 throughout
 void launch_gemm_f32(const float *A, int lda, const float *W, int ldw, float *C, int ldc, int M, int N, int K);

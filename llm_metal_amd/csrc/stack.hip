@@ -499,12 +499,17 @@ void stack_forward(LayerStack *st, StackRun *r, const int *tokens, int T, int po
 {
     const Rows rows{r->B, T, pos};
     const int n = rows.n();
-    // tokens travel through pinned memory, every position in a place of its own: only a new sequence writes a place again
-    if (pos == 0) HIP_CHECK(hipStreamSynchronize(stream()));
-    int *th = r->tok_host + (size_t)pos * r->B;
-    memcpy(th, tokens, (size_t)n * sizeof(int));
-    HIP_CHECK(hipMemcpyAsync(dptr(r->tok), th, (size_t)n * sizeof(int), hipMemcpyHostToDevice, stream()));
-    launch_embed_rows(ptr<float>(st->emb), ptr<int>(r->tok), st->cfg.emb_scale, ptr<float>(r->x), st->D, st->Dp, n);
+    if (n <= STACK_FEW) launch_embed_few(ptr<float>(st->emb), tokens, st->cfg.emb_scale, ptr<float>(r->x), st->D, st->Dp, n);
+    else {
+        // many tokens travel through pinned memory, every position in a place of its own: only a sequence that has gone back
+        // writes a place again, and waits for the copies from it
+        if (pos < r->tok_end) HIP_CHECK(hipStreamSynchronize(stream()));
+        r->tok_end = pos + T;
+        int *th = r->tok_host + (size_t)pos * r->B;
+        memcpy(th, tokens, (size_t)n * sizeof(int));
+        HIP_CHECK(hipMemcpyAsync(dptr(r->tok), th, (size_t)n * sizeof(int), hipMemcpyHostToDevice, stream()));
+        launch_embed_rows(ptr<float>(st->emb), ptr<int>(r->tok), st->cfg.emb_scale, ptr<float>(r->x), st->D, st->Dp, n);
+    }
     r->T = T; r->pending = 0;
     r->one = n == 1 && r->fused;
     if (r->one) { decode_layers(st, r, pos); return; }

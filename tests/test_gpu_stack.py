@@ -11,7 +11,7 @@ import pytest
 
 from llm_metal_amd.configs import C1
 from llm_metal_amd.sft import InferenceState
-from llm_metal_amd.synth import make_model
+from llm_metal_amd.synth import make_model, write_stack_checkpoint
 from oracle import stack_oracle as so
 from tests.stack_models import MODELS, Model, config, channel, delta, latent, logit_error, moe
 
@@ -245,6 +245,32 @@ def test_trace_runner(dtype, tmp_path):
             assert logit_error(got, ref[r][[lo + k for k in w]]) < TOL["f32" if dtype == "float32" else "f16"]
 
 
+def test_wide_layers_on_the_large_products(tmp_path):
+    """Sizes at which the products of a long prompt take the kernels for many rows: the 16-bit prompt, the 16-bit fused
+    decoding and the 32-bit state agree, whole and in portions.  (Every expert is chosen, so that no rounding decides.)"""
+    mlp = moe(4, 4, 320, 1024)
+    cfg = config([(channel(8, 8, 128, 128, 4), mlp), (latent(8, 128, 64, 128, 256, window=300, scale=0.07), mlp), (delta(8, 4, 128, 128, 4), mlp)],
+                 width=1024, vocab=512)
+    m = Model.__new__(Model)
+    m.cfg, m.path = cfg, str(tmp_path)
+    write_stack_checkpoint(m.path, cfg, seed=3, rank_a=64, rank_g=64)
+    n = 1150
+    toks = [int(t) for t in np.random.default_rng(4).integers(0, 512, n)]
+    at = [0, 1, 127, 128, 299, 300, 301, 512, 1022, 1023, 1024, 1100, n - 1]
+    with state(m, "f32", max_seq=n) as inf:
+        want = inf.forward_tokens(toks, at)
+    with state(m, "f16", max_seq=n) as inf:
+        whole = inf.forward_tokens(toks, at)
+        assert logit_error(whole, want) < TOL["f16"]
+        inf.reset()
+        rows = run_portions(inf, toks, [600, 15, 2, 1, 500])
+        assert logit_error(rows[at], want) < TOL["f16"]
+        inf.reset()
+        inf.forward_tokens(toks[:n - 60])
+        last = [inf.forward_token(t) for t in toks[n - 60:]][-1]
+        assert logit_error(last[None], want[-1:]) < TOL["f16"]
+
+
 def test_what_is_refused(tmp_path):
     cfg, ra, rg = MODELS["mixed"]
     m = Model(cfg, tmp_path, ra, rg)
@@ -270,6 +296,25 @@ def test_what_is_refused(tmp_path):
     with pytest.raises(RuntimeError):
         state(huge, "f16")
     state(huge, "f32").free()
+
+
+def test_states_give_their_memory_back(tmp_path):
+    import ctypes
+    from llm_metal_amd import lib
+    cfg, ra, rg = MODELS["mixed"]
+    m = Model(cfg, tmp_path, ra, rg)
+    prompt = m.tokens(40)
+    free = []
+    with state(m, "f32") as keep:                              # keeps the library's own scratch alive
+        keep.forward_tokens(prompt)
+        for _ in range(4):
+            with state(m, "f16") as inf:
+                inf.generate(prompt, 5)
+                inf.generate_batch(prompt, 5, 3)
+            f, t = ctypes.c_size_t(0), ctypes.c_size_t(0)
+            lib.load().hip_mem_info(ctypes.byref(f), ctypes.byref(t))
+            free.append(f.value)
+    assert free[1] == free[2] == free[3]
 
 
 def test_portions_of_the_other_models():
