@@ -344,16 +344,42 @@ __global__ __launch_bounds__(256) void k_cat_rows(CatRows a)
     const int m = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     for (int i = a.H * a.vdim + tid; i < a.ldk; i += 256) row[i] = 0.f;
     if (a.g_out) {
-        for (int h = wave; h < a.H; h += 4) {
-            const float *o = a.o + ((size_t)m * a.H + h) * a.vdim, *gt = a.gate + (size_t)m * a.ld_gate + h * a.vdim;
-            float ss = 0.f;
-            for (int d = lane; d < a.vdim; d += 64) ss += o[d] * o[d];
-            const float inv = 1.f / sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
-            for (int d = lane; d < a.vdim; d += 64) row[h * a.vdim + d] = o[d] * inv * a.g_out[d] * (a.gate_silu ? silu(gt[d]) : sigmoid(gt[d]));
+        // two heads of a wave at a time, up to 128 values of each requested together (longer heads: a second trip)
+        for (int h0 = wave * 2; h0 < a.H; h0 += 8) {
+            const float *o[2], *gt[2];
+            float ss[2] = {0.f, 0.f}, ov[2][2], gv[2][2], wv[2];
+#pragma unroll
+            for (int k = 0; k < 2; k++) {
+                const int h = min(h0 + k, a.H - 1);
+                o[k] = a.o + ((size_t)m * a.H + h) * a.vdim; gt[k] = a.gate + (size_t)m * a.ld_gate + h * a.vdim;
+#pragma unroll
+                for (int e = 0; e < 2; e++) {
+                    const int d = min(lane + 64 * e, a.vdim - 1);
+                    ov[k][e] = o[k][d]; gv[k][e] = gt[k][d]; wv[e] = a.g_out[d];
+                }
+            }
+#pragma unroll
+            for (int k = 0; k < 2; k++) {
+#pragma unroll
+                for (int e = 0; e < 2; e++) if (lane + 64 * e < a.vdim) ss[k] += ov[k][e] * ov[k][e];
+                for (int d = lane + 128; d < a.vdim; d += 64) ss[k] += o[k][d] * o[k][d];
+            }
+#pragma unroll
+            for (int k = 0; k < 2; k++) {
+                const float inv = 1.f / sqrtf(wave_total(ss[k]) / (float)a.vdim + a.eps);
+                if (h0 + k >= a.H) break;
+                float *out = row + (h0 + k) * a.vdim;
+#pragma unroll
+                for (int e = 0; e < 2; e++)
+                    if (lane + 64 * e < a.vdim) out[lane + 64 * e] = ov[k][e] * inv * wv[e] * (a.gate_silu ? silu(gv[k][e]) : sigmoid(gv[k][e]));
+                for (int d = lane + 128; d < a.vdim; d += 64) out[d] = o[k][d] * inv * a.g_out[d] * (a.gate_silu ? silu(gt[k][d]) : sigmoid(gt[k][d]));
+            }
         }
     } else
+#pragma unroll 8
         for (int i = tid; i < a.H * a.vdim; i += 256) row[i] = a.o[(size_t)m * a.H * a.vdim + i];
     __syncthreads();                                      // the zeros are down before the shared part overwrites some
+#pragma unroll 4
     for (int i = tid; i < a.shared_ff; i += 256) row[a.o_sh + i] = relu2(a.shared[(size_t)m * a.ld_shared + i]);
     __syncthreads();
     if (a.cat)

@@ -4,41 +4,50 @@
 
 namespace lmhip {
 
-// One wave: softmax over all E <= 1024 experts, the `top` largest scores in order (of equals the lower index), not
-// renormalised.  A lane holds experts lane, lane + 64, ...
-__device__ __forceinline__ void route_row(const float *z, int E, int top, int lane, int *out_idx, float *out_w)
+// One wave: softmax over all E experts, the `top` largest scores in order (of equals the lower index), not renormalised.
+// A lane holds experts lane, lane + 64, ... (NI of them).
+template <int NI>
+__device__ __forceinline__ void route_experts(const float *z, int E, int top, int lane, int *out_idx, float *out_w)
 {
-    float v[16], mx = -3.0e38f;
+    float v[NI], mx = -3.0e38f;
 #pragma unroll
-    for (int i = 0; i < 16; i++) {
+    for (int i = 0; i < NI; i++) {
         const int e = lane + 64 * i;
         v[i] = e < E ? z[e] : -3.0e38f;
         mx = fmaxf(mx, v[i]);
     }
-    mx = wave_max(mx);
+    mx = wave_peak(mx);
     float sum = 0.f;
 #pragma unroll
-    for (int i = 0; i < 16; i++) {
+    for (int i = 0; i < NI; i++) {
         const bool in = lane + 64 * i < E;
         v[i] = in ? expf(v[i] - mx) : -1.f;
         sum += in ? v[i] : 0.f;
     }
-    sum = wave_sum(sum);
+    sum = wave_total(sum);
     for (int s = 0; s < top; s++) {
-        float best = -2.f;
-        int idx = 0x7fffffff;
+        float best = v[0];
 #pragma unroll
-        for (int i = 0; i < 16; i++) if (v[i] > best) { best = v[i]; idx = lane + 64 * i; }
+        for (int i = 1; i < NI; i++) best = fmaxf(best, v[i]);
+        best = wave_peak(best);
+        int idx = E - 1;                                  // (what scores that are not numbers choose)
 #pragma unroll
-        for (int o = 32; o > 0; o >>= 1) {
-            const float ob = __shfl_xor(best, o, WAVE);
-            const int oi = __shfl_xor(idx, o, WAVE);
-            if (ob > best || (ob == best && oi < idx)) { best = ob; idx = oi; }
+        for (int i = NI - 1; i >= 0; i--) {
+            const unsigned long long has = __ballot(v[i] == best);
+            if (has) idx = 64 * i + __ffsll(has) - 1;
         }
-        if (lane == 0) { out_idx[s] = min(idx, E - 1); out_w[s] = best / sum; }   // (scores that are not numbers choose the last)
+        idx = min(idx, E - 1);
+        if (lane == 0) { out_idx[s] = idx; out_w[s] = best / sum; }
 #pragma unroll
-        for (int i = 0; i < 16; i++) if (lane + 64 * i == idx) v[i] = -1.f;
+        for (int i = 0; i < NI; i++) if (lane + 64 * i == idx) v[i] = -1.f;
     }
+}
+// E <= 1024
+__device__ __forceinline__ void route_row(const float *z, int E, int top, int lane, int *out_idx, float *out_w)
+{
+    if (E <= 64) route_experts<1>(z, E, top, lane, out_idx, out_w);
+    else if (E <= 256) route_experts<4>(z, E, top, lane, out_idx, out_w);
+    else route_experts<16>(z, E, top, lane, out_idx, out_w);
 }
 
 template <typename WT> struct Vec8;

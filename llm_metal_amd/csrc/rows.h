@@ -59,4 +59,19 @@ __device__ __forceinline__ float wave_total(float v)
     return swap32_add(group_sum<32>(v));
 }
 
+// largest over the wave, left in every lane
+template <int CTRL>
+__device__ __forceinline__ float dpp_max(float v)
+{
+    return fmaxf(v, __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, true)));
+}
+__device__ __forceinline__ float wave_peak(float v)
+{
+    v = dpp_max<0xB1>(v); v = dpp_max<0x4E>(v); v = dpp_max<0x141>(v); v = dpp_max<0x140>(v);
+    const auto t = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    v = fmaxf(__uint_as_float(t[0]), __uint_as_float(t[1]));
+    const auto u = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    return fmaxf(__uint_as_float(u[0]), __uint_as_float(u[1]));
+}
+
 }  // namespace lmhip
