@@ -120,7 +120,7 @@ def make_batch(c: SFTConfig, seed=1):
 
 # ---------------------------------------------------------------- models described layer by layer (Nevurax)
 
-def stack_shapes(cfg, rank_a=24, rank_g=24):
+def stack_shapes(cfg, rank_a=16, rank_g=16):
     """Tensor names and shapes of a layer-by-layer model; cfg is the dictionary that becomes its config.json.  rank_a and
     rank_g: widths of the two low-rank products of a per-channel decay (tensor shapes, not configuration)."""
     D = cfg["width"]
@@ -181,7 +181,7 @@ def to_bf16_bits(a):
     return ((b + np.uint32(0x7FFF) + ((b >> np.uint32(16)) & np.uint32(1))) >> np.uint32(16)).astype(np.uint16)
 
 
-def write_stack_checkpoint(path, cfg, seed=0, rank_a=24, rank_g=24, keep=False, edit=None, repeat=False):
+def write_stack_checkpoint(path, cfg, seed=0, rank_a=16, rank_g=16, keep=False, edit=None, repeat=False):
     """config.json and model.safetensors (bfloat16) of a random model in the folder `path`.  keep: return the values the
     file holds, fp32 by name.  edit(name, array): may replace a tensor before it is rounded.  repeat: every matrix of the
     experts is the same one (large models for timing, written in a fraction of the time)."""
