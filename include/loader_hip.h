@@ -52,6 +52,8 @@ WMat *model_file_load_wmat(ModelFile *f, const char *name, int use_fp16);
  * says nothing or is absent.  A design that lists its layers is recognised by its "architecture". */
 ModelType model_type_detect(const char *path);
 const char *model_type_name(ModelType model_type);
+/* 1 for a design whose config.json lists its layers (MODEL_NEVURAX, MODEL_PAPOSUN) */
+int model_type_layered(ModelType model_type);
 
 /* qwen3_load_safetensors / qwen3_load_gguf (src/nn/qwen3.c:211-371) and gemma3_load_safetensors
  * (src/nn/gemma3.c:176-285) up to the point where the model struct is filled: every tensor as fp32, the LM head tied to

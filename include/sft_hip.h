@@ -43,7 +43,7 @@ extern "C" {
  *      translation unit of the reference declares these types and functions ---- */
 #ifndef WMAT_H
 #define WMAT_H
-typedef enum { MODEL_QWEN3, MODEL_GEMMA3, MODEL_NEVURAX } ModelType;   /* the last: generation only (inference_hip.h) */
+typedef enum { MODEL_QWEN3, MODEL_GEMMA3, MODEL_NEVURAX, MODEL_PAPOSUN } ModelType;   /* the last two: generation only (inference_hip.h) */
 
 typedef struct WMat {
     MetalBuf *mbuf;

@@ -5,7 +5,7 @@ NL layers, D hidden, Hq/Hkv heads, hd head dim, IS FFN width, V vocab.
 """
 from dataclasses import dataclass, replace
 
-QWEN3, GEMMA3, NEVURAX = 0, 1, 2     # ModelType of include/sft_hip.h
+QWEN3, GEMMA3, NEVURAX, PAPOSUN = 0, 1, 2, 3     # ModelType of include/sft_hip.h
 
 
 @dataclass(frozen=True)

@@ -68,12 +68,19 @@ struct NormIn {
     const float *xr, *br, *g;
     float *x_out;
     float eps;
-    int dim;                             // layer norm only: entries of xr that count
+    int dim;                             // layer norm and norms around: entries of xr that count
+    const float *g_br, *b_br;            // norms around: RMS norm weight and bias (may be null) of br
 };
 // infer_kernels.hip: y = W . RMSNorm(xr + br; g) (glu 0), or the gated pair product of matvec_glu over it (1 SiLU, 2 GELU)
 void matvec_norm(MetalBuf *W, const NormIn &nin, MetalBuf *y, int rows, int cols, int q8, int glu);
 // infer_kernels.hip: y = W . LayerNorm(x; g) over the first dim of cols entries (F16 rows)
 void matvec_layernorm(MetalBuf *W, const float *x, const float *g, int dim, float eps, float *y, int rows, int cols);
+
+// infer_kernels.hip: y = W . RMSNorm(v; g) with v = xr + RMSNorm(br + b_br; g_br) (br may be null) over the first dim of cols
+// entries, v also to x_out (F16 rows); gelu: y = tanh-GELU of it
+void matvec_norms_around(MetalBuf *W, const NormIn &nin, float *y, int rows, int cols, int gelu);
+// infer_kernels.hip: y = W . x (F16 rows, cols a multiple of 8)
+void matvec_rows(MetalBuf *W, const float *x, float *y, int rows, int cols);
 
 }  // namespace lmhip
 

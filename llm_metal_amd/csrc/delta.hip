@@ -343,11 +343,17 @@ __global__ __launch_bounds__(256) void k_cat_rows(CatRows a)
     __shared__ float sm[16];
     const int m = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     for (int i = a.H * a.vdim + tid; i < a.ldk; i += 256) row[i] = 0.f;
-    if (a.g_out) {
+    if (!a.g_out && a.gate) {
+#pragma unroll 4
+        for (int i = tid; i < a.H * a.vdim; i += 256) {
+            const float g = a.gate[(size_t)m * a.ld_gate + i];
+            row[i] = a.o[(size_t)m * a.H * a.vdim + i] * (a.gate_silu ? silu(g) : sigmoid(g));
+        }
+    } else if (a.g_out) {
         // two heads of a wave at a time, up to 128 values of each requested together (longer heads: a second trip)
         for (int h0 = wave * 2; h0 < a.H; h0 += 8) {
             const float *o[2], *gt[2];
-            float ss[2] = {0.f, 0.f}, ov[2][2], gv[2][2], wv[2];
+            float ss[2] = {0.f, 0.f}, ov[2][2], gv[2][2], wv[2][2];
 #pragma unroll
             for (int k = 0; k < 2; k++) {
                 const int h = min(h0 + k, a.H - 1);
@@ -355,7 +361,7 @@ __global__ __launch_bounds__(256) void k_cat_rows(CatRows a)
 #pragma unroll
                 for (int e = 0; e < 2; e++) {
                     const int d = min(lane + 64 * e, a.vdim - 1);
-                    ov[k][e] = o[k][d]; gv[k][e] = gt[k][d]; wv[e] = a.g_out[d];
+                    ov[k][e] = o[k][d]; gv[k][e] = gt[k][d]; wv[k][e] = a.g_out[h * a.g_stride + d];
                 }
             }
 #pragma unroll
@@ -371,8 +377,8 @@ __global__ __launch_bounds__(256) void k_cat_rows(CatRows a)
                 float *out = row + (h0 + k) * a.vdim;
 #pragma unroll
                 for (int e = 0; e < 2; e++)
-                    if (lane + 64 * e < a.vdim) out[lane + 64 * e] = ov[k][e] * inv * wv[e] * (a.gate_silu ? silu(gv[k][e]) : sigmoid(gv[k][e]));
-                for (int d = lane + 128; d < a.vdim; d += 64) out[d] = o[k][d] * inv * a.g_out[d] * (a.gate_silu ? silu(gt[k][d]) : sigmoid(gt[k][d]));
+                    if (lane + 64 * e < a.vdim) out[lane + 64 * e] = ov[k][e] * inv * wv[k][e] * (a.gate_silu ? silu(gv[k][e]) : sigmoid(gv[k][e]));
+                for (int d = lane + 128; d < a.vdim; d += 64) out[d] = o[k][d] * inv * a.g_out[(h0 + k) * a.g_stride + d] * (a.gate_silu ? silu(gt[k][d]) : sigmoid(gt[k][d]));
             }
         }
     } else

@@ -98,8 +98,10 @@ const int8_t *q8_split_of(MetalBuf *W, int rows, int nb, const half_t **scales)
 // factor rsqrt(mean + eps) onto the finished sums; workgroup 0 also writes v to x_out (not xr: the others still read it).
 // residual_add + rms_norm of shaders/q8_kernels.metal:133-158, 369-375 without a launch of their own.  NORM 2: a layer norm
 // of the first `dim` entries of xr instead (mean taken off, no branch, the padding behind them zero).
+// NORM 3: RMSNorm of v = xr + RMSNorm(br + b_br; g_br) over the first `dim` entries, v kept as above.
+// ACT 1: y[row] = tanh-GELU of the sum.
 // REPS (NORM only): row groups a wave takes one after the other, so that fewer workgroups form the vector.
-template <int FMT, int R, int U, int XLDS, int GLU = 0, int NORM = 0, int REPS = 1>
+template <int FMT, int R, int U, int XLDS, int GLU = 0, int NORM = 0, int REPS = 1, int ACT = 0>
 __global__ __launch_bounds__(TB) void k_matvec(const void *__restrict__ Wp, const half_t *__restrict__ scales,
                                                const float *__restrict__ x, float *__restrict__ y, int rows, int cols, NormIn nin)
 {
@@ -202,6 +204,34 @@ __global__ __launch_bounds__(TB) void k_matvec(const void *__restrict__ Wp, cons
             *reinterpret_cast<float4v *>(&xs[i]) = v * gg;
         }
         norm_inv = 1.f / sqrtf(block_sum(ss, red) / (float)nin.dim + nin.eps);
+    } else if (NORM == 3) {
+        float post = 0.f;
+        if (nin.br) {
+            float ss = 0.f;
+            for (int i = tid * 4; i < cols; i += TB * 4) {
+                float4v v = *reinterpret_cast<const float4v *>(&nin.br[i]);
+                if (nin.b_br) v += *reinterpret_cast<const float4v *>(&nin.b_br[i]);
+#pragma unroll
+                for (int e = 0; e < 4; e++) { v[e] = i + e < nin.dim ? v[e] : 0.f; ss += v[e] * v[e]; }
+                *reinterpret_cast<float4v *>(&xs[i]) = v;
+            }
+            post = 1.f / sqrtf(block_sum(ss, red) / (float)nin.dim + nin.eps);
+        }
+        float ss = 0.f;
+        for (int i = tid * 4; i < cols; i += TB * 4) {          // the thread's own entries
+            float4v v = *reinterpret_cast<const float4v *>(&nin.xr[i]);
+            const float4v gg = *reinterpret_cast<const float4v *>(&nin.g[i]);
+            if (nin.br) {
+                const float4v b = *reinterpret_cast<const float4v *>(&xs[i]), w = *reinterpret_cast<const float4v *>(&nin.g_br[i]);
+#pragma unroll
+                for (int e = 0; e < 4; e++) v[e] = fmaf(b[e] * post, w[e], v[e]);
+                if (blockIdx.x == 0 && nin.x_out) *reinterpret_cast<float4v *>(&nin.x_out[i]) = v;
+            }
+#pragma unroll
+            for (int e = 0; e < 4; e++) ss += v[e] * v[e];      // (zeros behind dim)
+            *reinterpret_cast<float4v *>(&xs[i]) = v * gg;
+        }
+        norm_inv = 1.f / sqrtf(block_sum(ss, red) / (float)nin.dim + nin.eps);
     } else if (NORM) {
         float ss = 0.f;
         for (int i0 = tid * 4; i0 < cols; i0 += TB * 16) {      // four groups of a thread requested together
@@ -250,7 +280,7 @@ __global__ __launch_bounds__(TB) void k_matvec(const void *__restrict__ Wp, cons
 #pragma unroll
             for (int r = 0; r < R; r++) {
                 const float s = wave_sum(acc[r]) * norm_inv;
-                if (lane == 0 && row0 + r < rows) y[row0 + r] = s;
+                if (lane == 0 && row0 + r < rows) y[row0 + r] = ACT ? 0.5f * s * (1.0f + tanhf(gelu_inner(s))) : s;
             }
         }
     }
@@ -964,6 +994,34 @@ void matvec_layernorm(MetalBuf *W, const float *x, const float *g, int dim, floa
     HIP_CHECK(hipGetLastError()); } while (0)
     if (rows >= 16384) LN_LAUNCH(4); else LN_LAUNCH(1);      // many rows: fewer workgroups form the vector
 #undef LN_LAUNCH
+}
+
+void matvec_norms_around(MetalBuf *W, const NormIn &nin, float *y, int rows, int cols, int gelu)
+{
+    bool ok = rows > 0 && nin.dim > 0 && nin.dim <= cols && !(cols & 7) && cols <= 15360 && aligned16(dptr(W)) && nin.xr && nin.g && nin.x_out != nin.xr;
+    for (const void *p : {(const void *)nin.xr, (const void *)nin.g, (const void *)nin.br, (const void *)nin.g_br, (const void *)nin.b_br, (const void *)nin.x_out})
+        ok = ok && aligned16(p);
+    if (!ok || (nin.br && !nin.g_br)) { fprintf(stderr, "[fast_hip] matvec_norms_around: unsupported shape %d x %d or operands\n", rows, cols); abort(); }
+    REQUIRE_BYTES(W, (size_t)rows * cols * 2, "matvec_norms_around");
+    hipEvent_t ev_a = nullptr, ev_b = nullptr;
+    const bool prof = gemm_prof_begin(2.0 * rows * cols, 2.0 * rows * cols, &ev_a, &ev_b);
+    const size_t lds = (size_t)cols * 4;
+    const half_t *scales = nullptr;
+#define AROUND_LAUNCH(REPS_, ACT_) do { \
+    const dim3 grid((rows + 8 * REPS_ - 1) / (8 * REPS_)); \
+    if (prof) hipExtLaunchKernelGGL((k_matvec<0, 2, 2, 1, 0, 3, REPS_, ACT_>), grid, dim3(TB), lds, stream(), ev_a, ev_b, 0, dptr(W), scales, nullptr, y, rows, cols, nin); \
+    else hipLaunchKernelGGL((k_matvec<0, 2, 2, 1, 0, 3, REPS_, ACT_>), grid, dim3(TB), lds, stream(), dptr(W), scales, nullptr, y, rows, cols, nin); \
+    HIP_CHECK(hipGetLastError()); } while (0)
+    if (gelu) { if (rows >= 16384) AROUND_LAUNCH(4, 1); else AROUND_LAUNCH(1, 1); }
+    else { if (rows >= 16384) AROUND_LAUNCH(4, 0); else AROUND_LAUNCH(1, 0); }
+#undef AROUND_LAUNCH
+}
+
+void matvec_rows(MetalBuf *W, const float *x, float *y, int rows, int cols)
+{
+    if (rows <= 0 || cols <= 0 || (cols & 7) || !aligned16(dptr(W)) || !aligned16(x)) { fprintf(stderr, "[fast_hip] matvec_rows: unsupported shape %d x %d\n", rows, cols); abort(); }
+    REQUIRE_BYTES(W, (size_t)rows * cols * 2, "matvec_rows");
+    launch_matvec<0>(dptr(W), nullptr, x, y, rows, cols);
 }
 
 // The same products (glu 0: y[i] = W_i . ln for `rows` rows) over ln = RMSNorm(xr + br; g), the sum and the norm formed

@@ -480,7 +480,7 @@ extern "C" {
 
 InferenceState *inference_state_create_from_ref(const SFTModelRef *m, int max_seq_len, int use_fp16)
 {
-    if (m->model_type == MODEL_NEVURAX) { fprintf(stderr, "[FastGen] Nevurax models are created by inference_state_create_from_file\n"); return nullptr; }
+    if (model_type_layered(m->model_type)) { fprintf(stderr, "[FastGen] %s models are created by inference_state_create_from_file\n", model_type_name(m->model_type)); return nullptr; }
     InferenceState *s = new_state(m->model_type, m->d_model, m->n_q_heads, m->n_kv_heads, m->head_dim, m->intermediate_size,
                                   m->vocab_size, m->n_layers, max_seq_len, use_fp16, m->rope_thetas);
     if (!s) return nullptr;
@@ -522,11 +522,11 @@ InferenceState *inference_state_create_from_ref(const SFTModelRef *m, int max_se
 
 // Straight from the file to HBM: every matrix is uploaded as stored and converted on the GPU (F16 and Q8_0 tensors that
 // already have the wanted format are used bit for bit); Q|K|V and gate|up are joined by device copies of whole rows.
-static InferenceState *stack_state_from_file(const char *path, int max_seq_len, int weight_format);
+static InferenceState *stack_state_from_file(const char *path, ModelType model_type, int max_seq_len, int weight_format);
 
 InferenceState *inference_state_create_from_file(const char *path, ModelType model_type, int max_seq_len, int use_fp16)
 {
-    if (model_type == MODEL_NEVURAX) return stack_state_from_file(path, max_seq_len, use_fp16);
+    if (model_type_layered(model_type)) return stack_state_from_file(path, model_type, max_seq_len, use_fp16);
     if (use_fp16 == 2) { fprintf(stderr, "[FastGen] %s weights are F16 or Q8_0\n", model_type_name(model_type)); return nullptr; }
     ModelFile *f = model_file_open(path);
     if (!f) return nullptr;
@@ -610,9 +610,9 @@ InferenceState *inference_state_create_from_file(const char *path, ModelType mod
 }
 
 // A model described layer by layer: config.json beside the weights says what the layers are.
-static InferenceState *stack_state_from_file(const char *path, int max_seq_len, int weight_format)
+static InferenceState *stack_state_from_file(const char *path, ModelType model_type, int max_seq_len, int weight_format)
 {
-    if (weight_format != 1 && weight_format != 2) { fprintf(stderr, "[FastGen] Nevurax weights are F16 or 32-bit\n"); return nullptr; }
+    if (weight_format != 1 && weight_format != 2) { fprintf(stderr, "[FastGen] %s weights are F16 or 32-bit\n", model_type_name(model_type)); return nullptr; }
     if (max_seq_len <= 0) return nullptr;
     const std::string cfg_path = config_path_of(path);
     std::ifstream in(cfg_path);
@@ -620,7 +620,7 @@ static InferenceState *stack_state_from_file(const char *path, int max_seq_len, 
     if (in) text << in.rdbuf();
     StackConfig cfg;
     std::string why;
-    if (!in || !read_stack_config(text.str(), cfg, why)) {
+    if (!in || !read_stack_config(text.str(), model_type, cfg, why)) {
         fprintf(stderr, "[FastGen] %s: %s\n", cfg_path.c_str(), in ? why.c_str() : "cannot be read");
         return nullptr;
     }
@@ -629,7 +629,7 @@ static InferenceState *stack_state_from_file(const char *path, int max_seq_len, 
     LayerStack *st = f ? stack_load(f, cfg, weight_format == 2, max_seq_len) : nullptr;
     model_file_close(f);
     if (!st) { fast_metal_shutdown(); return nullptr; }
-    InferenceState *s = base_state(MODEL_NEVURAX, cfg.width, cfg.vocab, (int)cfg.layers.size(), max_seq_len, st);
+    InferenceState *s = base_state(model_type, cfg.width, cfg.vocab, (int)cfg.layers.size(), max_seq_len, st);
     s->use_fp16 = weight_format;
     return s;
 }

@@ -13,14 +13,6 @@ namespace {
 
 constexpr int HG = 4;        // heads that share the reading of a key row
 
-__global__ __launch_bounds__(256) void k_rope_interleaved(float2 *tab, int n, int pairs, int dims, double base)
-{
-    const int i = blockIdx.x * 256 + threadIdx.x;
-    if (i >= n) return;
-    const double angle = (double)(i / pairs) * pow(base, -2.0 * (double)(i % pairs) / (double)dims);
-    tab[i] = make_float2((float)cos(angle), (float)sin(angle));
-}
-
 // grid (rows)
 __global__ __launch_bounds__(256) void k_latent_cache(LatentRows a)
 {
@@ -166,12 +158,6 @@ __global__ __launch_bounds__(256) void k_latent_values(LatentRows a, int m0, int
 }
 
 }  // namespace
-
-void launch_rope_interleaved(float2 *tab, int max_seq, int dims, double base)
-{
-    const int n = max_seq * (dims / 2);
-    if (n > 0) LAUNCH(k_rope_interleaved, dim3((n + 255) / 256), dim3(256), 0, tab, n, dims / 2, dims, base);
-}
 
 void launch_latent_cache(const LatentRows &a) { LAUNCH(k_latent_cache, dim3(a.r.n()), dim3(256), 0, a); }
 

@@ -3,7 +3,7 @@
 // of a head per workgroup.  Scores, running maximum and sums are fp32; the operands of the two products are F16.
 #include "stack.h"
 #include "latent_rows.h"
-#include "lds_copy.h"
+#include "prompt_attn.h"
 #include <algorithm>
 
 namespace lmhip {
@@ -11,8 +11,6 @@ namespace {
 
 #define LAUNCH(kern, grid, block, lds, ...) do { \
     hipLaunchKernelGGL(kern, grid, block, lds, stream(), __VA_ARGS__); HIP_CHECK(hipGetLastError()); } while (0)
-
-typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 
 struct PromptArgs {
     LatentRows a;
@@ -36,9 +34,7 @@ __global__ __launch_bounds__(256) void k_latent_operand(PromptArgs p, half_t *a1
     if (threadIdx.x == 0) inv[m] = 1.f / s;
 }
 
-// grid (blocks, H, B): fragments of 32 keys of one head.  K fragment j: lane -> key lane & 31, dimensions 16 j + 8 (lane >> 5)
-// .. + 7.  V fragment (db, u): lane -> value column 32 db + (lane & 31), the keys that lane half holds of the score tile's
-// rows 8 u .. 8 u + 7.
+// grid (blocks, H, B): fragments of 32 keys of one head (prompt_attn.h)
 template <int NJ, int NDB>
 __global__ __launch_bounds__(256) void k_latent_frags(PromptArgs p)
 {
@@ -72,9 +68,7 @@ __global__ __launch_bounds__(256) void k_latent_frags(PromptArgs p)
     }
 }
 
-// grid (blocks of 128 queries, H, B), block 256: a wave owns 32 queries; key blocks pass through LDS, the next one on its
-// way while one is multiplied.  S^T = K Q^T leaves a query's scores in one lane pair, the running softmax needs one
-// exchange, and the weights are already the operand of O^T += V^T P^T.
+// grid (blocks of 128 queries, H, B), block 256
 template <int NJ, int NDB>
 __global__ __launch_bounds__(256) void k_latent_prompt(PromptArgs p)
 {
@@ -85,9 +79,12 @@ __global__ __launch_bounds__(256) void k_latent_prompt(PromptArgs p)
     const int q0 = (gridDim.x - 1 - blockIdx.x) * 128, h = blockIdx.y, b = blockIdx.z, T = a.r.T;
     const int qw = q0 + 32 * wave, qi = min(qw + l31, T - 1);
     const int off = a.r.pos - p.first;                    // key index of the step's first token
-    const int last = off + qi, lo = last - a.window + 1;  // this lane's visible keys: max(lo, 0) .. last
-    const int w_hi = off + min(qw + 31, T - 1), w_lo = off + min(qw, T - 1) - a.window + 1;
-    const bool w_live = qw < T;
+    PromptSpan sp;
+    sp.live = qw < T;
+    sp.last = off + qi; sp.lo = sp.last - a.window + 1;
+    sp.w_hi = off + min(qw + 31, T - 1); sp.w_lo = off + min(qw, T - 1) - a.window + 1;
+    sp.all_hi = off + qw; sp.all_lo = off + qw + 31 - a.window + 1;
+    sp.kb0 = max(0, off + q0 - a.window + 1) >> 5; sp.kb1 = (off + min(q0 + 127, T - 1)) >> 5;
     const size_t m = (size_t)b * T + qi;
     half8 qf[NJ];
     {
@@ -102,73 +99,10 @@ __global__ __launch_bounds__(256) void k_latent_prompt(PromptArgs p)
                 qf[j][e] = (half_t)(d < a.dim ? q[d] * f : d < a.dim + a.rot ? rotated(q + a.dim, d - a.dim, a.rot_dims, cs) * f : 0.f);
             }
     }
-    float16v O[NDB];
-#pragma unroll
-    for (int i = 0; i < NDB; i++)
-#pragma unroll
-        for (int v = 0; v < 16; v++) O[i][v] = 0.f;
-    float m_run = -1e30f, l_run = 0.f;
-    const int kb0 = max(0, off + q0 - a.window + 1) >> 5, kb1 = (off + min(q0 + 127, T - 1)) >> 5;
     const uint4 *src = reinterpret_cast<const uint4 *>(p.frags) + ((size_t)b * a.H + h) * p.blocks * NF * 64 + lane;
-    auto request = [&](int kb, uint4 *buf) __attribute__((always_inline)) {
-#pragma unroll
-        for (int f = 0; f < (NF + 3) / 4; f++)
-            if (wave + 4 * f < NF) copy_to_lds_1k(src + ((size_t)kb * NF + wave + 4 * f) * 64, buf + (wave + 4 * f) * 64);
-    };
-    auto step = [&](int kb, const uint4 *cur) __attribute__((always_inline)) {
-        const int k0 = kb * 32;
-        if (!w_live || k0 > w_hi || k0 + 31 < w_lo) return;
-        float16v s;
-#pragma unroll
-        for (int v = 0; v < 16; v++) s[v] = 0.f;
-#pragma unroll
-        for (int j = 0; j < NJ; j++) s = __builtin_amdgcn_mfma_f32_32x32x16_f16(__builtin_bit_cast(half8, cur[j * 64 + lane]), qf[j], s, 0, 0, 0);
-        if (k0 + 31 > off + qw || k0 < off + qw + 31 - a.window + 1) {    // a key of the block is hidden from some query of the wave
-#pragma unroll
-            for (int v = 0; v < 16; v++) {
-                const int k = k0 + 8 * (v >> 2) + 4 * hh + (v & 3);
-                if (k > last || k < lo) s[v] = -INFINITY;
-            }
-        }
-        float mx = s[0];
-#pragma unroll
-        for (int v = 1; v < 16; v++) mx = fmaxf(mx, s[v]);
-        mx = fmaxf(mx, __shfl_xor(mx, 32, WAVE));
-        const float m_new = fmaxf(m_run, mx);
-        if (__any(m_new > m_run)) {
-            const float alpha = exp2f(m_run - m_new);
-            l_run *= alpha;
-#pragma unroll
-            for (int i = 0; i < NDB; i++)
-#pragma unroll
-                for (int v = 0; v < 16; v++) O[i][v] *= alpha;
-            m_run = m_new;
-        }
-        half8 pf[2];
-#pragma unroll
-        for (int v = 0; v < 16; v++) {
-            const float e = __builtin_amdgcn_exp2f(s[v] - m_run);
-            l_run += e;
-            pf[v >> 3][v & 7] = (half_t)e;
-        }
-#pragma unroll
-        for (int i = 0; i < NDB; i++)
-#pragma unroll
-            for (int u = 0; u < 2; u++)
-                O[i] = __builtin_amdgcn_mfma_f32_32x32x16_f16(__builtin_bit_cast(half8, cur[(NJ + 2 * i + u) * 64 + lane]), pf[u], O[i], 0, 0, 0);
-    };
-    request(kb0, buf0);
-    FA_WAIT_AND_BARRIER();
-    for (int kb = kb0; kb <= kb1; kb += 2) {
-        if (kb + 1 <= kb1) request(kb + 1, buf1);
-        step(kb, buf0);
-        FA_WAIT_AND_BARRIER();
-        if (kb + 1 > kb1) break;
-        if (kb + 2 <= kb1) request(kb + 2, buf0);
-        step(kb + 1, buf1);
-        FA_WAIT_AND_BARRIER();
-    }
-    l_run += __shfl_xor(l_run, 32, WAVE);
+    float16v O[NDB];
+    float l_run;
+    prompt_attend<NJ, NDB>(qf, src, sp, buf0, buf1, O, l_run);
     if (qw + l31 >= T) return;
     const float inv = 1.f / l_run;
     float *out = a.o + (m * a.H + h) * a.vdim;

@@ -478,7 +478,7 @@ WMat *model_file_load_wmat(ModelFile *f, const char *name, int use_fp16)
 
 SFTModelRef *model_ref_load(const char *path, ModelType model_type)
 {
-    if (model_type == MODEL_NEVURAX) { fprintf(stderr, "[Loader] Nevurax models are created by inference_state_create_from_file\n"); return nullptr; }
+    if (model_type_layered(model_type)) { fprintf(stderr, "[Loader] %s models are created by inference_state_create_from_file\n", model_type_name(model_type)); return nullptr; }
     ModelFile *f = model_file_open(path);
     if (!f) return nullptr;
     const bool gg = f->gguf;

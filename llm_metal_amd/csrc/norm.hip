@@ -1,5 +1,5 @@
-// The residual row kernels of a layer-by-layer model: embedding rows, and the residual sum with the layer norm that
-// feeds a product.
+// The row kernels of a layer-by-layer model around its products: embedding rows, the residual sum with the norm that feeds
+// a product, the dense feed-forward's activation, rotation tables.
 #include "stack.h"
 #include "rows.h"
 
@@ -74,7 +74,123 @@ __global__ __launch_bounds__(256) void k_norm_rows(NormRows a)
     }
 }
 
+// One workgroup per row: the norm behind a sublayer, the residual sum, the norm ahead of the next one.
+__global__ __launch_bounds__(256) void k_norms_around(AroundRows a)
+{
+    extern __shared__ float row[];                        // [Dp]
+    __shared__ float sm[32];
+    const int m = blockIdx.x, src = a.want ? a.want[m] : m * a.step + a.first, tid = threadIdx.x;
+    const size_t off = (size_t)src * a.Dp;
+    float post = 0.f;
+    if (a.cout) {
+        float ss = 0.f;
+        for (int i = tid * 4; i < a.Dp; i += 1024) {
+            float4 y = *reinterpret_cast<const float4 *>(a.cout + off + i);
+            if (a.post_b) {
+                const float4 b = *reinterpret_cast<const float4 *>(a.post_b + i);
+                y.x += b.x; y.y += b.y; y.z += b.z; y.w += b.w;
+            }
+            *reinterpret_cast<float4 *>(row + i) = y;     // (the weight's padding rows are zero)
+            ss += (y.x * y.x + y.y * y.y) + (y.z * y.z + y.w * y.w);
+        }
+        post = 1.f / sqrtf(block_sum(ss, sm) / (float)a.D + a.eps);
+    }
+    float ss = 0.f, mx = 0.f;
+    for (int i = tid * 4; i < a.Dp; i += 1024) {          // the thread's own entries
+        float4 v = *reinterpret_cast<const float4 *>(a.x + off + i);
+        const float4 g = *reinterpret_cast<const float4 *>(a.g + i);
+        if (a.cout) {
+            const float4 y = *reinterpret_cast<const float4 *>(row + i), w = *reinterpret_cast<const float4 *>(a.post_g + i);
+            v.x = fmaf(y.x * post, w.x, v.x); v.y = fmaf(y.y * post, w.y, v.y); v.z = fmaf(y.z * post, w.z, v.z); v.w = fmaf(y.w * post, w.w, v.w);
+            if (a.keep) *reinterpret_cast<float4 *>(a.x + off + i) = v;
+        }
+        ss += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+        const float4 h = make_float4(v.x * g.x, v.y * g.y, v.z * g.z, v.w * g.w);
+        *reinterpret_cast<float4 *>(row + i) = h;
+        mx = fmaxf(mx, fmaxf(fmaxf(fabsf(h.x), fabsf(h.y)), fmaxf(fabsf(h.z), fabsf(h.w))));
+    }
+    block_sum_max(ss, mx, sm);                            // its barriers also publish the row
+    const float inv = 1.f / sqrtf(ss / (float)a.D + a.eps);
+    if (a.h)
+        for (int i = tid; i < a.Dp; i += 256) a.h[(size_t)m * a.Dp + i] = row[i] * inv;
+    if (a.a16) {
+        const float s = row_scale_for(mx * inv);
+        store_row_f16(row, a.Dp, a.a16, m, tiled_kb(a.Dp), s * inv);
+        if (tid == 0) a.inv[m] = 1.f / s;
+    }
+}
+
+// One workgroup per row.  The operand's rows wait in LDS (staged) or, when they are too long, are formed twice.
+__global__ __launch_bounds__(256) void k_gelu_rows(ActRows a, int staged)
+{
+    extern __shared__ float row[];                        // [K] when staged
+    __shared__ float sm[16];
+    const int m = blockIdx.x, tid = threadIdx.x;
+    const float *up = a.up + (size_t)m * a.ld;
+    if (a.h) {
+        for (int i = tid; i < a.K; i += 256) a.h[(size_t)m * a.K + i] = i < a.n ? gelu_tanh_exact(up[i]) : 0.f;
+        return;
+    }
+    auto eight = [&](int k, float (&v)[8]) __attribute__((always_inline)) {
+        const float4 p = *reinterpret_cast<const float4 *>(up + k), q = *reinterpret_cast<const float4 *>(up + k + 4);
+        v[0] = p.x; v[1] = p.y; v[2] = p.z; v[3] = p.w; v[4] = q.x; v[5] = q.y; v[6] = q.z; v[7] = q.w;
+#pragma unroll
+        for (int e = 0; e < 8; e++) v[e] = k + e < a.n ? gelu_tanh(v[e]) : 0.f;
+    };
+    float mx = 0.f;
+#pragma unroll 2
+    for (int k = tid * 8; k < a.K; k += 2048) {
+        float v[8];
+        eight(k, v);
+#pragma unroll
+        for (int e = 0; e < 8; e++) mx = fmaxf(mx, fabsf(v[e]));
+        if (staged) {
+            *reinterpret_cast<float4 *>(row + k) = make_float4(v[0], v[1], v[2], v[3]);
+            *reinterpret_cast<float4 *>(row + k + 4) = make_float4(v[4], v[5], v[6], v[7]);
+        }
+    }
+    const float s = row_scale_for(block_max(mx, sm));     // its barriers publish the row
+    const int Kb = tiled_kb(a.K);
+    if (staged) store_row_f16(row, a.K, a.a16, m, Kb, s);
+    else
+        for (int k = tid * 8; k < Kb * 64; k += 2048) {
+            float v[8] = {};
+            if (k < a.K) eight(k, v);
+            half8 h;
+#pragma unroll
+            for (int e = 0; e < 8; e++) h[e] = f2h(v[e] * s);
+            *reinterpret_cast<half8 *>(&a.a16[tiled_a_index(m, k, Kb)]) = h;
+        }
+    if (tid == 0) a.inv[m] = 1.f / s;
+}
+
+__global__ __launch_bounds__(256) void k_rope_table(float2 *tab, int n, int pairs, const double *__restrict__ freq)
+{
+    const int i = blockIdx.x * 256 + threadIdx.x;
+    if (i >= n) return;
+    const double angle = (double)(i / pairs) * freq[i % pairs];
+    tab[i] = make_float2((float)cos(angle), (float)sin(angle));
+}
+
 }  // namespace
+
+void launch_norms_around(const AroundRows &a, int rows) { LAUNCH(k_norms_around, dim3(rows), dim3(256), (size_t)a.Dp * 4, a); }
+
+void launch_gelu_rows(const ActRows &a, int rows)
+{
+    const size_t lds = (size_t)a.K * 4;
+    const int staged = !a.h && lds <= 60 * 1024;
+    LAUNCH(k_gelu_rows, dim3(rows), dim3(256), staged ? lds : 0, a, staged);
+}
+
+void launch_rope_table(float2 *tab, int max_seq, const std::vector<double> &freqs)
+{
+    const int pairs = (int)freqs.size(), n = max_seq * pairs;
+    if (n <= 0) return;
+    MetalBuf *f = metal_buf_from_data(freqs.data(), freqs.size() * sizeof(double));
+    LAUNCH(k_rope_table, dim3((n + 255) / 256), dim3(256), 0, tab, n, pairs, dptr_as<double>(f));
+    metal_buf_free(f);                                    // synchronises the stream first
+}
 
 void launch_embed_rows(const float *emb, const int *tok, float scale, float *x, int D, int Dp, int rows)
 {

@@ -21,6 +21,16 @@ __device__ __forceinline__ void store_row_f16(const float *row, int n, half_t *a
 __device__ __forceinline__ float softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 __device__ __forceinline__ float sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
 __device__ __forceinline__ float silu(float z) { return z / (1.f + expf(-z)); }
+// tanh form of GELU; the tanh as a quotient of exponentials, or as the library has it
+__device__ __forceinline__ float gelu_tanh(float z)
+{
+    const float in = 0.7978845608f * fmaf(0.044715f * z * z, z, z);
+    return z * __builtin_amdgcn_rcpf(1.f + __expf(-2.f * in));
+}
+__device__ __forceinline__ float gelu_tanh_exact(float z)
+{
+    return 0.5f * z * (1.f + tanhf(0.79788456080286536f * (z + 0.044715f * z * z * z)));
+}
 __device__ __forceinline__ float relu2(float z) { const float r = fmaxf(z, 0.f); return r * r; }
 
 // sum over the G lanes of an aligned group (G = 4, 8, 16 or 32), left in every one of them; cross-lane moves ride on

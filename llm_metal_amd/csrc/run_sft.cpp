@@ -44,7 +44,7 @@ void usage(const char *prog)
            "  --mode sft|generate   train (default), or emit greedy tokens after a prompt\n"
            "generate: --prompt <ids>  token ids with commas between them\n"
            "          --max-gen <n>   tokens to emit (default 64);  --max-seq <n>  positions to reserve\n"
-           "          --q8 | --f32    Q8_0 or 32-bit weights instead of F16 (32-bit: Nevurax models)\n", prog);
+           "          --q8 | --f32    Q8_0 or 32-bit weights instead of F16 (32-bit: Nevurax and Paposun models)\n", prog);
 }
 
 // which model the path holds, reported as the reference reports it (main.c:286-324)
@@ -127,7 +127,7 @@ int main(int argc, char **argv)
     if (o.seq_len <= 0 || o.batch <= 0 || o.max_steps < 0 || o.log_interval <= 0) { fprintf(stderr, "[SFT] Error: --seq, --batch, --log-interval must be positive\n"); return 2; }
     const float lr = o.lr > 0 ? o.lr : 1e-5f;
     const ModelType mtype = detect_model_type(o.model);
-    if (mtype == MODEL_NEVURAX) { fprintf(stderr, "[SFT] %s has no training path (--mode generate)\n", model_type_name(mtype)); return 2; }
+    if (model_type_layered(mtype)) { fprintf(stderr, "[SFT] %s has no training path (--mode generate)\n", model_type_name(mtype)); return 2; }
     printf("=== %s Fast %s SFT ===\n", model_type_name(mtype), o.full_param ? "Full-param SGD" : "LoRA");
     printf("  Model: %s\n", o.model.c_str());
     if (!o.full_param) printf("  LoRA rank: %d, alpha: %.1f\n", o.lora_rank, o.lora_alpha);

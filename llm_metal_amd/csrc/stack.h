@@ -1,6 +1,8 @@
 // A decoder described layer by layer: every layer names its mixer (gated delta rule with one decay per head or per key
-// channel, latent attention) and its feed-forward (mixture of experts, or none), both fed by one norm.  This header is
-// the configuration, the weights as the kernels read them, what a sequence keeps between steps, and the launches.
+// channel, latent attention, grouped attention inside chunks of positions, mLSTM) and its feed-forward (mixture of experts,
+// dense, or none).  Either one norm feeds both and their sum joins the residual, or each sublayer has a norm ahead of it
+// and another behind it.  This header is the configuration, the weights as the kernels read them, what a sequence keeps
+// between steps, and the launches.
 // The steps themselves are driven by the generation state (inference.hip) like those of the other models.
 #pragma once
 #include "backend.h"
@@ -14,28 +16,48 @@ namespace lmhip {
 
 // ---------------------------------------------------------------- configuration (config.json)
 
-enum MixerKind { MIX_DELTA, MIX_CHANNEL_DELTA, MIX_LATENT };
+enum MixerKind { MIX_DELTA, MIX_CHANNEL_DELTA, MIX_LATENT, MIX_GROUPED, MIX_MLSTM };
+// NORM_SHARED: one layer norm per layer, x += mixer(h) + ff(h).  NORMS_AROUND: RMS norms, x += m post(sublayer(pre(x))) twice.
+enum NormPlace { NORM_SHARED, NORMS_AROUND };
+
+// Rotary angles per position of `dims` / 2 pairs: base^(-2i / dims), with factor > 0 stretched for wavelengths above
+// original / low, kept below original / high, mixed in between.
+struct Rotation {
+    int dims = 0;
+    double base = 0.0, factor = 0.0, low = 0.0, high = 0.0, original = 0.0;
+    bool operator==(const Rotation &o) const
+    {
+        return dims == o.dims && base == o.base && factor == o.factor && low == o.low && high == o.high && original == o.original;
+    }
+    std::vector<double> frequencies() const;
+};
 
 struct LayerConfig {
     int mixer = MIX_DELTA;
     int heads = 0, dim = 0, vdim = 0;
     int kv_heads = 0, taps = 0;                          // delta rule
-    int rot_dim = 0, kv_rank = 0, window = 0, rot_dims = 0;   // latent attention; rot_dims: how many of the rot_dim turn
-    double rot_base = 0.0;
+    int rot_dim = 0, kv_rank = 0, window = 0;            // latent attention (rot.dims: how many of the rot_dim turn)
+    Rotation rot;                                        // both attentions
     float scale = 0.f;
+    int chunk = 0, kv_from = -1;                         // grouped attention: positions per chunk; layer whose keys and values are read (-1: own)
+    float gate_cap = 0.f;                                // mLSTM
+    int dense_ff = 0;                                    // dense feed-forward of this width
     int experts = 0, top = 0, ff = 0, shared_ff = 0;     // experts == 0: no feed-forward; shared_ff == 0: no shared expert
 };
 
 struct StackConfig {
     int vocab = 0, width = 0;
     float emb_scale = 1.f, eps = 0.f;
+    NormPlace norms = NORM_SHARED;
+    float residual_mult = 1.f, logit_scale = 1.f;        // NORMS_AROUND
+    bool tied = false;                                   // the head is the embedding table
     std::vector<LayerConfig> layers;
 };
 
 // config.json inside `path` when that is a directory, else next to it
 std::string config_path_of(const char *path);
 // false, with the reason in `why`, when the text is not a description this build can run
-bool read_stack_config(const std::string &json_text, StackConfig &out, std::string &why);
+bool read_stack_config(const std::string &json_text, ModelType type, StackConfig &out, std::string &why);
 
 // ---------------------------------------------------------------- weights
 
@@ -52,8 +74,13 @@ struct StackLayer {
     MetalBuf *g_norm = nullptr;                          // [width padded]
     // One product serves everything that reads the normed vector; each part starts at a multiple of four rows.
     //   delta: q | k | v | b | a (or a1) | g (or g1);  latent: q | dkv;  then router | shared up
+    //   grouped: q | k | v (its own only) | g;  mLSTM: q | k | v | g | i | f
     StackMat in;
-    int o_q = 0, o_k = 0, o_v = 0, o_b = 0, o_a = 0, o_g = 0, o_dkv = 0, o_router = 0, o_shared = 0;
+    int o_q = 0, o_k = 0, o_v = 0, o_b = 0, o_a = 0, o_g = 0, o_dkv = 0, o_router = 0, o_shared = 0, o_i = 0, o_f = 0;
+    MetalBuf *b_in = nullptr, *b_out = nullptr;          // fp32 biases of both products by output row (zeros where there is none)
+    // norms behind the sublayers and ahead of the feed-forward; those behind carry the residual's factor
+    MetalBuf *g_post = nullptr, *g_ff = nullptr, *g_ff_post = nullptr;
+    StackMat ff_up, ff_down;                             // dense feed-forward [pad8(ff), D], [Dp, ff]
     int rank_a = 0, rank_g = 0;                          // per-channel decay: widths of the two low-rank products
     // One product for everything added to the residual by the dense part: columns [mixer output | shared activation]
     StackMat out;
@@ -65,7 +92,7 @@ struct StackLayer {
     StackMat up, down;                                   // experts one after the other: [E * up_rows, width], [E * down_rows, ff]
     int up_rows = 0, down_rows = 0;                      // ff and width padded to the 32 rows of a tile
     int channels() const { return 2 * c.kv_heads * c.dim + c.heads * c.vdim; }
-    bool delta() const { return c.mixer != MIX_LATENT; }
+    bool delta() const { return c.mixer == MIX_DELTA || c.mixer == MIX_CHANNEL_DELTA; }
 };
 
 struct LayerStack {
@@ -98,8 +125,14 @@ struct StackRun {
     // per layer.  delta: state [B][heads][vdim][dim] and the last `taps` inputs of the convolutions [B][taps][channels];
     // latent: ring of (latent | rotated key) rows [B][ring][row width].  Row of position p: p % taps, p % ring.
     // Nothing is cleared between sequences: what lies before position 0 is never read.
-    struct Layer { MetalBuf *S = nullptr, *conv = nullptr, *ring = nullptr; int ring_rows = 0; };
+    // grouped: rings of rotated keys [B][kv_heads][ring][dim padded to 4] and of values; a layer that reads another's has
+    // none.  mLSTM: S [B][heads][vdim][dim padded to 4] and, in two slots that alternate with the parity of the position,
+    // the normaliser [2][B][heads][dim padded] and the running maximum [2][B][heads].
+    struct Layer { MetalBuf *S = nullptr, *conv = nullptr, *ring = nullptr, *vring = nullptr, *n = nullptr, *m = nullptr; int ring_rows = 0; };
     std::vector<Layer> layers;
+    MetalBuf *x2 = nullptr;                              // the residual's other place (fused steps of NORMS_AROUND)
+    float *xr = nullptr;                                 // where the fused steps left it
+    const float *post_g = nullptr, *post_b = nullptr;    // NORMS_AROUND: norm weight and bias of the sum that waits in cout
     MetalBuf *tok = nullptr, *want = nullptr;
     int *tok_host = nullptr, *want_host = nullptr;       // pinned; tok_host [B * max_seq], each portion in its own place
     MetalBuf *x = nullptr, *h = nullptr, *cin = nullptr, *cat = nullptr, *cout = nullptr;
@@ -146,6 +179,18 @@ struct NormRows {
     const float *moe_y, *route_w; const int *moe_pos; int top;
 };
 void launch_norm_rows(const NormRows &a, int rows);
+// The same where norms lie around the sublayers: y = cout + post_b, x += y / rms(y) * post_g (cout null: x as it is), kept
+// in x when `keep`; then RMS norm with weight g.
+struct AroundRows {
+    float *x; const float *cout, *post_b, *post_g;
+    const float *g; half_t *a16; float *inv, *h;
+    const int *want;
+    int step, first, D, Dp, keep; float eps;
+};
+void launch_norms_around(const AroundRows &a, int rows);
+// tanh-GELU of up rows [rows][ld] (n columns, the rest of K zero) as the operand a16 with inv, or (exact) as fp32 h [rows][K]
+struct ActRows { const float *up; int ld, n, K; half_t *a16; float *inv, *h; };
+void launch_gelu_rows(const ActRows &a, int rows);
 void launch_embed_rows(const float *emb, const int *tok, float scale, float *x, int D, int Dp, int rows);
 constexpr int STACK_FEW = 32;
 void launch_embed_few(const float *emb, const int *tok, float scale, float *x, int D, int Dp, int rows);   // tok: host array of at most STACK_FEW
@@ -175,7 +220,8 @@ void launch_delta_scan(const DeltaRows &a);              // the recurrence; also
 // up product, as fp32 cat [rows][ldk] and / or as a16 with inv
 struct CatRows {
     const float *o; int H, vdim;                         // mixer output [rows][H * vdim]
-    const float *g_out, *gate; int ld_gate, gate_silu; float eps;   // head norm weight, gate rows (silu or sigmoid)
+    const float *g_out, *gate; int ld_gate, gate_silu; float eps;   // head norm weight (either may be null), gate rows (silu or sigmoid)
+    int g_stride;                                        // from one head's norm weight to the next (0: one for all)
     const float *shared; int ld_shared, shared_ff, o_sh; // shared up rows
     float *cat; half_t *a16; float *inv; int ldk;
 };
@@ -210,7 +256,45 @@ size_t latent_prompt_frag_halfs(const LatentRows &a, int B, int n_keys);
 void launch_latent_operand(const LatentRows &a, half_t *a16, float *inv);        // the visible latents as a product's operand
 void launch_latent_prompt(const LatentRows &a, const float *kv, half_t *frags);
 
-void launch_rope_interleaved(float2 *tab, int max_seq, int dims, double base);
+// group_attn.hip: queries of H heads over G heads of keys; position i sees the positions of its chunk up to itself
+struct GroupRows {
+    Rows r;
+    int H, G, dim, vdim, chunk, ring_rows, rot_dims, own; // own: this layer writes the rings
+    float scale;
+    const float *cin, *bias; int ldc, o_q, o_k, o_v, o_g; // the input product and its biases
+    const float2 *rope;
+    float *kring, *vring;
+    float *part_o, *part_ml;                             // slices (scratch of the launch)
+    float *o;                                            // [rows][H * vdim]
+    int gated;                                           // single-token steps: o times sigmoid of the gate
+};
+void launch_group_cache(const GroupRows &a);             // rotated keys and values into the rings
+void launch_group_attend(const GroupRows &a);            // any number of rows in fp32; a step of one token also writes the rings
+// group_prompt.hip: many rows in 16-bit precision on the matrix cores, over the rings
+bool group_prompt_fits(const GroupRows &a);
+inline int group_prompt_first(const GroupRows &a) { return a.r.pos / a.chunk * a.chunk; }
+size_t group_prompt_frag_halfs(const GroupRows &a, int B, int n_keys);
+void launch_group_prompt(const GroupRows &a, half_t *frags);
+
+// mlstm.hip
+constexpr int MLSTM_CHUNK = 64;
+struct MlstmRows {
+    Rows r;
+    int H, dim, vdim; float cap;
+    const float *cin, *bias; int ldc, o_q, o_k, o_v, o_g, o_i, o_f;
+    float *S, *n, *m;                                    // state
+    // prompts: per (sequence, head) and token the parts of the gates, per chunk its decay, the state ahead of it (with the
+    // normaliser as a further row) and the pair products
+    float2 *u, *w; float *cf, *wk, *em, *qf, *gk, *Sc, *P;
+    float *o;                                            // [rows][H * vdim]
+    float *gate;                                         // single-token steps: the output gate as a factor, when wanted
+};
+inline int mlstm_chunks(int T) { return (T + MLSTM_CHUNK - 1) / MLSTM_CHUNK; }
+inline int pad4(int n) { return (n + 3) & ~3; }
+void launch_mlstm(const MlstmRows &a);
+
+// norm.hip: (cos, sin) of position * frequency, [max_seq][frequencies]
+void launch_rope_table(float2 *tab, int max_seq, const std::vector<double> &freqs);
 
 // moe.hip
 struct MoeRows {

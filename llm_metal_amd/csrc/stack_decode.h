@@ -21,7 +21,7 @@ struct DecodeDelta {
 
 struct DecodeOut {
     CatRows cat;                                         // gate: factors as k_delta_decode leaves them
-    const half_t *out; float *x; int D;
+    const half_t *out; float *x, *y; int D;               // y: the sum goes there instead of onto x
 };
 
 constexpr size_t DECODE_LDS = 152 * 1024;

@@ -161,8 +161,8 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentRows a, DecodeMoe e
     else experts_up(e, blockIdx.x - a.H - 1, lds);
 }
 
-// x[d] += out[d] . (mixer output | shared activation) + sum over the chosen experts of w * down_e[d] . act_e; a wave takes
-// PER values of d.  lds: [ldk] then [top * ffp]
+// x[d] += out[d] . (mixer output | shared activation) + sum over the chosen experts of w * down_e[d] . act_e (or y[d] = the
+// sum, when a norm lies behind it); a wave takes PER values of d.  lds: [ldk] then [top * ffp]
 template <int TPB, int PER>
 __global__ __launch_bounds__(TPB) void k_out_decode(DecodeOut a, DecodeMoe e)
 {
@@ -179,7 +179,7 @@ __global__ __launch_bounds__(TPB) void k_out_decode(DecodeOut a, DecodeMoe e)
             float ss = 0.f;
             for (int d = lane; d < c.vdim; d += 64) ss += o[d] * o[d];
             const float inv = 1.f / sqrtf(wave_total(ss) / (float)c.vdim + c.eps);
-            for (int d = lane; d < c.vdim; d += 64) cat[h * c.vdim + d] = o[d] * inv * c.g_out[d] * gt[d];
+            for (int d = lane; d < c.vdim; d += 64) cat[h * c.vdim + d] = o[d] * inv * c.g_out[h * c.g_stride + d] * gt[d];
         }
     } else
         for (int i = tid; i < c.H * c.vdim; i += TPB) cat[i] = c.o[i];
@@ -220,7 +220,7 @@ __global__ __launch_bounds__(TPB) void k_out_decode(DecodeOut a, DecodeMoe e)
 #pragma unroll
     for (int k = 0; k < PER; k++) {
         const float t = wave_total(y[k]);
-        if (lane == 0 && d0 + k < a.D) a.x[d0 + k] += t;
+        if (lane == 0 && d0 + k < a.D) { if (a.y) a.y[d0 + k] = t; else a.x[d0 + k] += t; }
     }
 }
 

@@ -153,7 +153,7 @@ def load():
         "inference_forward_token_argmax": (i, [vp, i]), "inference_state_set_lora": (None, [vp, vp]),
         "inference_state_set_eos": (None, [vp, vp, i]), "inference_state_load_eos": (None, [vp, C.c_char_p]),
         "inference_state_position": (i, [vp]), "inference_forward_tokens": (i, [vp, vp, i, vp, i, vp]),
-        "model_type_detect": (i, [C.c_char_p]), "model_type_name": (C.c_char_p, [i]),
+        "model_type_detect": (i, [C.c_char_p]), "model_type_layered": (i, [i]), "model_type_name": (C.c_char_p, [i]),
         "inference_state_create_from_file": (vp, [C.c_char_p, i, i, i]),
         "model_file_open": (vp, [C.c_char_p]), "model_file_close": (None, [vp]), "model_file_is_gguf": (i, [vp]),
         "model_file_count": (i, [vp]), "model_file_name": (C.c_char_p, [vp, i]),

@@ -1,11 +1,14 @@
-"""Plain restatement, in numpy and one token at a time, of a decoder whose layers are listed one by one (Nevurax):
-short causal convolutions, the gated delta rule with one decay per head or per key channel, latent attention with a
-sliding window and interleaved rotation, squared-ReLU experts behind a softmax router, one layer norm per layer whose
-output both sublayers read.  Test infrastructure only: nothing here is used by the package, and nothing of the package
-is used here.  Everything runs in the dtype of the weights handed in (float64 for pinning).
+"""Plain restatement, in numpy and one token at a time, of decoders whose layers are listed one by one.
 
-A model is a config dictionary (vocab, width, embedding.scale, norm.eps, layers[]: type, mixer, mlp) and a dictionary of
-numpy arrays by tensor name.
+Nevurax: short causal convolutions, the gated delta rule with one decay per head or per key channel, latent attention with
+a sliding window and interleaved rotation, squared-ReLU experts behind a softmax router, one layer norm per layer whose
+output both sublayers read.  Paposun: grouped attention inside fixed chunks of positions with biases, half-split rotation
+of scaled frequencies, an output gate and keys that later layers may share, the mLSTM matrix memory, a dense tanh-GELU
+feed-forward, RMS norms before and after each sublayer.
+
+Test infrastructure only: nothing here is used by the package, and nothing of the package is used here.  Everything runs in
+the dtype of the weights handed in (float64 for pinning).  A model is a config dictionary (its config.json) and a
+dictionary of numpy arrays by tensor name.
 """
 import numpy as np
 
@@ -27,6 +30,10 @@ def softplus(z):
 def relu2(z):
     r = np.maximum(z, 0.0)
     return r * r
+
+
+def gelu_tanh(z):
+    return 0.5 * z * (1.0 + np.tanh(np.sqrt(2.0 / np.pi) * (z + 0.044715 * z ** 3)))
 
 
 # ---------------------------------------------------------------- norms and rotation
@@ -52,6 +59,32 @@ def rotate_interleaved(x, pos, dims, base):
         c, s = np.cos(a), np.sin(a)
         u, v = x[2 * i], x[2 * i + 1]
         y[2 * i], y[2 * i + 1] = u * c - v * s, v * c + u * s
+    return y
+
+
+def scaled_frequencies(rot):
+    """Angles per position of the pairs.  Wavelengths above original / low are stretched by `factor`, those below
+    original / high are kept, a linear mix in between."""
+    out, sc = [], rot.get("scaling")
+    for i in range(rot["dims"] // 2):
+        f = float(rot["base"]) ** (-2.0 * i / rot["dims"])
+        if sc:
+            turns = sc["original"] * f / (2.0 * np.pi)          # turns within the original context
+            if turns < sc["low"]:
+                f = f / sc["factor"]
+            elif turns <= sc["high"]:
+                mix = (turns - sc["low"]) / (sc["high"] - sc["low"])
+                f = (1.0 - mix) * f / sc["factor"] + mix * f
+        out.append(f)
+    return out
+
+
+def rotate_halves(x, pos, rot):
+    """Entry i turned together with entry i + dims / 2, i < dims / 2."""
+    y, n = x.copy(), rot["dims"] // 2
+    for i, f in enumerate(scaled_frequencies(rot)):
+        c, s = np.cos(pos * f), np.sin(pos * f)
+        y[i], y[i + n] = x[i] * c - x[i + n] * s, x[i + n] * c + x[i] * s
     return y
 
 
@@ -122,6 +155,54 @@ def latent_attention(W, p, mx, eps, state, h, pos):
     return W[p + "o"] @ out.reshape(-1)
 
 
+def linear(W, name, h):
+    return W[name] @ h + W[name + ".b"]
+
+
+def chunk_attention(W, p, mx, state, cache, h, pos):
+    """`cache`: state of the layer whose keys and values are read (its own, or an earlier layer's)."""
+    H, G, d, dv = mx["heads"], mx["kv_heads"], mx["dim"], mx["vdim"]
+    q = linear(W, p + "q", h).reshape(H, d)
+    if cache is state:
+        ks, vs = state.setdefault("k", []), state.setdefault("v", [])
+        ks.append(np.stack([rotate_halves(r, pos, mx["rot"]) for r in linear(W, p + "k", h).reshape(G, d)]))
+        vs.append(linear(W, p + "v", h).reshape(G, dv))
+    first = pos // mx["mask"]["size"] * mx["mask"]["size"]
+    k, v = np.stack(cache["k"][first:pos + 1]), np.stack(cache["v"][first:pos + 1])
+    out = np.zeros((H, dv), dtype=h.dtype)
+    for i in range(H):
+        g = i // (H // G)
+        s = k[:, g] @ rotate_halves(q[i], pos, mx["rot"]) * mx["scale"]
+        w = np.exp(s - s.max())
+        out[i] = (w / w.sum()) @ v[:, g]
+    return linear(W, p + "o", out.reshape(-1) * sigmoid(W[p + "g"] @ h))
+
+
+def mlstm_step(S, n, m, q, k, v, i, f):
+    """One head, one token; i, f: logarithms of the gates.  Returns S [dim, vdim], n, m and the output."""
+    new = max(f + m, i)
+    keep, write = np.exp(f + m - new), np.exp(i - new)
+    S = keep * S + write * np.outer(k, v)
+    n = keep * n + write * k
+    return S, n, new, S.T @ q / (max(abs(n @ q), np.exp(-new)) + 1e-6)
+
+
+def mlstm_mixer(W, p, mx, eps, state, h):
+    H, d, dv, cap = mx["heads"], mx["dim"], mx["vdim"], mx["gate_cap"]
+    q = (W[p + "q"] @ h).reshape(H, d) * d ** -0.5
+    k, v = (W[p + "k"] @ h).reshape(H, d), (W[p + "v"] @ h).reshape(H, dv)
+    i = cap * np.tanh(linear(W, p + "i", h) / cap)
+    f = -softplus(-cap * np.tanh(linear(W, p + "f", h) / cap))
+    heads = state.setdefault("heads", [(np.zeros((d, dv), h.dtype), np.zeros(d, h.dtype), 0.0)] * H)
+    new, out = [], np.zeros((H, dv), h.dtype)
+    for x in range(H):
+        S, n, m, out[x] = mlstm_step(*heads[x], q[x], k[x], v[x], i[x], f[x])
+        new.append((S, n, m))
+        out[x] = rms_norm(out[x], 1.0, eps)
+    state["heads"] = new
+    return W[p + "o"] @ (out.reshape(-1) * W[p + "norm"] * sigmoid(W[p + "g"] @ h))
+
+
 # ---------------------------------------------------------------- feed-forward
 
 def expert(W, p, h):
@@ -157,6 +238,10 @@ def copy_state(state):
 
 def step(cfg, W, state, token, trace=None):
     """One token through every layer; returns the logits.  `trace`: list that receives x after each layer."""
+    return (step_norms_around if cfg["architecture"] == "Paposun" else step_one_norm)(cfg, W, state, token, trace)
+
+
+def step_one_norm(cfg, W, state, token, trace):
     eps, pos = cfg["norm"]["eps"], state["pos"]
     x = W["embed"][token] * cfg["embedding"]["scale"]
     for i, L in enumerate(cfg["layers"]):
@@ -174,6 +259,27 @@ def step(cfg, W, state, token, trace=None):
             trace.append(x.copy())
     state["pos"] = pos + 1
     return W["head"] @ layer_norm(x, W["final.norm"], eps)
+
+
+def step_norms_around(cfg, W, state, token, trace):
+    eps, pos, r = cfg["norm"]["eps"], state["pos"], cfg["residual_mult"]
+    x = W["embed"][token]
+    for i, L in enumerate(cfg["layers"]):
+        p = f"l{i}."
+        h = rms_norm(x, W[p + "norm1"], eps)
+        st, mx = state["layers"][i], L["mixer"]
+        if L["type"] == "attention":
+            y = chunk_attention(W, p + "mix.", mx, st, state["layers"][mx["kv_from"]] if mx.get("kv_from") is not None else st, h, pos)
+        else:
+            y = mlstm_mixer(W, p + "mix.", mx, eps, st, h)
+        x = x + r * rms_norm(y, W[p + "norm1b"], eps)
+        if L.get("mlp"):
+            y = W[p + "mlp.down"] @ gelu_tanh(W[p + "mlp.up"] @ rms_norm(x, W[p + "norm2"], eps))
+            x = x + r * rms_norm(y, W[p + "norm2b"], eps)
+        if trace is not None:
+            trace.append(x.copy())
+    state["pos"] = pos + 1
+    return W["embed"] @ rms_norm(x, W["final.norm"], eps) * cfg["logit_scale"]
 
 
 def run(cfg, W, tokens, state=None):
