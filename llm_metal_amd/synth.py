@@ -118,11 +118,13 @@ def make_batch(c: SFTConfig, seed=1):
     return tok.reshape(-1).copy(), tgt.reshape(-1).copy()
 
 
-# ---------------------------------------------------------------- models described layer by layer (Nevurax)
+# ---------------------------------------------------------------- models described layer by layer (Nevurax, Paposun)
 
 def stack_shapes(cfg, rank_a=16, rank_g=16):
     """Tensor names and shapes of a layer-by-layer model; cfg is the dictionary that becomes its config.json.  rank_a and
     rank_g: widths of the two low-rank products of a per-channel decay (tensor shapes, not configuration)."""
+    if cfg["architecture"] == "Paposun":
+        return around_shapes(cfg)
     D = cfg["width"]
     out = {"embed": (cfg["vocab"], D)}
     for i, L in enumerate(cfg["layers"]):
@@ -156,12 +158,43 @@ def stack_shapes(cfg, rank_a=16, rank_g=16):
     return out
 
 
+def around_shapes(cfg):
+    """The same for norms around the sublayers: grouped attention with biases, mLSTM, dense feed-forward, tied head."""
+    D = cfg["width"]
+    out = {"embed": (cfg["vocab"], D)}
+    for i, L in enumerate(cfg["layers"]):
+        m, p = L["mixer"], f"l{i}."
+        H, d, dv, x = m["heads"], m["dim"], m["vdim"], p + "mix."
+        out.update({p + "norm1": (D,), p + "norm1b": (D,)})
+
+        def biased(name, rows):
+            out.update({x + name: (rows, D), x + name + ".b": (rows,)})
+        if L["type"] == "attention":
+            biased("q", H * d)
+            if m.get("kv_from") is None:
+                biased("k", m["kv_heads"] * d)
+                biased("v", m["kv_heads"] * dv)
+            out.update({x + "g": (H * dv, D), x + "o": (D, H * dv), x + "o.b": (D,)})
+        else:
+            out.update({x + "q": (H * d, D), x + "k": (H * d, D), x + "v": (H * dv, D), x + "g": (H * dv, D), x + "o": (D, H * dv), x + "norm": (H * dv,)})
+            biased("i", H)
+            biased("f", H)
+        if L.get("mlp"):
+            out.update({p + "norm2": (D,), p + "norm2b": (D,), p + "mlp.up": (L["mlp"]["ff"], D), p + "mlp.down": (D, L["mlp"]["ff"])})
+    out["final.norm"] = (D,)
+    return out
+
+
 def make_stack_tensor(name, shape, rng):
     """Matrices ~ N(0, 1 / columns) (down and output projections half of that), norms around 1, filters and decay
-    parameters spread so that states remember from a few tokens to a few hundred."""
+    parameters and gate biases spread so that states remember from a few tokens to a few hundred, other biases small."""
     leaf = name.rsplit(".", 1)[-1]
-    if leaf in ("norm", "norm1"):
+    if leaf in ("norm", "norm1", "norm1b", "norm2", "norm2b"):
         return (1.0 + 0.1 * rng.standard_normal(shape)).astype(np.float32)
+    if leaf == "b" and len(shape) == 1:
+        if name.endswith(".f.b"):
+            return rng.uniform(1.0, 6.0, shape).astype(np.float32)
+        return (0.3 * rng.standard_normal(shape)).astype(np.float32)
     if leaf == "conv":
         return (rng.standard_normal(shape) / np.sqrt(shape[1])).astype(np.float32)
     if leaf == "A_log":

@@ -1,4 +1,4 @@
-"""Models described layer by layer (Nevurax) on the GPU through the generation API, against the plain numpy restatement in
+"""Models described layer by layer (Nevurax, Paposun) on the GPU through the generation API, against the plain numpy restatement in
 oracle/stack_oracle.py: every mechanism alone, prompts against decoding, portions, batches, reused states, window edges,
 rings that wrap, greedy generation, the command line and the trace runner."""
 import json
@@ -18,6 +18,7 @@ from tests.stack_models import MODELS, Model, config, channel, delta, latent, lo
 pytestmark = pytest.mark.gpu
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 TOL = {"f32": 2e-5, "f16": 4e-3}
+MIXED = pytest.mark.parametrize("mixed", ["mixed", "norms around, mixed"])
 
 
 def say(*a):
@@ -55,11 +56,12 @@ def test_prompt_and_decoding_match_the_oracle(name, fmt, tmp_path):
         assert logit_error(single, want) < TOL[fmt]
 
 
+@MIXED
 @pytest.mark.parametrize("fmt", ["f32", "f16"])
 @pytest.mark.parametrize("sizes", [[2], [3, 2, 5, 7, 2, 11], [40, 1, 1, 1, 20, 2], [1, 33, 16, 17], [64, 2, 1], [5, 70]])
-def test_portions_of_any_size(sizes, fmt, tmp_path):
-    say("portions", sizes, fmt)
-    cfg, ra, rg = MODELS["mixed"]
+def test_portions_of_any_size(sizes, fmt, mixed, tmp_path):
+    say("portions", mixed, sizes, fmt)
+    cfg, ra, rg = MODELS[mixed]
     m = Model(cfg, tmp_path, ra, rg)
     toks = m.tokens(90, seed=2)
     want = so.run(cfg, m.W, toks)
@@ -67,9 +69,10 @@ def test_portions_of_any_size(sizes, fmt, tmp_path):
         assert logit_error(run_portions(inf, toks, sizes), want) < TOL[fmt]
 
 
+@MIXED
 @pytest.mark.parametrize("fmt", ["f32", "f16"])
-def test_first_tokens_and_a_sequence_of_one(fmt, tmp_path):
-    cfg, ra, rg = MODELS["mixed"]
+def test_first_tokens_and_a_sequence_of_one(fmt, mixed, tmp_path):
+    cfg, ra, rg = MODELS[mixed]
     m = Model(cfg, tmp_path, ra, rg)
     with state(m, fmt) as inf:
         for n in (1, 2, 3, 4, 5):
@@ -78,9 +81,10 @@ def test_first_tokens_and_a_sequence_of_one(fmt, tmp_path):
             assert logit_error(inf.forward_tokens(toks, range(n)), so.run(cfg, m.W, toks)) < TOL[fmt]
 
 
-def test_states_are_used_again(tmp_path):
+@MIXED
+def test_states_are_used_again(mixed, tmp_path):
     """A second sequence in the same state sees nothing of the first, whatever its length: bit-identical to a fresh state."""
-    cfg, ra, rg = MODELS["mixed"]
+    cfg, ra, rg = MODELS[mixed]
     m = Model(cfg, tmp_path, ra, rg)
     prompts = [m.tokens(n, seed=n) for n in (60, 3, 1, 41, 2)]
     for fmt in ("f32", "f16"):
@@ -92,9 +96,10 @@ def test_states_are_used_again(tmp_path):
                     assert np.array_equal(got, run_portions(fresh, p, [17, 2, 1]))
 
 
+@MIXED
 @pytest.mark.parametrize("fmt", ["f32", "f16"])
-def test_lock_step_batches_against_each_alone(fmt, tmp_path):
-    cfg, ra, rg = MODELS["mixed"]
+def test_lock_step_batches_against_each_alone(fmt, mixed, tmp_path):
+    cfg, ra, rg = MODELS[mixed]
     m = Model(cfg, tmp_path, ra, rg)
     seqs = np.array([m.tokens(45, seed=50 + b) for b in range(5)])
     want = np.stack([so.run(cfg, m.W, s) for s in seqs])
@@ -193,11 +198,23 @@ def test_strong_decays_and_large_gates(tmp_path):
             assert logit_error(run_portions(inf, toks, [70, 2, 1]), want) < TOL[fmt]
 
 
-def test_greedy_generation_everywhere(tmp_path):
-    cfg, ra, rg = MODELS["mixed"]
-    m = Model(cfg, tmp_path, ra, rg)
-    prompt = m.tokens(23, seed=8)
+def moving_model(path):
+    """A tied head repeats its token: alternating signs on the final norm and larger sublayers make the sequence move."""
+    cfg = dict(MODELS["norms around, mixed"][0], residual_mult=1.7)
+    return Model(cfg, path, edit=lambda n, a: a * np.where(np.arange(a.size) % 2, 1, -1).astype(np.float32) if n == "final.norm" else a)
+
+
+@MIXED
+def test_greedy_generation_everywhere(mixed, tmp_path):
+    cfg, ra, rg = MODELS[mixed]
+    if mixed == "mixed":
+        m = Model(cfg, tmp_path, ra, rg)
+    else:
+        m = moving_model(tmp_path)
+        cfg = m.cfg
+    prompt = m.tokens(23, seed=8 if mixed == "mixed" else 10)
     want = so.generate(cfg, m.W, prompt, 40)
+    assert len(set(want)) >= 10
     logits = np.sort(so.run(cfg, m.W, prompt + want[:-1])[len(prompt) - 1:], axis=1)
     assert (logits[:, -1] - logits[:, -2]).min() > 10 * TOL["f32"] * logits.std()     # no close call in this sequence
     with state(m, "f32") as inf:
@@ -222,9 +239,10 @@ def test_greedy_generation_everywhere(tmp_path):
     assert [int(x) for x in line.split(":")[1].split()] == want
 
 
+@MIXED
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_trace_runner(dtype, tmp_path):
-    cfg, ra, rg = MODELS["mixed, odd"]
+def test_trace_runner(dtype, mixed, tmp_path):
+    cfg, ra, rg = MODELS[mixed + ", odd"]
     m = Model(cfg, tmp_path / "model", ra, rg)
     reqs = {"a": m.tokens(37, seed=1), "b": m.tokens(5, seed=2)}
     steps = [("a", 0, 20, [0, 19]), ("a", 20, 22, []), ("a", 22, 23, [0]), ("a", 23, 37, [13, 2]), ("b", 0, 4, [3]), ("b", 4, 5, [0])]
