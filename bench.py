@@ -215,18 +215,18 @@ def decode_bench(args, cfg, L):
     emit(out)
 
 
-def nevurax_bench(args, L):
-    """Prompt and decoding throughput of Nevurax models (random weights), each beside the Qwen3 shape of the same width: its
-    greedy decoding, and as its many-row pass the training state's forward over as many rows (generation takes Qwen3 prompts
-    token by token).  One JSON line for all sizes."""
+def layered_bench(args, L, design, sizes, names):
+    """Prompt and decoding throughput of models that are described layer by layer (random weights), each beside the Qwen3 shape
+    of the same width: its greedy decoding, and as its many-row pass the training state's forward over as many rows (generation
+    takes Qwen3 prompts token by token).  One JSON line for all sizes."""
     import tempfile
-    from llm_metal_amd.configs import NEVURAX_SIZES, qwen3_beside
+    from llm_metal_amd.configs import qwen3_beside
     from llm_metal_amd.sft import InferenceState, SFTState
     from llm_metal_amd.synth import write_stack_checkpoint
-    rows, rng = args.nevurax_prompt, np.random.default_rng(5)
+    rows, rng = args.layered_prompt, np.random.default_rng(5)
     out = []
-    for size in args.nevurax.split(","):
-        cfg = NEVURAX_SIZES[size]
+    for size in names.split(","):
+        cfg = sizes[size]
         toks = rng.integers(0, cfg["vocab"], rows)
 
         def decode_ms(inf, tok):
@@ -253,11 +253,11 @@ def nevurax_bench(args, L):
         res["decode_ms"] = round(decode_ms(inf, 1), 4)
         res["decode_tokens_per_s"] = round(1e3 / res["decode_ms"], 1)
         inf.free()
-        if not args.nevurax_alone:
+        if not args.layered_alone:
             q = qwen3_beside(cfg)
             model = make_model(q, seed=0, lora_b_std=0.0)
             inf = InferenceState(q, model, max_seq=max_seq)
-            for t in toks[:args.nevurax_context]:
+            for t in toks[:args.layered_context]:
                 tok = inf.forward_token_argmax(int(t))
             ref = {"ffn_width": q.IS, "decode_ms": round(decode_ms(inf, tok), 4)}
             inf.free()
@@ -274,7 +274,7 @@ def nevurax_bench(args, L):
             del model
             res["qwen3"] = ref
         out.append(res)
-    emit({"metric": "Nevurax prompt and greedy decode tokens/s", "unit": "tokens/s", "n_gpus": 1, "data": "synthetic", "steps": args.steps,
+    emit({"metric": f"{design} prompt and greedy decode tokens/s", "unit": "tokens/s", "n_gpus": 1, "data": "synthetic", "steps": args.steps,
           "dtype": "f16 weights, f32 accumulate", "sizes": out})
 
 
@@ -351,9 +351,11 @@ def _main():
                     help="with --decode: also time this many copies of one prompt decoded in lock step")
     ap.add_argument("--nevurax", nargs="?", const="1k,2k,4k", default=None, metavar="SIZES",
                     help="time prompts and decoding of Nevurax models of these sizes (1k,2k,4k) beside a Qwen3 shape of equal size")
-    ap.add_argument("--nevurax-prompt", type=int, default=2048, help="with --nevurax: tokens of the prompt")
-    ap.add_argument("--nevurax-context", type=int, default=256, help="with --nevurax: tokens before the Qwen3 shape's timed decoding")
-    ap.add_argument("--nevurax-alone", action="store_true", help="with --nevurax: without the Qwen3 shape")
+    ap.add_argument("--paposun", nargs="?", const="1k,2k,4k", default=None, metavar="SIZES", help="the same for Paposun models")
+    ap.add_argument("--layered-prompt", "--nevurax-prompt", type=int, default=2048, help="with --nevurax / --paposun: tokens of the prompt")
+    ap.add_argument("--layered-context", "--nevurax-context", type=int, default=256,
+                    help="with --nevurax / --paposun: tokens before the Qwen3 shape's timed decoding")
+    ap.add_argument("--layered-alone", "--nevurax-alone", action="store_true", help="with --nevurax / --paposun: without the Qwen3 shape")
     ap.add_argument("--gemm-shapes", action="store_true",
                     help="time every product shape of the configuration alone, with cold weights: the weight loads only, gemm_ring, gemm_tiled")
     ap.add_argument("--copy-calibration", action="store_true",
@@ -361,9 +363,9 @@ def _main():
                          "the known-size reference for scaling FETCH_SIZE / WRITE_SIZE counters")
     args = ap.parse_args()
     if args.steps is None:
-        args.steps = 20 if args.decode or args.nevurax else 200
+        args.steps = 20 if args.decode or args.nevurax or args.paposun else 200
     if args.warmup is None:
-        args.warmup = 3 if args.decode or args.nevurax else 20
+        args.warmup = 3 if args.decode or args.nevurax or args.paposun else 20
     if args.gpus != 1:
         print("bench.py: this build runs on one GPU only (the step has no multi-GPU path); use --gpus 1",
               file=sys.stderr)
@@ -391,8 +393,11 @@ def _main():
                                    "bytes_written_per_launch": 4 * n, "launches": 5}})
         return
 
-    if args.nevurax:
-        return nevurax_bench(args, L)
+    if args.nevurax or args.paposun:
+        from llm_metal_amd.configs import NEVURAX_SIZES, PAPOSUN_SIZES
+        if args.nevurax:
+            return layered_bench(args, L, "Nevurax", NEVURAX_SIZES, args.nevurax)
+        return layered_bench(args, L, "Paposun", PAPOSUN_SIZES, args.paposun)
     if args.decode:
         return decode_bench(args, cfg, L)
     if args.gemm_shapes:

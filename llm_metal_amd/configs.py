@@ -99,10 +99,32 @@ NEVURAX_SIZES = {
 }
 
 
+def paposun_config(width, heads, ff, memory_heads, memory_dim, vocab=32768, head_dim=128, chunk=1024):
+    """config.json of a Paposun model with layers of a real model's proportions: attention, attention on the same keys, mLSTM
+    (values twice as wide as keys, as wide together as the model), attention."""
+    def attention(**kw):
+        return {"type": "attention", "mlp": {"kind": "dense", "ff": ff},
+                "mixer": {"heads": heads, "kv_heads": max(1, heads // 4), "dim": head_dim, "vdim": head_dim, "mask": {"size": chunk}, "scale": head_dim ** -0.5,
+                          "rot": {"base": 5e5, "dims": head_dim, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}, **kw}}
+    memory = {"type": "mlstm", "mlp": None, "mixer": {"heads": memory_heads, "dim": memory_dim, "vdim": 2 * memory_dim, "gate_cap": 15.0}}
+    return {"architecture": "Paposun", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "residual_mult": 0.5, "logit_scale": 0.25,
+            "layers": [attention(), attention(kv_from=0), memory, attention()]}
+
+
+PAPOSUN_SIZES = {
+    "1k": paposun_config(1024, 8, 4096, 4, 128),
+    "2k": paposun_config(2048, 16, 8192, 4, 256),
+    "4k": paposun_config(4096, 32, 16384, 8, 256),
+}
+
+
 def qwen3_beside(cfg):
-    """The Qwen3 shape with a Nevurax configuration's width, layers, heads and feed-forward weights per token."""
-    L = cfg["layers"][0]["mlp"]
-    active = 2 * (L["router"]["top"] * L["expert"]["ff"] + L["shared"]["ff"])
-    heads = cfg["layers"][0]["mixer"]["heads"]
-    return SFTConfig("qwen3_beside_nevurax", QWEN3, NL=len(cfg["layers"]), D=cfg["width"], Hq=heads, Hkv=max(1, heads // 4),
-                     hd=cfg["layers"][0]["mixer"]["dim"], IS=active // 3 // 64 * 64, V=cfg["vocab"])
+    """The Qwen3 shape with a layer-by-layer configuration's width, layers, heads and feed-forward weights per token."""
+    active = 0
+    for L in cfg["layers"]:
+        m = L["mlp"]
+        if m:
+            active += 2 * (m["ff"] if m["kind"] == "dense" else m["router"]["top"] * m["expert"]["ff"] + m["shared"]["ff"])
+    NL, mx = len(cfg["layers"]), cfg["layers"][0]["mixer"]
+    return SFTConfig("qwen3_beside_layered", QWEN3, NL=NL, D=cfg["width"], Hq=mx["heads"], Hkv=max(1, mx["heads"] // 4),
+                     hd=mx["dim"], IS=active // NL // 3 // 64 * 64, V=cfg["vocab"])

@@ -2,6 +2,7 @@
 // Everything here is fp32, the matrix instructions of the recurrence included.
 #include "stack.h"
 #include "delta_rows.h"
+#include "planes.h"
 
 namespace lmhip {
 namespace {
@@ -341,7 +342,7 @@ __global__ __launch_bounds__(256) void k_cat_rows(CatRows a)
 {
     extern __shared__ float row[];                        // [ldk]
     __shared__ float sm[16];
-    const int m = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int m = xcd_block_row(blockIdx.x, gridDim.x), tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     for (int i = a.H * a.vdim + tid; i < a.ldk; i += 256) row[i] = 0.f;
     if (!a.g_out && a.gate) {
 #pragma unroll 4

@@ -17,15 +17,35 @@ __device__ __forceinline__ int up4(int n) { return (n + 3) & ~3; }
 __device__ __forceinline__ float *key_ring(const GroupRows &a, int b, int g) { return a.kring + (size_t)(b * a.G + g) * a.ring_rows * up4(a.dim); }
 __device__ __forceinline__ float *value_ring(const GroupRows &a, int b, int g) { return a.vring + (size_t)(b * a.G + g) * a.ring_rows * up4(a.vdim); }
 
-// grid (rows, G)
-__global__ __launch_bounds__(256) void k_group_cache(GroupRows a)
+// a thread per four entries of a row's keys | values of all key heads.  grid (ceil(G * (dp + vp) / 1024), rows); vec: four
+// entries lie on 16 bytes and turn with four others, or pass, together
+__global__ __launch_bounds__(256) void k_group_cache(GroupRows a, int vec)
 {
-    const int m = blockIdx.x, g = blockIdx.y, b = m / a.r.T, p = a.r.pos + m % a.r.T, slot = p % a.ring_rows;
-    const int dp = up4(a.dim), vp = up4(a.vdim);
-    float *k = key_ring(a, b, g) + (size_t)slot * dp, *v = value_ring(a, b, g) + (size_t)slot * vp;
-    for (int i = threadIdx.x; i < dp + vp; i += 256)
-        if (i < dp) k[i] = group_key(a, m, p, g, i);
-        else v[i - dp] = group_value(a, m, g, i - dp);
+    const int m = blockIdx.y, b = m / a.r.T, p = a.r.pos + m % a.r.T, slot = p % a.ring_rows;
+    const int dp = up4(a.dim), vp = up4(a.vdim), x = (blockIdx.x * 256 + threadIdx.x) * 4;
+    if (x >= a.G * (dp + vp)) return;
+    const bool key = x < a.G * dp;
+    const int y = key ? x : x - a.G * dp, g = y / (key ? dp : vp), i = y % (key ? dp : vp);
+    float4 v;
+    if (vec) {
+        const int at = key ? a.o_k + g * a.dim : a.o_v + g * a.vdim, n = a.rot_dims >> 1;
+        const float *c = a.cin + (size_t)m * a.ldc + at, *bias = a.bias + at;
+        auto four = [&](int d) __attribute__((always_inline)) {
+            const float4 s = *reinterpret_cast<const float4 *>(c + d), t = *reinterpret_cast<const float4 *>(bias + d);
+            return make_float4(s.x + t.x, s.y + t.y, s.z + t.z, s.w + t.w);
+        };
+        v = four(i);
+        if (key && i < a.rot_dims) {
+            const int o = i < n ? i + n : i - n;
+            const float4 w = four(o), *cs = reinterpret_cast<const float4 *>(group_angles(a, p) + (i < n ? i : o)), c0 = cs[0], c1 = cs[1];
+            const float s = i < n ? -1.f : 1.f;
+            v = make_float4(v.x * c0.x + s * w.x * c0.y, v.y * c0.z + s * w.y * c0.w, v.z * c1.x + s * w.z * c1.y, v.w * c1.z + s * w.w * c1.w);
+        }
+    } else
+#pragma unroll
+        for (int e = 0; e < 4; e++) (&v.x)[e] = key ? group_key(a, m, p, g, i + e) : group_value(a, m, g, i + e);
+    float *to = key ? key_ring(a, b, g) + (size_t)slot * dp : value_ring(a, b, g) + (size_t)slot * vp;
+    *reinterpret_cast<float4 *>(to + i) = v;
 }
 
 // SLK (up to 64): keys per workgroup.  grid (slices, G * ceil(H / G / HG), rows): softmax statistics and weighted value sum
@@ -170,7 +190,11 @@ __global__ __launch_bounds__(256) void k_group_merge(GroupRows a, int m0, int ns
 
 }  // namespace
 
-void launch_group_cache(const GroupRows &a) { LAUNCH(k_group_cache, dim3(a.r.n(), a.G), dim3(256), 0, a); }
+void launch_group_cache(const GroupRows &a)
+{
+    const int n = a.G * (pad4(a.dim) + pad4(a.vdim)), vec = a.dim % 4 == 0 && a.vdim % 4 == 0 && a.rot_dims % 8 == 0;
+    LAUNCH(k_group_cache, dim3((n + 1023) / 1024, a.r.n()), dim3(256), 0, a, vec);
+}
 
 void launch_group_attend(const GroupRows &in)
 {

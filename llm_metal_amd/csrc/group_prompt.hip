@@ -49,6 +49,16 @@ __global__ __launch_bounds__(256) void k_group_frags(PromptArgs p)
     }
 }
 
+// eight consecutive values with their biases (both on 16 bytes)
+__device__ __forceinline__ void biased8(const float *x, const float *b, float (&y)[8])
+{
+#pragma unroll
+    for (int i = 0; i < 8; i += 4) {
+        const float4 v = *reinterpret_cast<const float4 *>(x + i), w = *reinterpret_cast<const float4 *>(b + i);
+        y[i] = v.x + w.x; y[i + 1] = v.y + w.y; y[i + 2] = v.z + w.z; y[i + 3] = v.w + w.w;
+    }
+}
+
 // grid (blocks of 128 queries, H, B), block 256
 template <int NJ, int NDB>
 __global__ __launch_bounds__(256) void k_group_prompt(PromptArgs p)
@@ -74,28 +84,47 @@ __global__ __launch_bounds__(256) void k_group_prompt(PromptArgs p)
         const float *q = a.cin + m * a.ldc + at, *bias = a.bias + at;
         const float2 *cs = group_angles(a, a.r.pos + qi);
         const float f = a.scale * 1.44269504f;
+        if (a.dim % 8 == 0 && a.rot_dims % 16 == 0) {     // eight dimensions turn with eight others, or pass, together
+            const int n = a.rot_dims >> 1;
 #pragma unroll
-        for (int j = 0; j < NJ; j++)
+            for (int j = 0; j < NJ; j++) {
+                const int d = 16 * j + 8 * hh;
+                if (d >= a.dim) {
 #pragma unroll
-            for (int e = 0; e < 8; e++) {
-                const int d = 16 * j + 8 * hh + e;
-                qf[j][e] = (half_t)(d < a.dim ? rotated_half(q, bias, d, a.rot_dims, cs) * f : 0.f);
+                    for (int e = 0; e < 8; e++) qf[j][e] = (half_t)0.f;
+                    continue;
+                }
+                float x[8], w[8];
+                biased8(q + d, bias + d, x);
+                if (d < a.rot_dims) {
+                    const int o = d < n ? d + n : d - n;
+                    const float4 *c4 = reinterpret_cast<const float4 *>(cs + (d < n ? d : o));
+                    biased8(q + o, bias + o, w);
+#pragma unroll
+                    for (int e = 0; e < 8; e += 2) {
+                        const float4 c = c4[e >> 1];
+                        x[e] = x[e] * c.x + (d < n ? -w[e] : w[e]) * c.y;
+                        x[e + 1] = x[e + 1] * c.z + (d < n ? -w[e + 1] : w[e + 1]) * c.w;
+                    }
+                }
+#pragma unroll
+                for (int e = 0; e < 8; e++) qf[j][e] = (half_t)(x[e] * f);
             }
+        } else
+#pragma unroll
+            for (int j = 0; j < NJ; j++)
+#pragma unroll
+                for (int e = 0; e < 8; e++) {
+                    const int d = 16 * j + 8 * hh + e;
+                    qf[j][e] = (half_t)(d < a.dim ? rotated_half(q, bias, d, a.rot_dims, cs) * f : 0.f);
+                }
     }
     const uint4 *src = reinterpret_cast<const uint4 *>(p.frags) + ((size_t)b * a.G + h / (a.H / a.G)) * p.blocks * NF * 64 + lane;
     float16v O[NDB];
     float l_run;
     prompt_attend<NJ, NDB>(qf, src, sp, buf0, buf1, O, l_run);
     if (qw + l31 >= T) return;
-    const float inv = 1.f / l_run;
-    float *out = a.o + (m * a.H + h) * a.vdim;
-#pragma unroll
-    for (int i = 0; i < NDB; i++)
-#pragma unroll
-        for (int v = 0; v < 16; v++) {
-            const int d = 32 * i + 8 * (v >> 2) + 4 * hh + (v & 3);
-            if (d < a.vdim) out[d] = O[i][v] * inv;
-        }
+    prompt_store<NDB>(O, l_run, a.o + (m * a.H + h) * a.vdim, a.vdim);
 }
 
 int nj_of(const GroupRows &a)

@@ -104,15 +104,7 @@ __global__ __launch_bounds__(256) void k_latent_prompt(PromptArgs p)
     float l_run;
     prompt_attend<NJ, NDB>(qf, src, sp, buf0, buf1, O, l_run);
     if (qw + l31 >= T) return;
-    const float inv = 1.f / l_run;
-    float *out = a.o + (m * a.H + h) * a.vdim;
-#pragma unroll
-    for (int i = 0; i < NDB; i++)
-#pragma unroll
-        for (int v = 0; v < 16; v++) {
-            const int d = 32 * i + 8 * (v >> 2) + 4 * hh + (v & 3);
-            if (d < a.vdim) out[d] = O[i][v] * inv;
-        }
+    prompt_store<NDB>(O, l_run, a.o + (m * a.H + h) * a.vdim, a.vdim);
 }
 
 int nj_of(const LatentRows &a)

@@ -100,15 +100,16 @@ __global__ __launch_bounds__(256) void k_mlstm_token(MlstmRows a, int nb, int dq
 
 // ---------------------------------------------------------------- many tokens
 
-// grid (H, B), block 256: a wave takes a chunk of 64 tokens, a lane one of them.  Per token: u = F - m and w = i - F as sums
+// grid (H, B), block 64 NW: a wave takes a chunk of 64 tokens, a lane one of them.  Per token: u = F - m and w = i - F as sums
 // of two floats, cf = e^(F + m_c - m), wk = e^(F_L - F + i - m_L), em = e^(-m); per chunk gk = e^(F_L + m_c - m_L).
-__global__ __launch_bounds__(256) void k_mlstm_gates(MlstmRows a, int chunks)
+template <int NW>
+__global__ __launch_bounds__(64 * NW) void k_mlstm_gates(MlstmRows a, int chunks)
 {
-    __shared__ float wa[4], wb[4];
+    __shared__ float wa[NW], wb[NW];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.x, b = blockIdx.y, T = a.r.T;
     const size_t base = ((size_t)b * a.H + h) * chunks * CT;
     float carry = a.r.pos > 0 ? *m_slot(a, a.r.pos, b, h) : 0.f;
-    for (int t0 = 0; t0 < T; t0 += 256) {
+    for (int t0 = 0; t0 < T; t0 += 64 * NW) {
         const int t = t0 + tid;
         float2 g = make_float2(NONE, 0.f);                // tokens past the end change nothing
         if (t < T) g = log_gates(a, (size_t)b * T + t, h);
@@ -125,7 +126,7 @@ __global__ __launch_bounds__(256) void k_mlstm_gates(MlstmRows a, int chunks)
         float mc = carry;
         for (int w = 0; w < wave; w++) mc = fmaxf(wa[w] + mc, wb[w]);
         const float m = fmaxf(A + mc, M);
-        for (int w = 0; w < 4; w++) carry = fmaxf(wa[w] + carry, wb[w]);
+        for (int w = 0; w < NW; w++) carry = fmaxf(wa[w] + carry, wb[w]);
         const double FL = __shfl(F, 63, 64);
         const float mL = __shfl(m, 63, 64);
         const int ck = t0 / CT + wave;
@@ -145,14 +146,28 @@ __global__ __launch_bounds__(256) void k_mlstm_gates(MlstmRows a, int chunks)
     if (tid == 0) *m_slot(a, a.r.pos + T, b, h) = carry;
 }
 
-// four consecutive entries from column d on of a row of n, zeros behind it; vec: the rows start on 16 bytes and n % 4 == 0
-__device__ __forceinline__ float4 take4(const float *row, int d, int n, bool vec)
+// Workgroup ids go to the eight XCDs in turn.  Place of this workgroup in a list of n of which each XCD takes a contiguous
+// share, so that what neighbours of the list read lies in one L2.
+__device__ __forceinline__ int xcd_share(int id, int n)
 {
-    if (vec) return d < n ? *reinterpret_cast<const float4 *>(row + d) : make_float4(0.f, 0.f, 0.f, 0.f);
+    const int x = id & 7, rest = n & 7;
+    return x * (n >> 3) + min(x, rest) + (id >> 3);
+}
+
+// Four consecutive entries from column d on of a row of n: asked for at places that exist (nothing waits here), and those
+// behind the row's end zeroed when they are used.  VEC: rows start on 16 bytes and n % 4 == 0.
+template <bool VEC>
+__device__ __forceinline__ float4 ask4(const float *row, int d, int n)
+{
+    if (VEC) return *reinterpret_cast<const float4 *>(row + min(d, n - 4));
     float4 v;
 #pragma unroll
-    for (int e = 0; e < 4; e++) (&v.x)[e] = d + e < n ? row[d + e] : 0.f;
+    for (int e = 0; e < 4; e++) (&v.x)[e] = row[min(d + e, n - 1)];
     return v;
+}
+__device__ __forceinline__ float4 kept4(float4 v, int d, int n, float f)
+{
+    return make_float4(d < n ? v.x * f : 0.f, d + 1 < n ? v.y * f : 0.f, d + 2 < n ? v.z * f : 0.f, d + 3 < n ? v.w * f : 0.f);
 }
 
 // Operands in LDS for v_mfma_f32_16x16x4_f32 (A: lane -> row lane & 15; B: lane -> column lane & 15; both: reduction index
@@ -161,88 +176,104 @@ __device__ __forceinline__ float4 take4(const float *row, int d, int n, bool vec
 //   by steps [index][LDS_]: sixteen rows lie side by side
 constexpr int LDR = CT + 4, LDK = CT + 16;
 
-// grid (tiles of 64 columns, tiles of 64 dimensions, H * B), block 256: a workgroup takes one 64 x 64 tile of a head's
+// The state ahead of a chunk lies in tiles of 16 columns x 16 dimensions, [column tile][dimension tile][lane][4]: lane ->
+// column lane & 15, dimensions 4 (lane >> 4) + 0 .. 3 -- as the accumulators that make it and the operand that takes it hold
+// it.  Columns 0 .. vdim - 1, then the normaliser; what lies beyond is zero.
+__device__ __forceinline__ int v_tiles(const MlstmRows &a) { return a.vdim / 16 + 1; }
+__device__ __forceinline__ int d_tiles(const MlstmRows &a) { return (a.dim + 15) / 16; }
+__device__ __forceinline__ float *state_ahead(const MlstmRows &a, int chunks, int b, int ck, int h)
+{
+    return a.Sc + (((size_t)b * chunks + ck) * a.H + h) * v_tiles(a) * d_tiles(a) * 256;
+}
+
+// grid (nv tiles of 64 columns * nd tiles of 64 dimensions * H * B), block 256: a workgroup takes one 64 x 64 tile of a head's
 // state (columns 0 .. vdim - 1, column vdim the normaliser) through the chunks in order, a wave a quarter of it.
-__global__ __launch_bounds__(256) void k_mlstm_states(MlstmRows a, int chunks)
+template <bool VEC>
+__global__ __launch_bounds__(256) void k_mlstm_states(MlstmRows a, int chunks, int nv, int nd)
 {
     __shared__ float Ks[CT * LDK], Vs[CT * LDK];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, r4 = lane >> 4;
-    const int h = blockIdx.z % a.H, b = blockIdx.z / a.H, T = a.r.T, ds = up4(a.dim), V1 = a.vdim + 1;
-    const int v0 = blockIdx.x * 64, d0 = blockIdx.y * 64, wv = v0 + (wave & 1) * 32, wd = d0 + (wave >> 1) * 32;
-    const bool kvec = a.dim % 4 == 0, vvec = a.vdim % 4 == 0;
-    float4v S[2][2];
+    const int id = xcd_share(blockIdx.x, gridDim.x), hb = id / (nv * nd), h = hb % a.H, b = hb / a.H, T = a.r.T, ds = up4(a.dim);
+    const int v0 = id % nv * 64, d0 = id / nv % nd * 64, wv = v0 + (wave & 1) * 32, wd = d0 + (wave >> 1) * 32;
+    const int VT = v_tiles(a), DT = d_tiles(a);
+    // dimensions d .. d + 3 of column v of the lasting state
+    auto place = [&](int p, int v, int d) __attribute__((always_inline)) {
+        return reinterpret_cast<float4v *>((v < a.vdim ? a.S + (((size_t)b * a.H + h) * a.vdim + v) * ds : n_slot(a, p, b, h)) + d);
+    };
+    float4v S[2][2];                                      // [dimensions][columns]
 #pragma unroll
     for (int i = 0; i < 2; i++)
 #pragma unroll
-        for (int j = 0; j < 2; j++)
-#pragma unroll
-            for (int x = 0; x < 4; x++) {
-                const int v = wv + 16 * i + 4 * r4 + x, d = wd + 16 * j + c;
-                float s = 0.f;
-                if (a.r.pos > 0 && d < ds && v <= a.vdim)
-                    s = v < a.vdim ? a.S[(((size_t)b * a.H + h) * a.vdim + v) * ds + d] : n_slot(a, a.r.pos, b, h)[d];
-                S[i][j][x] = s;
-            }
-    float4 kr[4], vr[4];
+        for (int j = 0; j < 2; j++) {
+            const int v = wv + 16 * j + c, d = wd + 16 * i + 4 * r4;
+            S[i][j] = float4v{0.f, 0.f, 0.f, 0.f};
+            if (a.r.pos > 0 && d < ds && v <= a.vdim) S[i][j] = *place(a.r.pos, v, d);
+        }
     const int tok = tid >> 4, at = (tid & 15) * 4;        // four tokens of a thread, sixteen apart
-    auto fetch = [&](int ck) __attribute__((always_inline)) {
+    struct Set { float4 k[4], v[4]; float w[4], g; };
+    auto fetch = [&](Set &x, int ck_) __attribute__((always_inline)) {
+        const int ck = min(ck_, chunks - 1);
+        const size_t part = ((size_t)b * a.H + h) * chunks + ck;
 #pragma unroll
         for (int i = 0; i < 4; i++) {
-            const int t = ck * CT + tok + 16 * i;
-            const float *row = a.cin + ((size_t)b * T + min(t, T - 1)) * a.ldc;
-            kr[i] = take4(row + a.o_k + h * a.dim, d0 + at, a.dim, kvec);
-            vr[i] = take4(row + a.o_v + h * a.vdim, v0 + at, a.vdim, vvec);
-#pragma unroll
-            for (int e = 0; e < 4; e++) if (v0 + at + e == a.vdim) (&vr[i].x)[e] = 1.f;
-            const float w = a.wk[(((size_t)b * a.H + h) * chunks + ck) * CT + tok + 16 * i];      // 0 past the end
-            kr[i].x *= w; kr[i].y *= w; kr[i].z *= w; kr[i].w *= w;
+            const float *row = a.cin + ((size_t)b * T + min(ck * CT + tok + 16 * i, T - 1)) * a.ldc;
+            x.k[i] = ask4<VEC>(row + a.o_k + h * a.dim, d0 + at, a.dim);
+            x.v[i] = ask4<VEC>(row + a.o_v + h * a.vdim, v0 + at, a.vdim);
+            x.w[i] = a.wk[part * CT + tok + 16 * i];      // 0 past the end
         }
+        x.g = a.gk[part];
     };
-    fetch(0);
-    for (int ck = 0; ck < chunks; ck++) {
+    auto take = [&](const Set &x, int ck) __attribute__((always_inline)) {
         __syncthreads();
 #pragma unroll
         for (int i = 0; i < 4; i++) {
-            *reinterpret_cast<float4 *>(&Ks[(tok + 16 * i) * LDK + at]) = kr[i];
-            *reinterpret_cast<float4 *>(&Vs[(tok + 16 * i) * LDK + at]) = vr[i];
+            float4 v = kept4(x.v[i], v0 + at, a.vdim, 1.f);
+#pragma unroll
+            for (int e = 0; e < 4; e++) if (v0 + at + e == a.vdim) (&v.x)[e] = 1.f;
+            *reinterpret_cast<float4 *>(&Ks[(tok + 16 * i) * LDK + at]) = kept4(x.k[i], d0 + at, a.dim, x.w[i]);
+            *reinterpret_cast<float4 *>(&Vs[(tok + 16 * i) * LDK + at]) = v;
         }
+        const float g = x.g;
         __syncthreads();
-        if (ck + 1 < chunks) fetch(ck + 1);
-        const float g = a.gk[((size_t)b * a.H + h) * chunks + ck];
-        float *out = a.Sc + (((size_t)b * chunks + ck) * a.H + h) * V1 * ds;
+        float *out = state_ahead(a, chunks, b, ck, h) + lane * 4;
 #pragma unroll
         for (int i = 0; i < 2; i++)
 #pragma unroll
-            for (int j = 0; j < 2; j++)
-#pragma unroll
-                for (int x = 0; x < 4; x++) {             // the state ahead of the chunk
-                    const int v = wv + 16 * i + 4 * r4 + x, d = wd + 16 * j + c;
-                    if (v < V1 && d < ds) out[(size_t)v * ds + d] = S[i][j][x];
-                    S[i][j][x] *= g;
-                }
+            for (int j = 0; j < 2; j++) {
+                const int vt = (wv >> 4) + j, dt = (wd >> 4) + i;
+                if (vt < VT && dt < DT) *reinterpret_cast<float4v *>(out + (size_t)(vt * DT + dt) * 256) = S[i][j];
+                S[i][j] *= g;
+            }
         const float *kp = Ks + r4 * LDK + (wave >> 1) * 32 + c, *vp = Vs + r4 * LDK + (wave & 1) * 32 + c;
-#pragma unroll 4
+#pragma unroll
         for (int s = 0; s < CT / 4; s++) {
             float av[2], bv[2];
 #pragma unroll
-            for (int i = 0; i < 2; i++) { av[i] = vp[4 * s * LDK + 16 * i]; bv[i] = kp[4 * s * LDK + 16 * i]; }
+            for (int i = 0; i < 2; i++) { av[i] = kp[4 * s * LDK + 16 * i]; bv[i] = vp[4 * s * LDK + 16 * i]; }
 #pragma unroll
             for (int i = 0; i < 2; i++)
 #pragma unroll
                 for (int j = 0; j < 2; j++) S[i][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(av[i], bv[j], S[i][j], 0, 0, 0);
         }
-    }
+    };
+    constexpr int SETS = 3;                               // a chunk is asked for two chunks ahead
+    Set x[SETS];
+#pragma unroll
+    for (int n = 0; n < SETS - 1; n++) fetch(x[n], n);
+    for (int ck = 0; ck < chunks; ck += SETS)
+#pragma unroll
+        for (int n = 0; n < SETS; n++) {
+            if (ck + n >= chunks) break;                  // uniform
+            fetch(x[(n + SETS - 1) % SETS], ck + n + SETS - 1);
+            take(x[n], ck + n);
+        }
 #pragma unroll
     for (int i = 0; i < 2; i++)
 #pragma unroll
-        for (int j = 0; j < 2; j++)
-#pragma unroll
-            for (int x = 0; x < 4; x++) {
-                const int v = wv + 16 * i + 4 * r4 + x, d = wd + 16 * j + c;
-                if (d >= ds || v > a.vdim) continue;
-                if (v < a.vdim) a.S[(((size_t)b * a.H + h) * a.vdim + v) * ds + d] = S[i][j][x];
-                else n_slot(a, a.r.pos + T, b, h)[d] = S[i][j][x];
-            }
+        for (int j = 0; j < 2; j++) {
+            const int v = wv + 16 * j + c, d = wd + 16 * i + 4 * r4;
+            if (d < ds && v <= a.vdim) *place(a.r.pos + T, v, d) = S[i][j];
+        }
 }
 
 // acc[2][2] += rows A[32 of them] x rows B[32 of them] of two LDS tiles held by rows, over 16 `blocks` of reduction indices
@@ -268,35 +299,41 @@ __device__ __forceinline__ void tile_product(const float *A, const float *B, int
 
 // grid (chunks, H, B), block 256: weights of the chunk's pairs over their denominators, P [token][token], and qf, the factor
 // of the state's part of a token's output
+template <bool VEC>
 __global__ __launch_bounds__(256) void k_mlstm_pairs(MlstmRows a, int chunks)
 {
     __shared__ float Qs[CT * LDR], Ks[CT * LDR], ns[CT], sums[2][CT], qn[CT], rd[CT];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, r4 = lane >> 4;
-    const int ck = blockIdx.x, h = blockIdx.y, b = blockIdx.z, T = a.r.T, ds = up4(a.dim), nt = min(CT, T - ck * CT);
+    const int ck = blockIdx.x, h = blockIdx.y, b = blockIdx.z, T = a.r.T, nt = min(CT, T - ck * CT);
     const size_t g0 = (((size_t)b * a.H + h) * chunks + ck) * CT;
-    const float *nc = a.Sc + ((((size_t)b * chunks + ck) * a.H + h) * (a.vdim + 1) + a.vdim) * ds;
-    const bool vec = a.dim % 4 == 0;
+    const float *nc = state_ahead(a, chunks, b, ck, h) + (size_t)(a.vdim >> 4) * d_tiles(a) * 256 + (a.vdim & 15) * 4;
     const int wi = wave >> 1, wj = wave & 1, tok = tid >> 4, at = (tid & 15) * 4;
     const float scale = 1.f / sqrtf((float)a.dim);
     float4v acc[2][2] = {};
     float dot = 0.f;
-    for (int d0 = 0; d0 < a.dim; d0 += 64) {
-        float4 q[4], k[4];
+    float4 q[4], k[4];
+    float nv = 0.f;
+    auto fetch = [&](int d0) __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < 4; i++) {
             const float *row = a.cin + ((size_t)b * T + min(ck * CT + tok + 16 * i, T - 1)) * a.ldc;
-            q[i] = take4(row + a.o_q + h * a.dim, d0 + at, a.dim, vec);
-            k[i] = take4(row + a.o_k + h * a.dim, d0 + at, a.dim, vec);
+            q[i] = ask4<VEC>(row + a.o_q + h * a.dim, d0 + at, a.dim);
+            k[i] = ask4<VEC>(row + a.o_k + h * a.dim, d0 + at, a.dim);
         }
-        const float nv = tid < 64 && d0 + tid < ds ? nc[d0 + tid] : 0.f;
+        const int d = min(d0 + (tid & 63), a.dim - 1);
+        nv = nc[(d >> 4) * 256 + ((d & 15) >> 2) * 64 + (d & 3)];
+    };
+    fetch(0);
+    for (int d0 = 0; d0 < a.dim; d0 += 64) {
         __syncthreads();
 #pragma unroll
         for (int i = 0; i < 4; i++) {
-            *reinterpret_cast<float4 *>(&Qs[(tok + 16 * i) * LDR + at]) = q[i];
-            *reinterpret_cast<float4 *>(&Ks[(tok + 16 * i) * LDR + at]) = k[i];
+            *reinterpret_cast<float4 *>(&Qs[(tok + 16 * i) * LDR + at]) = kept4(q[i], d0 + at, a.dim, 1.f);
+            *reinterpret_cast<float4 *>(&Ks[(tok + 16 * i) * LDR + at]) = kept4(k[i], d0 + at, a.dim, 1.f);
         }
-        if (tid < 64) ns[tid] = nv;
+        if (tid < 64) ns[tid] = d0 + tid < a.dim ? nv : 0.f;
         __syncthreads();
+        if (d0 + 64 < a.dim) fetch(d0 + 64);
         if (wj <= wi) tile_product<4>(Qs + 32 * wi * LDR, Ks + 32 * wj * LDR, c, r4, acc);
         // four threads per token, every fourth dimension each
 #pragma unroll
@@ -342,50 +379,70 @@ __global__ __launch_bounds__(256) void k_mlstm_pairs(MlstmRows a, int chunks)
         }
 }
 
-// grid (tiles of 64 columns, chunks, H * B), block 256: outputs of a chunk's tokens in 64 columns, a wave 32 x 32 of them
-__global__ __launch_bounds__(256) void k_mlstm_outputs(MlstmRows a, int chunks)
+// grid (nv tiles of 64 columns * chunks * H * B), block 256: outputs of a chunk's tokens in 64 columns, a wave 32 x 32 of them
+template <bool VEC>
+__global__ __launch_bounds__(256) void k_mlstm_outputs(MlstmRows a, int chunks, int nv)
 {
     __shared__ float As[CT * LDR], Bs[CT * LDR];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, r4 = lane >> 4;
-    const int v0 = blockIdx.x * 64, ck = blockIdx.y, h = blockIdx.z % a.H, b = blockIdx.z / a.H, T = a.r.T, ds = up4(a.dim);
-    const size_t g0 = (((size_t)b * a.H + h) * chunks + ck) * CT, part = ((size_t)b * chunks + ck) * a.H + h;
-    const float *Sc = a.Sc + part * (a.vdim + 1) * ds, *P = a.P + part * CT * CT;
-    const bool qvec = a.dim % 4 == 0, vvec = a.vdim % 4 == 0;
-    const int wi = wave >> 1, wj = wave & 1, tok = tid >> 4, at = (tid & 15) * 4;
-    float4v acc[2][2] = {};
-    float4 x[4], y[4];
-    auto fetch = [&](int d0) __attribute__((always_inline)) {      // d0 < dim: queries and state; behind: pairs and values
+    const int id = xcd_share(blockIdx.x, gridDim.x), hb = id / (nv * chunks), h = hb % a.H, b = hb / a.H, T = a.r.T;
+    const int v0 = id % nv * 64, ck = id / nv % chunks;
+    const size_t g0 = (((size_t)b * a.H + h) * chunks + ck) * CT;
+    const int wi = wave >> 1, wj = wave & 1, tok = tid >> 4, at = (tid & 15) * 4, VT = v_tiles(a), DT = d_tiles(a);
+    const float *P = a.P + (((size_t)b * chunks + ck) * a.H + h) * CT * CT;
+    const float *Sc[2];
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const int t = tok + 16 * i;
-            const float *row = a.cin + ((size_t)b * T + min(ck * CT + t, T - 1)) * a.ldc;
-            if (d0 < a.dim) {
-                x[i] = take4(row + a.o_q + h * a.dim, d0 + at, a.dim, qvec);
-                const float f = a.qf[g0 + t];
-                x[i].x *= f; x[i].y *= f; x[i].z *= f; x[i].w *= f;
-                y[i] = take4(Sc + (size_t)min(v0 + t, a.vdim) * ds, d0 + at, ds, true);
-            } else {
-                x[i] = *reinterpret_cast<const float4 *>(P + t * CT + at);
-                y[i] = take4(row + a.o_v + h * a.vdim, v0 + at, a.vdim, vvec);
-            }
-        }
+    for (int j = 0; j < 2; j++) Sc[j] = state_ahead(a, chunks, b, ck, h) + (size_t)min((v0 >> 4) + 2 * wj + j, VT - 1) * DT * 256 + lane * 4;
+    float4v acc[2][2] = {}, B0[4][2], B1[4][2];
+    float4 x[4], y[4], p[4];
+    float f[4];
+#pragma unroll
+    for (int i = 0; i < 4; i++) f[i] = a.qf[g0 + tok + 16 * i];
+    auto row = [&](int i) __attribute__((always_inline)) { return a.cin + ((size_t)b * T + min(ck * CT + tok + 16 * i, T - 1)) * a.ldc; };
+    auto ask = [&](int d0, float4v (&B)[4][2]) __attribute__((always_inline)) {        // queries, and the state as an operand
+#pragma unroll
+        for (int i = 0; i < 4; i++) x[i] = ask4<VEC>(row(i) + a.o_q + h * a.dim, d0 + at, a.dim);
+#pragma unroll
+        for (int kb = 0; kb < 4; kb++)
+#pragma unroll
+            for (int j = 0; j < 2; j++) B[kb][j] = *reinterpret_cast<const float4v *>(Sc[j] + (size_t)min((d0 >> 4) + kb, DT - 1) * 256);
     };
-    auto stage = [&]() __attribute__((always_inline)) {
+    auto use = [&](int d0, const float4v (&B)[4][2], float4v (&next)[4][2]) __attribute__((always_inline)) {
         __syncthreads();
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            *reinterpret_cast<float4 *>(&As[(tok + 16 * i) * LDR + at]) = x[i];
-            *reinterpret_cast<float4 *>(&Bs[(tok + 16 * i) * LDR + at]) = y[i];
-        }
+        for (int i = 0; i < 4; i++) *reinterpret_cast<float4 *>(&As[(tok + 16 * i) * LDR + at]) = kept4(x[i], d0 + at, a.dim, f[i]);
         __syncthreads();
+        if (d0 + 64 < a.dim) ask(d0 + 64, next);
+#pragma unroll
+        for (int kb = 0; kb < 4; kb++) {                  // (dimensions beyond the head's: the queries are zero)
+            float4v av[2];
+#pragma unroll
+            for (int i = 0; i < 2; i++) av[i] = *reinterpret_cast<const float4v *>(As + (32 * wi + 16 * i + c) * LDR + 16 * kb + 4 * r4);
+#pragma unroll
+            for (int e = 0; e < 4; e++)
+#pragma unroll
+                for (int i = 0; i < 2; i++)
+#pragma unroll
+                    for (int j = 0; j < 2; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(av[i][e], B[kb][j][e], acc[i][j], 0, 0, 0);
+        }
     };
-    fetch(0);
-    for (int d0 = 0; d0 < a.dim; d0 += 64) {
-        stage();
-        fetch(d0 + 64);
-        tile_product<4>(As + 32 * wi * LDR, Bs + 32 * wj * LDR, c, r4, acc);
+    ask(0, B0);
+#pragma unroll
+    for (int i = 0; i < 4; i++) {                         // pairs and values, for the end
+        p[i] = *reinterpret_cast<const float4 *>(P + (tok + 16 * i) * CT + at);
+        y[i] = ask4<VEC>(row(i) + a.o_v + h * a.vdim, v0 + at, a.vdim);
     }
-    stage();                                              // pairs by rows, values by steps
+    for (int d0 = 0; d0 < a.dim; d0 += 128) {
+        use(d0, B0, B1);
+        if (d0 + 64 < a.dim) use(d0 + 64, B1, B0);
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < 4; i++) {                         // pairs by rows, values by steps
+        *reinterpret_cast<float4 *>(&As[(tok + 16 * i) * LDR + at]) = p[i];
+        *reinterpret_cast<float4 *>(&Bs[(tok + 16 * i) * LDR + at]) = kept4(y[i], v0 + at, a.vdim, 1.f);
+    }
+    __syncthreads();
     const float *A = As + 32 * wi * LDR, *B = Bs + 32 * wj;
     for (int kb = 0; kb < 2 + 2 * wi; kb++) {             // later tokens weigh nothing
         float4v av[2];
@@ -434,10 +491,14 @@ void launch_mlstm(const MlstmRows &a)
         return;
     }
     const int chunks = mlstm_chunks(a.r.T);
-    LAUNCH(k_mlstm_gates, dim3(a.H, a.r.B), dim3(256), 0, a, chunks);
-    LAUNCH(k_mlstm_states, dim3((a.vdim + 64) / 64, (a.dim + 63) / 64, a.H * a.r.B), dim3(256), 0, a, chunks);
-    LAUNCH(k_mlstm_pairs, dim3(chunks, a.H, a.r.B), dim3(256), 0, a, chunks);
-    LAUNCH(k_mlstm_outputs, dim3((a.vdim + 63) / 64, chunks, a.H * a.r.B), dim3(256), 0, a, chunks);
+    if (chunks <= 4) LAUNCH(k_mlstm_gates<4>, dim3(a.H, a.r.B), dim3(256), 0, a, chunks);
+    else LAUNCH(k_mlstm_gates<16>, dim3(a.H, a.r.B), dim3(1024), 0, a, chunks);
+    const int nv = (a.vdim + 63) / 64, nv1 = (a.vdim + 64) / 64, nd = (a.dim + 63) / 64;      // (the normaliser is one more column)
+    const dim3 states(nv1 * nd * a.H * a.r.B), pairs(chunks, a.H, a.r.B), outputs(nv * chunks * a.H * a.r.B);
+#define CHUNKS(VEC_) do { LAUNCH((k_mlstm_states<VEC_>), states, dim3(256), 0, a, chunks, nv1, nd); LAUNCH((k_mlstm_pairs<VEC_>), pairs, dim3(256), 0, a, chunks); \
+                          LAUNCH((k_mlstm_outputs<VEC_>), outputs, dim3(256), 0, a, chunks, nv); } while (0)
+    if (a.dim % 4 == 0 && a.vdim % 4 == 0) CHUNKS(true); else CHUNKS(false);
+#undef CHUNKS
 }
 
 }  // namespace lmhip

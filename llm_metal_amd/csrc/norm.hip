@@ -2,6 +2,7 @@
 // a product, the dense feed-forward's activation, rotation tables.
 #include "stack.h"
 #include "rows.h"
+#include "planes.h"
 
 namespace lmhip {
 namespace {
@@ -79,7 +80,7 @@ __global__ __launch_bounds__(256) void k_norms_around(AroundRows a)
 {
     extern __shared__ float row[];                        // [Dp]
     __shared__ float sm[32];
-    const int m = blockIdx.x, src = a.want ? a.want[m] : m * a.step + a.first, tid = threadIdx.x;
+    const int m = xcd_block_row(blockIdx.x, gridDim.x), src = a.want ? a.want[m] : m * a.step + a.first, tid = threadIdx.x;
     const size_t off = (size_t)src * a.Dp;
     float post = 0.f;
     if (a.cout) {
@@ -120,48 +121,53 @@ __global__ __launch_bounds__(256) void k_norms_around(AroundRows a)
     }
 }
 
-// One workgroup per row.  The operand's rows wait in LDS (staged) or, when they are too long, are formed twice.
-__global__ __launch_bounds__(256) void k_gelu_rows(ActRows a, int staged)
+// One workgroup of NT threads per row.  A thread holds P pieces of eight columns in registers; what a row has beyond them is
+// formed twice.
+template <int NT, int P>
+__global__ __launch_bounds__(NT) void k_gelu_rows(ActRows a)
 {
-    extern __shared__ float row[];                        // [K] when staged
     __shared__ float sm[16];
-    const int m = blockIdx.x, tid = threadIdx.x;
+    const int m = xcd_block_row(blockIdx.x, gridDim.x), tid = threadIdx.x;
     const float *up = a.up + (size_t)m * a.ld;
-    if (a.h) {
-        for (int i = tid; i < a.K; i += 256) a.h[(size_t)m * a.K + i] = i < a.n ? gelu_tanh_exact(up[i]) : 0.f;
-        return;
-    }
-    auto eight = [&](int k, float (&v)[8]) __attribute__((always_inline)) {
-        const float4 p = *reinterpret_cast<const float4 *>(up + k), q = *reinterpret_cast<const float4 *>(up + k + 4);
-        v[0] = p.x; v[1] = p.y; v[2] = p.z; v[3] = p.w; v[4] = q.x; v[5] = q.y; v[6] = q.z; v[7] = q.w;
+    auto ask = [&](int k, float4 (&p)[2]) __attribute__((always_inline)) {
 #pragma unroll
-        for (int e = 0; e < 8; e++) v[e] = k + e < a.n ? gelu_tanh(v[e]) : 0.f;
+        for (int e = 0; e < 2; e++) p[e] = k < a.K ? *reinterpret_cast<const float4 *>(up + k + 4 * e) : make_float4(0.f, 0.f, 0.f, 0.f);
     };
-    float mx = 0.f;
-#pragma unroll 2
-    for (int k = tid * 8; k < a.K; k += 2048) {
-        float v[8];
-        eight(k, v);
+    auto act = [&](int k, float4 (&p)[2]) __attribute__((always_inline)) {
+        float mx = 0.f;
 #pragma unroll
-        for (int e = 0; e < 8; e++) mx = fmaxf(mx, fabsf(v[e]));
-        if (staged) {
-            *reinterpret_cast<float4 *>(row + k) = make_float4(v[0], v[1], v[2], v[3]);
-            *reinterpret_cast<float4 *>(row + k + 4) = make_float4(v[4], v[5], v[6], v[7]);
+        for (int e = 0; e < 8; e++) {
+            float &v = (&p[e >> 2].x)[e & 3];
+            v = k + e < a.n ? gelu_tanh(v) : 0.f;
+            mx = fmaxf(mx, fabsf(v));
         }
-    }
-    const float s = row_scale_for(block_max(mx, sm));     // its barriers publish the row
+        return mx;
+    };
     const int Kb = tiled_kb(a.K);
-    if (staged) store_row_f16(row, a.K, a.a16, m, Kb, s);
-    else
-        for (int k = tid * 8; k < Kb * 64; k += 2048) {
-            float v[8] = {};
-            if (k < a.K) eight(k, v);
-            half8 h;
+    auto put = [&](int k, const float4 (&p)[2], float s) __attribute__((always_inline)) {
+        half8 h;
 #pragma unroll
-            for (int e = 0; e < 8; e++) h[e] = f2h(v[e] * s);
-            *reinterpret_cast<half8 *>(&a.a16[tiled_a_index(m, k, Kb)]) = h;
-        }
+        for (int e = 0; e < 8; e++) h[e] = f2h((&p[e >> 2].x)[e & 3] * s);
+        if (k < Kb * 64) *reinterpret_cast<half8 *>(&a.a16[tiled_a_index(m, k, Kb)]) = h;
+    };
+    float4 v[P][2], x[2];
+    float mx = 0.f;
+#pragma unroll
+    for (int i = 0; i < P; i++) ask((i * NT + tid) * 8, v[i]);
+#pragma unroll
+    for (int i = 0; i < P; i++) mx = fmaxf(mx, act((i * NT + tid) * 8, v[i]));
+    for (int k = (P * NT + tid) * 8; k < a.K; k += NT * 8) { ask(k, x); mx = fmaxf(mx, act(k, x)); }
+    const float s = row_scale_for(block_max(mx, sm));
+#pragma unroll
+    for (int i = 0; i < P; i++) put((i * NT + tid) * 8, v[i], s);
+    for (int k = (P * NT + tid) * 8; k < Kb * 64; k += NT * 8) { ask(k, x); act(k, x); put(k, x, s); }
     if (tid == 0) a.inv[m] = 1.f / s;
+}
+
+__global__ __launch_bounds__(256) void k_gelu_rows_f32(ActRows a)
+{
+    const size_t m = blockIdx.x;
+    for (int i = threadIdx.x; i < a.K; i += 256) a.h[m * a.K + i] = i < a.n ? gelu_tanh_exact(a.up[m * a.ld + i]) : 0.f;
 }
 
 __global__ __launch_bounds__(256) void k_rope_table(float2 *tab, int n, int pairs, const double *__restrict__ freq)
@@ -178,9 +184,9 @@ void launch_norms_around(const AroundRows &a, int rows) { LAUNCH(k_norms_around,
 
 void launch_gelu_rows(const ActRows &a, int rows)
 {
-    const size_t lds = (size_t)a.K * 4;
-    const int staged = !a.h && lds <= 60 * 1024;
-    LAUNCH(k_gelu_rows, dim3(rows), dim3(256), staged ? lds : 0, a, staged);
+    if (a.h) LAUNCH(k_gelu_rows_f32, dim3(rows), dim3(256), 0, a);
+    else if (a.K <= 4096) LAUNCH((k_gelu_rows<256, 2>), dim3(rows), dim3(256), 0, a);
+    else LAUNCH((k_gelu_rows<512, 4>), dim3(rows), dim3(512), 0, a);
 }
 
 void launch_rope_table(float2 *tab, int max_seq, const std::vector<double> &freqs)

@@ -95,4 +95,23 @@ __device__ __forceinline__ void prompt_attend(const half8 (&qf)[NJ], const uint4
     l_run += __shfl_xor(l_run, 32, WAVE);
 }
 
+// a lane's query row divided by its weight sum, columns below vdim
+template <int NDB>
+__device__ __forceinline__ void prompt_store(const float16v (&O)[NDB], float l_run, float *out, int vdim)
+{
+    const float inv = 1.f / l_run;
+    const int hh = (threadIdx.x & 63) >> 5;
+    const bool vec = vdim % 4 == 0;                      // rows of a multiple of four columns start on 16 bytes
+#pragma unroll
+    for (int i = 0; i < NDB; i++)
+#pragma unroll
+        for (int v = 0; v < 16; v += 4) {
+            const int d = 32 * i + 8 * (v >> 2) + 4 * hh;
+            if (vec) { if (d < vdim) *reinterpret_cast<float4 *>(out + d) = make_float4(O[i][v] * inv, O[i][v + 1] * inv, O[i][v + 2] * inv, O[i][v + 3] * inv); }
+            else
+#pragma unroll
+                for (int e = 0; e < 4; e++) if (d + e < vdim) out[d + e] = O[i][v + e] * inv;
+        }
+}
+
 }  // namespace lmhip

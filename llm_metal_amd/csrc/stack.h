@@ -290,6 +290,7 @@ struct MlstmRows {
     float *gate;                                         // single-token steps: the output gate as a factor, when wanted
 };
 inline int mlstm_chunks(int T) { return (T + MLSTM_CHUNK - 1) / MLSTM_CHUNK; }
+inline size_t mlstm_state_floats(int dim, int vdim) { return (size_t)(vdim / 16 + 1) * ((dim + 15) / 16) * 256; }   // of one head ahead of a chunk
 inline int pad4(int n) { return (n + 3) & ~3; }
 void launch_mlstm(const MlstmRows &a);
 

@@ -316,7 +316,7 @@ MlstmAux mlstm_aux(Aux &x, const LayerConfig &c, int B, int T)
     if (T == 1) return d;
     d.u = (float2 *)x.take(2 * at); d.w = (float2 *)x.take(2 * at);
     d.cf = x.take(at); d.wk = x.take(at); d.em = x.take(at); d.qf = x.take(at); d.gk = x.take(parts);
-    d.Sc = x.take(parts * (c.vdim + 1) * pad4(c.dim)); d.P = x.take(at * MLSTM_CHUNK);
+    d.Sc = x.take(parts * mlstm_state_floats(c.dim, c.vdim)); d.P = x.take(at * MLSTM_CHUNK);
     return d;
 }
 
