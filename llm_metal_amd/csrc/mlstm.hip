@@ -2,7 +2,7 @@
 // running maximum m_t = max(f_t + m_(t-1), i_t),
 //     S_t = e^(f_t + m_(t-1) - m_t) S_(t-1) + e^(i_t - m_t) k_t v_t^T         n_t likewise with k_t alone
 //     o_t = S_t^T q_t / (max(|n_t . q_t|, e^(-m_t)) + 1e-6)
-// Everything here is fp32, the matrix instructions included.  n is carried as one more column of S (with v = 1).
+// Everything here is fp32, the matrix instructions included.
 //
 // Prompts go in chunks of 64 tokens.  The gates are scalars that do not depend on the state, so all m_t are known ahead of
 // the recurrence (k_mlstm_gates).  With F_t the sum of f from a chunk's first token to t, c the token ahead of the chunk
@@ -178,16 +178,17 @@ constexpr int LDR = CT + 4, LDK = CT + 16;
 
 // The state ahead of a chunk lies in tiles of 16 columns x 16 dimensions, [column tile][dimension tile][lane][4]: lane ->
 // column lane & 15, dimensions 4 (lane >> 4) + 0 .. 3 -- as the accumulators that make it and the operand that takes it hold
-// it.  Columns 0 .. vdim - 1, then the normaliser; what lies beyond is zero.
-__device__ __forceinline__ int v_tiles(const MlstmRows &a) { return a.vdim / 16 + 1; }
+// it; what lies beyond the head is zero.  Behind the tiles the normaliser, in four parts of [dimension tiles][16].
+__device__ __forceinline__ int v_tiles(const MlstmRows &a) { return (a.vdim + 15) / 16; }
 __device__ __forceinline__ int d_tiles(const MlstmRows &a) { return (a.dim + 15) / 16; }
 __device__ __forceinline__ float *state_ahead(const MlstmRows &a, int chunks, int b, int ck, int h)
 {
-    return a.Sc + (((size_t)b * chunks + ck) * a.H + h) * v_tiles(a) * d_tiles(a) * 256;
+    return a.Sc + (((size_t)b * chunks + ck) * a.H + h) * (v_tiles(a) * 256 + 64) * d_tiles(a);
 }
 
 // grid (nv tiles of 64 columns * nd tiles of 64 dimensions * H * B), block 256: a workgroup takes one 64 x 64 tile of a head's
-// state (columns 0 .. vdim - 1, column vdim the normaliser) through the chunks in order, a wave a quarter of it.
+// state through the chunks in order, a wave a quarter of it.  Those of the first columns also take their dimensions of the
+// normaliser along, each wave over a quarter of the tokens: their sum is left to whoever reads it.
 template <bool VEC>
 __global__ __launch_bounds__(256) void k_mlstm_states(MlstmRows a, int chunks, int nv, int nd)
 {
@@ -196,9 +197,11 @@ __global__ __launch_bounds__(256) void k_mlstm_states(MlstmRows a, int chunks, i
     const int id = xcd_share(blockIdx.x, gridDim.x), hb = id / (nv * nd), h = hb % a.H, b = hb / a.H, T = a.r.T, ds = up4(a.dim);
     const int v0 = id % nv * 64, d0 = id / nv % nd * 64, wv = v0 + (wave & 1) * 32, wd = d0 + (wave >> 1) * 32;
     const int VT = v_tiles(a), DT = d_tiles(a);
+    const bool norm = v0 == 0;
+    float n = norm && wave == 0 && a.r.pos > 0 && d0 + lane < a.dim ? n_slot(a, a.r.pos, b, h)[d0 + lane] : 0.f;
     // dimensions d .. d + 3 of column v of the lasting state
-    auto place = [&](int p, int v, int d) __attribute__((always_inline)) {
-        return reinterpret_cast<float4v *>((v < a.vdim ? a.S + (((size_t)b * a.H + h) * a.vdim + v) * ds : n_slot(a, p, b, h)) + d);
+    auto place = [&](int v, int d) __attribute__((always_inline)) {
+        return reinterpret_cast<float4v *>(a.S + (((size_t)b * a.H + h) * a.vdim + v) * ds + d);
     };
     float4v S[2][2];                                      // [dimensions][columns]
 #pragma unroll
@@ -207,7 +210,7 @@ __global__ __launch_bounds__(256) void k_mlstm_states(MlstmRows a, int chunks, i
         for (int j = 0; j < 2; j++) {
             const int v = wv + 16 * j + c, d = wd + 16 * i + 4 * r4;
             S[i][j] = float4v{0.f, 0.f, 0.f, 0.f};
-            if (a.r.pos > 0 && d < ds && v <= a.vdim) S[i][j] = *place(a.r.pos, v, d);
+            if (a.r.pos > 0 && d < ds && v < a.vdim) S[i][j] = *place(v, d);
         }
     const int tok = tid >> 4, at = (tid & 15) * 4;        // four tokens of a thread, sixteen apart
     struct Set { float4 k[4], v[4]; float w[4], g; };
@@ -227,11 +230,8 @@ __global__ __launch_bounds__(256) void k_mlstm_states(MlstmRows a, int chunks, i
         __syncthreads();
 #pragma unroll
         for (int i = 0; i < 4; i++) {
-            float4 v = kept4(x.v[i], v0 + at, a.vdim, 1.f);
-#pragma unroll
-            for (int e = 0; e < 4; e++) if (v0 + at + e == a.vdim) (&v.x)[e] = 1.f;
             *reinterpret_cast<float4 *>(&Ks[(tok + 16 * i) * LDK + at]) = kept4(x.k[i], d0 + at, a.dim, x.w[i]);
-            *reinterpret_cast<float4 *>(&Vs[(tok + 16 * i) * LDK + at]) = v;
+            *reinterpret_cast<float4 *>(&Vs[(tok + 16 * i) * LDK + at]) = kept4(x.v[i], v0 + at, a.vdim, 1.f);
         }
         const float g = x.g;
         __syncthreads();
@@ -244,6 +244,12 @@ __global__ __launch_bounds__(256) void k_mlstm_states(MlstmRows a, int chunks, i
                 if (vt < VT && dt < DT) *reinterpret_cast<float4v *>(out + (size_t)(vt * DT + dt) * 256) = S[i][j];
                 S[i][j] *= g;
             }
+        if (norm) {
+            if (d0 + lane < 16 * DT) (out - lane * 4)[(size_t)VT * DT * 256 + wave * DT * 16 + d0 + lane] = n;
+            n *= g;
+#pragma unroll
+            for (int t = 0; t < CT / 4; t++) n += Ks[(wave * (CT / 4) + t) * LDK + lane];
+        }
         const float *kp = Ks + r4 * LDK + (wave >> 1) * 32 + c, *vp = Vs + r4 * LDK + (wave & 1) * 32 + c;
 #pragma unroll
         for (int s = 0; s < CT / 4; s++) {
@@ -272,8 +278,13 @@ __global__ __launch_bounds__(256) void k_mlstm_states(MlstmRows a, int chunks, i
 #pragma unroll
         for (int j = 0; j < 2; j++) {
             const int v = wv + 16 * j + c, d = wd + 16 * i + 4 * r4;
-            if (d < ds && v <= a.vdim) *place(a.r.pos + T, v, d) = S[i][j];
+            if (d < ds && v < a.vdim) *place(v, d) = S[i][j];
         }
+    if (!norm) return;
+    __syncthreads();
+    Ks[tid] = n;
+    __syncthreads();
+    if (tid < 64 && d0 + tid < ds) n_slot(a, a.r.pos + T, b, h)[d0 + tid] = (Ks[tid] + Ks[64 + tid]) + (Ks[128 + tid] + Ks[192 + tid]);
 }
 
 // acc[2][2] += rows A[32 of them] x rows B[32 of them] of two LDS tiles held by rows, over 16 `blocks` of reduction indices
@@ -306,7 +317,8 @@ __global__ __launch_bounds__(256) void k_mlstm_pairs(MlstmRows a, int chunks)
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = lane & 15, r4 = lane >> 4;
     const int ck = blockIdx.x, h = blockIdx.y, b = blockIdx.z, T = a.r.T, nt = min(CT, T - ck * CT);
     const size_t g0 = (((size_t)b * a.H + h) * chunks + ck) * CT;
-    const float *nc = state_ahead(a, chunks, b, ck, h) + (size_t)(a.vdim >> 4) * d_tiles(a) * 256 + (a.vdim & 15) * 4;
+    const int DT16 = d_tiles(a) * 16;
+    const float *nc = state_ahead(a, chunks, b, ck, h) + (size_t)v_tiles(a) * DT16 * 16;
     const int wi = wave >> 1, wj = wave & 1, tok = tid >> 4, at = (tid & 15) * 4;
     const float scale = 1.f / sqrtf((float)a.dim);
     float4v acc[2][2] = {};
@@ -321,7 +333,7 @@ __global__ __launch_bounds__(256) void k_mlstm_pairs(MlstmRows a, int chunks)
             k[i] = ask4<VEC>(row + a.o_k + h * a.dim, d0 + at, a.dim);
         }
         const int d = min(d0 + (tid & 63), a.dim - 1);
-        nv = nc[(d >> 4) * 256 + ((d & 15) >> 2) * 64 + (d & 3)];
+        nv = (nc[d] + nc[DT16 + d]) + (nc[2 * DT16 + d] + nc[3 * DT16 + d]);
     };
     fetch(0);
     for (int d0 = 0; d0 < a.dim; d0 += 64) {
@@ -493,9 +505,9 @@ void launch_mlstm(const MlstmRows &a)
     const int chunks = mlstm_chunks(a.r.T);
     if (chunks <= 4) LAUNCH(k_mlstm_gates<4>, dim3(a.H, a.r.B), dim3(256), 0, a, chunks);
     else LAUNCH(k_mlstm_gates<16>, dim3(a.H, a.r.B), dim3(1024), 0, a, chunks);
-    const int nv = (a.vdim + 63) / 64, nv1 = (a.vdim + 64) / 64, nd = (a.dim + 63) / 64;      // (the normaliser is one more column)
-    const dim3 states(nv1 * nd * a.H * a.r.B), pairs(chunks, a.H, a.r.B), outputs(nv * chunks * a.H * a.r.B);
-#define CHUNKS(VEC_) do { LAUNCH((k_mlstm_states<VEC_>), states, dim3(256), 0, a, chunks, nv1, nd); LAUNCH((k_mlstm_pairs<VEC_>), pairs, dim3(256), 0, a, chunks); \
+    const int nv = (a.vdim + 63) / 64, nd = (a.dim + 63) / 64;
+    const dim3 states(nv * nd * a.H * a.r.B), pairs(chunks, a.H, a.r.B), outputs(nv * chunks * a.H * a.r.B);
+#define CHUNKS(VEC_) do { LAUNCH((k_mlstm_states<VEC_>), states, dim3(256), 0, a, chunks, nv, nd); LAUNCH((k_mlstm_pairs<VEC_>), pairs, dim3(256), 0, a, chunks); \
                           LAUNCH((k_mlstm_outputs<VEC_>), outputs, dim3(256), 0, a, chunks, nv); } while (0)
     if (a.dim % 4 == 0 && a.vdim % 4 == 0) CHUNKS(true); else CHUNKS(false);
 #undef CHUNKS

@@ -283,14 +283,14 @@ struct MlstmRows {
     int H, dim, vdim; float cap;
     const float *cin, *bias; int ldc, o_q, o_k, o_v, o_g, o_i, o_f;
     float *S, *n, *m;                                    // state
-    // prompts: per (sequence, head) and token the parts of the gates, per chunk its decay, the state ahead of it (with the
-    // normaliser as a further row) and the pair products
+    // prompts: per (sequence, head) and token the parts of the gates, per chunk its decay, the state and the
+    // normaliser ahead of it and the pair products
     float2 *u, *w; float *cf, *wk, *em, *qf, *gk, *Sc, *P;
     float *o;                                            // [rows][H * vdim]
     float *gate;                                         // single-token steps: the output gate as a factor, when wanted
 };
 inline int mlstm_chunks(int T) { return (T + MLSTM_CHUNK - 1) / MLSTM_CHUNK; }
-inline size_t mlstm_state_floats(int dim, int vdim) { return (size_t)(vdim / 16 + 1) * ((dim + 15) / 16) * 256; }   // of one head ahead of a chunk
+inline size_t mlstm_state_floats(int dim, int vdim) { return (size_t)((vdim + 15) / 16 * 256 + 64) * ((dim + 15) / 16); }   // of one head ahead of a chunk
 inline int pad4(int n) { return (n + 3) & ~3; }
 void launch_mlstm(const MlstmRows &a);
 
