@@ -32,11 +32,13 @@ InferenceState *inference_state_create_from_ref(const SFTModelRef *model, int ma
  * fp32 copy of the model in host memory: tensor bytes are uploaded as stored and converted on the GPU, and F16 / Q8_0
  * tensors that already have the wanted format are used bit for bit (no dequantise -> requantise). */
 InferenceState *inference_state_create_from_file(const char *path, ModelType model_type, int max_seq_len, int use_fp16);
-/* MODEL_NEVURAX: a decoder whose config.json (beside the weights) lists its layers one by one -- mixer 'delta' or
- * 'channel_delta' (gated delta rule, one decay per head or per key channel) or 'latent_attention' (sliding window), each
- * with an optional mixture of experts.  It is created from safetensors files only; use_fp16 is 1 (F16 weights, F16
- * operands of the products of several rows, everything else fp32) or 2 (weights, products and sums in 32-bit).  It has
- * no end tokens unless config.json gives eos_token_id (inference_state_load_eos) or the caller sets some, takes no
+/* MODEL_NEVURAX and MODEL_PAPOSUN: decoders whose config.json (beside the weights) lists their layers one by one.  Nevurax:
+ * mixer 'delta' or 'channel_delta' (gated delta rule, one decay per head or per key channel) or 'latent_attention' (sliding
+ * window), each with an optional mixture of experts.  Paposun: mixer 'attention' (grouped heads inside chunks of positions,
+ * with keys of its own or of an earlier layer) or 'mlstm' (matrix memory), each with an optional dense feed-forward, norms
+ * ahead of and behind every sublayer, a tied head.  Such a model is created from safetensors files only; use_fp16 is 1
+ * (F16 weights, F16 operands of the products of several rows, everything else fp32) or 2 (weights, products and sums in
+ * 32-bit).  It has no end tokens unless config.json gives eos_token_id (inference_state_load_eos) or the caller sets some, takes no
  * adapters, and has no training path. */
 
 /* src/nn/fast_inference.h:49 (impl src/nn/fast_inference.c:527-610, owns_weights = 0 at :596-603): the state owns no
@@ -78,8 +80,8 @@ int inference_generate_batch(InferenceState *state, const uint32_t *prompt_token
 int inference_step_batch(InferenceState *state, const int *tokens, int batch_size, int pos, float *logits);
 
 /* The next n tokens at the current position, which advances by n, and the logits [n_want][vocab] (host) at the places
- * want[0 .. n_want) among them, ascending; n_want may be 0.  A prompt may be cut into calls anywhere.  MODEL_NEVURAX runs
- * them as one step (long prompts: a few), the other models token by token.  No counterpart in the reference.  Returns 0,
+ * want[0 .. n_want) among them, ascending; n_want may be 0.  A prompt may be cut into calls anywhere.  MODEL_NEVURAX and
+ * MODEL_PAPOSUN run them as one step (long prompts: a few), the other models token by token.  No counterpart in the reference.  Returns 0,
  * -1 when the arguments do not fit. */
 int  inference_forward_tokens(InferenceState *state, const int *tokens, int n, const int *want, int n_want, float *logits);
 

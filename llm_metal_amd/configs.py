@@ -105,9 +105,9 @@ def paposun_config(width, heads, ff, memory_heads, memory_dim, vocab=32768, head
     def attention(**kw):
         return {"type": "attention", "mlp": {"kind": "dense", "ff": ff},
                 "mixer": {"heads": heads, "kv_heads": max(1, heads // 4), "dim": head_dim, "vdim": head_dim, "mask": {"size": chunk}, "scale": head_dim ** -0.5,
-                          "rot": {"base": 5e5, "dims": head_dim, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}, **kw}}
+                          "rot": {"base": 1e6, "dims": head_dim, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}, **kw}}
     memory = {"type": "mlstm", "mlp": None, "mixer": {"heads": memory_heads, "dim": memory_dim, "vdim": 2 * memory_dim, "gate_cap": 15.0}}
-    return {"architecture": "Paposun", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "residual_mult": 0.5, "logit_scale": 0.25,
+    return {"architecture": "Paposun", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "residual_mult": 0.5, "logit_scale": 0.5,
             "layers": [attention(), attention(kv_from=0), memory, attention()]}
 
 

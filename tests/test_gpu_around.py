@@ -231,8 +231,8 @@ def test_generated_batches_equal_the_single_sequence(fmt, tmp_path):
 def test_wide_layers_on_the_large_products(tmp_path):
     """Sizes at which a long prompt takes the kernels for many rows: the 16-bit prompt, the 16-bit fused decoding and the
     32-bit state agree, whole and in portions."""
-    cfg = around([(grouped(16, 4, 128, 128, 300, scale=0.07, dims=64, base=5e5), dense(4096)), (mlstm(4, 256, 192, 12.0), dense(3000)),
-                  (grouped(16, 4, 128, 128, 512, scale=0.09, dims=64, base=5e5, kv_from=0), None), (mlstm(8, 128, 128, 12.0), None)], width=1024, vocab=512)
+    cfg = around([(grouped(16, 4, 128, 128, 300, scale=0.07, dims=64, base=2e5), dense(4096)), (mlstm(4, 256, 192, 12.0), dense(3000)),
+                  (grouped(16, 4, 128, 128, 512, scale=0.09, dims=64, base=2e5, kv_from=0), None), (mlstm(8, 128, 128, 12.0), None)], width=1024, vocab=512)
     m = Model.__new__(Model)
     m.cfg, m.path = cfg, str(tmp_path)
     write_stack_checkpoint(m.path, cfg, seed=3)
